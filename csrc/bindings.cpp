@@ -1,3 +1,4 @@
+#include <map>
 #include <mutex>
 // PyTorch bindings for the gfx950 kernel library.
 //
@@ -5,37 +6,12 @@
 // shape must never reach a kernel: an out-of-bounds access can reset the whole node), then
 // launches on the current HIP stream of the tensor's device -- so each op is capturable in a
 // torch.cuda.CUDAGraph (= hipGraph on ROCm).
-#include <torch/extension.h>
-#include <ATen/hip/impl/HIPStreamMasqueradingAsCUDA.h>
-#include <c10/core/DeviceGuard.h>
+#include "bindings_common.h"
 
-#include "kernels/vwa_kernels.h"
+// bindings_stack.cpp: the ops of layer stacks with an f32 residual stream
+void bind_stack(pybind11::module_& m);
 
 namespace {
-
-using at::Tensor;
-
-// torch-ROCm exposes GPUs as device type "cuda"; the masquerading accessor returns the stream
-// torch itself launches on (including the capture stream inside torch.cuda.graph).
-hipStream_t cur_stream(const Tensor& t) {
-  return c10::hip::getCurrentHIPStreamMasqueradingAsCUDA(t.device().index()).stream();
-}
-
-const uint16_t* bfp(const Tensor& t) { return reinterpret_cast<const uint16_t*>(t.data_ptr()); }
-uint16_t* bfp_mut(const Tensor& t) { return reinterpret_cast<uint16_t*>(t.data_ptr()); }
-const uint16_t* bfp_opt(const c10::optional<Tensor>& t) { return t.has_value() ? bfp(*t) : nullptr; }
-
-void check_bf16(const Tensor& t, const char* name) {
-  TORCH_CHECK(t.is_cuda(), name, " must be a GPU tensor");
-  TORCH_CHECK(t.scalar_type() == at::kBFloat16, name, " must be bf16");
-}
-void check_contig_rows(const Tensor& t, const char* name) {
-  TORCH_CHECK(t.dim() == 2, name, " must be 2-D");
-  TORCH_CHECK(t.stride(1) == 1, name, " must be row-contiguous");
-  TORCH_CHECK(t.stride(0) % 8 == 0, name, " row stride must be a multiple of 8 elements");
-  TORCH_CHECK((reinterpret_cast<uintptr_t>(t.data_ptr()) & 15) == 0, name, " must be 16-byte aligned");
-}
-void check_rc(int rc, const char* what) { TORCH_CHECK(rc == 0, what, " launch failed with code ", rc); }
 
 // skinny GEMM dispatch: 1 = persistent streaming kernel when the shape fits (default), 0 = one-tile kernel
 int g_skinny_mode = 1;
@@ -137,32 +113,57 @@ void set_ln_fold(SkinnyParams& p, const c10::optional<Tensor>& ln_c, int epi) {
   p.ln_c = ln_c->data_ptr<float>();
 }
 
-// epi: 0 store, 1 residual add, 3 gelu
+// f32 residual stream: an f32 residual goes with f32 output rows (y_f32 2), else bf16
+template <class P>
+void set_f32_residual(P& p, const Tensor& residual, int y_f32) {
+  if (residual.scalar_type() == at::kFloat) {
+    TORCH_CHECK(residual.is_cuda() && y_f32, "an f32 residual needs f32 output rows");
+    p.y_f32 = 2;
+  } else {
+    check_bf16(residual, "residual");
+  }
+}
+
+// split epilogue: y takes the first y.size(1) columns, y2 (bf16) relu(.)^2 of the others
+void set_split(uint16_t*& ptr, int& ld, int& n_split, const c10::optional<Tensor>& y2, const Tensor& y, const Tensor& w) {
+  TORCH_CHECK(y2.has_value() && y.scalar_type() == at::kBFloat16, "split epilogue: bf16 y and y2");
+  check_bf16(*y2, "y2");
+  check_contig_rows(*y2, "y2");
+  TORCH_CHECK(y.size(1) % 16 == 0 && y2->size(0) == y.size(0) && y.size(1) + y2->size(1) == w.size(0),
+              "split epilogue: y and y2 columns must add up to the weight's rows, y a multiple of 16");
+  ptr = bfp_mut(*y2);
+  ld = (int)y2->stride(0);
+  n_split = (int)y.size(1);
+}
+
+// epi: 0 store, 1 residual add, 3 gelu, 5 split (y | relu^2 -> y2)
 // col_mask (epi 0): int32 token bitmask rows [>= rows_used, words]; column n of y is the mask's bit
 // col_mask_off * 32 + n (vocab shard offset under TP) -- tiles without an admissible bit in any of
 // the first mask_rows rows are not computed (their y columns are left as they were)
 void skinny_gemm(Tensor x, Tensor w, c10::optional<Tensor> bias, Tensor y, int64_t epi, bool fuse_rms, double eps,
                  c10::optional<Tensor> residual, c10::optional<Tensor> w_scale, c10::optional<Tensor> ln_c,
-                 bool w_tiled, c10::optional<Tensor> col_mask, int64_t col_mask_off, int64_t mask_rows) {
+                 bool w_tiled, c10::optional<Tensor> col_mask, int64_t col_mask_off, int64_t mask_rows,
+                 c10::optional<Tensor> y2) {
   c10::DeviceGuard g(x.device());
   SkinnyParams p = base_params(x, w, bias, fuse_rms, eps, w_scale, w_tiled);
-  TORCH_CHECK(epi == 0 || epi == 1 || epi == 3, "bad epilogue");
+  TORCH_CHECK(epi == 0 || epi == 1 || epi == 3 || epi == 5, "bad epilogue");
   set_ln_fold(p, ln_c, (int)epi);
   TORCH_CHECK(y.is_cuda() && y.dim() == 2 && y.stride(1) == 1, "y must be a 2-D row-contiguous GPU tensor");
-  TORCH_CHECK(y.size(0) == x.size(0) && y.size(1) == w.size(0), "y shape mismatch");
+  TORCH_CHECK(y.size(0) == x.size(0) && (epi == 5 || y.size(1) == w.size(0)), "y shape mismatch");
   TORCH_CHECK(y.scalar_type() == at::kBFloat16 || y.scalar_type() == at::kFloat, "y must be bf16 or f32");
   p.Y = y.data_ptr();
   p.ldy = (int)y.stride(0);
   p.y_f32 = y.scalar_type() == at::kFloat;
   if (epi == 1) {
     TORCH_CHECK(residual.has_value(), "residual epilogue needs residual");
-    check_bf16(*residual, "residual");
+    set_f32_residual(p, *residual, p.y_f32);
     TORCH_CHECK(residual->dim() == 2 && residual->size(0) == x.size(0) && residual->size(1) == w.size(0) &&
                     residual->stride(1) == 1,
                 "residual shape mismatch");
     p.R = bfp(*residual);
     p.ldr = (int)residual->stride(0);
   }
+  if (epi == 5) set_split(p.q_out, p.ldq, p.n_q_heads, y2, y, w);
   if (col_mask.has_value()) {
     const Tensor& cm = *col_mask;
     TORCH_CHECK(epi == 0, "col_mask needs the store epilogue");
@@ -234,13 +235,13 @@ void set_ss(GemmParams& p, int64_t epi, const c10::optional<Tensor>& ss_out, con
 // workspace (the launcher splits K only when the output tiles alone cannot fill the CUs).
 void gemm(Tensor x, Tensor w, c10::optional<Tensor> bias, Tensor y, int64_t epi, c10::optional<Tensor> rstd,
           c10::optional<Tensor> residual, bool w_tiled, c10::optional<Tensor> ws, c10::optional<Tensor> ss_out,
-          c10::optional<Tensor> ss_zero, c10::optional<Tensor> ss_in, double ss_eps) {
+          c10::optional<Tensor> ss_zero, c10::optional<Tensor> ss_in, double ss_eps, c10::optional<Tensor> y2) {
   c10::DeviceGuard g(x.device());
   check_bf16(x, "x");
   check_bf16(w, "w");
   check_contig_rows(x, "x");
   TORCH_CHECK(w.is_contiguous() && w.dim() == 2 && w.size(1) == x.size(1), "w must be contiguous [N, K] with x's K");
-  TORCH_CHECK(epi >= 0 && epi <= 3, "gemm: bad epilogue");
+  TORCH_CHECK((epi >= 0 && epi <= 3) || epi == 6, "gemm: bad epilogue");
   GemmParams p{};
   p.X = bfp(x);
   p.ldx = (int)x.stride(0);
@@ -252,7 +253,7 @@ void gemm(Tensor x, Tensor w, c10::optional<Tensor> bias, Tensor y, int64_t epi,
   TORCH_CHECK(p.N % 16 == 0 && p.K % 128 == 0, "gemm: N % 16 == 0 and K % 128 == 0 required");
   if (epi == 2) TORCH_CHECK(p.N % 32 == 0, "gemm SwiGLU: gate/up rows must be a multiple of 32");
   TORCH_CHECK(y.is_cuda() && y.dim() == 2 && y.stride(1) == 1 && y.size(0) == p.M &&
-                  y.size(1) == (epi == 2 ? p.N / 2 : p.N),
+                  (epi == 6 || y.size(1) == (epi == 2 ? p.N / 2 : p.N)),
               "y shape");
   TORCH_CHECK(y.scalar_type() == at::kBFloat16 || (y.scalar_type() == at::kFloat && epi != 2), "y bf16 (or f32)");
   p.Y = y.data_ptr();
@@ -271,11 +272,11 @@ void gemm(Tensor x, Tensor w, c10::optional<Tensor> bias, Tensor y, int64_t epi,
                     (reinterpret_cast<uintptr_t>(residual->data_ptr()) & 15) == 0,
                 "gemm: residual rows must be 16-byte aligned");
     TORCH_CHECK(residual.has_value(), "residual epilogue needs residual");
-    check_bf16(*residual, "residual");
+    set_f32_residual(p, *residual, p.y_f32);
     TORCH_CHECK(residual->dim() == 2 && residual->size(0) == p.M && residual->size(1) == p.N &&
                     residual->stride(1) == 1,
                 "residual shape");
-    TORCH_CHECK(!p.y_f32, "residual epilogue writes bf16");
+    TORCH_CHECK(p.y_f32 != 1, "an f32 output row needs an f32 residual");
     p.R = bfp(*residual);
     p.ldr = (int)residual->stride(0);
   }
@@ -291,6 +292,7 @@ void gemm(Tensor x, Tensor w, c10::optional<Tensor> bias, Tensor y, int64_t epi,
     p.ws_cap = ws->numel();
   }
   p.cus = device_cus(x);
+  if (epi == 6) set_split(p.Y2, p.ldy2, p.n_split, y2, y, w);
   set_ss(p, epi, ss_out, ss_zero, ss_in, ss_eps);
   check_rc(vwa_gemm((int)epi, &p, cur_stream(x)), "gemm");
 }
@@ -600,7 +602,7 @@ void chain_schedule(ChainParams& cp) {
   }
 }
 
-// ---- chained decode layer tail (skinny_stream.hip, vwa_chain_*): descriptor built once on the
+// ---- chained decode layer tail (chain.hip, vwa_chain_*): descriptor built once on the
 // host and copied to a device tensor (graph replays then only launch); M <= 4, bf16, one GPU.
 void set_resid(SkinnyParams& p, const Tensor& h) {
   p.Y = h.data_ptr();
@@ -740,7 +742,7 @@ std::tuple<Tensor, int64_t> chain_make(Tensor h, Tensor att, Tensor act, Tensor 
                                     (s_o.has_value() ? (int64_t)1 << 25 : 0) | (cp.o_nt2 ? (int64_t)1 << 26 : 0)};
 }
 
-// Whisper decoder chains (skinny_stream.hip chain_kernel SEQ 1 / 2): phase i computes
+// Whisper decoder chains (chain.hip chain_kernel SEQ 1 / 2): phase i computes
 // Y[i] (=|+=) X[i] . W[i]^T + bias[i] with the epilogue epi[i] (0 store, 1 residual into Y, 3 GELU,
 // 4 QKV + self-KV write, no RoPE); ln_c[i] set = LayerNorm folded into W[i] (fuse_rms 2).
 std::tuple<Tensor, int64_t> chain_make_seq(int64_t seq, std::vector<Tensor> X, std::vector<Tensor> W,
@@ -819,31 +821,39 @@ void decode_advance(Tensor tokens, Tensor positions, Tensor ctx_lens, Tensor slo
 }
 
 // Device memory the L2 does not cache (hipDeviceMallocUncached): chain barrier words polled with
-// scalar loads.  Returned as an int32 tensor whose deleter DEFERS the hipFree to the next
-// allocation: the tensor may die in a garbage collection that runs inside another model's graph
-// capture, where a hipFree is not permitted (seen: the whole process aborted in the GC of an
-// earlier test's model during the next test's capture).
+// scalar loads.  The memory is never freed once kernels have read it (tensors allocated over freed
+// uncached memory can hold wrong values): a dead tensor's buffer goes to a per-(device, size) list
+// that the next allocation takes from, so repeated model builds do not grow it -- and no hipFree can
+// run in a garbage collection inside another model's graph capture.
 static std::mutex g_uncached_mu;
-static std::vector<void*> g_uncached_pending;
+static std::map<std::pair<int, int64_t>, std::vector<void*>> g_uncached_idle;
 
 Tensor alloc_uncached_i32(int64_t n, Tensor like) {
   c10::DeviceGuard g(like.device());
+  const auto key = std::make_pair((int)like.device().index(), n);
+  void* ptr = nullptr;
   {
     std::lock_guard<std::mutex> lk(g_uncached_mu);
-    for (void* p : g_uncached_pending) (void)hipFree(p);
-    g_uncached_pending.clear();
+    auto& idle = g_uncached_idle[key];
+    if (!idle.empty()) {
+      ptr = idle.back();
+      idle.pop_back();
+    }
   }
-  void* ptr = nullptr;
-  TORCH_CHECK(hipExtMallocWithFlags(&ptr, (size_t)n * 4, hipDeviceMallocUncached) == hipSuccess, "uncached malloc");
+  if (ptr) {  // (its last owner's launches are over)
+    TORCH_CHECK(hipDeviceSynchronize() == hipSuccess, "sync");
+  } else {
+    TORCH_CHECK(hipExtMallocWithFlags(&ptr, (size_t)n * 4, hipDeviceMallocUncached) == hipSuccess, "uncached malloc");
+  }
   TORCH_CHECK(hipMemset(ptr, 0, (size_t)n * 4) == hipSuccess, "memset");
-  return torch::from_blob(ptr, {n}, [](void* p) {
+  return torch::from_blob(ptr, {n}, [key](void* p) {
         std::lock_guard<std::mutex> lk(g_uncached_mu);
-        g_uncached_pending.push_back(p);
+        g_uncached_idle[key].push_back(p);
       }, torch::dtype(torch::kInt).device(like.device()));
 }
 
 // n_layers > 1: desc holds n_layers consecutive descriptors (torch.cat of chain_make outputs of
-// consecutive layers, same flags) run by ONE launch (skinny_stream.hip chain_kernel MULTI)
+// consecutive layers, same flags) run by ONE launch (chain.hip chain_kernel MULTI)
 void chain_run(Tensor desc, int64_t n_phases, int64_t lds, Tensor like, int64_t attn_g, int64_t seq, int64_t n_layers) {
   c10::DeviceGuard g(like.device());
   TORCH_CHECK(n_layers >= 1 && desc.is_cuda() && desc.is_contiguous() &&
@@ -1499,7 +1509,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("skinny_gemm", &skinny_gemm, py::arg("x"), py::arg("w"), py::arg("bias"), py::arg("y"), py::arg("epi"),
         py::arg("fuse_rms"), py::arg("eps"), py::arg("residual"), py::arg("w_scale") = py::none(),
         py::arg("ln_c") = py::none(), py::arg("w_tiled") = false, py::arg("col_mask") = py::none(),
-        py::arg("col_mask_off") = 0, py::arg("mask_rows") = 1);
+        py::arg("col_mask_off") = 0, py::arg("mask_rows") = 1, py::arg("y2") = py::none());
   m.def("skinny_gemm_swiglu", &skinny_gemm_swiglu, py::arg("x"), py::arg("w_gu"), py::arg("bias"), py::arg("h"),
         py::arg("fuse_rms"), py::arg("eps"), py::arg("w_scale") = py::none(), py::arg("w_tiled") = false);
   m.def("skinny_gemm_qkv", &skinny_gemm_qkv, py::arg("x"), py::arg("w_qkv"), py::arg("bias"), py::arg("fuse_rms"),
@@ -1538,7 +1548,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("gemm", &gemm, py::arg("x"), py::arg("w"), py::arg("bias"), py::arg("y"), py::arg("epi"),
         py::arg("rstd") = py::none(), py::arg("residual") = py::none(), py::arg("w_tiled") = false,
         py::arg("ws") = py::none(), py::arg("ss_out") = py::none(), py::arg("ss_zero") = py::none(),
-        py::arg("ss_in") = py::none(), py::arg("ss_eps") = 1e-5);
+        py::arg("ss_in") = py::none(), py::arg("ss_eps") = 1e-5, py::arg("y2") = py::none());
   m.def("row_rstd", &row_rstd);
   m.def("gemm_qkv", &gemm_qkv, py::arg("x"), py::arg("sx"), py::arg("w"), py::arg("sw"), py::arg("bias"),
         py::arg("rstd"), py::arg("w_tiled"), py::arg("ws"), py::arg("n_q_heads"), py::arg("n_kv_heads"),
@@ -1568,4 +1578,5 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         py::arg("w_first") = 2);
   m.def("attention_split_tokens", []() { return vwa_attention_split_tokens(); });
   m.def("set_attention_impl", [](int64_t impl) { vwa_set_attention_impl((int)impl); });
+  bind_stack(m);
 }

@@ -24,7 +24,7 @@
 // hipIpcGetMemHandle / hipIpcOpenMemHandle (dmabuf).
 //
 // Behind the gather region: two f32 regions of the chained decode layer's in-launch all-reduce
-// rounds (skinny_stream.hip chain_tp_reduce; vwa_ar_chain_tp hands the pointers to the chain).
+// rounds (chain.hip chain_tp_reduce; vwa_ar_chain_tp hands the pointers to the chain).
 //
 // The same buffers also carry a one-shot ALL-GATHER of small int32 payloads (vwa_ar_gather: the
 // vocab-parallel sampler's per-rank partial (value, index) maxima, SURVEY.md §2.8 C4 as [B, 2]
@@ -278,8 +278,8 @@ void vwa_ar_destroy(void* st) {
       (void)hipIpcCloseMemHandle(s->peers.flags[p]);
     }
   }
-  (void)hipFree(s->staging);
-  (void)hipFree(s->flags);
+  // (staging / flags are uncached memory that kernels have read: they stay allocated until the process
+  // ends -- tensors allocated over freed uncached memory can hold wrong values)
   (void)hipFree(s->epochs);
   (void)hipFree(s->error);
   delete s;

@@ -206,6 +206,8 @@ __global__ __launch_bounds__(256) void logmel_norm_kernel(const float* __restric
   out[(int64_t)f * ld_out + m] = f2bf(v);
 }
 
+__global__ void logmel_reset_kernel(int* mb) { *mb = (int)0x80808080; }
+
 }  // namespace
 
 extern "C" int vwa_pcm16_to_f32(const int16_t* pcm, float* out, int n_in, int n_out, float ratio, hipStream_t st) {
@@ -218,8 +220,9 @@ extern "C" int vwa_log_mel(const float* audio, int n_samples, int n_frames, cons
                            int ld_out, hipStream_t st) {
   if (n_mels < 1 || n_mels > 16 * kLmWaves || n_frames < 1 || n_samples <= kNFFT / 2) return -1;
   int* mb = reinterpret_cast<int*>(max_buf);
-  // order-preserving encoding of -inf is a large negative int; reset every call (graph-safe memset node)
-  hipMemsetAsync(mb, 0x80, sizeof(int), st);
+  // order-preserving encoding of -inf is a large negative int; reset every call (a kernel, not a memset
+  // node: those have replayed wrongly from captured graphs)
+  hipLaunchKernelGGL(logmel_reset_kernel, dim3(1), dim3(1), 0, st, mb);
   hipLaunchKernelGGL(logmel_mfma_kernel, dim3((n_frames + kLmFrames - 1) / kLmFrames), dim3(kLmWaves * 64), 0, st,
                      audio, n_samples, n_frames, window, reinterpret_cast<const float4*>(basis),
                      reinterpret_cast<const float4*>(fb_frag), n_mels, mel_out, mb);

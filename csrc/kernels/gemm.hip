@@ -31,6 +31,8 @@
 //   0 store (+bias; bf16 or f32 out)   1 residual add (+bias)   2 SwiGLU over gate/up tiles
 //   interleaved per 16 rows (ops.interleave_gate_up)   3 GELU (+bias)   4 GELU (+bias) then a
 //   residual add (the Whisper conv stem's positional embedding: y = gelu(conv + b) + pos)
+//   5 QKV (rotary + paged KV write)   6 split: the first n_split columns stored, relu^2 of the others
+//   to a second matrix (one projection feeding a layer's mixers and its feed-forward)
 //
 // Implicit-GEMM convolution (K3, ops.conv1d_gelu): X rows are ldx apart and K long, so a k=3
 // conv over a zero-padded channels-last buffer is X row t = padded rows t*stride .. t*stride+2
@@ -42,7 +44,7 @@ using namespace vwa;
 
 namespace {
 
-enum Epi { EPI_STORE = 0, EPI_RESID = 1, EPI_SWIGLU = 2, EPI_GELU = 3, EPI_GELU_RESID = 4, EPI_QKV = 5 };
+enum Epi { EPI_STORE = 0, EPI_RESID = 1, EPI_SWIGLU = 2, EPI_GELU = 3, EPI_GELU_RESID = 4, EPI_QKV = 5, EPI_SPLIT = 6 };
 template <int EPI> constexpr bool kResid = EPI == EPI_RESID || EPI == EPI_GELU_RESID;
 template <int EPI> constexpr bool kGelu = EPI == EPI_GELU || EPI == EPI_GELU_RESID;
 
@@ -312,9 +314,18 @@ VWA_DEVICE float row_scale(const GemmParams& p, int m) {
   return 1.f;
 }
 
+VWA_DEVICE float resid_at(const GemmParams& p, int m, int n) {
+  return p.y_f32 == 2 ? reinterpret_cast<const float*>(p.R)[(size_t)m * p.ldr + n] : bf2f(p.R[(size_t)m * p.ldr + n]);
+}
+
+VWA_DEVICE float relu2(float v) {
+  v = fmaxf(v, 0.f);
+  return v * v;
+}
+
 template <int EPI>
 VWA_DEVICE void store_out(const GemmParams& p, int m, int n, float v) {
-  if constexpr (kResid<EPI>) v += bf2f(p.R[(size_t)m * p.ldr + n]);
+  if constexpr (kResid<EPI>) v += resid_at(p, m, n);
   if (p.y_f32)
     reinterpret_cast<float*>(p.Y)[(size_t)m * p.ldy + n] = v;
   else
@@ -439,6 +450,14 @@ VWA_DEVICE float finish_item(const GemmParams& p, int m, int c, const float (&a)
 #pragma unroll
       for (int e = 0; e < 8; ++e) b[e] = b[e] * rs * (p.sw ? p.sw[n1 + e] : 1.f) + bias_at(p, n1 + e);
       qkv_store(p, m, c, v, b);
+      return 0.f;
+    }
+  }
+  if constexpr (EPI == EPI_SPLIT) {
+    if (c >= p.n_split) {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[e] = relu2(v[e]);
+      *reinterpret_cast<uint4*>(p.Y2 + (size_t)m * p.ldy2 + c - p.n_split) = pack8(v);
       return 0.f;
     }
   }
@@ -678,7 +697,7 @@ __global__ __launch_bounds__(C::THREADS, C::NW == 4 ? 2 : 1) void gemm_kernel(Ge
           if (n >= p.N) continue;
           float v = acc[i][j][r] * rsv[i][r] * cz[j] + bz[j];
           if constexpr (kGelu<EPI>) v = gelu_erf(v);
-          if constexpr (kResid<EPI>) v += bf2f(p.R[(size_t)m * p.ldr + n]);
+          if constexpr (kResid<EPI>) v += resid_at(p, m, n);
           reinterpret_cast<float*>(p.Y)[(size_t)m * p.ldy + n] = v;
         }
       }
@@ -706,6 +725,7 @@ __global__ __launch_bounds__(C::THREADS, C::NW == 4 ? 2 : 1) void gemm_kernel(Ge
         for (int j = 0; j < FN; ++j) {
           float v = acc[i][j][r] * rsv[i][r] * cz[j] + bz[j];
           if constexpr (kGelu<EPI>) v = gelu_erf(v);
+          if constexpr (EPI == EPI_SPLIT) v = col0 + j * 16 >= p.n_split ? relu2(v) : v;  // (uniform per fragment)
           *reinterpret_cast<u16*>(wl + rl * RS + (j * 16 + (l & 15)) * 2) = f2bf(v);
         }
       }
@@ -742,7 +762,10 @@ __global__ __launch_bounds__(C::THREADS, C::NW == 4 ? 2 : 1) void gemm_kernel(Ge
         for (int e = 0; e < 8; ++e) sqv[it] += a[e] * a[e];
       }
     }
-    *reinterpret_cast<uint4*>(reinterpret_cast<u16*>(p.Y) + (size_t)m * p.ldy + n) = v;
+    if (EPI == EPI_SPLIT && n >= p.n_split)
+      *reinterpret_cast<uint4*>(p.Y2 + (size_t)m * p.ldy2 + n - p.n_split) = v;
+    else
+      *reinterpret_cast<uint4*>(reinterpret_cast<u16*>(p.Y) + (size_t)m * p.ldy + n) = v;
   }
   if (kResid<EPI> && p.ss_out) {  // one atomic per (row, wave): the CPR lanes of a row reduce first
 #pragma unroll
@@ -864,6 +887,10 @@ extern "C" int vwa_gemm(int epi, const GemmParams* pp, hipStream_t st) {
   if (epi == EPI_QKV && (p.y_f32 || p.head_dim % 16 || p.N != (p.n_q_heads + 2 * p.n_kv_heads) * p.head_dim ||
                          !p.q_out || !p.k_cache || !p.v_cache || !p.slots || (p.use_rope && (!p.rope || !p.positions))))
     return -16;
+  if (p.y_f32 == 2 && epi != EPI_RESID) return -18;
+  if (epi == EPI_SPLIT && (p.y_f32 || !p.Y2 || p.n_split % 16 || p.n_split < 0 || p.n_split > p.N || p.ldy2 % 8 ||
+                           (reinterpret_cast<uintptr_t>(p.Y2) & 15)))
+    return -19;
   if (p.splits < 1) p.splits = 1;
   // 8-phase 256^2 kernel (mode 2, measured rule, tools/bench_gemm.py): the prompt-sized shapes
   // whose 256^2 tiles alone fill the CUs (>= 256 tiles, e.g. the 1011-row gate/up), or fill them
@@ -893,6 +920,7 @@ extern "C" int vwa_gemm(int epi, const GemmParams* pp, hipStream_t st) {
     case EPI_GELU: return launch_epi<EPI_GELU>(p, st, p8);
     case EPI_GELU_RESID: return launch_epi<EPI_GELU_RESID>(p, st, p8);
     case EPI_QKV: return launch_epi<EPI_QKV>(p, st, p8);
+    case EPI_SPLIT: return launch_epi<EPI_SPLIT>(p, st, p8);
     default: return -3;
   }
 }

@@ -1,5 +1,5 @@
 // Multi-query MFMA decode attention body + the paged-KV / sc1 helpers it uses, shared by the
-// standalone decode kernel (attention.hip) and the chained decode-layer launch (skinny_stream.hip).
+// standalone decode kernel (attention.hip) and the chained decode-layer launch (chain.hip).
 #pragma once
 #include "common.h"
 #include "vwa_kernels.h"

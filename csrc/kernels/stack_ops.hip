@@ -1,0 +1,196 @@
+// Row kernels of layer stacks with an f32 residual stream.
+//
+//  layernorm_f32 : y (T) = (x - mean) * rstd * w + b of f32 rows, two-pass statistics in f32
+//  embedding_f32 : f32 residual rows from a T table
+//  qkv_cache     : partial rotation of q / k heads + paged cache write (V transposed inside a block)
+#include "common.h"
+#include "stack_kernels.h"
+
+using namespace vwa;
+
+namespace {
+
+template <class T> VWA_DEVICE float ldv(const T* p);
+template <> VWA_DEVICE float ldv<u16>(const u16* p) { return bf2f(*p); }
+template <> VWA_DEVICE float ldv<float>(const float* p) { return *p; }
+VWA_DEVICE void stv(u16* p, float v) { *p = f2bf(v); }
+VWA_DEVICE void stv(float* p, float v) { *p = v; }
+
+// four consecutive values
+VWA_DEVICE void st4(u16* p, const float (&v)[4]) {
+  uint2 o;
+  o.x = pack2(v[0], v[1]);
+  o.y = pack2(v[2], v[3]);
+  *reinterpret_cast<uint2*>(p) = o;
+}
+VWA_DEVICE void st4(float* p, const float (&v)[4]) { *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]); }
+
+VWA_DEVICE float block_sum(float v, float* red) {
+  v = wave_sum(v);
+  __syncthreads();  // (red may still be read from the previous sum)
+  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+  __syncthreads();
+  return (red[0] + red[1]) + (red[2] + red[3]);
+}
+
+// one workgroup per row, the row held in registers (D <= 8192): 4 columns per thread and step
+constexpr int kLnSteps = 8;
+template <class T>
+__global__ __launch_bounds__(256) void layernorm_f32_kernel(const float* __restrict__ x, int ldx,
+                                                            const float* __restrict__ w, const float* __restrict__ b,
+                                                            T* __restrict__ y, int ldy, int D, int Dpad, float eps) {
+  __shared__ float red[4];
+  const float* xr = x + (size_t)blockIdx.x * ldx;
+  T* yr = y + (size_t)blockIdx.x * ldy;
+  float v[kLnSteps][4];
+  float s = 0.f;
+#pragma unroll
+  for (int i = 0; i < kLnSteps; ++i) {
+    const int c = (i * 256 + threadIdx.x) * 4;
+    if (i * 1024 >= D) break;
+    if (c < D) {  // (rows are padded to a multiple of 4 and the padding is zero or never read back)
+      const float4 f = *reinterpret_cast<const float4*>(xr + c);
+      v[i][0] = f.x;
+      v[i][1] = c + 1 < D ? f.y : 0.f;
+      v[i][2] = c + 2 < D ? f.z : 0.f;
+      v[i][3] = c + 3 < D ? f.w : 0.f;
+    } else {
+      v[i][0] = v[i][1] = v[i][2] = v[i][3] = 0.f;
+    }
+    s += (v[i][0] + v[i][1]) + (v[i][2] + v[i][3]);
+  }
+  const float mu = block_sum(s, red) / (float)D;
+  float q = 0.f;
+#pragma unroll
+  for (int i = 0; i < kLnSteps; ++i) {
+    if (i * 1024 >= D) break;
+    const int c = (i * 256 + threadIdx.x) * 4;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const float d = c + j < D ? v[i][j] - mu : 0.f;
+      q += d * d;
+    }
+  }
+  const float rstd = 1.f / sqrtf(block_sum(q, red) / (float)D + eps);
+#pragma unroll
+  for (int i = 0; i < kLnSteps; ++i) {
+    if (i * 1024 >= D) break;
+    const int c = (i * 256 + threadIdx.x) * 4;
+    if (c >= D) continue;
+    float o[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) o[j] = c + j < D ? (v[i][j] - mu) * rstd * w[c + j] + b[c + j] : 0.f;
+    st4(yr + c, o);
+  }
+  for (int c = ((D + 3) & ~3) + threadIdx.x; c < Dpad; c += 256) stv(yr + c, 0.f);
+}
+
+template <class T>
+__global__ __launch_bounds__(256) void embedding_f32_kernel(const int* __restrict__ ids, const T* __restrict__ table,
+                                                            int ld, float* __restrict__ out, int ldo, int D, int Dpad,
+                                                            int vocab) {
+  const int row = blockIdx.x;
+  const int id = ids[row];
+  const bool ok = id >= 0 && id < vocab;
+  for (int c = threadIdx.x; c < Dpad; c += 256)
+    out[(size_t)row * ldo + c] = ok && c < D ? ldv(table + (size_t)id * ld + c) : 0.f;
+}
+
+// One workgroup per row.  VEC consecutive dimensions per thread (8 when the half rotation is a
+// multiple of 8, else 1): a rotated chunk reads its partner chunk rot_dims / 2 away.
+template <class T, int VEC>
+__global__ __launch_bounds__(256) void qkv_cache_kernel(QkvCacheParams p) {
+  const int row = blockIdx.x;
+  const T* x = reinterpret_cast<const T*>(p.x) + (size_t)row * p.ldx;
+  const int64_t slot = p.slots[row];
+  const int pos = min(max(p.positions[row], 0), p.max_pos - 1);
+  const int64_t blk = slot >= 0 ? slot / p.block_size : 0;
+  const int off = slot >= 0 ? (int)(slot % p.block_size) : 0;
+  const int half = p.rot_dims >> 1;
+  const float* cs = p.rope + (size_t)pos * p.rot_dims;
+  const int cph = p.dk / VEC, nqk = (p.H + p.G) * cph;
+  T* kc = reinterpret_cast<T*>(p.k) + blk * p.k_sb + (int64_t)off * p.dk;
+  for (int u = blockIdx.y * 256 + threadIdx.x; u < nqk; u += gridDim.y * 256) {
+    const int head = u / cph, e = (u % cph) * VEC;
+    const T* xh = x + head * p.dk;
+    float o[VEC];
+    if (e < p.rot_dims) {
+      const bool hi = e >= half;
+      const int i0 = hi ? e - half : e, pe = hi ? e - half : e + half;
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) {
+        const float a = ldv(xh + e + j), b = ldv(xh + pe + j);
+        const float c = cs[2 * (i0 + j)], s = cs[2 * (i0 + j) + 1];
+        o[j] = hi ? a * c + b * s : a * c - b * s;
+      }
+    } else {
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) o[j] = ldv(xh + e + j);
+    }
+    T* dst;
+    if (head < p.H) {
+      dst = reinterpret_cast<T*>(p.q_out) + (size_t)row * p.ldq + head * p.dk + e;
+    } else {
+      if (slot < 0) continue;
+      dst = kc + (int64_t)(head - p.H) * p.k_sh + e;
+    }
+    if constexpr (VEC == 8) {
+      const float lo[4] = {o[0], o[1], o[2], o[3]}, hi4[4] = {o[4], o[5], o[6], o[7]};
+      st4(dst, lo);
+      st4(dst + 4, hi4);
+    } else {
+      stv(dst, o[0]);
+    }
+  }
+  if (slot < 0) return;
+  const T* xv = x + (p.H + p.G) * p.dk;
+  T* vc = reinterpret_cast<T*>(p.v) + blk * p.v_sb + off;
+  for (int u = blockIdx.y * 256 + threadIdx.x; u < p.G * p.dv; u += gridDim.y * 256) {
+    const int g = u / p.dv, d = u % p.dv;
+    vc[(int64_t)g * p.v_sh + (int64_t)d * p.block_size] = xv[u];
+  }
+}
+
+}  // namespace
+
+extern "C" int vwa_layernorm_f32(const float* x, int ldx, const float* w, const float* b, void* y, int ldy, int rows,
+                                 int D, int Dpad, float eps, int f32, hipStream_t st) {
+  if (rows < 1 || D < 1 || D > kLnSteps * 1024 || Dpad < D || ldx % 4 || ldy % 4 || ldx < ((D + 3) & ~3) || ldy < Dpad ||
+      Dpad % 4)
+    return -1;
+  if (f32)
+    hipLaunchKernelGGL((layernorm_f32_kernel<float>), dim3(rows), dim3(256), 0, st, x, ldx, w, b,
+                       reinterpret_cast<float*>(y), ldy, D, Dpad, eps);
+  else
+    hipLaunchKernelGGL((layernorm_f32_kernel<u16>), dim3(rows), dim3(256), 0, st, x, ldx, w, b,
+                       reinterpret_cast<u16*>(y), ldy, D, Dpad, eps);
+  return (int)hipGetLastError();
+}
+
+extern "C" int vwa_embedding_f32(const int* ids, const void* table, int ld, float* out, int ldo, int rows, int D, int Dpad,
+                                 int vocab, int f32, hipStream_t st) {
+  if (rows < 1 || D < 1 || ld < D || Dpad < D || ldo < Dpad) return -1;
+  if (f32)
+    hipLaunchKernelGGL((embedding_f32_kernel<float>), dim3(rows), dim3(256), 0, st, ids,
+                       reinterpret_cast<const float*>(table), ld, out, ldo, D, Dpad, vocab);
+  else
+    hipLaunchKernelGGL((embedding_f32_kernel<u16>), dim3(rows), dim3(256), 0, st, ids,
+                       reinterpret_cast<const u16*>(table), ld, out, ldo, D, Dpad, vocab);
+  return (int)hipGetLastError();
+}
+
+extern "C" int vwa_qkv_cache(const QkvCacheParams* p, hipStream_t st) {
+  if (p->rows < 1 || p->H < 1 || p->G < 1 || p->dk < 1 || p->dv < 1 || p->rot_dims % 2 || p->rot_dims > p->dk ||
+      p->max_pos < 1 || p->block_size < 1)
+    return -1;
+  const bool vec = (p->rot_dims / 2) % 8 == 0 && p->dk % 8 == 0 && p->ldq % 8 == 0 && p->ldx % 8 == 0;
+  const dim3 grid(p->rows, p->rows <= 64 ? 4 : 1), block(256);
+  if (p->f32) {
+    if (vec) hipLaunchKernelGGL((qkv_cache_kernel<float, 8>), grid, block, 0, st, *p);
+    else hipLaunchKernelGGL((qkv_cache_kernel<float, 1>), grid, block, 0, st, *p);
+  } else {
+    if (vec) hipLaunchKernelGGL((qkv_cache_kernel<u16, 8>), grid, block, 0, st, *p);
+    else hipLaunchKernelGGL((qkv_cache_kernel<u16, 1>), grid, block, 0, st, *p);
+  }
+  return (int)hipGetLastError();
+}

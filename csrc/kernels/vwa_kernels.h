@@ -11,8 +11,10 @@ struct SkinnyParams {
   int M, N, K;
   const uint16_t* bias;
   int fuse_rms; float eps;
-  void* Y; int ldy; int y_f32;
+  void* Y; int ldy; int y_f32;      // y_f32: 0 bf16 out, 1 f32 out, 2 f32 out and R holds f32 (f32 residual stream)
   const uint16_t* R; int ldr;
+  // (split epilogue: output columns n < n_q_heads go to Y, the others as relu(v)^2 to q_out rows of
+  // ldq elements, column n - n_q_heads -- the QKV epilogue's fields, so descriptors keep their size)
   int n_q_heads, n_kv_heads, head_dim, use_rope;
   const int* positions;
   const int64_t* slots;
@@ -74,10 +76,10 @@ struct DecodeAttnParams {
   int* plan; int plan_mode;
 };
 
-// Chained decode GEMM phases in one persistent launch (skinny_stream.hip, vwa_chain): each phase
+// Chained decode GEMM phases in one persistent launch (chain.hip, vwa_chain): each phase
 // is a streaming-GEMM SkinnyParams + epilogue id (1 residual, 2 SwiGLU, 4 QKV, 0 store); the
 // launcher fills nt / nb.  bar: >= 1536 zero-initialised bytes of monotonic ticket counters and
-// the timeout flag (skinny_stream.hip chain_arrive), valid across launches.
+// the timeout flag (chain.hip chain_arrive), valid across launches.
 constexpr int kChainMaxPhases = 4;
 struct ChainPhase {
   SkinnyParams p;
@@ -103,7 +105,7 @@ struct ChainTP {
 struct alignas(64) ChainParams {
   ChainPhase ph[kChainMaxPhases];
   int n;
-  int seq;                 // 0 Llama tail, 1 Whisper tail, 2 Whisper middle (skinny_stream.hip chain_kernel)
+  int seq;                 // 0 Llama tail, 1 Whisper tail, 2 Whisper middle (chain.hip chain_kernel)
   int pre2;                // issue a phase's first two weight items before the barrier wait (else one)
   int next0;               // phase 1's item 0 rides in the register set a 1-item phase 0 leaves free
   int xdma;                // X staged by one wave with LDS-DMA while the others stream (chain_phase)
@@ -153,7 +155,7 @@ struct GemmParams {
   const uint16_t* X; int ldx;       // [M, K] bf16 row-major
   const uint16_t* W; int w_tiled;   // [N, K] bf16: pre-tiled (ops.tile_weight) or row-major
   int M, N, K;
-  void* Y; int ldy; int y_f32;      // [M, N] (SwiGLU: [M, N/2]) bf16 or f32
+  void* Y; int ldy; int y_f32;      // [M, N] (SwiGLU: [M, N/2]) bf16 or f32; 2: f32 and R holds f32
   const uint16_t* bias;             // [N] or null
   const uint16_t* R; int ldr;       // residual (epilogue 1), may alias Y
   const float* rstd;                // [M] per-row scale (RMSNorm with gamma folded into W) or null
@@ -184,6 +186,9 @@ struct GemmParams {
   // reproducible (f32 atomics were not: tools/repro_check.py)
   unsigned long long* ss_out; unsigned long long* ss_zero; int ss_zero_n; const unsigned long long* ss_in;
   float ss_eps;
+  // epilogue 6 (split, bf16): columns n < n_split (a multiple of 16) go to Y, the others as relu(v)^2
+  // to Y2[m][n - n_split] -- one projection of a normed row feeding the mixers and the feed-forward
+  int n_split; uint16_t* Y2; int ldy2;
 };
 
 struct FlashAttnParams {
@@ -252,7 +257,7 @@ int vwa_skinny_stream(int epi, const SkinnyParams* p, int grid_cap, int ks, hipS
 void vwa_skinny_set_x_skew(int skew);  // LDS-staged X rows: 64-B skew every 4 rows (default) or none (0)
 int vwa_chain_prepare(ChainParams* cp, int grid);
 // n_layers > 1: d_cp is an array of n_layers descriptors of consecutive 4-phase Llama tails with the
-// attention phase, run by ONE launch (skinny_stream.hip chain_kernel MULTI)
+// attention phase, run by ONE launch (chain.hip chain_kernel MULTI)
 int vwa_chain_launch(const ChainParams* d_cp, int seq, int n_phases, int attn_g, int lds, int grid, hipStream_t st,
                      int xg2 = 0, int f8 = 0, int o2 = 0, int n_layers = 1);
 // -10: a shape / role table the kernel does not take (the caller keeps per-kernel launches)

@@ -158,7 +158,7 @@ def test_llama_fp8_gpu_engine_matches_cpu_emulation():
     ids=["small", "llama8b-layers", "llama70b-tp8-rank-griddiv8"])
 def test_chained_layer_tail_matches_per_kernel_path(cfg, grid_div, monkeypatch):
     """The chained decode launch (o_proj -> gate/up -> down -> next layer's QKV behind grid
-    barriers, skinny_stream.hip chain_kernel) against the per-kernel path on the same weights,
+    barriers, chain.hip chain_kernel) against the per-kernel path on the same weights,
     for 1, 2 and 4 rows (the small config leaves most workgroups without a tile; the 8B-shaped
     one gives them several items per phase)."""
     ops.ext()
@@ -223,7 +223,7 @@ def test_chained_layer_tail_matches_per_kernel_path(cfg, grid_div, monkeypatch):
                  ffn=28672, max_pos=2048), "bf16")],
     ids=["llama8b-4layers", "llama8b-4layers-fp8", "llama70b-3layers-gqa8"])
 def test_multi_layer_chained_launch_matches_per_layer_launches(cfg, wdtype, monkeypatch):
-    """All layers in ONE chained launch (skinny_stream.hip chain_kernel MULTI: the QKV phase
+    """All layers in ONE chained launch (chain.hip chain_kernel MULTI: the QKV phase
     feeds the next layer's attention through an in-launch barrier that only attention workgroups
     wait on) give the SAME bits as one chained launch per layer, and match the per-kernel path,
     over steps of 1, 2, 4 and 1 rows and a second session (contexts that differ per row)."""
@@ -421,7 +421,7 @@ def test_prefix_cached_prefill_decode_attention_slices(monkeypatch):
 @pytest.mark.parametrize("name", ["whisper-test", "whisper-tiny", "whisper-large-v3"])
 def test_whisper_chained_decoder_matches_per_kernel_path(name, monkeypatch):
     """The chained Whisper decoder launches (out-proj -> LN cross query; out-proj -> LN fc1 GELU
-    -> fc2 -> next layer's LN QKV + self-KV write, skinny_stream.hip chain_kernel SEQ 2 / 1)
+    -> fc2 -> next layer's LN QKV + self-KV write, chain.hip chain_kernel SEQ 2 / 1)
     against the per-kernel path on the same weights and caches, for 1, 2 and 4 rows over a few
     positions (large-v3: its layer shapes, 3 decoder layers)."""
     from voice_enabled_browser_automation_amd.asr.engine import WhisperRunner
@@ -726,7 +726,7 @@ def test_intent_engine_recovers_from_a_failed_chained_step(monkeypatch):
                                                   n_kv_heads=8, head_dim=128, ffn=14336, max_pos=2048)],
                          ids=["small", "llama8b-layers"])
 def test_fp8_chained_layer_is_w8a16(cfg, monkeypatch):
-    """fp8 tiled weights through the chained decode launch (skinny_stream.hip chain_kernel F8:
+    """fp8 tiled weights through the chained decode launch (chain.hip chain_kernel F8:
     e4m3 items converted to bf16 in registers, per-row scales in the epilogues) == a bf16 model
     holding the dequantised weights on the per-kernel path (W8A16 semantics), 1 / 2 / 4 rows."""
     ops.ext()

@@ -53,7 +53,7 @@ def _kernels(obj_name):
 
 
 def test_chain_kernels_do_not_spill():
-    ks = _kernels("skinny_stream.hip.o")
+    ks = _kernels("chain.hip.o")
     chains = {k: v for k, v in ks.items() if "chain_kernel" in k}
     assert chains
     # (every instantiation: bf16 and -- since its items are 8 loads -- the fp8 W8A16 chain)

@@ -1,5 +1,5 @@
 """Whisper transcription time split (encoder / decoder) with and without the chained decoder
-launches (models/whisper.py, skinny_stream.hip chain_kernel SEQ 1/2), fixed 40-token work on the
+launches (models/whisper.py, chain.hip chain_kernel SEQ 1/2), fixed 40-token work on the
 bench's synthetic 10 s utterance.  One JSON line per mode.
 python tools/asr_timing.py [--asr whisper-large-v3] [--reps 10]
 

@@ -1,6 +1,6 @@
 // Critical-load latency under a weight stream (diagnostic, not part of the framework).
 //
-// The chained decode layer (skinny_stream.hip chain_kernel) keeps HBM busy by issuing weight items
+// The chained decode layer (chain.hip chain_kernel) keeps HBM busy by issuing weight items
 // ahead of every grid barrier; its in-phase stamps (tools/chain_probe.py, profiles/r5_*) show the
 // phase's small activation read taking 3-6.5 us after each barrier release.  This probe asks how
 // the round trip of one such "critical" load depends on how many weight bytes every CU keeps in

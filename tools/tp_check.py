@@ -9,7 +9,7 @@ from a hipGraph -- with the one-shot IPC all-reduce for the vocab-parallel embed
 row-parallel outputs, and compares the (diagnostically gathered) logits with a TP=1 model run
 on the same device.  Decode steps of <= 4 rows run the chained layer (one launch per layer) with
 the row-parallel all-reduces as in-launch rounds over the same IPC buffers
-(skinny_stream.hip chain_tp_reduce).  Then the vocab-parallel sampler (partial maxima -> one-shot IPC all-gather
+(chain.hip chain_tp_reduce).  Then the vocab-parallel sampler (partial maxima -> one-shot IPC all-gather
 -> merge, ops.sample tp=...) is checked token for token against the TP=1 full-vocab sampler,
 under grammar-like random masks and temperature.  VWA_DIST_BACKEND selects the control /
 large-message backend (gloo when two ranks share one GPU, RCCL needs one GPU per rank); the

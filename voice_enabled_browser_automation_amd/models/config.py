@@ -5,6 +5,8 @@ north star names these on-node replacements.
 """
 from __future__ import annotations
 
+import json
+import os
 from dataclasses import dataclass, field, replace
 from typing import Optional
 
@@ -82,6 +84,90 @@ class WhisperConfig:
         return 4 * self.d_model
 
 
+@dataclass(frozen=True)
+class TalkAttentionConfig:
+    """Windowed grouped-query attention with kept first keys, partial rotation, softmax weights mixed
+    across the query heads and an output gate per head."""
+    heads: int
+    kv_heads: int
+    dim: int                 # query / key size of a head
+    vdim: int                # value size of a head
+    scale: float
+    window: int              # a position sees the last ``window`` positions (itself included) ...
+    keep_first: int          # ... and the first ``keep_first`` of the sequence
+    rot_base: float
+    rot_dims: int            # rotated dimensions of every query / key head (the first ones)
+
+
+@dataclass(frozen=True)
+class MinGRUConfig:
+    width: int
+
+
+@dataclass(frozen=True)
+class ParallelLayerConfig:
+    """One layer: two mixers side by side, and a feed-forward (0: none), all reading one normed input."""
+    left: TalkAttentionConfig
+    right: MinGRUConfig
+    left_scale: float = 1.0
+    right_scale: float = 1.0
+    ffn: int = 0
+
+
+@dataclass(frozen=True)
+class KabanexConfig:
+    name: str
+    vocab_size: int
+    hidden: int
+    layers: tuple            # of ParallelLayerConfig, in order (sizes may differ from layer to layer)
+    norm_eps: float = 1e-5
+    max_pos: int = 8192      # rotation table length to start with (it grows with the engine's contexts)
+    bos_id: int = 0
+    eos_ids: tuple = ()
+    init_std: float = 0.02
+
+    @property
+    def n_layers(self) -> int:
+        return len(self.layers)
+
+    @staticmethod
+    def from_json(j: dict, name: str = "kabanex") -> "KabanexConfig":
+        """The checkpoint's config.json.  A layer, feed-forward or norm kind this design does not have
+        is an error, never ignored."""
+        layers = []
+        for i, L in enumerate(j["layers"]):
+            if L["type"] != "parallel":
+                raise ValueError(f"layer {i}: unknown mixer type {L['type']!r}")
+            m, mlp = L["mixer"], L.get("mlp")
+            if mlp is not None and mlp["kind"] != "dense":
+                raise ValueError(f"layer {i}: unknown feed-forward kind {mlp['kind']!r}")
+            a = m["left"]
+            if a["heads"] % a["kv_heads"] or a["rot"]["dims"] % 2 or not 0 < a["rot"]["dims"] <= a["dim"]:
+                raise ValueError(f"layer {i}: head counts or rotated dimensions do not fit")
+            if a["mask"]["size"] < 1 or a["mask"]["keep_first"] < 0:
+                raise ValueError(f"layer {i}: window size must be positive, kept keys not negative")
+            layers.append(ParallelLayerConfig(
+                left=TalkAttentionConfig(heads=a["heads"], kv_heads=a["kv_heads"], dim=a["dim"], vdim=a["vdim"],
+                                         scale=float(a["scale"]), window=a["mask"]["size"],
+                                         keep_first=a["mask"]["keep_first"], rot_base=float(a["rot"]["base"]),
+                                         rot_dims=a["rot"]["dims"]),
+                right=MinGRUConfig(width=m["right"]["width"]), left_scale=float(m["left_scale"]),
+                right_scale=float(m["right_scale"]), ffn=mlp["ff"] if mlp is not None else 0))
+        return KabanexConfig(name=name, vocab_size=j["vocab"], hidden=j["width"], layers=tuple(layers),
+                             norm_eps=float(j["norm"]["eps"]))
+
+
+def kabanex_stack(name: str, *, vocab: int, hidden: int, n_layers: int, heads: int, kv_heads: int, dim: int, vdim: int,
+                  window: int, keep_first: int, width: int, ffn: int, rot_dims: Optional[int] = None,
+                  rot_base: float = 500000.0, **kw) -> KabanexConfig:
+    """A uniform stack (presets, benchmarks)."""
+    L = ParallelLayerConfig(
+        left=TalkAttentionConfig(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, scale=dim ** -0.5, window=window,
+                                 keep_first=keep_first, rot_base=rot_base, rot_dims=rot_dims or dim // 2),
+        right=MinGRUConfig(width=width), ffn=ffn)
+    return KabanexConfig(name=name, vocab_size=vocab, hidden=hidden, layers=(L,) * n_layers, **kw)
+
+
 LLAMA_PRESETS = {
     "llama3-8b": LlamaConfig(),
     "llama3-70b": LlamaConfig(name="llama3-70b", hidden=8192, n_layers=80, n_heads=64, n_kv_heads=8, ffn=28672),
@@ -108,8 +194,47 @@ WHISPER_PRESETS = {
 }
 
 
+KABANEX_PRESETS = {
+    # Llama-3.2-1B-sized layers (bench.py --design): its residual width, feed-forward and vocabulary
+    "kabanex-1b": kabanex_stack("kabanex-1b", vocab=128256, hidden=2048, n_layers=16, heads=16, kv_heads=4, dim=128, vdim=128,
+                                window=1024, keep_first=4, width=2048, ffn=8192, bos_id=128000, eos_ids=(128001, 128009)),
+    # small shapes for tests (vocab kept at the real tokenizer size so the grammar works)
+    "kabanex-tiny": kabanex_stack("kabanex-tiny", vocab=128256, hidden=192, n_layers=2, heads=6, kv_heads=2, dim=32, vdim=48,
+                                  window=640, keep_first=3, width=160, ffn=384, bos_id=128000,
+                                  eos_ids=(128001, 128009)),
+}
+
+
+def _llama_from_json(j: dict, name: str) -> LlamaConfig:
+    hd = j.get("head_dim") or j["hidden_size"] // j["num_attention_heads"]
+    return LlamaConfig(name=name, vocab_size=j["vocab_size"], hidden=j["hidden_size"], n_layers=j["num_hidden_layers"],
+                       n_heads=j["num_attention_heads"], n_kv_heads=j["num_key_value_heads"], head_dim=hd,
+                       ffn=j["intermediate_size"], rope_theta=j["rope_theta"], rms_eps=j["rms_norm_eps"],
+                       tie_embeddings=bool(j.get("tie_word_embeddings", False)))
+
+
+# config.json "architecture" (or the first of "architectures") -> configuration reader
+ARCHITECTURES = {
+    "Kabanex": KabanexConfig.from_json,
+    "LlamaForCausalLM": _llama_from_json,
+}
+
+
+def config_from_dir(path: str):
+    """The configuration of a checkpoint folder, by its config.json."""
+    with open(os.path.join(path, "config.json"), encoding="utf-8") as fh:
+        j = json.load(fh)
+    arch = j.get("architecture") or (j.get("architectures") or [None])[0]
+    if arch not in ARCHITECTURES:
+        raise KeyError(f"unknown model architecture {arch!r} (known: {', '.join(sorted(ARCHITECTURES))})")
+    return ARCHITECTURES[arch](j, os.path.basename(os.path.normpath(path)))
+
+
 def get_config(name: str):
-    for table in (LLAMA_PRESETS, GPT2_PRESETS, WHISPER_PRESETS):
+    """A preset by name, or the configuration of a checkpoint folder."""
+    if os.path.isfile(os.path.join(name, "config.json")):
+        return config_from_dir(name)
+    for table in (LLAMA_PRESETS, GPT2_PRESETS, KABANEX_PRESETS, WHISPER_PRESETS):
         if name in table:
             return table[name]
     raise KeyError(f"unknown model preset {name!r}")

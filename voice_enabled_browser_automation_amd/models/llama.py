@@ -234,7 +234,7 @@ class LlamaModel:
     # ---- chained layer tail (o_proj -> gate/up -> down -> next QKV in one launch; M <= 4 rows)
     def _chain_ok(self, M: int) -> bool:
         # 5..16 rows (jump-forward feeds, concurrent sessions): the chain without its attention
-        # phase, the down projection streaming X with the weights (skinny_stream.hip XG2)
+        # phase, the down projection streaming X with the weights (chain.hip XG2)
         # fp8: the W8A16 chain over the fp8 tiled weights (<= 4 rows: no X streaming)
         fp8_ok = self.wdtype == "fp8" and M <= 4 and isinstance(self.layers[0].o, ops.FP8Weight) and self.layers[0].o.tiled
         # TP > 1: the one-shot all-reduce buffers carry the in-launch rounds (chain_tp_reduce)
@@ -297,7 +297,7 @@ class LlamaModel:
         N = self.layers[li + 1] if nxt else None
         # the layer's decode attention as the launch's first phase (VWA_CHAIN_ATTN, default on;
         # same-box bench A/B/A: GPU time per decode step 3868 vs 3897 / 3907 us, p50 276 vs 284 /
-        # 285 ms, profiles/r1_bench_results.jsonl; skinny_stream.hip chain_kernel)
+        # 285 ms, profiles/r1_bench_results.jsonl; chain.hip chain_kernel)
         # (the chained attention addresses K/V through per-row copies of the block table, which
         # the step buffers keep for contexts of <= 128 blocks, in 16-token blocks: otherwise the
         # separate launch)
@@ -344,7 +344,7 @@ class LlamaModel:
 
     def _chain_multi(self, bufs, kv, M: int):
         """(descriptors, lds, attn_g, n) of ONE launch over all n = L layers (4-phase tails with the
-        attention phase, the last one a 3-phase tail; skinny_stream.hip chain_kernel MULTI), or None
+        attention phase, the last one a 3-phase tail; chain.hip chain_kernel MULTI), or None
         when some layer cannot take it (per-layer chained / per-kernel launches then).  The
         descriptors are the per-layer ones (_chain_desc) concatenated into one device array; layer
         0's writes the attention step plan that layers 1.. of the same launch read, so a plan can

@@ -417,7 +417,7 @@ class WhisperModel:
         return res
 
     # ------------------------------------------------------------------ decoder step
-    # ---- chained decode launches (skinny_stream.hip chain_kernel SEQ 2 / SEQ 1; M <= 4 rows).
+    # ---- chained decode launches (chain.hip chain_kernel SEQ 2 / SEQ 1; M <= 4 rows).
     # Opt-in (VWA_CHAIN_ASR=1): measured (tools/asr_timing.py, 1 row, 40 tokens) 2.32 vs 2.26 ms
     # per token for whisper-large-v3 and 260 vs 244 us for whisper-tiny -- the decoder's
     # phases are 0.3-13 MB each, so every phase is latency-bound and a grid barrier (~4-5 us,

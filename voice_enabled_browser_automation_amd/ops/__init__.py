@@ -19,6 +19,7 @@ Layout conventions shared by kernels, reference and models:
 from __future__ import annotations
 
 import math
+import os
 from typing import Dict, Optional, Tuple
 
 import torch
@@ -28,6 +29,21 @@ from . import reference as ref
 
 _EXT = None
 _EXT_ERR: Optional[BaseException] = None
+
+
+def _load_built():
+    """The in-tree library: the full one, or (a checkout where only that was built) the core one."""
+    import importlib.machinery
+    import importlib.util
+
+    from .build import CORE_SO, KERNEL_SO
+
+    path = KERNEL_SO if os.path.exists(KERNEL_SO) or not os.path.exists(CORE_SO) else CORE_SO
+    name = __name__ + "._vwa_kernels"
+    spec = importlib.util.spec_from_file_location(name, path, loader=importlib.machinery.ExtensionFileLoader(name, path))
+    m = importlib.util.module_from_spec(spec)
+    spec.loader.exec_module(m)
+    return m
 
 
 def ext():
@@ -49,7 +65,7 @@ def ext():
             m = importlib.util.module_from_spec(spec)
             spec.loader.exec_module(m)
         else:
-            from . import _vwa_kernels as m  # type: ignore
+            m = _load_built()
 
         # diagnostic overrides (utils/env.py Settings; defaults are the measured-best settings)
         impl = knob("VWA_ATTN_IMPL")
@@ -508,6 +524,11 @@ def gemm_fp8(x: torch.Tensor, w: "FP8Weight", out: torch.Tensor, *, epi: str = "
     return out
 
 
+def _f32_resid(out: torch.Tensor, residual: Optional[torch.Tensor]) -> bool:
+    """An f32 residual stream: both the residual and the output rows are f32."""
+    return residual is not None and residual.dtype == torch.float32 and out.dtype == torch.float32
+
+
 def gemm_fp8_ok(x: torch.Tensor, w, out: Optional[torch.Tensor] = None, residual: Optional[torch.Tensor] = None) -> bool:
     return (isinstance(w, FP8Weight) and w.tiled and _gpu(x) and x.dtype == torch.bfloat16 and w.shape[0] % 16 == 0
             and w.shape[1] % 128 == 0 and _rows16(x) and _rows16(out) and _rows16(residual))
@@ -584,6 +605,12 @@ def _linear_impl(x, w, bias, out, residual, act, fuse_rms, eps, out_dtype, ln_c,
         ss["used"] = True
         return dict(ss_out=ss["ss_out"], ss_zero=ss["ss_zero"], ss_in=ss["ss_in"])
 
+    if _gpu(x) and x.dtype == torch.float32:  # 32-bit models: the f32 MFMA GEMM
+        assert bias is None and act == "none" and not fuse_rms and ln_c is None, "f32 linear: plain or residual only"
+        if out is None:
+            out = torch.empty((M, w.shape[0]), dtype=torch.float32, device=x.device)
+        ext().gemm_f32(x, w, out, 1 if residual is not None else 0, residual)
+        return out
     mk = {}
     if col_mask is not None and residual is None and act == "none" and bias is None and ln_c is None:
         mk = dict(col_mask=col_mask, col_mask_off=col_mask_off, mask_rows=mask_rows)
@@ -602,7 +629,7 @@ def _linear_impl(x, w, bias, out, residual, act, fuse_rms, eps, out_dtype, ln_c,
         if ln_c is not None:
             return linear(_layernorm_plain(x, eps), w, bias, out=out, residual=residual, act=act, out_dtype=out_dtype)
         if _gpu(x) and gemm_ok(x, w, out, residual) and (act == "none" or residual is None) and \
-                (out.dtype == torch.bfloat16 or (residual is None and act == "none")):
+                (out.dtype == torch.bfloat16 or _f32_resid(out, residual) or (residual is None and act == "none")):
             e = "resid" if residual is not None else ("gelu" if act == "gelu" else "none")
             return gemm(x, w, out, epi=e, bias=bias, residual=residual, fuse_rms=fuse_rms, eps=eps, **ssk())
         w = w.dense()
@@ -877,7 +904,7 @@ def split_counters(device, n: int) -> torch.Tensor:
 
 def chain_buffers(device):
     """(barrier words, bar_mode, work) for one model's chained decode launches
-    (skinny_stream.hip chain_kernel): barrier words in L2-uncached memory polled with scalar
+    (chain.hip chain_kernel): barrier words in L2-uncached memory polled with scalar
     loads (bar_mode 2: the poll does not queue behind the next phase's weight loads), plain
     memory + vector polls (bar_mode 1) if the uncached allocation is unavailable; work = split-tile
     tickets + partial slots.  One set per model: launches sharing a set must be stream-ordered."""
@@ -893,7 +920,7 @@ def chain_buffers(device):
 
 
 def chain_error_word(bar: Optional[torch.Tensor]) -> Optional[torch.Tensor]:
-    """The device word a timed-out chain barrier sets (skinny_stream.hip chain_wait)."""
+    """The device word a timed-out chain barrier sets (chain.hip chain_wait)."""
     return None if bar is None else bar.view(torch.int64)[160:161]
 
 
@@ -1153,3 +1180,7 @@ def env_flag(name: str) -> bool:
 
 def env_int(name: str) -> int:
     return int(knob(name))
+
+
+from .stack import (TalkScratch, embedding_f32, layernorm_f32, linear_split, mingru, pad_talk, plan_runs,  # noqa: E402,F401
+                    qkv_cache_write, talk_attention)

@@ -109,6 +109,93 @@ def layernorm(x, w, b, *, eps=1e-5, residual=None, residual_out=None, out):
     return out
 
 
+# ----------------------------------------------------------------------------- layer stacks (ops/stack.py)
+def layernorm_f32(x, w, b, *, eps, out):
+    D = w.shape[0]
+    y = F.layer_norm(x[:, :D].float(), (D,), w.float(), b.float(), eps)
+    out.zero_()
+    out[:, :D] = y.to(out.dtype)
+    return out
+
+
+def embedding_f32(ids, table, *, out):
+    idl = ids[: out.shape[0]].long()
+    ok = (idl >= 0) & (idl < table.shape[0])
+    out.zero_()
+    out[:, : table.shape[1]] = table[idl.clamp(0, table.shape[0] - 1)].float() * ok[:, None]
+    return out
+
+
+def linear_split(x, w, *, out, out2):
+    y = x.float() @ w.float().t()
+    n = out.shape[1]
+    out.copy_(y[:, :n].to(out.dtype))
+    out2.copy_(torch.relu(y[:, n:]).square().to(out2.dtype))
+    return out
+
+
+def qkv_cache_write(x, *, n_q_heads, rot_dims, rope, positions, slots, q_out, k_cache, v_cache):
+    M, G, bs, dk, dv = q_out.shape[0], k_cache.shape[1], k_cache.shape[2], k_cache.shape[3], v_cache.shape[2]
+    nq = n_q_heads * dk
+    qk = x[:M, : nq + G * dk].float().view(M, n_q_heads + G, dk).clone()
+    half = rot_dims // 2
+    cs = rope[positions[:M].long()]
+    c, s = cs[..., 0][:, None, :], cs[..., 1][:, None, :]
+    u, v = qk[..., :half].clone(), qk[..., half:rot_dims].clone()
+    qk[..., :half], qk[..., half:rot_dims] = u * c - v * s, v * c + u * s
+    q_out.copy_(qk[:, :n_q_heads].reshape(M, nq).to(q_out.dtype))
+    vals = x[:M, nq + G * dk : nq + G * (dk + dv)].reshape(M, G, dv)
+    for m in range(M):
+        sl = int(slots[m])
+        if sl >= 0:
+            k_cache[sl // bs, :, sl % bs, :] = qk[m, n_q_heads:].to(k_cache.dtype)
+            v_cache[sl // bs, :, :, sl % bs] = vals[m].to(v_cache.dtype)
+    return q_out
+
+
+def talk_attention(q, k_cache, v_cache, block_table, positions, seq_ids, slots, *, n_q_heads, scale, window, keep, talk,
+                   gate, out_scale, out):
+    G, bs, dk, dv = k_cache.shape[1], k_cache.shape[2], k_cache.shape[3], v_cache.shape[2]
+    H, R = n_q_heads, n_q_heads // k_cache.shape[1]
+    for m in range(q.shape[0]):
+        if int(slots[m]) < 0:
+            out[m, : H * dv] = 0
+            continue
+        i, sid = int(positions[m]), int(seq_ids[m])
+        blk = block_table[sid, : i // bs + 1].long()
+        K = k_cache[blk].transpose(0, 1).reshape(G, -1, dk)[:, : i + 1].float()
+        V = v_cache[blk].permute(1, 0, 3, 2).reshape(G, -1, dv)[:, : i + 1].float()
+        j = torch.arange(i + 1)
+        vis = ((i - j < window) | (j < keep)) if window > 0 else torch.ones(i + 1, dtype=torch.bool)
+        s = torch.einsum("grd,gnd->grn", q[m, : H * dk].float().view(G, R, dk), K) * scale
+        w = torch.softmax(s.masked_fill(~vis, float("-inf")), -1).view(H, i + 1)
+        if talk is not None:
+            w = talk.float() @ w
+        o = torch.einsum("grn,gnd->grd", w.view(G, R, i + 1), V).reshape(H, dv) * out_scale
+        if gate is not None:
+            o = o * torch.sigmoid(gate[m, :H].float())[:, None]
+        out[m, : H * dv] = o.reshape(-1).to(out.dtype)
+    return out
+
+
+def mingru(z, x, g, zb, xb, *, seq_ids, positions, slots, state, out_scale, out):
+    W = state.shape[1]
+    zf, xf, gf = z[:, :W].float(), x[:, :W].float(), g[:, :W].float()
+    zf = torch.sigmoid(zf if zb is None else zf + zb)
+    xf = xf if xb is None else xf + xb
+    cand = torch.where(xf >= 0, xf + 0.5, torch.sigmoid(xf))
+    for m in range(out.shape[0]):
+        if int(slots[m]) < 0:
+            out[m, :W] = 0
+            continue
+        sid = int(seq_ids[m])
+        S = state[sid] if int(positions[m]) > 0 else torch.zeros(W)
+        S = (1 - zf[m]) * S + zf[m] * cand[m]
+        state[sid] = S
+        out[m, :W] = (S * F.silu(gf[m]) * out_scale).to(out.dtype)
+    return out
+
+
 def embedding(ids, table, *, pos_table=None, positions=None, vocab_start=0, out):
     n = out.shape[0]
     idl = ids[:n].long() - vocab_start

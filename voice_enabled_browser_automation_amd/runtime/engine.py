@@ -79,7 +79,6 @@ class StepBuffers:
 
     def __init__(self, model, max_rows: int, max_seqs: int, max_blocks_per_seq: int, max_ctx: int, device):
         i32 = dict(dtype=torch.int32, device=device)
-        dt = model.dtype
         self.max_rows = max_rows
         self.max_ctx = max_ctx
         # all per-row metadata lives in ONE device buffer (and one pinned host mirror) so a step
@@ -108,7 +107,15 @@ class StepBuffers:
         self.ctx_lens.fill_(1)
         self.slots.fill_(-1)
         self.block_table = torch.zeros(max_seqs, max_blocks_per_seq, **i32)
-        d = model.cfg.hidden
+        if hasattr(model, "step_buffers"):  # models with activations of their own
+            for name, t in model.step_buffers(max_rows, max_ctx).items():
+                setattr(self, name, t)
+        else:
+            self._default_activations(model, max_rows, max_ctx, device)
+        self._host_staging(max_rows, max_seqs, max_blocks_per_seq, T, C, device)
+
+    def _default_activations(self, model, max_rows: int, max_ctx: int, device) -> None:
+        dt, d = model.dtype, model.cfg.hidden
         self.hidden = torch.zeros(max_rows, d, dtype=dt, device=device)
         self.hidden_sel = torch.zeros(max_rows, d, dtype=dt, device=device)
         self.q = torch.zeros(max_rows, model.nq * model.hd, dtype=dt, device=device)
@@ -120,6 +127,8 @@ class StepBuffers:
         self.part_o = torch.zeros(max_rows * ns * model.nq * model.hd, dtype=torch.float32, device=device)
         self.part_ml = torch.zeros(max_rows * ns * model.nq * 2, dtype=torch.float32, device=device)
         self.attn_cnt = torch.zeros(max_rows * model.nkv, dtype=torch.int32, device=device)  # chunk tickets
+
+    def _host_staging(self, R: int, max_seqs: int, max_blocks_per_seq: int, T: int, C: int, device) -> None:
         pin = torch.device(device).type == "cuda"
         self.h_meta_all = torch.zeros(T + R * C, dtype=torch.int32, pin_memory=pin)
         self.h_meta = self.h_meta_all[: 7 * R + 2]
@@ -167,6 +176,19 @@ class LLMEngine:
         self.max_model_len = max_model_len
         self.max_seqs = max_seqs
         cfg = model.cfg
+        # layers with their own cache sizes and recurrent state (else: one K / V shape for all)
+        layers = model.cache_layers() if hasattr(model, "cache_layers") else None
+        # a recurrent state cannot be resumed from prefix-cached blocks: no prefix matching
+        self.stateful = bool(getattr(model, "stateful", False))
+        elem = torch.empty(0, dtype=model.dtype).element_size()
+        per_block = PagedKVCache.layer_bytes_per_block(layers, block_size, elem) if layers else \
+            PagedKVCache.bytes_per_block(cfg.n_layers, model.nkv, model.hd, block_size)
+        if hasattr(model, "ensure_positions"):
+            model.ensure_positions(max_model_len)
+        if layers and kv_blocks is None and kv_gb is None and knob("VWA_KV_GB").strip().lower() == "auto":
+            # what is free now, minus headroom for step buffers, graphs, prompt scratch and a co-located service
+            free, _total = torch.cuda.mem_get_info(self.device) if self.device.type == "cuda" else (0, 0)
+            kv_blocks = max(4, int(free * 0.95 - 8e9 - knob("VWA_SHARED_GB") * 1e9) // per_block)
         if kv_blocks is None and kv_gb is None and knob("VWA_KV_GB").strip().lower() == "auto":
             # size the paged KV from the per-GPU HBM plan (runtime/memory_plan.py): what the weights,
             # step buffers and workspaces leave of the 288 GB
@@ -183,19 +205,22 @@ class LLMEngine:
                 # never more than the device has free now (other processes, fragmentation), minus
                 # headroom for what is allocated after the KV: step buffers, graph pools, GEMM and
                 # prefill scratch, and the co-located service
-                per = PagedKVCache.bytes_per_block(cfg.n_layers, model.nkv, model.hd, block_size)
                 head = plan.step_buffers + plan.workspace + int(4e9) + int(shared * 1e9)
-                kv_blocks = min(kv_blocks, max(0, int(free * 0.95) - head) // per)
+                kv_blocks = min(kv_blocks, max(0, int(free * 0.95) - head) // per_block)
             self.memory_plan = plan
         if kv_blocks is None:
             if kv_gb is None:
                 kv_gb = float(knob("VWA_KV_GB") or 0)
             if kv_gb > 0:
-                kv_blocks = PagedKVCache.blocks_for_budget(kv_gb * 1e9, cfg.n_layers, model.nkv, model.hd, block_size)
+                kv_blocks = max(4, int(kv_gb * 1e9 // per_block))
             else:
                 kv_blocks = max_seqs * (max_model_len // block_size) * 2 + 1
-        self.kv = PagedKVCache(cfg.n_layers, model.nkv, model.hd, block_size, kv_blocks, device=self.device,
-                               dtype=model.dtype)
+        if layers:
+            self.kv = PagedKVCache.from_layers(layers, block_size, kv_blocks, max_seqs, device=self.device,
+                                               dtype=model.dtype)
+        else:
+            self.kv = PagedKVCache(cfg.n_layers, model.nkv, model.hd, block_size, kv_blocks, device=self.device,
+                                   dtype=model.dtype)
         self.blocks = BlockManager(kv_blocks, block_size)
         self.max_blocks_per_seq = (max_model_len + block_size - 1) // block_size
         self.bufs = StepBuffers(model, max_rows, max_seqs, self.max_blocks_per_seq, max_model_len, self.device)
@@ -225,7 +250,7 @@ class LLMEngine:
             raise RuntimeError("too many concurrent sequences")
         sid = self.free_sids.pop()
         seq = Sequence_(sid=sid, tokens=list(tokens))
-        if use_prefix_cache:
+        if use_prefix_cache and not self.stateful:
             blocks, n = self.blocks.match_prefix(seq.tokens)
             seq.blocks = blocks
             seq.n_computed = n
@@ -238,7 +263,7 @@ class LLMEngine:
     def free_sequence(self, seq: Sequence_, publish: bool = True, publish_upto: Optional[int] = None) -> None:
         """Release a sequence; publish its first ``publish_upto`` computed tokens (default all) to the
         prefix cache."""
-        if publish:
+        if publish and not self.stateful:
             n = seq.n_computed if publish_upto is None else min(seq.n_computed, publish_upto)
             self.blocks.register_prefix(seq.tokens, seq.blocks, n)
         self.blocks.release(seq.blocks)
@@ -301,11 +326,21 @@ class LLMEngine:
 
     def _capture(self, M: int, L: int):
         s = torch.cuda.Stream()
+        b, slots = self.bufs, None
+        if self.stateful:
+            # the warm-up forwards below must not advance a recurrent state: they run this step's rows as
+            # inert ones (no slot), the replay after the capture runs them for real
+            torch.cuda.current_stream().synchronize()
+            slots = b.np_slots[:M].copy()
+            b.np_slots[:M] = -1
         s.wait_stream(torch.cuda.current_stream())
         with torch.cuda.stream(s):
             for _ in range(2):
                 self._forward_rows(M, L, upload_meta=True)
         torch.cuda.current_stream().wait_stream(s)
+        if slots is not None:
+            s.synchronize()  # (the warm-ups have read the staging rows)
+            b.np_slots[:M] = slots
         g = torch.cuda.CUDAGraph()
         if self.graph_pool is None:
             self.graph_pool = torch.cuda.graph_pool_handle()
@@ -583,7 +618,7 @@ class LLMEngine:
             todo = end - seq.n_computed
             if todo <= 0:
                 continue
-            if todo > seq.n_computed and todo > self.bufs.max_rows:
+            if todo > seq.n_computed and todo > self.bufs.max_rows and not self.stateful:
                 self.prefill(seq, upto=end)
                 continue
             rows += [(seq, t) for t in seq.tokens[seq.n_computed:end]]
@@ -595,15 +630,54 @@ class LLMEngine:
             self.run_rows(rows, logits_for=[len(rows) - 1], check=True, defer_head=True)
             self._head_rows = None
             return
-        if self._staging_inflight and self.device.type == "cuda":
-            torch.cuda.current_stream().synchronize()
-            self._staging_inflight = False
+        self._sync_staging()
         for i in range(0, len(rows), chunk):
             self._ragged_forward(rows[i : i + chunk])
 
-    def _ragged_forward(self, rows: List[Tuple[Sequence_, int]]) -> None:
-        """One eager forward of ragged rows (more than the step buckets hold): the decode-mode
-        model forward over scratch buffers sized for them; attention in 64-row slices."""
+    def step_batch(self, entries: List[Tuple[Sequence_, List[int]]], want: Sequence[int] = (),
+                   chunk: int = 4096) -> Optional[torch.Tensor]:
+        """One step over any mix of prompt portions and single decoded tokens: every entry's next tokens
+        are appended to its sequence and all of them run together (the step graphs when they fit a row
+        bucket, one ragged forward otherwise).  ``want``: places in the concatenated tokens whose logits
+        are returned, f32 [len(want), V] (None when there are none)."""
+        rows: List[Tuple[Sequence_, int]] = []
+        for seq, toks in entries:
+            if seq.n_computed != len(seq.tokens):
+                # (a prompt given to new_sequence: its next tokens are the uncomputed ones)
+                assert seq.tokens[seq.n_computed : seq.n_computed + len(toks)] == list(toks), "tokens out of order"
+            else:
+                seq.tokens.extend(toks)
+            rows += [(seq, t) for t in toks]
+        want = list(want)
+        if not rows:
+            return None
+        if len(rows) <= min(self.bufs.max_rows, BUCKETS[-1]):
+            if want:
+                return self.run_rows(rows, logits_for=want)
+            self.run_rows(rows, logits_for=[len(rows) - 1], defer_head=True)
+            self._head_rows = None
+            return None
+        self._sync_staging()
+        hidden = []
+        for i in range(0, len(rows), chunk):
+            part = rows[i : i + chunk]
+            hs = self._ragged_forward(part, [w - i for w in want if i <= w < i + len(part)])
+            if hs is not None:
+                hidden.append(hs)
+        if not want:
+            return None
+        hs = torch.cat(hidden) if len(hidden) > 1 else hidden[0]
+        return self.model.lm_logits(self.bufs, hs)
+
+    def _sync_staging(self) -> None:
+        if self._staging_inflight and self.device.type == "cuda":
+            torch.cuda.current_stream().synchronize()
+            self._staging_inflight = False
+
+    def _ragged_forward(self, rows: List[Tuple[Sequence_, int]], want: Sequence[int] = ()) -> Optional[torch.Tensor]:
+        """One eager forward of ragged rows (more than the step buffers hold): the decode-mode
+        model forward over scratch buffers sized for them; attention in 64-row slices, or by the
+        model's own row plan.  Returns the final hidden rows at the places ``want``."""
         n = len(rows)
         bs = self.block_size
         pending: Dict[int, int] = {}
@@ -620,26 +694,47 @@ class LLMEngine:
         if self.bufs.table_dirty:
             self.bufs.block_table.copy_(self.bufs.h_table, non_blocking=self.device.type == "cuda")
             self.bufs.table_dirty = False
+            self._staging_inflight = self.device.type == "cuda"  # (the copy reads the pinned table)
         dev, m = self.device, self.model
         i32 = dict(dtype=torch.int32)
         meta = torch.tensor([toks, poss, sids, [p + 1 for p in poss]], **i32)
         if dev.type == "cuda":
             meta = meta.pin_memory().to(dev, non_blocking=True)
-        d = m.cfg.hidden
         scratch = SimpleNamespace(
             tokens=meta[0], positions=meta[1], seq_ids=meta[2], ctx_lens=meta[3],
             slots=torch.tensor(slots, dtype=torch.int64).to(dev, non_blocking=dev.type == "cuda"),
-            block_table=self.bufs.block_table, max_ctx=self.bufs.max_ctx,
-            hidden=torch.empty(n, d, dtype=m.dtype, device=dev),
-            q=torch.empty(n, m.nq * m.hd, dtype=m.dtype, device=dev),
-            attn=torch.empty(n, m.nq * m.hd, dtype=m.dtype, device=dev),
-            act=torch.empty(n, getattr(m, "F", getattr(m.cfg, "ffn", d)), dtype=m.dtype, device=dev),
-            part_o=self.bufs.part_o, part_ml=self.bufs.part_ml, attn_cnt=self.bufs.attn_cnt,
-            logits_local=self.bufs.logits_local, logits=self.bufs.logits,
-            flash=self._ragged_flash(sids, poss) if dev.type == "cuda" else None)
-        m.forward(scratch, n, self.kv, head=False)
+            block_table=self.bufs.block_table, max_ctx=self.bufs.max_ctx, logits_local=self.bufs.logits_local)
+        if hasattr(m, "row_buffers"):
+            vars(scratch).update(m.row_buffers(n, self.bufs.max_ctx), talk=getattr(self.bufs, "talk", None),
+                                 plan=m.plan_rows(self._runs(sids, poss)))
+        else:
+            d = m.cfg.hidden
+            vars(scratch).update(
+                hidden=torch.empty(n, d, dtype=m.dtype, device=dev),
+                q=torch.empty(n, m.nq * m.hd, dtype=m.dtype, device=dev),
+                attn=torch.empty(n, m.nq * m.hd, dtype=m.dtype, device=dev),
+                act=torch.empty(n, getattr(m, "F", getattr(m.cfg, "ffn", d)), dtype=m.dtype, device=dev),
+                part_o=self.bufs.part_o, part_ml=self.bufs.part_ml, attn_cnt=self.bufs.attn_cnt,
+                logits=self.bufs.logits, flash=self._ragged_flash(sids, poss) if dev.type == "cuda" else None)
+        hs = m.forward(scratch, n, self.kv, head=False)
         for sid, ln in pending.items():
             self.seqs[sid].n_computed = ln
+        self.stats["steps"] += 1
+        self.stats["rows"] += n
+        if not want:
+            return None
+        return hs.index_select(0, torch.tensor(list(want), dtype=torch.int64, device=hs.device))
+
+    @staticmethod
+    def _runs(sids: List[int], poss: List[int]) -> List[Tuple[int, int]]:
+        """(first row, rows) of the runs of one sequence at consecutive positions."""
+        runs: List[List[int]] = []
+        for i, (sid, pos) in enumerate(zip(sids, poss)):
+            if runs and sids[i - 1] == sid and pos == poss[i - 1] + 1:
+                runs[-1][1] += 1
+            else:
+                runs.append([i, 1])
+        return [(a, n) for a, n in runs]
 
     def _ragged_flash(self, sids: List[int], poss: List[int]) -> Optional[SimpleNamespace]:
         """Ragged rows made of whole per-sequence runs (consecutive positions, one run per
@@ -687,6 +782,11 @@ class LLMEngine:
             if n <= self.bufs.max_rows:
                 toks = seq.tokens[start : start + n]
                 logits = self.run_rows([(seq, t) for t in toks], logits_for=[n - 1])
+                continue
+            if hasattr(self.model, "row_buffers"):
+                self._sync_staging()
+                hs = self._ragged_forward([(seq, t) for t in seq.tokens[start : start + n]], [n - 1])
+                logits = self.model.lm_logits(self.bufs, hs)
                 continue
             self._ensure_blocks(seq, start + n)
             if self.bufs.table_dirty:

@@ -13,9 +13,20 @@ from __future__ import annotations
 
 import hashlib
 from collections import OrderedDict
+from dataclasses import dataclass
 from typing import Dict, List, Optional, Sequence, Tuple
 
 import torch
+
+
+@dataclass(frozen=True)
+class CacheLayer:
+    """What one layer keeps of a sequence: paged keys and values, and ``state`` f32 channels."""
+    n_kv_heads: int
+    k_dim: int
+    v_dim: int
+    v_transposed: bool = False
+    state: int = 0
 
 
 class PagedKVCache:
@@ -28,6 +39,30 @@ class PagedKVCache:
         shape = (n_layers, num_blocks, n_kv_heads, block_size, head_dim)
         self.k = torch.zeros(shape, dtype=dtype, device=device)
         self.v = torch.zeros(shape, dtype=dtype, device=device)
+
+    @classmethod
+    def from_layers(cls, layers: Sequence["CacheLayer"], block_size: int, num_blocks: int, n_slots: int, device="cpu",
+                    dtype=torch.bfloat16) -> "PagedKVCache":
+        """A cache whose layers differ: ``k[layer]`` / ``v[layer]`` by each layer's own sizes (v
+        ``[num_blocks, n_kv_heads, v_dim, block_size]`` when v_transposed) and ``state[layer]``
+        ``[n_slots, channels]`` f32 recurrent state, one row per live sequence (its block-table row).
+        State is not cleared when a slot is given back: a sequence's first token starts from zero."""
+        self = cls.__new__(cls)
+        self.n_layers, self.block_size, self.num_blocks = len(layers), block_size, num_blocks
+        self.layers = tuple(layers)
+
+        def pages(L, dim, transposed):
+            shape = (num_blocks, L.n_kv_heads) + ((dim, block_size) if transposed else (block_size, dim))
+            return torch.zeros(shape, dtype=dtype, device=device)
+
+        self.k = [pages(L, L.k_dim, False) for L in layers]
+        self.v = [pages(L, L.v_dim, L.v_transposed) for L in layers]
+        self.state = [torch.zeros(n_slots, L.state, dtype=torch.float32, device=device) for L in layers]
+        return self
+
+    @staticmethod
+    def layer_bytes_per_block(layers: Sequence["CacheLayer"], block_size: int, elem: int = 2) -> int:
+        return sum(L.n_kv_heads * block_size * (L.k_dim + L.v_dim) * elem for L in layers)
 
     @staticmethod
     def bytes_per_block(n_layers: int, n_kv_heads: int, head_dim: int, block_size: int, elem: int = 2) -> int:

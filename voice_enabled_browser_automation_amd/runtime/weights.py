@@ -58,17 +58,21 @@ class LazySafetensors:
 
 
 def load_llm(name: str, *, device, tp=None, seed: int = 0, weights_path: Optional[str] = None,
-             wdtype: str = "bf16"):
-    """Build the intent LLM of preset ``name`` (random init, or from ``weights_path``); ``wdtype``
-    "fp8" quantises the Llama projections to OCP e4m3 on load."""
-    from ..models.config import GPT2Config, get_config
+             wdtype: str = "bf16", dtype: Optional[torch.dtype] = None):
+    """Build the LLM of preset ``name`` or of the checkpoint folder ``name`` (config.json +
+    safetensors): random init, or the folder's / ``weights_path``'s tensors.  ``wdtype`` "fp8" quantises
+    the Llama projections to OCP e4m3 on load; ``dtype`` overrides the compute dtype (torch.float32:
+    everything in 32-bit, for the models that have it)."""
+    from ..models import model_class
+    from ..models.config import GPT2Config, KabanexConfig, get_config
 
     cfg = get_config(name)
+    if weights_path is None and os.path.isdir(name):
+        weights_path = name
     w = LazySafetensors(weights_path) if weights_path else None
-    if isinstance(cfg, GPT2Config):
-        from ..models.gpt2 import GPT2Model
-
-        return GPT2Model(cfg, device=device, seed=seed, weights=w)
-    from ..models.llama import LlamaModel
-
-    return LlamaModel(cfg, device=device, tp=tp, seed=seed, weights=w, wdtype=wdtype)
+    cls = model_class(cfg)
+    if isinstance(cfg, (GPT2Config, KabanexConfig)):
+        return cls(cfg, device=device, seed=seed, weights=w, dtype=dtype)
+    if dtype not in (None, torch.bfloat16):
+        raise NotImplementedError(f"{cls.__name__} has no {dtype} kernels")
+    return cls(cfg, device=device, tp=tp, seed=seed, weights=w, wdtype=wdtype)

@@ -128,7 +128,7 @@ class Settings(BaseModel):
     VWA_SPIN_WAIT: bool = Field(True, description="wait for a step's tokens by polling the pinned readback")
     VWA_ZERO_COPY: bool = Field(True, description="grammar masks written straight into pinned step memory")
     VWA_ASR_DEVICE_LOOP: bool = Field(True, description="single-session Whisper greedy loop resident on the GPU")
-    VWA_CHAIN: bool = Field(True, description="chained Llama decode layer (skinny_stream.hip chain_kernel)")
+    VWA_CHAIN: bool = Field(True, description="chained Llama decode layer (chain.hip chain_kernel)")
     VWA_CHAIN_ATTN: bool = Field(True, description="decode attention as the chained launch's phase 0")
     VWA_CHAIN_MAX_ROWS: int = Field(4, description="rows per step the chained launch takes")
     VWA_CHAIN_TP: bool = Field(True, description="chained launch with in-launch TP all-reduce rounds")
@@ -138,7 +138,7 @@ class Settings(BaseModel):
     VWA_ASR_PERSIST: bool = Field(True, description="one-row Whisper decode steps (every width, tiny .. large) as ONE persistent launch: embedding, every decoder layer, LM head and, in the device loop, argmax + advance (csrc/kernels/whisper_dec.hip); needs every CU free: off when the GPU is shared with a persistent brain launch")
     VWA_CHAIN_GRID_DIV: Optional[str] = Field(None, description="chained launch on CUs / k workgroups (shared GPU)")
     VWA_CHAIN_PLAN: bool = Field(True, description="chained attention: layer 0 writes the step's work plan, layers 1.. read it")
-    VWA_CHAIN_MULTI: bool = Field(True, description="chained decode: all layers in ONE launch (skinny_stream.hip chain_kernel MULTI)")
+    VWA_CHAIN_MULTI: bool = Field(True, description="chained decode: all layers in ONE launch (chain.hip chain_kernel MULTI)")
     VWA_CHAIN_BAR_MODE: int = Field(2, description="chained launches' grid barrier: 2 two-level tickets + scalar polls (default), 4 no-return arrivals + polled sum of the 8 group counters")
     VWA_CHAIN_SCHED: Optional[str] = Field(None, description="DIAGNOSTIC: chained schedule override name=value,...")
     VWA_GEMM_QKV: bool = Field(True, description="> 16-row QKV: rotary + KV write in the tiled GEMM epilogue")
