@@ -147,6 +147,14 @@ def _build_kernels(force: bool, jobs: int, core: bool) -> str:
     return target
 
 
+def ensure_kernels(core: bool = True) -> None:
+    """Build a kernel library if this checkout has none that serves: the core one is enough for models
+    without chained or persistent launches (``core``)."""
+    if os.path.exists(KERNEL_SO) or (core and os.path.exists(CORE_SO)):
+        return
+    build_kernels(core=core)
+
+
 def build_native(force: bool = False) -> str:
     """CPU runtime library (grammar engine + block manager) -- g++ / pybind11."""
     srcs = sorted(glob.glob(os.path.join(CSRC, "runtime", "*.cpp")))
