@@ -23,9 +23,10 @@ def rotate(x, base, dims, first=0):
     """x [n, heads, dim]: pairs (i, i + dims/2) of the first ``dims`` dimensions turned by p * base^(-2i/dims)."""
     out = x.clone()
     half = dims // 2
-    for p in range(x.shape[0]):
-        for i in range(half):
-            a = (first + p) * base ** (-2.0 * i / dims)
+    for i in range(half):
+        f = base ** (-2.0 * i / dims)
+        for p in range(x.shape[0]):
+            a = (first + p) * f
             c, s = math.cos(a), math.sin(a)
             u, v = x[p, :, i], x[p, :, i + half]
             out[p, :, i] = u * c - v * s
@@ -129,3 +130,60 @@ def forward(cfg, weights, tokens, layers=False):
         res.append(x)
     logits = layer_norm(x, w["final.norm"], w["final.norm.b"], eps) @ w["head"].T
     return (logits, res) if layers else logits
+
+
+# ----------------------------------------------------------------------------- test models
+def layer_config(heads, kv_heads, dim, vdim, rot_dims, window, keep, width, ff, base=10000.0, scale=None, ls=0.9, rs=0.6):
+    return {"type": "parallel",
+            "mixer": {"left": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim,
+                               "mask": {"size": window, "keep_first": keep}, "rot": {"base": base, "dims": rot_dims},
+                               "scale": dim ** -0.5 if scale is None else scale},
+                      "right": {"width": width}, "left_scale": ls, "right_scale": rs},
+            "mlp": {"kind": "dense", "ff": ff} if ff else None}
+
+
+def model_config(width, vocab, layers, eps=1e-5):
+    return {"architecture": "Kabanex", "vocab": vocab, "width": width, "norm": {"eps": eps}, "layers": layers}
+
+
+def random_weights(cfg, seed=0, dtype=torch.bfloat16):
+    """Weights that keep every mechanism visible: spread-out scores, strong mixing and gates, slow and
+    fast recurrent channels."""
+    gen = torch.Generator().manual_seed(seed)
+    r = lambda *s, std=1.0: (torch.randn(*s, generator=gen) * std).to(dtype)  # noqa: E731
+    d = cfg["width"]
+    w = {"embed": r(cfg["vocab"], d), "final.norm": (1 + r(d, std=0.2).float()).to(dtype), "final.norm.b": r(d, std=0.2),
+         "head": r(cfg["vocab"], d, std=d ** -0.5)}
+    for i, L in enumerate(cfg["layers"]):
+        a, W, p = L["mixer"]["left"], L["mixer"]["right"]["width"], f"l{i}."
+        w[p + "norm1"], w[p + "norm1.b"] = (1 + r(d, std=0.2).float()).to(dtype), r(d, std=0.2)
+        H, G, m = a["heads"], a["kv_heads"], p + "mix."
+        s = d ** -0.5
+        w.update({m + "left.q": r(H * a["dim"], d, std=1.6 * s), m + "left.k": r(G * a["dim"], d, std=1.6 * s),
+                  m + "left.v": r(G * a["vdim"], d, std=s), m + "left.talk": (torch.eye(H) + r(H, H, std=0.4).float()).to(dtype),
+                  m + "left.g": r(H, d, std=s), m + "left.o": r(d, H * a["vdim"], std=(H * a["vdim"]) ** -0.5),
+                  m + "right.z": r(W, d, std=2 * s), m + "right.z.b": r(W, std=3.0), m + "right.x": r(W, d, std=s),
+                  m + "right.x.b": r(W, std=0.3), m + "right.g": r(W, d, std=s), m + "right.o": r(d, W, std=W ** -0.5)})
+        if L["mlp"]:
+            f = L["mlp"]["ff"]
+            w.update({p + "mlp.up": r(f, d, std=s), p + "mlp.down": r(d, f, std=f ** -0.5)})
+    return w
+
+
+def save_model(path, cfg, weights):
+    import json
+    import os
+
+    from safetensors.torch import save_file
+
+    os.makedirs(path, exist_ok=True)
+    with open(os.path.join(path, "config.json"), "w") as fh:
+        json.dump(cfg, fh)
+    save_file({k: v.contiguous() for k, v in weights.items()}, os.path.join(path, "model.safetensors"))
+
+
+def logit_error(got, want):
+    """Per row: RMS over the vocabulary of the difference (its mean taken off), relative to the logits' spread."""
+    d = got.double().cpu() - want
+    d = d - d.mean(-1, keepdim=True)
+    return d.pow(2).mean(-1).sqrt() / want.std()
