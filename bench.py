@@ -199,10 +199,19 @@ def main():
                          "intent decoding); reported under 'concurrent', outside the headline value")
     ap.add_argument("--dtype", default=knob("VWA_DTYPE"), choices=("bf16", "fp8"),
                     help="LLM weight dtype: bf16 (headline config) or fp8 (W8A8 on the fp8 MFMA, config 5)")
+    ap.add_argument("--design", choices=("kabanex",), help="instead of the headline: prefill / decode throughput of a model "
+                    "design beside Llama layers of equal size (tools/design_bench.py)")
+    ap.add_argument("--design-size", default="s1,s2,s4")
+    ap.add_argument("--design-only", choices=("kabanex", "llama"))
+    ap.add_argument("--design-rounds", type=int, default=3)
     ap.add_argument("--no-graphs", action="store_true")
     ap.add_argument("--verbose", action="store_true")
     args = ap.parse_args()
 
+    if args.design:
+        from tools.design_bench import run as design_run
+
+        return design_run(args)
     env_world = os.environ.get("WORLD_SIZE")
     if env_world is None and args.gpus > 1:
         sys.exit(spawn_ranks(args.gpus))

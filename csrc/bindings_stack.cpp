@@ -239,8 +239,8 @@ void talk_attention(Tensor q, Tensor k, Tensor v, Tensor table, Tensor positions
 }
 
 void talk_prefill(Tensor q, Tensor k, Tensor v, Tensor table, Tensor positions, Tensor seq_ids, Tensor slots, Tensor tiles,
-                  int64_t H, double scale, int64_t window, int64_t keep, Tensor talk_pad, c10::optional<Tensor> gate,
-                  double out_scale, int64_t max_ctx, Tensor out) {
+                  int64_t H, double scale, int64_t window, int64_t keep, Tensor talk_frag, c10::optional<Tensor> gate,
+                  double out_scale, int64_t max_ctx, int64_t splits, Tensor lse, Tensor part, Tensor tickets, Tensor out) {
   c10::DeviceGuard g(q.device());
   TalkPrefillParams p{};
   p.a = attn_params(q, k, v, table, positions, seq_ids, slots, q.size(0), H, scale, window, keep, c10::nullopt, gate, out_scale,
@@ -250,14 +250,21 @@ void talk_prefill(Tensor q, Tensor k, Tensor v, Tensor table, Tensor positions, 
   TORCH_CHECK(tiles.dim() == 2 && tiles.size(1) == 2 && tiles.size(0) >= 1, "tiles int32 [n, 2]");
   p.tiles = i32p(tiles, tiles.numel(), "tiles");
   p.n_tiles = (int)tiles.size(0);
-  auto up = [](int64_t n) {
-    int64_t r = 1;
-    while (r < n) r <<= 1;
-    return r;
-  };
-  p.GP = (int)up(p.a.G);
-  p.RP = (int)up(H / p.a.G);
-  p.talk_pad = f32p(talk_pad, (int64_t)p.GP * p.RP * p.GP * p.RP, "talk_pad");
+  TORCH_CHECK(talk_frag.is_cuda() && talk_frag.scalar_type() == at::kBFloat16 && talk_frag.is_contiguous() &&
+                  talk_frag.numel() >= (H > 16 ? 1024 : 512),
+              "talk_frag bf16 [tiles, 64, 8] (ops.talk_fragment)");
+  check_aligned(talk_frag, "talk_frag");
+  p.talk_frag = bfp(talk_frag);
+  p.lse = f32p(lse, q.size(0) * H, "lse");
+  p.splits = (int)splits;
+  if (splits > 1) {
+    const int64_t per = vwa_talk_prefill_part((int)H, p.a.G, p.a.dk, p.a.dv);
+    TORCH_CHECK(per > 0, "talk_prefill does not take these sizes");
+    p.part = f32p(part, p.n_tiles * splits * per, "part");
+    check_aligned(part, "part");
+    i32p(tickets, p.n_tiles, "tickets");
+    p.tickets = tickets.data_ptr<int>();
+  }
   TORCH_CHECK((reinterpret_cast<uintptr_t>(out.data_ptr()) & 7) == 0, "out rows must be 8-byte aligned");
   check_rc(vwa_talk_prefill(&p, cur_stream(q)), "talk_prefill");
 }
@@ -317,8 +324,8 @@ void bind_stack(py::module_& m) {
   m.def("embedding_f32", &embedding_f32);
   m.def("qkv_cache", &qkv_cache);
   m.def("talk_chunks", &talk_chunks);
-  m.def("talk_prefill_fits", [](int64_t H, int64_t G, int64_t dk, int64_t dv) {
-    return vwa_talk_prefill_fits((int)H, (int)G, (int)dk, (int)dv) != 0;
+  m.def("talk_prefill_part", [](int64_t H, int64_t G, int64_t dk, int64_t dv) {
+    return vwa_talk_prefill_part((int)H, (int)G, (int)dk, (int)dv);
   });
   m.def("talk_attention", &talk_attention, py::arg("q"), py::arg("k"), py::arg("v"), py::arg("table"), py::arg("positions"),
         py::arg("seq_ids"), py::arg("slots"), py::arg("row_list"), py::arg("n_rows"), py::arg("H"), py::arg("scale"),
@@ -326,7 +333,8 @@ void bind_stack(py::module_& m) {
         py::arg("s"), py::arg("stat"), py::arg("part"), py::arg("counters"), py::arg("out"));
   m.def("talk_prefill", &talk_prefill, py::arg("q"), py::arg("k"), py::arg("v"), py::arg("table"), py::arg("positions"),
         py::arg("seq_ids"), py::arg("slots"), py::arg("tiles"), py::arg("H"), py::arg("scale"), py::arg("window"),
-        py::arg("keep"), py::arg("talk_pad"), py::arg("gate"), py::arg("out_scale"), py::arg("max_ctx"), py::arg("out"));
+        py::arg("keep"), py::arg("talk_frag"), py::arg("gate"), py::arg("out_scale"), py::arg("max_ctx"), py::arg("splits"),
+        py::arg("lse"), py::arg("part"), py::arg("tickets"), py::arg("out"));
   m.def("mingru", &mingru, py::arg("z"), py::arg("x"), py::arg("g"), py::arg("zb"), py::arg("xb"), py::arg("seq_ids"),
         py::arg("positions"), py::arg("slots"), py::arg("state"), py::arg("out_scale"), py::arg("out"),
         py::arg("chunks") = py::none(), py::arg("scratch") = py::none());

@@ -59,8 +59,15 @@ struct TalkPrefillParams {
   TalkAttnParams a;                 // (row_list / nch / s / stat / part / counters unused)
   const int* tiles;                 // [n_tiles][2]: first row, rows (1..16) -- one sequence, consecutive positions
   int n_tiles;
-  const float* talk_pad;            // [GP * RP][GP * RP] talk in the padded head order (identity if not mixed)
-  int GP, RP;                       // kv heads and q heads per kv head, padded to powers of two
+  // talk (identity if not mixed) as the MFMA A operand over the padded heads h = c * RP + r (kv heads GP
+  // and query heads per kv head RP rounded up to powers of two, HT = GP * RP): bf16 [HT > 16 ? 2 : 1]
+  // [64 lanes][8], lane (row rl, group b), element e: talk[16 mt + rl][head of k], k = 8 b + e -- HT 32:
+  // head k; 16: k mod 16; 8: k mod 8 for k < 16, else 0; <= 4: k mod 4 for k < 8, else 0
+  const uint16_t* talk_frag;
+  float* lse;                       // [rows of q][H] scratch
+  int splits;                       // workgroups per tile over its keys
+  float* part;                      // [n_tiles][splits][vwa_talk_prefill_part floats] (splits > 1)
+  int* tickets;                     // [n_tiles], zero between launches (splits > 1)
 };
 
 // Gated recurrence of one layer over a step's rows: z = sigmoid(zp + zb), u = xp + xb,
@@ -92,7 +99,8 @@ int vwa_embedding_f32(const int* ids, const void* table, int ld, float* out, int
 int vwa_qkv_cache(const QkvCacheParams* p, hipStream_t st);
 int vwa_talk_attention(const TalkAttnParams* p, hipStream_t st);
 int vwa_talk_prefill(const TalkPrefillParams* p, hipStream_t st);
-int vwa_talk_prefill_fits(int H, int G, int dk, int dv);  // 1 if vwa_talk_prefill takes these sizes
+// partial floats per (tile, split) of vwa_talk_prefill, < 0 if it does not take these sizes
+int64_t vwa_talk_prefill_part(int H, int G, int dk, int dv);
 int vwa_mingru_rows(const MinGruParams* p, hipStream_t st);
 int vwa_mingru_scan(const MinGruParams* p, hipStream_t st);
 #ifdef __cplusplus

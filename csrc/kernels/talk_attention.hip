@@ -15,10 +15,10 @@
 //     of every head, mixes the chunk's weights into LDS in B-operand order and multiplies by V^T,
 //     which the cache stores transposed (its A operand, no staging).  Chunks of a row are added in
 //     chunk order by the last-arriving workgroup (sc1 hand-off + ticket, as decode attention).
-//  2) prefill form (bf16): a workgroup per 16 consecutive queries, its waves owning key tiles in the
-//     score pass (all heads of a tile in one wave's registers: the mixing is lane-local, talk read
-//     through scalar loads) and (kv head, 16 value columns) tiles in the value pass; the mixed weights
-//     pass between them through LDS in B-operand order.
+//  2) prefill form (bf16), per 16 consecutive queries: launch A reduces the scores to log-sum-exps;
+//     launch B recomputes them, a wave holding every head of its key tile, mixes the heads on the MFMA
+//     and hands the mixed weights through LDS (B-operand order) to the waves' (kv head, 16 value
+//     columns) tiles.
 #include "common.h"
 #include "mq_attention.h"
 #include "stack_kernels.h"
@@ -297,221 +297,404 @@ __global__ __launch_bounds__(256) void talk_mix_kernel(TalkAttnParams p) {
 
 // ------------------------------------------------------------------------------------------ prefill form
 constexpr int kTab = 1024;                  // block-table entries kept in LDS
-constexpr int kMaxKS = 8;                   // 32-wide steps over the q / k dimensions (dk <= 256)
+constexpr int kNone = -1;
 
-// GP, RP: kv heads and query heads per kv head in the padded head order h = c * RP + r
-// NV: (kv head, 16 value columns) tiles per wave; NW waves; QL: query fragments in LDS (else read
-// from the q rows, L1 / L2)
-template <int GP, int RP, int NV, int NW, bool QL>
+VWA_DEVICE void st_sc1_x4(__amdgpu_buffer_rsrc_t r, int off, const f32x4& v) {
+  __builtin_amdgcn_raw_buffer_store_b128(__builtin_bit_cast(u32x4, v), r, off, 0, 16);
+}
+VWA_DEVICE f32x4 ld_sc1_x4(__amdgpu_buffer_rsrc_t r, int off) {
+  return __builtin_bit_cast(f32x4, __builtin_amdgcn_raw_buffer_load_b128(r, off, 0, 16));
+}
+
+// every key of the tile visible to every query p0 .. p1 (no per-key masks needed)
+VWA_DEVICE bool all_visible(int p0, int p1, int key0, int window, int keep) {
+  return key0 + kTile - 1 <= p0 && (window <= 0 || p1 - key0 < window || key0 + kTile - 1 < keep);
+}
+
+// Pass 1: log2-sum-exp of every (query, head): a workgroup per (16 queries, kv head, RB query heads),
+// the query fragments in registers, its 4 waves taking every fourth key tile (next tile's keys in
+// flight).  lse[row][H] = max + log2(sum) of the scaled scores in log2 units.
+template <int RB, int KSN>
+__global__ __launch_bounds__(256) void talk_lse_kernel(TalkPrefillParams pp) {
+  const TalkAttnParams& p = pp.a;
+  __shared__ float red[4][RB][16][2];
+  const int lane = lane_id(), w = threadIdx.x >> 6, rl = lane & 15, b = lane >> 4;
+  const int lt = xcd_remap((int)blockIdx.x, pp.n_tiles * p.G);  // (a kv head's tiles share an XCD's L2)
+  const int c = lt / pp.n_tiles, tile = lt % pp.n_tiles;
+  const int row0 = pp.tiles[2 * tile], nq = pp.tiles[2 * tile + 1];
+  const int R = p.H / p.G, r0 = blockIdx.y * RB, nr = min(RB, R - r0), nst = p.dk >> 5;
+  const int pos0 = p.positions[row0], pos1 = pos0 + nq - 1, seq = p.seq_ids[row0];
+  const int qrow = row0 + min(rl, nq - 1), qpos = pos0 + min(rl, nq - 1);
+  const Vis v = vis_tiles(pos0, pos1, p.window, p.keep);
+  const float sl2 = p.scale * kLog2e;
+  const int* gtab = p.block_table + (int64_t)seq * p.table_stride;
+  uint4 qf[RB][KSN];
+#pragma unroll
+  for (int r = 0; r < RB; ++r)
+#pragma unroll
+    for (int s = 0; s < KSN; ++s)
+      if (s < nst)
+        qf[r][s] = ld128(reinterpret_cast<const u16*>(p.q) + (size_t)qrow * p.ldq + (size_t)(c * R + r0 + min(r, nr - 1)) * p.dk +
+                         b * 8 + s * 32);
+  auto load_k = [&](uint4 (&kf)[KSN], int t) {
+    const int key0 = tile_of(v, t) * kTile;
+    const u16* kp = reinterpret_cast<const u16*>(p.k) + (int64_t)gtab[key0 / p.block_size] * p.k_sb + (int64_t)c * p.k_sh +
+                    (int64_t)(key0 % p.block_size + rl) * p.dk + b * 8;
+#pragma unroll
+    for (int s = 0; s < KSN; ++s)
+      if (s < nst) kf[s] = ld128(kp + s * 32);
+  };
+  float m[RB], l[RB];
+#pragma unroll
+  for (int r = 0; r < RB; ++r) {
+    m[r] = -1e30f;
+    l[r] = 0.f;
+  }
+  auto add_tile = [&](const uint4 (&kf)[KSN], int t) {
+    const int key0 = tile_of(v, t) * kTile;
+    const bool full = all_visible(pos0, pos1, key0, p.window, p.keep);
+    bool vis[4] = {true, true, true, true};
+    if (!full) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) vis[i] = sees(qpos, key0 + 4 * b + i, p.window, p.keep);
+    }
+#pragma unroll
+    for (int r = 0; r < RB; ++r) {
+      f32x4 a = {};
+#pragma unroll
+      for (int s = 0; s < KSN; ++s)
+        if (s < nst) a = mfma16(as_bf16x8(kf[s]), as_bf16x8(qf[r][s]), a);
+      float s[4], mn = m[r];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        s[i] = vis[i] ? a[i] * sl2 : -1e30f;
+        mn = fmaxf(mn, s[i]);
+      }
+      float x = l[r] * __builtin_amdgcn_exp2f(m[r] - mn);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) x += vis[i] ? __builtin_amdgcn_exp2f(s[i] - mn) : 0.f;
+      l[r] = x;
+      m[r] = mn;
+    }
+  };
+  uint4 ka[KSN], kb[KSN];
+  if (w < v.n) load_k(ka, w);
+  for (int t = w; t < v.n; t += 8) {
+    if (t + 4 < v.n) load_k(kb, t + 4);
+    add_tile(ka, t);
+    if (t + 4 >= v.n) break;
+    if (t + 8 < v.n) load_k(ka, t + 8);
+    add_tile(kb, t + 4);
+  }
+#pragma unroll
+  for (int r = 0; r < RB; ++r) {
+#pragma unroll
+    for (int o = 16; o < 64; o <<= 1) {
+      const float mo = __shfl_xor(m[r], o, 64), lo = __shfl_xor(l[r], o, 64), mn = fmaxf(m[r], mo);
+      l[r] = l[r] * __builtin_amdgcn_exp2f(m[r] - mn) + lo * __builtin_amdgcn_exp2f(mo - mn);
+      m[r] = mn;
+    }
+    if (b == 0) {
+      red[w][r][rl][0] = m[r];
+      red[w][r][rl][1] = l[r];
+    }
+  }
+  __syncthreads();
+  const int r = threadIdx.x >> 4, q = threadIdx.x & 15;
+  if (r >= nr || q >= nq) return;
+  float mm = -1e30f, ll = 0.f;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) mm = fmaxf(mm, red[i][r][q][0]);
+#pragma unroll
+  for (int i = 0; i < 4; ++i) ll += red[i][r][q][1] * __builtin_amdgcn_exp2f(red[i][r][q][0] - mm);
+  pp.lse[(size_t)(row0 + q) * p.H + c * R + r0 + r] = mm + __log2f(ll);
+}
+
+// rows [0 1 2 3] of 16 lanes of four registers, transposed: out_b row b' = in_b' row b
+VWA_DEVICE void transpose4(unsigned& a, unsigned& b, unsigned& c, unsigned& d) {
+  const auto r = __builtin_amdgcn_permlane32_swap(a, c, false, false);
+  const auto s = __builtin_amdgcn_permlane32_swap(b, d, false, false);
+  const auto x = __builtin_amdgcn_permlane16_swap(r[0], s[0], false, false);
+  const auto y = __builtin_amdgcn_permlane16_swap(r[1], s[1], false, false);
+  a = x[0];
+  b = x[1];
+  c = y[0];
+  d = y[1];
+}
+
+// Pass 2.  GP, RP: kv heads and query heads per kv head in the padded head order h = c * RP + r; NV: (kv
+// head, 16 value columns) tiles per wave; NW waves; KSN: 32-wide steps over the q / k dimensions.
+// Heads are mixed on the MFMA: a weight x = hi + lo (two bf16, 16 mantissa bits) is one B operand with
+// k = (hi | lo, head) against the talk matrix (bf16 as stored) repeated for both halves; the lanes hold
+// every head of their own (query, key), so the operand is a 4 x 4 transpose of 16-lane groups.
+// A tile's key rows enter the score product in the order 4 i + b (row 4 b + i), so the four results of one
+// key element i are four consecutive keys.
+// The tile's keys may be split over workgroups (blockIdx.y): their sums are added in order by the last
+// one to finish.
+template <int GP, int RP, int NV, int NW, int KSN>
 struct PrefillCfg {
   static constexpr int HT = GP * RP, KEYS = NW * kTile, KG = KEYS / 32;
+  static constexpr int MT = HT > 16 ? 2 : 1;                         // 16-row tiles of the mixed heads
+  static constexpr int KM = HT > 16 ? 2 : 1;                         // 32-deep steps of the mixing
   static constexpr int P_BYTES = HT * KEYS * 16 * 2;                 // mixed weights
-  static constexpr int RED_BYTES = NW * HT * 16 * 2 * 4;             // statistics of the waves (before P is used)
-  static constexpr int PR = P_BYTES > RED_BYTES ? P_BYTES : RED_BYTES;
-  static size_t lds(int dk) { return PR + HT * 16 * 4 + kTab * 4 + (QL ? (size_t)HT * dk * 16 * 2 : 0); }
+  static constexpr bool QL = HT * KSN <= 64;                         // query fragments in LDS (else L1 / L2)
+  static size_t lds(int dk) { return P_BYTES + HT * 16 * 4 + kTab * 4 + (QL ? (size_t)HT * dk * 16 * 2 : 0); }
 };
 
-template <int GP, int RP, int NV, int NW, bool QL>
+template <int GP, int RP, int NV, int NW, int KSN>
 __global__ __launch_bounds__(NW * 64) void talk_prefill_kernel(TalkPrefillParams pp) {
-  using C = PrefillCfg<GP, RP, NV, NW, QL>;
-  constexpr int HT = C::HT;
+  using C = PrefillCfg<GP, RP, NV, NW, KSN>;
+  constexpr int HT = C::HT, KG = C::KG, HX = HT < 4 ? 4 : HT;
+  constexpr int HS = KG * 4 * 16 * 16;                               // bytes of a head's mixed weights
   const TalkAttnParams& p = pp.a;
   extern __shared__ __attribute__((aligned(16))) char smem[];
-  char* pm = smem;                                                   // [HT][KG][4][16 q][16 B]
-  float* red = reinterpret_cast<float*>(smem);                       // [NW][HT][16][2]
-  float* lse = reinterpret_cast<float*>(smem + C::PR);               // [HT][16]
+  __shared__ int s_last;
+  char* pm = smem;                                                   // [HT][KG][4][16 q][8 keys]
+  float* lse = reinterpret_cast<float*>(smem + C::P_BYTES);          // [HT][16]
   int* btab = reinterpret_cast<int*>(lse + HT * 16);
   uint4* qs = reinterpret_cast<uint4*>(btab + kTab);                 // [HT][dk / 32][64]
   const int lane = lane_id(), w = threadIdx.x >> 6, rl = lane & 15, b = lane >> 4;
   const int bt = xcd_remap((int)blockIdx.x, pp.n_tiles);
   const int row0 = pp.tiles[2 * bt], nq = pp.tiles[2 * bt + 1];
   const int R = p.H / p.G, nst = p.dk >> 5;
-  const int pos0 = p.positions[row0], seq = p.seq_ids[row0];
+  const int pos0 = p.positions[row0], pos1 = pos0 + nq - 1, seq = p.seq_ids[row0];
   const int qrow = row0 + min(rl, nq - 1), qpos = pos0 + min(rl, nq - 1);
-  const Vis v = vis_tiles(pos0, pos0 + nq - 1, p.window, p.keep);
+  const Vis v = vis_tiles(pos0, pos1, p.window, p.keep);
+  const int nit = (v.n + NW - 1) / NW, per = (nit + pp.splits - 1) / pp.splits;
+  const int nact = (nit + per - 1) / per;                            // splits with work
+  const int split = blockIdx.y;
+  if (split >= nact) return;
+  const int it0 = split * per, it1 = min(nit, it0 + per);
   const float sl2 = p.scale * kLog2e;
   const int* gtab = p.block_table + (int64_t)seq * p.table_stride;
-  const int nblk = (pos0 + nq - 1) / p.block_size + 1;
+  const int nblk = pos1 / p.block_size + 1;
   const bool tab = nblk <= kTab;
   if (tab)
     for (int i = threadIdx.x; i < nblk; i += NW * 64) btab[i] = gtab[i];
+  for (int u = threadIdx.x; u < p.H * 16; u += NW * 64) {
+    const int h = u >> 4, q = u & 15;
+    lse[((h / R) * RP + h % R) * 16 + q] = pp.lse[(size_t)(row0 + min(q, nq - 1)) * p.H + h];
+  }
   const u16* qp = reinterpret_cast<const u16*>(p.q) + (size_t)qrow * p.ldq + b * 8;
-  if constexpr (QL) {
+  if constexpr (C::QL) {
     for (int u = w; u < p.H * nst; u += NW) {
       const int h = u / nst, s = u % nst;
       qs[((size_t)((h / R) * RP + h % R) * nst + s) * 64 + lane] = ld128(qp + (size_t)h * p.dk + s * 32);
     }
   }
+  uint4 tf[C::MT];                                                   // talk, A operand (both mixing steps use it)
+#pragma unroll
+  for (int mt = 0; mt < C::MT; ++mt) tf[mt] = reinterpret_cast<const uint4*>(pp.talk_frag)[mt * 64 + lane];
   __syncthreads();
   auto blk_of = [&](int key) -> int64_t {
     const int i = key / p.block_size;
     return tab ? btab[i] : gtab[i];
   };
-  auto load_k = [&](uint4 (&kf)[kMaxKS], int c, int key0) {
+  auto load_k = [&](uint4 (&kf)[KSN], int c, int t) {
+    const int key0 = tile_of(v, t) * kTile;
     const u16* kp = reinterpret_cast<const u16*>(p.k) + blk_of(key0) * p.k_sb + (int64_t)c * p.k_sh +
-                    (int64_t)(key0 % p.block_size + rl) * p.dk + b * 8;
+                    (int64_t)(key0 % p.block_size + 4 * (rl & 3) + (rl >> 2)) * p.dk + b * 8;
 #pragma unroll
-    for (int s = 0; s < kMaxKS; ++s)
+    for (int s = 0; s < KSN; ++s)
       if (s < nst) kf[s] = ld128(kp + s * 32);
   };
-  // S^T tile of head (c, r): lane = query rl, keys 4b .. 4b+3
-  auto score = [&](const uint4 (&kf)[kMaxKS], int c, int r) {
-    f32x4 a = {};
+  const int ndv = p.dv >> 4, nvt = p.G * ndv, nvw = (nvt + NW - 1) / NW, v0 = w * nvw;
+  // value tiles of a wave in chunks of NC; a step is one chunk of one 32-key group
+  constexpr int NC = NV < 4 ? NV : 4, CH = NV / NC, STEPS = KG * CH;
+  static_assert(NV % NC == 0, "whole chunks");
+  auto load_v = [&](uint4 (&vf)[NC], int it, int step) {
+    const int key = tile_of(v, min(it * NW + 2 * (step / CH) + (b >> 1), v.n - 1)) * kTile;
+    const u16* vp = reinterpret_cast<const u16*>(p.v) + blk_of(key) * p.v_sb + (int64_t)rl * p.block_size +
+                    key % p.block_size + (b & 1) * 8;
 #pragma unroll
-    for (int s = 0; s < kMaxKS; ++s)
-      if (s < nst) {
-        uint4 qf;
-        if constexpr (QL) qf = qs[((size_t)(c * RP + r) * nst + s) * 64 + lane];
-        else qf = ld128(qp + (size_t)(c * R + r) * p.dk + s * 32);
-        a = mfma16(as_bf16x8(kf[s]), as_bf16x8(qf), a);
-      }
-    return a;
+    for (int n = 0; n < NC; ++n) {
+      const int idx = min(v0 + min((step % CH) * NC + n, nvw - 1), nvt - 1);
+      vf[n] = ld128(vp + (int64_t)(idx / ndv) * p.v_sh + (int64_t)(idx % ndv) * 16 * p.block_size);
+    }
   };
 
-  // ---- pass 1: per-lane running (max, sum) of every head over this wave's tiles
-  {
-    float m[HT], l[HT];
-#pragma unroll
-    for (int h = 0; h < HT; ++h) {
-      m[h] = -INFINITY;
-      l[h] = 0.f;
-    }
-    for (int t = w; t < v.n; t += NW) {
-      const int key0 = tile_of(v, t) * kTile;
-      bool vis[4];
-#pragma unroll
-      for (int i = 0; i < 4; ++i) vis[i] = sees(qpos, key0 + 4 * b + i, p.window, p.keep);
-#pragma unroll
-      for (int c = 0; c < GP; ++c) {
-        if (c >= p.G) break;
-        uint4 kf[kMaxKS];
-        load_k(kf, c, key0);
-#pragma unroll
-        for (int r = 0; r < RP; ++r) {
-          if (r >= R) break;
-          const f32x4 a = score(kf, c, r);
-          float s[4];
-#pragma unroll
-          for (int i = 0; i < 4; ++i) s[i] = vis[i] ? a[i] * sl2 : -INFINITY;
-          float& mh = m[c * RP + r];
-          const float mn = fmaxf(fmaxf(mh, fmaxf(s[0], s[1])), fmaxf(s[2], s[3]));
-          const float ms = mn == -INFINITY ? 0.f : mn;
-          float x = l[c * RP + r] * __builtin_amdgcn_exp2f(mh - ms);
-#pragma unroll
-          for (int i = 0; i < 4; ++i) x += __builtin_amdgcn_exp2f(s[i] - ms);
-          l[c * RP + r] = x;
-          mh = mn;
-        }
-      }
-    }
-#pragma unroll
-    for (int h = 0; h < HT; ++h) {
-#pragma unroll
-      for (int o = 16; o < 64; o <<= 1) {
-        const float mo = __shfl_xor(m[h], o, 64), lo = __shfl_xor(l[h], o, 64);
-        const float mn = fmaxf(m[h], mo), ms = mn == -INFINITY ? 0.f : mn;
-        l[h] = l[h] * __builtin_amdgcn_exp2f(m[h] - ms) + lo * __builtin_amdgcn_exp2f(mo - ms);
-        m[h] = mn;
-      }
-      if (b == 0) {
-        red[((w * HT + h) * 16 + rl) * 2] = m[h];
-        red[((w * HT + h) * 16 + rl) * 2 + 1] = l[h];
-      }
-    }
-  }
-  __syncthreads();
-  for (int u = threadIdx.x; u < HT * 16; u += NW * 64) {
-    float m = -INFINITY, s = 0.f;
-#pragma unroll
-    for (int i = 0; i < NW; ++i) m = fmaxf(m, red[(i * HT * 16 + u) * 2]);
-#pragma unroll
-    for (int i = 0; i < NW; ++i) {
-      const float li = red[(i * HT * 16 + u) * 2 + 1];
-      s += li > 0.f ? li * __builtin_amdgcn_exp2f(red[(i * HT * 16 + u) * 2] - m) : 0.f;
-    }
-    lse[u] = s > 0.f ? m + __log2f(s) : 0.f;
-  }
-  __syncthreads();
-
-  // ---- pass 2
   f32x4 acc[NV][RP] = {};
-  const int ndv = p.dv >> 4, nvt = p.G * ndv;
-  for (int it = 0; it * NW < v.n; ++it) {
+  uint4 kf[2][KSN];
+  if (it0 * NW + w < v.n) load_k(kf[0], 0, it0 * NW + w);
+  for (int it = it0; it < it1; ++it) {
     const int t = it * NW + w;
-    char* pw = pm + ((((w >> 1) * 4 + 2 * (w & 1) + (b >> 1)) * 16 + rl) * 16) + (b & 1) * 8;
-    constexpr int HS = C::KG * 4 * 16 * 16;  // bytes per head
+    char* pw = pm + (((w >> 1) * 4 + 2 * (w & 1)) * 16 + rl) * 16;   // [head][..][key chunk][q]
+    uint4 vf[2][NC];
     if (t < v.n) {
       const int key0 = tile_of(v, t) * kTile;
-      bool vis[4];
+      const bool full = all_visible(pos0, pos1, key0, p.window, p.keep);
+      bool vis[4] = {true, true, true, true};
+      if (!full) {
 #pragma unroll
-      for (int i = 0; i < 4; ++i) vis[i] = sees(qpos, key0 + 4 * b + i, p.window, p.keep);
-      float x[HT][4];
+        for (int i = 0; i < 4; ++i) vis[i] = sees(qpos, key0 + 4 * i + b, p.window, p.keep);
+      }
+      // hi / lo parts of the weights, [key i][heads pairwise]
+      unsigned xh[4][HX / 2], xl[4][HX / 2];
+      float px[4] = {0.f, 0.f, 0.f, 0.f};  // the even head of a pair
 #pragma unroll
       for (int c = 0; c < GP; ++c) {
-        uint4 kf[kMaxKS];
-        if (c < p.G) load_k(kf, c, key0);
+        if (c + 1 < GP && c + 1 < p.G) load_k(kf[(c + 1) & 1], c + 1, t);
 #pragma unroll
         for (int r = 0; r < RP; ++r) {
+          const int h = c * RP + r;
           f32x4 a = {};
           const bool real = c < p.G && r < R;
-          if (real) a = score(kf, c, r);
-          const float ls = lse[(c * RP + r) * 16 + rl];
+          if (real) {
 #pragma unroll
-          for (int i = 0; i < 4; ++i)
-            x[c * RP + r][i] = real && vis[i] ? __builtin_amdgcn_exp2f(a[i] * sl2 - ls) : 0.f;
+            for (int s = 0; s < KSN; ++s)
+              if (s < nst) {
+                uint4 qf;
+                if constexpr (C::QL) qf = qs[((size_t)h * nst + s) * 64 + lane];
+                else qf = ld128(qp + (size_t)(c * R + r) * p.dk + s * 32);
+                a = mfma16(as_bf16x8(kf[c & 1][s]), as_bf16x8(qf), a);
+              }
+          }
+          const float ls = lse[h * 16 + rl];
+          float x[4];
+#pragma unroll
+          for (int i = 0; i < 4; ++i) x[i] = real && vis[i] ? __builtin_amdgcn_exp2f(a[i] * sl2 - ls) : 0.f;
+          if (HT == 1 || (h & 1)) {
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+              const float e = HT == 1 ? x[i] : px[i], o = HT == 1 ? 0.f : x[i];
+              const unsigned hi = pack2(e, o);
+              xh[i][h >> 1] = hi;
+              xl[i][h >> 1] = pack2(e - __uint_as_float(hi << 16), o - __uint_as_float(hi & 0xffff0000u));
+            }
+          } else {
+#pragma unroll
+            for (int i = 0; i < 4; ++i) px[i] = x[i];
+          }
+          // (bounds how far ahead the query fragments are read: unbounded, their registers spill)
+          if ((r & 1) == 1 || RP == 1) __builtin_amdgcn_sched_barrier(0);
         }
       }
-#pragma unroll 1
-      for (int h = 0; h < HT; ++h) {
-        const float* tk = pp.talk_pad + h * HT;  // (uniform: scalar loads)
-        float y[4] = {0.f, 0.f, 0.f, 0.f};
+      if constexpr (HT < 4) {
 #pragma unroll
-        for (int g = 0; g < HT; ++g) {
-          const float tg = tk[g];
+        for (int i = 0; i < 4; ++i) xh[i][1] = xl[i][1] = 0u;
+      }
+      // next iteration's first keys, this one's first values
+      if (t + NW < v.n && it + 1 < it1) load_k(kf[0], 0, t + NW);
+      load_v(vf[0], it, 0);
+      // per key element: B operands by transposing the lane groups' blocks of 8 heads (4 registers), the
+      // mixed weights of keys 4 i .. 4 i + 3 of every head, and their bf16 quads to LDS
 #pragma unroll
-          for (int i = 0; i < 4; ++i) y[i] += tg * x[g][i];
+      for (int i = 0; i < 4; ++i) {
+        uint4 bm[C::KM][4];  // [mixing step][source lane group]
+#pragma unroll
+        for (int ks = 0; ks < C::KM; ++ks) {
+          unsigned o[4][4];  // [source group][register]
+#pragma unroll
+          for (int g = 0; g < 4; ++g) {
+            unsigned q0, q1, q2, q3;
+            if constexpr (HT == 32) {
+              const unsigned (&x)[HX / 2] = ks ? xl[i] : xh[i];
+              q0 = x[g], q1 = x[4 + g], q2 = x[8 + g], q3 = x[12 + g];
+            } else if constexpr (HT == 16) {
+              q0 = xh[i][g], q1 = xh[i][4 + g], q2 = xl[i][g], q3 = xl[i][4 + g];
+            } else if constexpr (HT == 8) {
+              q0 = xh[i][g], q1 = xl[i][g], q2 = 0u, q3 = 0u;
+            } else {
+              q0 = g < 2 ? xh[i][g & 1] : xl[i][g & 1], q1 = 0u, q2 = 0u, q3 = 0u;
+            }
+            transpose4(q0, q1, q2, q3);
+            o[0][g] = q0, o[1][g] = q1, o[2][g] = q2, o[3][g] = q3;
+          }
+#pragma unroll
+          for (int g = 0; g < 4; ++g) bm[ks][g] = make_uint4(o[g][0], o[g][1], o[g][2], o[g][3]);
         }
-        *reinterpret_cast<uint2*>(pw + h * HS) = make_uint2(pack2(y[0], y[1]), pack2(y[2], y[3]));
+#pragma unroll
+        for (int mt = 0; mt < C::MT; ++mt) {
+          f32x4 y[4];
+#pragma unroll
+          for (int g = 0; g < 4; ++g) {
+            f32x4 a = {};
+#pragma unroll
+            for (int ks = 0; ks < C::KM; ++ks) a = mfma16(as_bf16x8(tf[mt]), as_bf16x8(bm[ks][g]), a);
+            y[g] = a;
+          }
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            const int h = 16 * mt + 4 * b + e;
+            if (HT >= 16 || h < HT)
+              *reinterpret_cast<uint2*>(pw + h * HS + (i >> 1) * 256 + (i & 1) * 8) =
+                  make_uint2(pack2(y[0][e], y[1][e]), pack2(y[2][e], y[3][e]));
+          }
+        }
       }
     } else {
+      load_v(vf[0], it, 0);
 #pragma unroll
-      for (int h = 0; h < HT; ++h) *reinterpret_cast<uint2*>(pw + h * HS) = make_uint2(0u, 0u);
+      for (int mt = 0; mt < C::MT; ++mt)
+#pragma unroll
+        for (int ch = 0; ch < 2; ++ch)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            const int h = 16 * mt + 4 * b + i;
+            if (HT >= 16 || h < HT) *reinterpret_cast<uint4*>(pw + h * HS + ch * 256) = make_uint4(0, 0, 0, 0);
+          }
     }
-    __syncthreads();
+    lds_sync();
+    uint4 pf[RP];
 #pragma unroll
-    for (int kg = 0; kg < C::KG; ++kg) {
+    for (int st = 0; st < STEPS; ++st) {
+      const int kg = st / CH;
       if (it * NW + 2 * kg >= v.n) break;
-      const int tt = min(it * NW + 2 * kg + (b >> 1), v.n - 1);
-      const int key = tile_of(v, tt) * kTile;
-      const u16* vp = reinterpret_cast<const u16*>(p.v) + blk_of(key) * p.v_sb + (int64_t)rl * p.block_size +
-                      key % p.block_size + (b & 1) * 8;
-      uint4 vf[NV];
+      if (st + 1 < STEPS && it * NW + 2 * ((st + 1) / CH) < v.n) load_v(vf[(st + 1) & 1], it, st + 1);
 #pragma unroll
-      for (int n = 0; n < NV; ++n) {
-        const int idx = min(w + NW * n, nvt - 1);
-        vf[n] = ld128(vp + (int64_t)(idx / ndv) * p.v_sh + (int64_t)(idx % ndv) * 16 * p.block_size);
-      }
-#pragma unroll
-      for (int n = 0; n < NV; ++n) {
-        const int idx = w + NW * n;
-        if (idx >= nvt) break;
+      for (int n = 0; n < NC; ++n) {
+        const int u = (st % CH) * NC + n, idx = v0 + u;
+        if (u >= nvw || idx >= nvt) break;
         const int c = idx / ndv;
+        if (u == 0 || c != (idx - 1) / ndv) {  // (the kv head's mixed weights serve all of its value tiles)
 #pragma unroll
-        for (int r = 0; r < RP; ++r) {
-          if (r >= R) break;
-          const uint4 pf = *reinterpret_cast<const uint4*>(pm + (c * RP + r) * HS + ((kg * 4 + b) * 16 + rl) * 16);
-          acc[n][r] = mfma16(as_bf16x8(vf[n]), as_bf16x8(pf), acc[n][r]);
+          for (int r = 0; r < RP; ++r)
+            if (r < R) pf[r] = *reinterpret_cast<const uint4*>(pm + (c * RP + r) * HS + ((kg * 4 + b) * 16 + rl) * 16);
         }
+#pragma unroll
+        for (int r = 0; r < RP; ++r)
+          if (r < R) acc[u][r] = mfma16(as_bf16x8(vf[st & 1][n]), as_bf16x8(pf[r]), acc[u][r]);
       }
     }
+    lds_sync();
+  }
+  if (nact > 1) {
+    // ---- every split's sums out (sc1), a ticket, and the last one adds them in order
+    constexpr int kWave = NV * RP * 64 * 16, kPart = NW * kWave;     // bytes per wave / workgroup
+    float* base = pp.part + (size_t)bt * pp.splits * (kPart / 4);
+    const __amdgpu_buffer_rsrc_t rp = rsrc_f32(base, (int64_t)pp.splits * (kPart / 4));
+    const int at = w * kWave + lane * 16;
+#pragma unroll
+    for (int n = 0; n < NV; ++n)
+#pragma unroll
+      for (int r = 0; r < RP; ++r) st_sc1_x4(rp, split * kPart + at + (n * RP + r) * 1024, acc[n][r]);
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     __syncthreads();
+    if (threadIdx.x == 0) {
+      const int ticket = __hip_atomic_fetch_add(pp.tickets + bt, 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+      const int last = ticket == nact - 1;
+      if (last) __hip_atomic_store(pp.tickets + bt, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+      s_last = last;
+    }
+    __syncthreads();
+    if (!s_last) return;
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+#pragma unroll
+    for (int n = 0; n < NV; ++n)
+#pragma unroll
+      for (int r = 0; r < RP; ++r) acc[n][r] = ld_sc1_x4(rp, at + (n * RP + r) * 1024);
+    for (int s = 1; s < nact; ++s)
+#pragma unroll
+      for (int n = 0; n < NV; ++n)
+#pragma unroll
+        for (int r = 0; r < RP; ++r) acc[n][r] += ld_sc1_x4(rp, s * kPart + at + (n * RP + r) * 1024);
   }
   // ---- gate, scale, store: lane (query rl, value columns 4b .. 4b+3 of the tile)
   if (rl >= nq) return;
 #pragma unroll
   for (int n = 0; n < NV; ++n) {
-    const int idx = w + NW * n;
-    if (idx >= nvt) break;
+    const int idx = v0 + n;
+    if (n >= nvw || idx >= nvt) break;
     const int c = idx / ndv, d = (idx % ndv) * 16 + 4 * b;
 #pragma unroll
     for (int r = 0; r < RP; ++r) {
@@ -534,55 +717,64 @@ int pow2_up(int n) {
 
 constexpr size_t kMaxLds = 160 * 1024;
 
-template <int GP, int RP, int NV, int NW, bool QL>
-int launch_prefill(const TalkPrefillParams& p, hipStream_t st) {
-  hipLaunchKernelGGL((talk_prefill_kernel<GP, RP, NV, NW, QL>), dim3(p.n_tiles), dim3(NW * 64),
-                     (PrefillCfg<GP, RP, NV, NW, QL>::lds(p.a.dk)), st, p);
+// what a call wants: only whether the sizes have an instantiation, its partial floats per tile and split,
+// or the launch
+enum Want { WANT_FIT, WANT_PART, WANT_LAUNCH };
+
+template <int GP, int RP, int NV, int NW, int KSN>
+int64_t prefill_cfg(const TalkPrefillParams& p, hipStream_t st, Want want) {
+  using C = PrefillCfg<GP, RP, NV, NW, KSN>;
+  if (C::lds(p.a.dk) > kMaxLds - 64) return -10;
+  if (want == WANT_FIT) return 0;
+  if (want == WANT_PART) return (int64_t)NW * NV * RP * 256;
+  const int R = p.a.H / p.a.G;
+  constexpr int RB = RP < 4 ? RP : 4;
+  hipLaunchKernelGGL((talk_lse_kernel<RB, KSN>), dim3(p.n_tiles * p.a.G, (R + RB - 1) / RB), dim3(256), 0, st, p);
+  hipLaunchKernelGGL((talk_prefill_kernel<GP, RP, NV, NW, KSN>), dim3(p.n_tiles, p.splits), dim3(NW * 64),
+                     (C::lds(p.a.dk)), st, p);
   return 0;
 }
 
-// launch = null: only whether these sizes have an instantiation
 template <int GP, int RP>
-int prefill_sizes(const TalkPrefillParams& p, hipStream_t st, bool launch) {
+int64_t prefill_sizes(const TalkPrefillParams& p, hipStream_t st, Want want) {
   constexpr int HT = GP * RP;
   constexpr int NW = HT > 16 ? 4 : 8;       // 32 heads: 4 waves with twice the registers
   constexpr int N1 = (GP * 8 + NW - 1) / NW, N2 = (GP * 16 + NW - 1) / NW;   // dv <= 128 / <= 256
   const int need = (p.a.G * (p.a.dv >> 4) + NW - 1) / NW;
-  const bool ql = PrefillCfg<GP, RP, N1, NW, true>::lds(p.a.dk) <= kMaxLds;
   if (need <= N1) {
-    if (!launch) return 0;
-    return ql ? launch_prefill<GP, RP, N1, NW, true>(p, st) : launch_prefill<GP, RP, N1, NW, false>(p, st);
+    if (p.a.dk <= 128) return prefill_cfg<GP, RP, N1, NW, 4>(p, st, want);
+    return prefill_cfg<GP, RP, N1, NW, 8>(p, st, want);
   }
   if constexpr (HT <= 16) {
     if (need <= N2) {
-      if (!launch) return 0;
-      return ql ? launch_prefill<GP, RP, N2, NW, true>(p, st) : launch_prefill<GP, RP, N2, NW, false>(p, st);
+      if (p.a.dk <= 128) return prefill_cfg<GP, RP, N2, NW, 4>(p, st, want);
+      return prefill_cfg<GP, RP, N2, NW, 8>(p, st, want);
     }
   }
   return -10;
 }
 
-int dispatch_prefill(const TalkPrefillParams& p, hipStream_t st, bool launch) {
+int64_t dispatch_prefill(const TalkPrefillParams& p, hipStream_t st, Want want) {
   const TalkAttnParams& a = p.a;
-  if (a.H < 1 || a.G < 1 || a.H % a.G || a.dk % 32 || a.dk > 32 * kMaxKS || a.dv % 16 || a.dv < 16) return -10;
+  if (a.H < 1 || a.G < 1 || a.H % a.G || a.dk % 32 || a.dk > 256 || a.dv % 16 || a.dv < 16) return -10;
   switch (pow2_up(a.G) * 100 + pow2_up(a.H / a.G)) {
-    case 101: return prefill_sizes<1, 1>(p, st, launch);
-    case 102: return prefill_sizes<1, 2>(p, st, launch);
-    case 104: return prefill_sizes<1, 4>(p, st, launch);
-    case 108: return prefill_sizes<1, 8>(p, st, launch);
-    case 201: return prefill_sizes<2, 1>(p, st, launch);
-    case 202: return prefill_sizes<2, 2>(p, st, launch);
-    case 204: return prefill_sizes<2, 4>(p, st, launch);
-    case 208: return prefill_sizes<2, 8>(p, st, launch);
-    case 401: return prefill_sizes<4, 1>(p, st, launch);
-    case 402: return prefill_sizes<4, 2>(p, st, launch);
-    case 404: return prefill_sizes<4, 4>(p, st, launch);
-    case 408: return prefill_sizes<4, 8>(p, st, launch);
-    case 801: return prefill_sizes<8, 1>(p, st, launch);
-    case 802: return prefill_sizes<8, 2>(p, st, launch);
-    case 804: return prefill_sizes<8, 4>(p, st, launch);
-    case 1601: return prefill_sizes<16, 1>(p, st, launch);
-    case 1602: return prefill_sizes<16, 2>(p, st, launch);
+    case 101: return prefill_sizes<1, 1>(p, st, want);
+    case 102: return prefill_sizes<1, 2>(p, st, want);
+    case 104: return prefill_sizes<1, 4>(p, st, want);
+    case 108: return prefill_sizes<1, 8>(p, st, want);
+    case 201: return prefill_sizes<2, 1>(p, st, want);
+    case 202: return prefill_sizes<2, 2>(p, st, want);
+    case 204: return prefill_sizes<2, 4>(p, st, want);
+    case 208: return prefill_sizes<2, 8>(p, st, want);
+    case 401: return prefill_sizes<4, 1>(p, st, want);
+    case 402: return prefill_sizes<4, 2>(p, st, want);
+    case 404: return prefill_sizes<4, 4>(p, st, want);
+    case 408: return prefill_sizes<4, 8>(p, st, want);
+    case 801: return prefill_sizes<8, 1>(p, st, want);
+    case 802: return prefill_sizes<8, 2>(p, st, want);
+    case 804: return prefill_sizes<8, 4>(p, st, want);
+    case 1601: return prefill_sizes<16, 1>(p, st, want);
+    case 1602: return prefill_sizes<16, 2>(p, st, want);
     default: return -10;
   }
 }
@@ -613,22 +805,24 @@ extern "C" int vwa_talk_attention(const TalkAttnParams* p, hipStream_t st) {
   return (int)hipGetLastError();
 }
 
-extern "C" int vwa_talk_prefill_fits(int H, int G, int dk, int dv) {
+extern "C" int64_t vwa_talk_prefill_part(int H, int G, int dk, int dv) {
   TalkPrefillParams p{};
   p.a.H = H;
   p.a.G = G;
   p.a.dk = dk;
   p.a.dv = dv;
-  return dispatch_prefill(p, nullptr, false) == 0;
+  return dispatch_prefill(p, nullptr, WANT_PART);
 }
 
 extern "C" int vwa_talk_prefill(const TalkPrefillParams* p, hipStream_t st) {
   const int rc = check_attn(p->a);
   if (rc) return rc;
-  if (p->a.f32 || p->n_tiles < 1 || !p->tiles || !p->talk_pad || p->GP != pow2_up(p->a.G) ||
-      p->RP != pow2_up(p->a.H / p->a.G) || p->a.ldo % 4)
-    return -6;
-  const int r = dispatch_prefill(*p, st, true);
-  if (r) return r;
+  if (p->a.f32 || p->n_tiles < 1 || !p->tiles || !p->talk_frag || !p->lse || p->splits < 1 || p->a.ldo % 4) return -6;
+  if (p->splits > 1) {
+    const int64_t part = dispatch_prefill(*p, st, WANT_PART);
+    if (!p->part || !p->tickets || part < 0 || part * p->splits * 4 >= (1ll << 31)) return -7;
+  }
+  const int64_t r = dispatch_prefill(*p, st, WANT_LAUNCH);
+  if (r) return (int)r;
   return (int)hipGetLastError();
 }

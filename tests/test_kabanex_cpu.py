@@ -275,11 +275,32 @@ def test_cache_with_unequal_layers():
     assert PagedKVCache.layer_bytes_per_block(layers, 16) == 2 * 16 * (2 * 48 + 112)
 
 
-def test_pad_talk_order():
-    T = torch.arange(36.0).view(6, 6)
-    P = ops.pad_talk(T, 2)  # 2 kv heads x 3 -> 2 x 4
-    assert P.shape == (8, 8) and P[3].abs().sum() == 0 and P[:, 7].abs().sum() == 0
-    assert P[4, 6] == T[3, 5] and P[2, 4] == T[2, 3]
+@pytest.mark.parametrize("H,G", [(1, 1), (2, 1), (4, 2), (6, 2), (8, 8), (16, 4), (12, 3), (32, 8), (24, 2)])
+def test_talk_fragment_is_the_matrix_for_both_halves(H, G):
+    """The A operand times (hi | lo) stacked heads is talk @ (hi + lo), in the padded head order."""
+    T = torch.randn(H, H).to(torch.bfloat16).float()
+    fr = ops.talk_fragment(T, G).float()
+    R = H // G
+    up = lambda n: 1 << (n - 1).bit_length()  # noqa: E731
+    HT = up(G) * up(R)
+    A = fr.view(-1, 4, 16, 8).permute(0, 2, 1, 3).reshape(-1, 32)          # [rows, k]
+    order = [(h // R) * up(R) + h % R for h in range(H)]
+    hi, lo = torch.zeros(max(HT, 4)), torch.zeros(max(HT, 4))
+    hi[order], lo[order] = torch.randn(H), torch.randn(H) * 0.01
+    if HT == 32:
+        got = A @ hi + A @ lo
+    else:
+        x = torch.zeros(32)
+        x[: 2 * max(HT, 4)] = torch.cat([hi, lo])
+        got = A @ x
+    assert torch.allclose(got[order], T @ (hi + lo)[order], atol=1e-4)
+
+
+def test_prefill_splits():
+    from voice_enabled_browser_automation_amd.ops.stack import prefill_splits
+
+    assert prefill_splits(128, 2047, 1024, 4, 256) == 2 and prefill_splits(300, 5000, 0, 0, 256) == 1
+    assert prefill_splits(4, 63, 1024, 0, 256) == 1 and prefill_splits(4, 4095, 1024, 4, 256) == 9
 
 
 def test_trace_replay_command(folder, weights, tmp_path):

@@ -133,6 +133,10 @@ ATT = [  # H, G, dk, dv, window, keep, bs, n
 ]
 
 
+def pads(n):
+    return 1 << (n - 1).bit_length()
+
+
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("mixed", [True, False])
 @pytest.mark.parametrize("case", ATT, ids=[str(c) for c in ATT])
@@ -151,7 +155,7 @@ def test_talk_attention(dtype, mixed, case):
             k[j] += (3.0 + float(torch.rand(1, generator=gen))) * u
     v = rnd(n, G, dv, seed=4)
     q, k, v = q.to(dtype), k.to(dtype), v.to(dtype)
-    T = (torch.eye(H) + rnd(H, H, seed=5, std=0.4)) if mixed else torch.eye(H)
+    T = (torch.eye(H) + rnd(H, H, seed=5, std=0.4)).to(BF16).float() if mixed else torch.eye(H)
     gate = rnd(n, H + 8, seed=6, dtype=dtype)
     scale = 0.7
     m = O.mask(n, window, keep)
@@ -166,7 +170,7 @@ def test_talk_attention(dtype, mixed, case):
     max_ctx = len(perm) * bs
     sc = ops.TalkScratch([(H, G, dv, window, keep)], max_ctx, DEV)
     kw = dict(n_q_heads=H, scale=scale, window=window, keep=keep, talk=T.to(DEV) if mixed else None,
-              talk_pad=ops.pad_talk(T, G).to(DEV), out_scale=0.8, max_ctx=max_ctx, scratch=sc)
+              talk_frag=ops.talk_fragment(T, G).to(DEV) if pads(G) * pads(H // G) <= 32 else None, out_scale=0.8, max_ctx=max_ctx, scratch=sc)
     pos = torch.arange(n, dtype=torch.int32, device=DEV)
     sid = torch.full((n,), 2, dtype=torch.int32, device=DEV)
     slots = torch.zeros(n, dtype=torch.int64, device=DEV)
@@ -186,7 +190,7 @@ def test_talk_attention(dtype, mixed, case):
             c = min(c, n - a)
             runs.append((len(sel), c))
             sel += list(range(a, a + c))
-        got = run(sel, ops.plan_runs(runs, DEV))
+        got = run(sel, ops.plan_runs(runs, DEV, n - 1))
         assert rel(got, want[sel]) < tol
     # inert rows of a padded step are zero and touch nothing
     slots[5] = -1
@@ -196,10 +200,10 @@ def test_talk_attention(dtype, mixed, case):
 
 
 def test_prefill_form_takes_the_usual_sizes():
-    E = ops.ext()
+    part = ops.ext().talk_prefill_part
     for H, G, dk, dv in [(4, 2, 64, 128), (16, 4, 128, 128), (32, 8, 128, 128), (6, 2, 96, 192), (8, 1, 256, 64), (12, 12, 64, 64)]:
-        assert E.talk_prefill_fits(H, G, dk, dv)
-    assert not E.talk_prefill_fits(40, 1, 64, 64)
+        assert part(H, G, dk, dv) > 0
+    assert part(40, 1, 64, 64) < 0
 
 
 def test_attention_with_every_key_visible():
@@ -212,10 +216,10 @@ def test_attention_with_every_key_visible():
     kc, vc = paged(k, v, perm, 16, BF16)
     table = torch.tensor([perm], dtype=torch.int32, device=DEV)
     pos = torch.arange(n, dtype=torch.int32, device=DEV)
-    for plan in (None, ops.plan_runs([(0, n)], DEV)):
+    for plan in (None, ops.plan_runs([(0, n)], DEV, n - 1)):
         out = torch.zeros(n, H * dv, dtype=BF16, device=DEV)
         ops.talk_attention(q.reshape(n, -1).to(DEV), kc, vc, table, pos, torch.zeros_like(pos), pos.long(), n_q_heads=H,
-                           scale=0.125, window=0, keep=0, talk=None, talk_pad=ops.pad_talk(torch.eye(H), G).to(DEV), gate=None,
+                           scale=0.125, window=0, keep=0, talk=None, talk_frag=ops.talk_fragment(torch.eye(H), G).to(DEV), gate=None,
                            out_scale=1.0, max_ctx=112, scratch=ops.TalkScratch([(H, G, dv, 0, 0)], 112, DEV), out=out, plan=plan)
         assert rel(out, want) < 1.5e-2
 
@@ -239,7 +243,7 @@ def test_mingru(dtype, W):
     y = torch.cat([z, x, g], 1).to(DEV)
     ids = torch.cat([torch.full((n,), s) for s, _, n, _ in R]).int().to(DEV)
     pos = torch.cat([torch.arange(p, p + n) for _, p, n, _ in R]).int().to(DEV)
-    for plan in (None, ops.plan_runs([(r0, n) for _, _, n, r0 in R], DEV)):
+    for plan in (None, ops.plan_runs([(r0, n) for _, _, n, r0 in R], DEV, 200)):
         st = st0.clone().to(DEV)
         out = torch.zeros(tot, W + 8, dtype=dtype, device=DEV)
         ops.mingru(y[:, :W], y[:, W : 2 * W], y[:, 2 * W :], zb.to(DEV), xb.to(DEV), seq_ids=ids, positions=pos,

@@ -34,6 +34,10 @@ def _up(n: int, m: int) -> int:
     return (n + m - 1) // m * m
 
 
+def _padded_heads(a) -> int:
+    return (1 << (a.kv_heads - 1).bit_length()) * (1 << (a.heads // a.kv_heads - 1).bit_length())
+
+
 @dataclass(frozen=True)
 class LayerDims:
     """Padded section sizes of a layer's fused projections."""
@@ -81,7 +85,7 @@ class KabanexLayerWeights:
     w_in: object             # [n_mix + f, d]   (TiledWeight on a bf16 GPU model)
     w_out: object            # [hidden padded to 16, n_cat]
     talk: torch.Tensor       # f32 [H, H]
-    talk_pad: torch.Tensor   # the same in the prefill kernel's padded head order
+    talk_frag: Optional[torch.Tensor]  # the same as the prefill kernel's A operand (None: too many heads for it)
     zb: torch.Tensor         # f32 [width]
     xb: torch.Tensor
 
@@ -151,7 +155,7 @@ class KabanexModel:
                 raise ValueError(f"{p}mix.left.talk: shape {tuple(talk.shape)}, expected {(a.heads, a.heads)}")
             self.layers.append(KabanexLayerWeights(
                 norm_w=vec(p + "norm1"), norm_b=vec(p + "norm1.b"), w_in=place(w_in), w_out=place(w_out), talk=talk,
-                talk_pad=ops.pad_talk(talk, a.kv_heads), zb=vec(p + "mix.right.z.b"), xb=vec(p + "mix.right.x.b")))
+                talk_frag=ops.talk_fragment(talk, a.kv_heads) if tiled and _padded_heads(a) <= 32 else None, zb=vec(p + "mix.right.z.b"), xb=vec(p + "mix.right.x.b")))
         self.final_w, self.final_b = vec("final.norm"), vec("final.norm.b")
         head = torch.zeros(self.v_pad, self.d_pad, dtype=dt, device=dev)
         head[: cfg.vocab_size, : cfg.hidden] = mat("head", cfg.vocab_size, cfg.hidden)
@@ -196,8 +200,8 @@ class KabanexModel:
                                        for L, D in zip(self.cfg.layers, self.dims)], max_ctx, dev))
         return b
 
-    def plan_rows(self, runs: Sequence[Tuple[int, int]]) -> SimpleNamespace:
-        return ops.plan_runs(runs, self.device)
+    def plan_rows(self, runs: Sequence[Tuple[int, int]], max_pos: int) -> SimpleNamespace:
+        return ops.plan_runs(runs, self.device, max_pos)
 
     # ------------------------------------------------------------------ forward
     def forward(self, bufs, M: int, kv, *, n_sel: Optional[int] = None, head: bool = True) -> torch.Tensor:
@@ -227,7 +231,7 @@ class KabanexModel:
                                 positions=rows["positions"], slots=rows["slots"],
                                 q_out=bufs.q[: M * D.H * D.dk].view(M, D.H * D.dk), k_cache=kv.k[li], v_cache=kv.v[li])
         ops.talk_attention(q, kv.k[li], kv.v[li], bufs.block_table, n_q_heads=D.H, scale=a.scale, window=a.window,
-                           keep=a.keep_first, talk=L.talk, talk_pad=L.talk_pad, gate=y[:, g0 : g0 + D.gate],
+                           keep=a.keep_first, talk=L.talk, talk_frag=L.talk_frag, gate=y[:, g0 : g0 + D.gate],
                            out_scale=C.left_scale, max_ctx=bufs.max_ctx, scratch=bufs.talk, out=cat[:, : D.heads_out],
                            plan=plan, **rows)
         W = C.right.width

@@ -1182,5 +1182,5 @@ def env_int(name: str) -> int:
     return int(knob(name))
 
 
-from .stack import (TalkScratch, embedding_f32, layernorm_f32, linear_split, mingru, pad_talk, plan_runs,  # noqa: E402,F401
-                    qkv_cache_write, talk_attention)
+from .stack import (TalkScratch, embedding_f32, layernorm_f32, linear_split, mingru, plan_runs,  # noqa: E402,F401
+                    qkv_cache_write, talk_attention, talk_fragment)

@@ -27,9 +27,9 @@ def _ext():
 
 
 # ----------------------------------------------------------------------------- row plans
-def plan_runs(runs: Sequence[Tuple[int, int]], device) -> SimpleNamespace:
+def plan_runs(runs: Sequence[Tuple[int, int]], device, max_pos: int) -> SimpleNamespace:
     """Launch tables of a ragged step with many rows.  runs: (first row, rows), each of one sequence at
-    consecutive positions.  tiles: prefill attention tiles of the runs longer than one row; singles:
+    consecutive positions; max_pos: the largest position of the step.  tiles: prefill attention tiles of the runs longer than one row; singles:
     the rows that are a run of their own (decoded tokens beside prompt portions); chunks: recurrence
     scan chunks of every run."""
     tiles: List[List[int]] = []
@@ -47,7 +47,7 @@ def plan_runs(runs: Sequence[Tuple[int, int]], device) -> SimpleNamespace:
         t = torch.tensor(x, dtype=torch.int32).view(-1, cols)
         return t.pin_memory().to(device, non_blocking=True) if torch.device(device).type == "cuda" else t
 
-    return SimpleNamespace(tiles=dev(tiles, 2) if tiles else None, chunks=dev(chunks, 4),
+    return SimpleNamespace(max_pos=max_pos, tiles=dev(tiles, 2) if tiles else None, chunks=dev(chunks, 4),
                            singles=dev(singles, 1).view(-1) if singles else None)
 
 
@@ -129,7 +129,7 @@ def qkv_cache_write(x: torch.Tensor, *, n_q_heads: int, rot_dims: int, rope: tor
 
 def talk_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor,
                    positions: torch.Tensor, seq_ids: torch.Tensor, slots: torch.Tensor, *, n_q_heads: int, scale: float,
-                   window: int, keep: int, talk: Optional[torch.Tensor], talk_pad: Optional[torch.Tensor],
+                   window: int, keep: int, talk: Optional[torch.Tensor], talk_frag: Optional[torch.Tensor],
                    gate: Optional[torch.Tensor], out_scale: float, max_ctx: int, scratch: Optional[TalkScratch],
                    out: torch.Tensor, plan: Optional[SimpleNamespace] = None) -> torch.Tensor:
     """Attention of ragged rows over their sequences' cached keys: row i sees key j if j <= i and
@@ -147,10 +147,16 @@ def talk_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor
                          gt, out_scale, max_ctx, scratch.s, scratch.stat, scratch.part, scratch.counters, o)
 
     G, dk, dv = k_cache.shape[1], k_cache.shape[3], v_cache.shape[2]
-    if plan is not None and q.dtype == torch.bfloat16 and talk_pad is not None and E.talk_prefill_fits(n_q_heads, G, dk, dv):
+    part = E.talk_prefill_part(n_q_heads, G, dk, dv) if plan is not None and talk_frag is not None else -1
+    if part > 0 and q.dtype == torch.bfloat16:
         if plan.tiles is not None:
+            from . import scratch as ws
+
+            nt = plan.tiles.shape[0]
+            splits = prefill_splits(nt, plan.max_pos, window, keep, E.device_cus(q))
             E.talk_prefill(q, k_cache, v_cache, block_table, positions, seq_ids, slots, plan.tiles, n_q_heads, scale, window,
-                           keep, talk_pad, gate, out_scale, max_ctx, out)
+                           keep, talk_frag, gate, out_scale, max_ctx, splits, ws(q.device, "talk_lse", rows * n_q_heads),
+                           ws(q.device, "talk_part", nt * splits * part if splits > 1 else 1), _tickets(q.device, nt), out)
         if plan.singles is not None:
             n = plan.singles.shape[0]
             for i in range(0, n, ROW_SLICE):
@@ -163,17 +169,46 @@ def talk_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor
     return out
 
 
-def pad_talk(talk: torch.Tensor, n_kv_heads: int) -> torch.Tensor:
-    """talk [H, H] in the prefill kernel's padded head order h = c * RP + r (kv heads and query heads per
-    kv head rounded up to powers of two; padding zero)."""
+def prefill_splits(n_tiles: int, max_pos: int, window: int, keep: int, cus: int) -> int:
+    """Workgroups per 16-query tile over its keys: enough to give every CU one, and no more than leaves
+    each a round of its waves (128 keys)."""
+    keys = max_pos + 1
+    if window > 0:
+        keys = min(keys, window + keep + 2 * TILE_ROWS)
+    return max(1, min(-(-keys // 128), cus // n_tiles))
+
+
+_TICKETS: dict = {}
+
+
+def _tickets(device, n: int) -> torch.Tensor:
+    """Zeroed chunk tickets of the prefill form (the kernel leaves them zero)."""
+    t = _TICKETS.get(str(device))
+    if t is None or t.numel() < n:
+        t = _TICKETS[str(device)] = torch.zeros(max(n, 4096), dtype=torch.int32, device=device)
+    return t
+
+
+def talk_fragment(talk: torch.Tensor, n_kv_heads: int) -> torch.Tensor:
+    """talk [H, H] as the prefill kernel's A operand (stack_kernels.h TalkPrefillParams::talk_frag), in its
+    padded head order h = c * RP + r (kv heads and query heads per kv head rounded up to powers of two)."""
     H = talk.shape[0]
     R = H // n_kv_heads
     up = lambda n: 1 << (n - 1).bit_length()  # noqa: E731
     GP, RP = up(n_kv_heads), up(R)
-    idx = torch.tensor([(h // R) * RP + h % R for h in range(H)], device=talk.device)
-    out = torch.zeros(GP * RP, GP * RP, dtype=torch.float32, device=talk.device)
-    out[idx[:, None], idx[None, :]] = talk.float()
-    return out
+    HT = GP * RP
+    idx = torch.tensor([(h // R) * RP + h % R for h in range(H)])
+    rows, cols = max(16, -(-HT // 16) * 16), max(HT, 4)
+    T = torch.zeros(rows, cols)
+    T[idx[:, None], idx[None, :]] = talk.detach().float().cpu()
+    k = torch.arange(32)
+    head = k % max(HT, 4) if HT < 32 else k
+    live = k < 2 * max(HT, 4)                    # (hi and lo halves of the weights share the matrix)
+    A = T[:, head] * live                        # [rows, 32]
+    if HT > 32:
+        raise ValueError(f"{HT} padded heads: the prefill kernel takes 32")
+    A = A.view(rows // 16, 16, 4, 8).permute(0, 2, 1, 3)   # [mt][lane group b][row rl][e]
+    return A.reshape(rows // 16, 64, 8).contiguous().to(device=talk.device, dtype=torch.bfloat16)
 
 
 def mingru(z: torch.Tensor, x: torch.Tensor, g: torch.Tensor, zb: Optional[torch.Tensor], xb: Optional[torch.Tensor], *,

@@ -706,7 +706,7 @@ class LLMEngine:
             block_table=self.bufs.block_table, max_ctx=self.bufs.max_ctx, logits_local=self.bufs.logits_local)
         if hasattr(m, "row_buffers"):
             vars(scratch).update(m.row_buffers(n, self.bufs.max_ctx), talk=getattr(self.bufs, "talk", None),
-                                 plan=m.plan_rows(self._runs(sids, poss)))
+                                 plan=m.plan_rows(self._runs(sids, poss), max(poss)))
         else:
             d = m.cfg.hidden
             vars(scratch).update(
