@@ -117,9 +117,8 @@ void check_caches(const Tensor& k, const Tensor& v, bool f32, int64_t G, int64_t
   check_aligned(v, "v cache");
 }
 
-void qkv_cache(Tensor x, int64_t H, int64_t G, int64_t dk, int64_t dv, int64_t rot_dims, Tensor rope, Tensor positions,
-               Tensor slots, Tensor q_out, Tensor k, Tensor v) {
-  c10::DeviceGuard g(x.device());
+QkvCacheParams qkv_params(const Tensor& x, int64_t H, int64_t G, int64_t dk, int64_t dv, int64_t rot_dims, const Tensor& rope,
+                          const Tensor& positions, const Tensor& slots, const Tensor& q_out, const Tensor& k, const Tensor& v) {
   const bool f32 = t_is_f32(x, "x");
   const int64_t rows = q_out.size(0);
   check_rows(x, rows, H * dk + G * (dk + dv), "x");
@@ -154,6 +153,13 @@ void qkv_cache(Tensor x, int64_t H, int64_t G, int64_t dk, int64_t dv, int64_t r
   p.v_sb = v.stride(0);
   p.v_sh = v.stride(1);
   p.block_size = (int)k.size(2);
+  return p;
+}
+
+void qkv_cache(Tensor x, int64_t H, int64_t G, int64_t dk, int64_t dv, int64_t rot_dims, Tensor rope, Tensor positions,
+               Tensor slots, Tensor q_out, Tensor k, Tensor v) {
+  c10::DeviceGuard g(x.device());
+  const QkvCacheParams p = qkv_params(x, H, G, dk, dv, rot_dims, rope, positions, slots, q_out, k, v);
   check_rc(vwa_qkv_cache(&p, cur_stream(x)), "qkv_cache");
 }
 
@@ -255,6 +261,7 @@ void talk_prefill(Tensor q, Tensor k, Tensor v, Tensor table, Tensor positions, 
               "talk_frag bf16 [tiles, 64, 8] (ops.talk_fragment)");
   check_aligned(talk_frag, "talk_frag");
   p.talk_frag = bfp(talk_frag);
+  p.max_tiles = (int)max_tiles(max_ctx, window > 0 ? window + 15 : 0, keep);
   p.lse = f32p(lse, q.size(0) * H, "lse");
   p.splits = (int)splits;
   if (splits > 1) {
@@ -269,9 +276,9 @@ void talk_prefill(Tensor q, Tensor k, Tensor v, Tensor table, Tensor positions, 
   check_rc(vwa_talk_prefill(&p, cur_stream(q)), "talk_prefill");
 }
 
-void mingru(Tensor z, Tensor x, Tensor gt, c10::optional<Tensor> zb, c10::optional<Tensor> xb, Tensor seq_ids, Tensor positions,
-            Tensor slots, Tensor state, double out_scale, Tensor out, c10::optional<Tensor> chunks, c10::optional<Tensor> scratch) {
-  c10::DeviceGuard g(z.device());
+MinGruParams mingru_params(const Tensor& z, const Tensor& x, const Tensor& gt, const c10::optional<Tensor>& zb,
+                           const c10::optional<Tensor>& xb, const Tensor& seq_ids, const Tensor& positions, const Tensor& slots,
+                           const Tensor& state, double out_scale, const Tensor& out) {
   const bool f32 = t_is_f32(z, "z");
   const int64_t rows = out.size(0), width = state.size(1);
   for (const Tensor* t : {&z, &x, &gt}) {
@@ -300,6 +307,14 @@ void mingru(Tensor z, Tensor x, Tensor gt, c10::optional<Tensor> zb, c10::option
   p.out_scale = (float)out_scale;
   p.out = out.data_ptr();
   p.ldo = (int)out.stride(0);
+  return p;
+}
+
+void mingru(Tensor z, Tensor x, Tensor gt, c10::optional<Tensor> zb, c10::optional<Tensor> xb, Tensor seq_ids, Tensor positions,
+            Tensor slots, Tensor state, double out_scale, Tensor out, c10::optional<Tensor> chunks, c10::optional<Tensor> scratch) {
+  c10::DeviceGuard g(z.device());
+  MinGruParams p = mingru_params(z, x, gt, zb, xb, seq_ids, positions, slots, state, out_scale, out);
+  const int64_t width = p.width;
   if (!chunks.has_value()) {
     check_rc(vwa_mingru_rows(&p, cur_stream(z)), "mingru_rows");
     return;
@@ -315,6 +330,16 @@ void mingru(Tensor z, Tensor x, Tensor gt, c10::optional<Tensor> zb, c10::option
   check_rc(vwa_mingru_scan(&p, cur_stream(z)), "mingru_scan");
 }
 
+// a decode step's rows: rotation + cache write and the recurrence in one launch (arguments of both)
+void qkv_mingru(Tensor x, int64_t H, int64_t G, int64_t dk, int64_t dv, int64_t rot_dims, Tensor rope, Tensor positions,
+                Tensor slots, Tensor q_out, Tensor k, Tensor v, Tensor z, Tensor u, Tensor gt, c10::optional<Tensor> zb,
+                c10::optional<Tensor> xb, Tensor seq_ids, Tensor state, double out_scale, Tensor out) {
+  c10::DeviceGuard g(x.device());
+  const QkvCacheParams p = qkv_params(x, H, G, dk, dv, rot_dims, rope, positions, slots, q_out, k, v);
+  const MinGruParams m = mingru_params(z, u, gt, zb, xb, seq_ids, positions, slots, state, out_scale, out);
+  check_rc(vwa_qkv_mingru(&p, &m, cur_stream(x)), "qkv_mingru");
+}
+
 }  // namespace
 
 void bind_stack(py::module_& m) {
@@ -323,6 +348,7 @@ void bind_stack(py::module_& m) {
   m.def("layernorm_f32", &layernorm_f32);
   m.def("embedding_f32", &embedding_f32);
   m.def("qkv_cache", &qkv_cache);
+  m.def("qkv_mingru", &qkv_mingru);
   m.def("talk_chunks", &talk_chunks);
   m.def("talk_prefill_part", [](int64_t H, int64_t G, int64_t dk, int64_t dv) {
     return vwa_talk_prefill_part((int)H, (int)G, (int)dk, (int)dv);

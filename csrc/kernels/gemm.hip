@@ -461,6 +461,14 @@ VWA_DEVICE float finish_item(const GemmParams& p, int m, int c, const float (&a)
       return 0.f;
     }
   }
+  if (p.y_f32 == 2) {  // f32 residual stream: 16-byte accesses (rows are 32-byte aligned)
+    const float4* r = reinterpret_cast<const float4*>(reinterpret_cast<const float*>(p.R) + (size_t)m * p.ldr + c);
+    float4* y = reinterpret_cast<float4*>(reinterpret_cast<float*>(p.Y) + (size_t)m * p.ldy + c);
+    const float4 r0 = r[0], r1 = r[1];
+    y[0] = make_float4(v[0] + r0.x, v[1] + r0.y, v[2] + r0.z, v[3] + r0.w);
+    y[1] = make_float4(v[4] + r1.x, v[5] + r1.y, v[6] + r1.z, v[7] + r1.w);
+    return 0.f;
+  }
   if (p.y_f32) {
 #pragma unroll
     for (int e = 0; e < 8; ++e) store_out<EPI>(p, m, c + e, v[e]);

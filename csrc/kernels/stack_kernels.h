@@ -64,6 +64,7 @@ struct TalkPrefillParams {
   // [64 lanes][8], lane (row rl, group b), element e: talk[16 mt + rl][head of k], k = 8 b + e -- HT 32:
   // head k; 16: k mod 16; 8: k mod 8 for k < 16, else 0; <= 4: k mod 4 for k < 8, else 0
   const uint16_t* talk_frag;
+  int max_tiles;                    // key tiles a query tile can see at most (<= 1024)
   float* lse;                       // [rows of q][H] scratch
   int splits;                       // workgroups per tile over its keys
   float* part;                      // [n_tiles][splits][vwa_talk_prefill_part floats] (splits > 1)
@@ -97,6 +98,8 @@ int vwa_layernorm_f32(const float* x, int ldx, const float* w, const float* b, v
 int vwa_embedding_f32(const int* ids, const void* table, int ld, float* out, int ldo, int rows, int D, int Dpad, int vocab,
                       int f32, hipStream_t st);
 int vwa_qkv_cache(const QkvCacheParams* p, hipStream_t st);
+// a decode step's qkv_cache and mingru_rows over the same rows, one launch
+int vwa_qkv_mingru(const QkvCacheParams* p, const MinGruParams* g, hipStream_t st);
 int vwa_talk_attention(const TalkAttnParams* p, hipStream_t st);
 int vwa_talk_prefill(const TalkPrefillParams* p, hipStream_t st);
 // partial floats per (tile, split) of vwa_talk_prefill, < 0 if it does not take these sizes

@@ -3,18 +3,12 @@
 //  layernorm_f32 : y (T) = (x - mean) * rstd * w + b of f32 rows, two-pass statistics in f32
 //  embedding_f32 : f32 residual rows from a T table
 //  qkv_cache     : partial rotation of q / k heads + paged cache write (V transposed inside a block)
-#include "common.h"
-#include "stack_kernels.h"
+//  qkv_mingru    : qkv_cache and the recurrence's rows form of a decode step in one launch
+#include "recurrence.h"
 
 using namespace vwa;
 
 namespace {
-
-template <class T> VWA_DEVICE float ldv(const T* p);
-template <> VWA_DEVICE float ldv<u16>(const u16* p) { return bf2f(*p); }
-template <> VWA_DEVICE float ldv<float>(const float* p) { return *p; }
-VWA_DEVICE void stv(u16* p, float v) { *p = f2bf(v); }
-VWA_DEVICE void stv(float* p, float v) { *p = v; }
 
 // four consecutive values
 VWA_DEVICE void st4(u16* p, const float (&v)[4]) {
@@ -96,11 +90,10 @@ __global__ __launch_bounds__(256) void embedding_f32_kernel(const int* __restric
     out[(size_t)row * ldo + c] = ok && c < D ? ldv(table + (size_t)id * ld + c) : 0.f;
 }
 
-// One workgroup per row.  VEC consecutive dimensions per thread (8 when the half rotation is a
+// Part of one row.  VEC consecutive dimensions per thread (8 when the half rotation is a
 // multiple of 8, else 1): a rotated chunk reads its partner chunk rot_dims / 2 away.
 template <class T, int VEC>
-__global__ __launch_bounds__(256) void qkv_cache_kernel(QkvCacheParams p) {
-  const int row = blockIdx.x;
+VWA_DEVICE void qkv_cache_row(const QkvCacheParams& p, int row, int part, int parts) {
   const T* x = reinterpret_cast<const T*>(p.x) + (size_t)row * p.ldx;
   const int64_t slot = p.slots[row];
   const int pos = min(max(p.positions[row], 0), p.max_pos - 1);
@@ -110,7 +103,7 @@ __global__ __launch_bounds__(256) void qkv_cache_kernel(QkvCacheParams p) {
   const float* cs = p.rope + (size_t)pos * p.rot_dims;
   const int cph = p.dk / VEC, nqk = (p.H + p.G) * cph;
   T* kc = reinterpret_cast<T*>(p.k) + blk * p.k_sb + (int64_t)off * p.dk;
-  for (int u = blockIdx.y * 256 + threadIdx.x; u < nqk; u += gridDim.y * 256) {
+  for (int u = part * 256 + threadIdx.x; u < nqk; u += parts * 256) {
     const int head = u / cph, e = (u % cph) * VEC;
     const T* xh = x + head * p.dk;
     float o[VEC];
@@ -145,10 +138,23 @@ __global__ __launch_bounds__(256) void qkv_cache_kernel(QkvCacheParams p) {
   if (slot < 0) return;
   const T* xv = x + (p.H + p.G) * p.dk;
   T* vc = reinterpret_cast<T*>(p.v) + blk * p.v_sb + off;
-  for (int u = blockIdx.y * 256 + threadIdx.x; u < p.G * p.dv; u += gridDim.y * 256) {
+  for (int u = part * 256 + threadIdx.x; u < p.G * p.dv; u += parts * 256) {
     const int g = u / p.dv, d = u % p.dv;
     vc[(int64_t)g * p.v_sh + (int64_t)d * p.block_size] = xv[u];
   }
+}
+
+template <class T, int VEC>
+__global__ __launch_bounds__(256) void qkv_cache_kernel(QkvCacheParams p) {
+  qkv_cache_row<T, VEC>(p, blockIdx.x, blockIdx.y, gridDim.y);
+}
+
+// grid.y: kQkvParts parts of the row's heads, then its recurrence channels by 256
+constexpr int kQkvParts = 4;
+template <class T, int VEC>
+__global__ __launch_bounds__(256) void qkv_mingru_kernel(QkvCacheParams p, MinGruParams g) {
+  if (blockIdx.y < kQkvParts) qkv_cache_row<T, VEC>(p, blockIdx.x, blockIdx.y, kQkvParts);
+  else mingru_row<T>(g, blockIdx.x, (blockIdx.y - kQkvParts) * 256 + threadIdx.x);
 }
 
 }  // namespace
@@ -179,18 +185,40 @@ extern "C" int vwa_embedding_f32(const int* ids, const void* table, int ld, floa
   return (int)hipGetLastError();
 }
 
+namespace {
+int check_qkv(const QkvCacheParams* p) {
+  return p->rows < 1 || p->H < 1 || p->G < 1 || p->dk < 1 || p->dv < 1 || p->rot_dims % 2 || p->rot_dims > p->dk ||
+         p->max_pos < 1 || p->block_size < 1;
+}
+bool qkv_vec(const QkvCacheParams* p) {
+  return (p->rot_dims / 2) % 8 == 0 && p->dk % 8 == 0 && p->ldq % 8 == 0 && p->ldx % 8 == 0;
+}
+}  // namespace
+
 extern "C" int vwa_qkv_cache(const QkvCacheParams* p, hipStream_t st) {
-  if (p->rows < 1 || p->H < 1 || p->G < 1 || p->dk < 1 || p->dv < 1 || p->rot_dims % 2 || p->rot_dims > p->dk ||
-      p->max_pos < 1 || p->block_size < 1)
-    return -1;
-  const bool vec = (p->rot_dims / 2) % 8 == 0 && p->dk % 8 == 0 && p->ldq % 8 == 0 && p->ldx % 8 == 0;
-  const dim3 grid(p->rows, p->rows <= 64 ? 4 : 1), block(256);
+  if (check_qkv(p)) return -1;
+  const bool vec = qkv_vec(p);
+  const dim3 grid(p->rows, p->rows <= 64 ? kQkvParts : 1), block(256);
   if (p->f32) {
     if (vec) hipLaunchKernelGGL((qkv_cache_kernel<float, 8>), grid, block, 0, st, *p);
     else hipLaunchKernelGGL((qkv_cache_kernel<float, 1>), grid, block, 0, st, *p);
   } else {
     if (vec) hipLaunchKernelGGL((qkv_cache_kernel<u16, 8>), grid, block, 0, st, *p);
     else hipLaunchKernelGGL((qkv_cache_kernel<u16, 1>), grid, block, 0, st, *p);
+  }
+  return (int)hipGetLastError();
+}
+
+extern "C" int vwa_qkv_mingru(const QkvCacheParams* p, const MinGruParams* g, hipStream_t st) {
+  if (check_qkv(p) || g->rows != p->rows || g->width < 1 || g->f32 != p->f32) return -1;
+  const bool vec = qkv_vec(p);
+  const dim3 grid(p->rows, kQkvParts + (g->width + 255) / 256), block(256);
+  if (p->f32) {
+    if (vec) hipLaunchKernelGGL((qkv_mingru_kernel<float, 8>), grid, block, 0, st, *p, *g);
+    else hipLaunchKernelGGL((qkv_mingru_kernel<float, 1>), grid, block, 0, st, *p, *g);
+  } else {
+    if (vec) hipLaunchKernelGGL((qkv_mingru_kernel<u16, 8>), grid, block, 0, st, *p, *g);
+    else hipLaunchKernelGGL((qkv_mingru_kernel<u16, 1>), grid, block, 0, st, *p, *g);
   }
   return (int)hipGetLastError();
 }

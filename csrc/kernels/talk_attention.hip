@@ -16,9 +16,8 @@
 //     which the cache stores transposed (its A operand, no staging).  Chunks of a row are added in
 //     chunk order by the last-arriving workgroup (sc1 hand-off + ticket, as decode attention).
 //  2) prefill form (bf16), per 16 consecutive queries: launch A reduces the scores to log-sum-exps;
-//     launch B recomputes them, a wave holding every head of its key tile, mixes the heads on the MFMA
-//     and hands the mixed weights through LDS (B-operand order) to the waves' (kv head, 16 value
-//     columns) tiles.
+//     launch B recomputes them (a wave per few heads), mixes the heads on the MFMA and multiplies by V^T,
+//     the weights passing between the waves through LDS in B-operand order.
 #include "common.h"
 #include "mq_attention.h"
 #include "stack_kernels.h"
@@ -69,6 +68,13 @@ VWA_DEVICE bool sees(int i, int j, int window, int keep) {
   return j <= i && (window <= 0 || i - j < window || j < keep);
 }
 
+VWA_DEVICE void st_sc1_x4(__amdgpu_buffer_rsrc_t r, int off, const f32x4& v) {
+  __builtin_amdgcn_raw_buffer_store_b128(__builtin_bit_cast(u32x4, v), r, off, 0, 16);
+}
+VWA_DEVICE f32x4 ld_sc1_x4(__amdgpu_buffer_rsrc_t r, int off) {
+  return __builtin_bit_cast(f32x4, __builtin_amdgcn_raw_buffer_load_b128(r, off, 0, 16));
+}
+
 // ------------------------------------------------------------------------------------------ rows form
 template <class T>
 __global__ __launch_bounds__(256) void talk_scores_kernel(TalkAttnParams p) {
@@ -81,8 +87,9 @@ __global__ __launch_bounds__(256) void talk_scores_kernel(TalkAttnParams p) {
   const Vis v = vis_tiles(pos, pos, p.window, p.keep);
   if (chunk * kChunkTiles >= v.n) return;
   const int R = p.H / p.G, Rb = min(16, R - r0);
-  const int lane = lane_id(), w = threadIdx.x >> 6, rl = lane & 15, b = lane >> 4;
+  const int lane = lane_id(), w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), rl = lane & 15, b = lane >> 4;
   const T* q = reinterpret_cast<const T*>(p.q) + (size_t)row * p.ldq + (size_t)(c * R + r0 + min(rl, Rb - 1)) * p.dk + b * M::EPL;
+  const int lb = __builtin_ctz(p.block_size);
   const T* kp[2];
   int key0[2];
   bool ok[2];
@@ -91,9 +98,9 @@ __global__ __launch_bounds__(256) void talk_scores_kernel(TalkAttnParams p) {
     const int t = chunk * kChunkTiles + w * 2 + u;
     ok[u] = t < v.n;
     key0[u] = tile_of(v, ok[u] ? t : v.n - 1) * kTile;
-    const int64_t blk = p.block_table[(int64_t)seq * p.table_stride + key0[u] / p.block_size];
+    const int64_t blk = p.block_table[(int64_t)seq * p.table_stride + (key0[u] >> lb)];
     kp[u] = reinterpret_cast<const T*>(p.k) + blk * p.k_sb + (int64_t)c * p.k_sh +
-            (int64_t)(key0[u] % p.block_size + rl) * p.dk + b * M::EPL;
+            (int64_t)((key0[u] & (p.block_size - 1)) + rl) * p.dk + b * M::EPL;
   }
   f32x4 acc[2] = {};
 #pragma unroll 4
@@ -181,17 +188,53 @@ __global__ __launch_bounds__(256) void talk_mix_kernel(TalkAttnParams p) {
   float* hm = wt + p.H * kChunk;                                        // [H] max
   float* hl = hm + p.H;                                                 // [H] 1 / sum
   const int g0 = p.talk ? 0 : h0, g1 = p.talk ? p.H : h0 + Rb;          // heads whose weights are needed
+  const int lane = lane_id(), w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), rl = lane & 15, b = lane >> 4;
+  // ---- everything that is read is requested first: the scores of this thread's (key, heads), the first
+  // value tiles of this wave (16-column tiles w, w + 4, ...), the chunk statistics
+  constexpr int kPre = 8;
+  const int j = threadIdx.x & (kChunk - 1), hp = w >> 1;                // key, head parity
+  const float* srow = p.s + (size_t)ri * p.H * p.nch * kChunk + chunk * kChunk + j;
+  float sv[kPre];
+#pragma unroll
+  for (int k = 0; k < kPre; ++k) sv[k] = srow[(size_t)min(g0 + hp + 2 * k, g1 - 1) * p.nch * kChunk];
+  constexpr int TPS = M::KS / kTile;                 // tiles per step (bf16 2, f32 1)
+  constexpr int NST = kChunkTiles / TPS;
+  const int lb = __builtin_ctz(p.block_size);
+  const T* vb[NST];
+  bool vok[NST];
+#pragma unroll
+  for (int s = 0; s < NST; ++s) {
+    const int t = chunk * kChunkTiles + s * TPS + (TPS == 2 ? b >> 1 : 0);
+    vok[s] = t < v.n;
+    const int key = tile_of(v, vok[s] ? t : v.n - 1) * kTile;
+    const int64_t blk = p.block_table[(int64_t)seq * p.table_stride + (key >> lb)];
+    vb[s] = reinterpret_cast<const T*>(p.v) + blk * p.v_sb + (int64_t)c * p.v_sh + (int64_t)rl * p.block_size +
+            (key & (p.block_size - 1)) + (TPS == 2 ? (b & 1) : b) * M::EPL;
+  }
+  uint4 va[NST], vn[NST];
+  auto load_v = [&](uint4 (&x)[NST], int d) {
+#pragma unroll
+    for (int s = 0; s < NST; ++s)
+      x[s] = vok[s] ? *reinterpret_cast<const uint4*>(vb[s] + (int64_t)min(d, p.dv - 16) * p.block_size) : make_uint4(0, 0, 0, 0);
+  };
+  load_v(va, w * 16);
+  load_v(vn, w * 16 + 64);
   // ---- statistics of every needed head: 16 lanes per head
   for (int h = g0 + (threadIdx.x >> 4); h < g1; h += 16) {
     const float* st = p.stat + ((size_t)ri * p.H + h) * p.nch * 2;
-    float m = -INFINITY;
-    for (int k = threadIdx.x & 15; k < nact; k += 16) m = fmaxf(m, st[2 * k]);
+    float m = -INFINITY, s = 0.f;
+    for (int k = threadIdx.x & 15; k < nact; k += 16) {
+      const float2 ms = *reinterpret_cast<const float2*>(st + 2 * k);
+      const float mn = fmaxf(m, ms.x);
+      if (ms.y > 0.f) s = (s > 0.f ? s * __expf(m - mn) : 0.f) + ms.y * __expf(ms.x - mn);
+      m = mn;
+    }
 #pragma unroll
-    for (int o = 8; o > 0; o >>= 1) m = fmaxf(m, __shfl_xor(m, o, 64));
-    float s = 0.f;
-    for (int k = threadIdx.x & 15; k < nact; k += 16) s += st[2 * k + 1] > 0.f ? st[2 * k + 1] * __expf(st[2 * k] - m) : 0.f;
-#pragma unroll
-    for (int o = 8; o > 0; o >>= 1) s += __shfl_xor(s, o, 64);
+    for (int o = 8; o > 0; o >>= 1) {
+      const float mo = __shfl_xor(m, o, 64), so = __shfl_xor(s, o, 64), mn = fmaxf(m, mo);
+      s = (s > 0.f ? s * __expf(m - mn) : 0.f) + (so > 0.f ? so * __expf(mo - mn) : 0.f);
+      m = mn;
+    }
     if ((threadIdx.x & 15) == 0) {
       hm[h] = m;
       hl[h] = 1.f / s;
@@ -199,26 +242,20 @@ __global__ __launch_bounds__(256) void talk_mix_kernel(TalkAttnParams p) {
   }
   __syncthreads();
   // ---- normalised weights of the chunk's keys (0 past the last tile)
-  {
-    const int j = threadIdx.x & (kChunk - 1);
-    for (int h = g0 + (threadIdx.x >> 7); h < g1; h += 2) {
-      float x = 0.f;
-      if (j < nkey) {
-        const float s = p.s[((size_t)ri * p.H + h) * p.nch * kChunk + chunk * kChunk + j];
-        x = s == -INFINITY ? 0.f : __expf(s - hm[h]) * hl[h];
-      }
-      wt[h * kChunk + j] = x;
-    }
-  }
+  auto weight = [&](int h, float s) { wt[h * kChunk + j] = j < nkey && s != -INFINITY ? __expf(s - hm[h]) * hl[h] : 0.f; };
+#pragma unroll
+  for (int k = 0; k < kPre; ++k)
+    if (g0 + hp + 2 * k < g1) weight(g0 + hp + 2 * k, sv[k]);
+  for (int h = g0 + hp + 2 * kPre; h < g1; h += 2) weight(h, srow[(size_t)h * p.nch * kChunk]);
   __syncthreads();
   // ---- mixed weights of this kv head's query heads
   {
-    const int j = threadIdx.x & (kChunk - 1);
     const int idx = ((j / M::KS) * 64 + 16 * ((j % M::KS) / M::EPL)) * M::EPL + j % M::EPL;
-    for (int r = threadIdx.x >> 7; r < Rb; r += 2) {
+    for (int r = hp; r < Rb; r += 2) {
       float x = 0.f;
       if (p.talk) {
-        const float* tk = p.talk + (size_t)(h0 + r) * p.H;
+        const float* tk = p.talk + (size_t)(h0 + r) * p.H;  // (uniform per wave: scalar loads)
+#pragma unroll 8
         for (int g = 0; g < p.H; ++g) x += tk[g] * wt[g * kChunk + j];
       } else {
         x = wt[(h0 + r) * kChunk + j];
@@ -227,33 +264,18 @@ __global__ __launch_bounds__(256) void talk_mix_kernel(TalkAttnParams p) {
     }
   }
   __syncthreads();
-  // ---- O^T = V^T . P^T: wave w takes 16-column tiles w, w + 4, ... of the values
-  const int lane = lane_id(), w = threadIdx.x >> 6, rl = lane & 15, b = lane >> 4;
-  constexpr int TPS = M::KS / kTile;                 // tiles per step (bf16 2, f32 1)
-  constexpr int NST = kChunkTiles / TPS;
-  const T* vb[NST];
-  bool vok[NST];
-#pragma unroll
-  for (int s = 0; s < NST; ++s) {
-    const int t = chunk * kChunkTiles + s * TPS + (TPS == 2 ? b >> 1 : 0);
-    vok[s] = t < v.n;
-    const int key = tile_of(v, vok[s] ? t : v.n - 1) * kTile;
-    const int64_t blk = p.block_table[(int64_t)seq * p.table_stride + key / p.block_size];
-    vb[s] = reinterpret_cast<const T*>(p.v) + blk * p.v_sb + (int64_t)c * p.v_sh + (int64_t)rl * p.block_size +
-            key % p.block_size + (TPS == 2 ? (b & 1) : b) * M::EPL;
-  }
+  // ---- O^T = V^T . P^T
   const int nz = gridDim.z;
   float* prow = p.part + ((size_t)ri * p.nch) * p.H * p.dv;
   const __amdgpu_buffer_rsrc_t rp = rsrc_f32(prow, (int64_t)p.nch * p.H * p.dv);
   for (int d = w * 16; d < p.dv; d += 64) {
-    uint4 va[NST];
-#pragma unroll
-    for (int s = 0; s < NST; ++s)
-      va[s] = vok[s] ? *reinterpret_cast<const uint4*>(vb[s] + (int64_t)d * p.block_size) : make_uint4(0, 0, 0, 0);
     f32x4 acc = {};
 #pragma unroll
     for (int s = 0; s < NST; ++s)
       acc = M::mma(va[s], *reinterpret_cast<const uint4*>(pf + ((size_t)s * 64 + lane) * M::EPL), acc);
+#pragma unroll
+    for (int s = 0; s < NST; ++s) va[s] = vn[s];
+    if (d + 128 < p.dv) load_v(vn, d + 128);
     if (rl >= Rb) continue;
     const int h = h0 + rl;
     if (nact == 1) {
@@ -261,9 +283,7 @@ __global__ __launch_bounds__(256) void talk_mix_kernel(TalkAttnParams p) {
 #pragma unroll
       for (int i = 0; i < 4; ++i) stv(out + (size_t)h * p.dv + d + 4 * b + i, acc[i] * g);
     } else {
-      const int64_t o = ((int64_t)chunk * p.H + h) * p.dv + d + 4 * b;
-      st_sc1_f2(rp, o, acc[0], acc[1]);
-      st_sc1_f2(rp, o + 2, acc[2], acc[3]);
+      st_sc1_x4(rp, (int)((((int64_t)chunk * p.H + h) * p.dv + d + 4 * b) * 4), acc);
     }
   }
   if (nact == 1) return;
@@ -296,14 +316,16 @@ __global__ __launch_bounds__(256) void talk_mix_kernel(TalkAttnParams p) {
 }
 
 // ------------------------------------------------------------------------------------------ prefill form
-constexpr int kTab = 1024;                  // block-table entries kept in LDS
-constexpr int kNone = -1;
+constexpr int kTab = 1024;                  // tiles a query tile may see (their cache places are kept in LDS)
 
-VWA_DEVICE void st_sc1_x4(__amdgpu_buffer_rsrc_t r, int off, const f32x4& v) {
-  __builtin_amdgcn_raw_buffer_store_b128(__builtin_bit_cast(u32x4, v), r, off, 0, 16);
-}
-VWA_DEVICE f32x4 ld_sc1_x4(__amdgpu_buffer_rsrc_t r, int off) {
-  return __builtin_bit_cast(f32x4, __builtin_amdgcn_raw_buffer_load_b128(r, off, 0, 16));
+// cache place of every visible tile: block * (tiles per block) + tile in the block
+VWA_DEVICE void tile_table(const TalkAttnParams& p, const Vis& v, int seq, int* tab, int threads) {
+  const int* gtab = p.block_table + (int64_t)seq * p.table_stride;
+  const int lb = __builtin_ctz(p.block_size) - 4;           // log2 of the tiles per block
+  for (int t = threadIdx.x; t < v.n; t += threads) {
+    const int tl = tile_of(v, t);
+    tab[t] = (gtab[tl >> lb] << lb) + (tl & ((1 << lb) - 1));
+  }
 }
 
 // every key of the tile visible to every query p0 .. p1 (no per-key masks needed)
@@ -318,7 +340,7 @@ template <int RB, int KSN>
 __global__ __launch_bounds__(256) void talk_lse_kernel(TalkPrefillParams pp) {
   const TalkAttnParams& p = pp.a;
   __shared__ float red[4][RB][16][2];
-  const int lane = lane_id(), w = threadIdx.x >> 6, rl = lane & 15, b = lane >> 4;
+  const int lane = lane_id(), w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), rl = lane & 15, b = lane >> 4;
   const int lt = xcd_remap((int)blockIdx.x, pp.n_tiles * p.G);  // (a kv head's tiles share an XCD's L2)
   const int c = lt / pp.n_tiles, tile = lt % pp.n_tiles;
   const int row0 = pp.tiles[2 * tile], nq = pp.tiles[2 * tile + 1];
@@ -327,22 +349,26 @@ __global__ __launch_bounds__(256) void talk_lse_kernel(TalkPrefillParams pp) {
   const int qrow = row0 + min(rl, nq - 1), qpos = pos0 + min(rl, nq - 1);
   const Vis v = vis_tiles(pos0, pos1, p.window, p.keep);
   const float sl2 = p.scale * kLog2e;
-  const int* gtab = p.block_table + (int64_t)seq * p.table_stride;
+  __shared__ int tab[kTab];
+  tile_table(p, v, seq, tab, 256);
+  const int lb = __builtin_ctz(p.block_size) - 4;
+  // (steps past dk: the query fragment is zero, the key fragment repeats the last step)
   uint4 qf[RB][KSN];
 #pragma unroll
   for (int r = 0; r < RB; ++r)
 #pragma unroll
-    for (int s = 0; s < KSN; ++s)
-      if (s < nst)
-        qf[r][s] = ld128(reinterpret_cast<const u16*>(p.q) + (size_t)qrow * p.ldq + (size_t)(c * R + r0 + min(r, nr - 1)) * p.dk +
-                         b * 8 + s * 32);
+    for (int s = 0; s < KSN; ++s) {
+      qf[r][s] = ld128(reinterpret_cast<const u16*>(p.q) + (size_t)qrow * p.ldq + (size_t)(c * R + r0 + min(r, nr - 1)) * p.dk +
+                       b * 8 + min(s, nst - 1) * 32);
+      if (s >= nst) qf[r][s] = make_uint4(0, 0, 0, 0);
+    }
+  __syncthreads();
+  const u16* kbase = reinterpret_cast<const u16*>(p.k) + (int64_t)c * p.k_sh + rl * p.dk + b * 8;
   auto load_k = [&](uint4 (&kf)[KSN], int t) {
-    const int key0 = tile_of(v, t) * kTile;
-    const u16* kp = reinterpret_cast<const u16*>(p.k) + (int64_t)gtab[key0 / p.block_size] * p.k_sb + (int64_t)c * p.k_sh +
-                    (int64_t)(key0 % p.block_size + rl) * p.dk + b * 8;
+    const int ts = __builtin_amdgcn_readfirstlane(tab[min(t, v.n - 1)]);
+    const u16* kp = kbase + (int64_t)(ts >> lb) * p.k_sb + (ts & ((1 << lb) - 1)) * kTile * p.dk;
 #pragma unroll
-    for (int s = 0; s < KSN; ++s)
-      if (s < nst) kf[s] = ld128(kp + s * 32);
+    for (int s = 0; s < KSN; ++s) kf[s] = ld128(kp + min(s, nst - 1) * 32);
   };
   float m[RB], l[RB];
 #pragma unroll
@@ -362,8 +388,7 @@ __global__ __launch_bounds__(256) void talk_lse_kernel(TalkPrefillParams pp) {
     for (int r = 0; r < RB; ++r) {
       f32x4 a = {};
 #pragma unroll
-      for (int s = 0; s < KSN; ++s)
-        if (s < nst) a = mfma16(as_bf16x8(kf[s]), as_bf16x8(qf[r][s]), a);
+      for (int s = 0; s < KSN; ++s) a = mfma16(as_bf16x8(kf[s]), as_bf16x8(qf[r][s]), a);
       float s[4], mn = m[r];
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
@@ -378,12 +403,12 @@ __global__ __launch_bounds__(256) void talk_lse_kernel(TalkPrefillParams pp) {
     }
   };
   uint4 ka[KSN], kb[KSN];
-  if (w < v.n) load_k(ka, w);
+  load_k(ka, w);
   for (int t = w; t < v.n; t += 8) {
-    if (t + 4 < v.n) load_k(kb, t + 4);
+    load_k(kb, t + 4);
     add_tile(ka, t);
     if (t + 4 >= v.n) break;
-    if (t + 8 < v.n) load_k(ka, t + 8);
+    load_k(ka, t + 8);
     add_tile(kb, t + 4);
   }
 #pragma unroll
@@ -410,257 +435,239 @@ __global__ __launch_bounds__(256) void talk_lse_kernel(TalkPrefillParams pp) {
   pp.lse[(size_t)(row0 + q) * p.H + c * R + r0 + r] = mm + __log2f(ll);
 }
 
-// rows [0 1 2 3] of 16 lanes of four registers, transposed: out_b row b' = in_b' row b
-VWA_DEVICE void transpose4(unsigned& a, unsigned& b, unsigned& c, unsigned& d) {
-  const auto r = __builtin_amdgcn_permlane32_swap(a, c, false, false);
-  const auto s = __builtin_amdgcn_permlane32_swap(b, d, false, false);
-  const auto x = __builtin_amdgcn_permlane16_swap(r[0], s[0], false, false);
-  const auto y = __builtin_amdgcn_permlane16_swap(r[1], s[1], false, false);
-  a = x[0];
-  b = x[1];
-  c = y[0];
-  d = y[1];
-}
-
 // Pass 2.  GP, RP: kv heads and query heads per kv head in the padded head order h = c * RP + r; NV: (kv
-// head, 16 value columns) tiles per wave; NW waves; KSN: 32-wide steps over the q / k dimensions.
-// Heads are mixed on the MFMA: a weight x = hi + lo (two bf16, 16 mantissa bits) is one B operand with
-// k = (hi | lo, head) against the talk matrix (bf16 as stored) repeated for both halves; the lanes hold
-// every head of their own (query, key), so the operand is a 4 x 4 transpose of 16-lane groups.
-// A tile's key rows enter the score product in the order 4 i + b (row 4 b + i), so the four results of one
-// key element i are four consecutive keys.
+// head, 16 value columns) tiles per wave; KSN: 32-wide steps over the q / k dimensions.  8 waves walk
+// the keys 32 (few heads: 64) at a time, in three stages with two barriers:
+//   scores   a wave owns HW heads (their query fragments stay in its registers) and two key tiles; the
+//            normalised weights x go to LDS as hi + lo bf16 pairs (16 mantissa bits together), in the
+//            B-operand order of the mixing: k = (hi | lo, head), column = query, one block per key
+//   mixing   a wave takes 4 keys: talk (bf16 as stored, repeated for both halves) times that block on
+//            the MFMA; the mixed weights go back to LDS as bf16 in the B-operand order of the values
+//   values   a wave owns NV value tiles of a kv head's query heads: O^T += V^T . P^T
+// The values stage of one round and the scores of the next lie between the same two barriers.
 // The tile's keys may be split over workgroups (blockIdx.y): their sums are added in order by the last
 // one to finish.
-template <int GP, int RP, int NV, int NW, int KSN>
+constexpr int kPW = 8;                                               // waves
+template <int GP, int RP, int NV, int KSN>
 struct PrefillCfg {
-  static constexpr int HT = GP * RP, KEYS = NW * kTile, KG = KEYS / 32;
+  static constexpr int HT = GP * RP, HX = HT < 4 ? 4 : HT;
+  static constexpr int KT = HX == 4 ? 4 : 2, KEYS = KT * kTile, KG = KT / 2;   // tiles, keys, 32-key groups per round
+  static constexpr int HW = HX > kPW ? HX / kPW : 1;                 // heads per wave
+  static constexpr int HWAVES = HX / HW;                             // waves over the heads; the others take other tiles
+  static constexpr int NCW = HW > RP ? HW / RP : 1;                  // kv heads per wave
   static constexpr int MT = HT > 16 ? 2 : 1;                         // 16-row tiles of the mixed heads
   static constexpr int KM = HT > 16 ? 2 : 1;                         // 32-deep steps of the mixing
-  static constexpr int P_BYTES = HT * KEYS * 16 * 2;                 // mixed weights
-  static constexpr bool QL = HT * KSN <= 64;                         // query fragments in LDS (else L1 / L2)
-  static size_t lds(int dk) { return P_BYTES + HT * 16 * 4 + kTab * 4 + (QL ? (size_t)HT * dk * 16 * 2 : 0); }
+  // next keys requested after the values (not before the mixing): their registers would not fit beside
+  // the accumulators and query fragments
+  static constexpr bool LATE_K = NV * RP * 4 + HW * KSN * 4 > 128;
+  static constexpr int NC = LATE_K ? (NV < 2 ? NV : 2) : NV < 4 ? NV : 4;   // value tiles loaded ahead
+  static constexpr int X_BYTES = KEYS * KM * 1024, P_BYTES = HX * KEYS * 16 * 2;
+  static constexpr int LDS = X_BYTES + P_BYTES + 2 * HX * 16 * 4 + kTab * 4;
 };
 
-template <int GP, int RP, int NV, int NW, int KSN>
-__global__ __launch_bounds__(NW * 64) void talk_prefill_kernel(TalkPrefillParams pp) {
-  using C = PrefillCfg<GP, RP, NV, NW, KSN>;
-  constexpr int HT = C::HT, KG = C::KG, HX = HT < 4 ? 4 : HT;
+// ONE: every wave's value tiles belong to one kv head (its mixed weights are read once per 32 keys)
+template <int GP, int RP, int NV, int KSN, bool ONE>
+__global__ __launch_bounds__(kPW * 64) void talk_prefill_kernel(TalkPrefillParams pp) {
+  using C = PrefillCfg<GP, RP, NV, KSN>;
+  constexpr int HT = C::HT, HX = C::HX, HW = C::HW, KG = C::KG, KT = C::KT;
   constexpr int HS = KG * 4 * 16 * 16;                               // bytes of a head's mixed weights
+  constexpr int KB = C::KM * 1024;                                   // bytes of a key's mixing operand
   const TalkAttnParams& p = pp.a;
   extern __shared__ __attribute__((aligned(16))) char smem[];
   __shared__ int s_last;
-  char* pm = smem;                                                   // [HT][KG][4][16 q][8 keys]
-  float* lse = reinterpret_cast<float*>(smem + C::P_BYTES);          // [HT][16]
-  int* btab = reinterpret_cast<int*>(lse + HT * 16);
-  uint4* qs = reinterpret_cast<uint4*>(btab + kTab);                 // [HT][dk / 32][64]
-  const int lane = lane_id(), w = threadIdx.x >> 6, rl = lane & 15, b = lane >> 4;
+  char* xm = smem;                                                   // [KEYS][KM][64][16 B]
+  char* pm = smem + C::X_BYTES;                                      // [HX][KG][4][16 q][8 keys]
+  float* lse = reinterpret_cast<float*>(pm + C::P_BYTES);            // [HX][16]
+  float* gate = lse + HX * 16;                                       // [HX][16] output factors
+  int* btab = reinterpret_cast<int*>(gate + HX * 16);
+  const int lane = lane_id(), w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), rl = lane & 15, b = lane >> 4;
   const int bt = xcd_remap((int)blockIdx.x, pp.n_tiles);
   const int row0 = pp.tiles[2 * bt], nq = pp.tiles[2 * bt + 1];
   const int R = p.H / p.G, nst = p.dk >> 5;
   const int pos0 = p.positions[row0], pos1 = pos0 + nq - 1, seq = p.seq_ids[row0];
   const int qrow = row0 + min(rl, nq - 1), qpos = pos0 + min(rl, nq - 1);
   const Vis v = vis_tiles(pos0, pos1, p.window, p.keep);
-  const int nit = (v.n + NW - 1) / NW, per = (nit + pp.splits - 1) / pp.splits;
+  const int nit = (v.n + KT - 1) / KT, per = (nit + pp.splits - 1) / pp.splits;
   const int nact = (nit + per - 1) / per;                            // splits with work
   const int split = blockIdx.y;
   if (split >= nact) return;
   const int it0 = split * per, it1 = min(nit, it0 + per);
   const float sl2 = p.scale * kLog2e;
-  const int* gtab = p.block_table + (int64_t)seq * p.table_stride;
-  const int nblk = pos1 / p.block_size + 1;
-  const bool tab = nblk <= kTab;
-  if (tab)
-    for (int i = threadIdx.x; i < nblk; i += NW * 64) btab[i] = gtab[i];
-  for (int u = threadIdx.x; u < p.H * 16; u += NW * 64) {
+  tile_table(p, v, seq, btab, kPW * 64);
+  const int lb = __builtin_ctz(p.block_size) - 4, lm = (1 << lb) - 1;
+  // (padding heads: weights exp2(-huge) = 0)
+  for (int u = threadIdx.x; u < HX * 16; u += kPW * 64)
+    if ((u >> 4) / RP >= p.G || (u >> 4) % RP >= R) lse[u] = 1e30f;
+  for (int u = threadIdx.x; u < p.H * 16; u += kPW * 64) {
     const int h = u >> 4, q = u & 15;
-    lse[((h / R) * RP + h % R) * 16 + q] = pp.lse[(size_t)(row0 + min(q, nq - 1)) * p.H + h];
+    const int at = ((h / R) * RP + h % R) * 16 + q;
+    lse[at] = pp.lse[(size_t)(row0 + min(q, nq - 1)) * p.H + h];
+    gate[at] = head_gate<u16>(p, row0 + min(q, nq - 1), h);
   }
+  // (operand slots no head writes -- padding heads, blocks past 2 HT -- stay zero)
+  for (int u = threadIdx.x; u < C::X_BYTES / 16; u += kPW * 64) reinterpret_cast<uint4*>(xm)[u] = make_uint4(0, 0, 0, 0);
+  // this wave's heads and tiles of a round
+  const int hw0 = (w % C::HWAVES) * HW, tw0 = (w / C::HWAVES) * 2;
   const u16* qp = reinterpret_cast<const u16*>(p.q) + (size_t)qrow * p.ldq + b * 8;
-  if constexpr (C::QL) {
-    for (int u = w; u < p.H * nst; u += NW) {
-      const int h = u / nst, s = u % nst;
-      qs[((size_t)((h / R) * RP + h % R) * nst + s) * 64 + lane] = ld128(qp + (size_t)h * p.dk + s * 32);
+  uint4 qf[HW][KSN];
+  float ls[HW];
+#pragma unroll
+  for (int k = 0; k < HW; ++k) {
+    const int c = min((hw0 + k) / RP, p.G - 1), r = min((hw0 + k) % RP, R - 1);
+#pragma unroll
+    for (int s = 0; s < KSN; ++s) {  // (steps past dk: zero here, the key fragment repeats the last step)
+      qf[k][s] = ld128(qp + (size_t)(c * R + r) * p.dk + min(s, nst - 1) * 32);
+      if (s >= nst) qf[k][s] = make_uint4(0, 0, 0, 0);
     }
   }
   uint4 tf[C::MT];                                                   // talk, A operand (both mixing steps use it)
 #pragma unroll
   for (int mt = 0; mt < C::MT; ++mt) tf[mt] = reinterpret_cast<const uint4*>(pp.talk_frag)[mt * 64 + lane];
   __syncthreads();
-  auto blk_of = [&](int key) -> int64_t {
-    const int i = key / p.block_size;
-    return tab ? btab[i] : gtab[i];
-  };
-  auto load_k = [&](uint4 (&kf)[KSN], int c, int t) {
-    const int key0 = tile_of(v, t) * kTile;
-    const u16* kp = reinterpret_cast<const u16*>(p.k) + blk_of(key0) * p.k_sb + (int64_t)c * p.k_sh +
-                    (int64_t)(key0 % p.block_size + 4 * (rl & 3) + (rl >> 2)) * p.dk + b * 8;
 #pragma unroll
-    for (int s = 0; s < KSN; ++s)
-      if (s < nst) kf[s] = ld128(kp + s * 32);
+  for (int k = 0; k < HW; ++k) ls[k] = lse[(hw0 + k) * 16 + rl];
+  const unsigned klane = rl * p.dk + b * 8;                          // (scalar tile base + one lane offset)
+  auto load_k = [&](uint4 (&kf)[C::NCW][2][KSN], int it) {
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+      const int ts = __builtin_amdgcn_readfirstlane(btab[min(it * KT + tw0 + u, v.n - 1)]);
+      const u16* kp = reinterpret_cast<const u16*>(p.k) + (int64_t)(ts >> lb) * p.k_sb + (ts & lm) * kTile * p.dk;
+#pragma unroll
+      for (int c = 0; c < C::NCW; ++c)
+#pragma unroll
+        for (int s = 0; s < KSN; ++s)
+          kf[c][u][s] = ld128(kp + (int64_t)min(hw0 / RP + c, p.G - 1) * p.k_sh + min(s, nst - 1) * 32 + klane);
+    }
   };
-  const int ndv = p.dv >> 4, nvt = p.G * ndv, nvw = (nvt + NW - 1) / NW, v0 = w * nvw;
   // value tiles of a wave in chunks of NC; a step is one chunk of one 32-key group
-  constexpr int NC = NV < 4 ? NV : 4, CH = NV / NC, STEPS = KG * CH;
+  const int ndv = p.dv >> 4, nvt = p.G * ndv, nvw = (nvt + kPW - 1) / kPW, v0 = w * nvw;
+  constexpr int NC = C::NC, CH = NV / NC, STEPS = KG * CH;
   static_assert(NV % NC == 0, "whole chunks");
+  // (value tiles past the last compute something nobody stores)
+  auto tile_at = [&](int u) { return min(v0 + min(u, nvw - 1), nvt - 1); };
+  const u16* vbase = reinterpret_cast<const u16*>(p.v) + rl * p.block_size + (b & 1) * 8;
   auto load_v = [&](uint4 (&vf)[NC], int it, int step) {
-    const int key = tile_of(v, min(it * NW + 2 * (step / CH) + (b >> 1), v.n - 1)) * kTile;
-    const u16* vp = reinterpret_cast<const u16*>(p.v) + blk_of(key) * p.v_sb + (int64_t)rl * p.block_size +
-                    key % p.block_size + (b & 1) * 8;
+    const int ts = btab[min(it * KT + 2 * (step / CH) + (b >> 1), v.n - 1)];
+    const u16* vp = vbase + (int64_t)(ts >> lb) * p.v_sb + (ts & lm) * kTile;
 #pragma unroll
     for (int n = 0; n < NC; ++n) {
-      const int idx = min(v0 + min((step % CH) * NC + n, nvw - 1), nvt - 1);
+      const int idx = tile_at((step % CH) * NC + n);
       vf[n] = ld128(vp + (int64_t)(idx / ndv) * p.v_sh + (int64_t)(idx % ndv) * 16 * p.block_size);
     }
   };
 
   f32x4 acc[NV][RP] = {};
-  uint4 kf[2][KSN];
-  if (it0 * NW + w < v.n) load_k(kf[0], 0, it0 * NW + w);
+  uint4 kf[C::NCW][2][KSN];
+  load_k(kf, it0);
+  // The values of a round's first step (two steps when there are several: va, vb) are requested at the end
+  // of the round before it, its keys after the scores of the round before it
+  static_assert(STEPS == 1 || STEPS % 2 == 0, "register sets by step parity");
+  uint4 va[NC], vb[NC];
+  load_v(va, it0, 0);
+  if (STEPS > 1) load_v(vb, it0, 1);
   for (int it = it0; it < it1; ++it) {
-    const int t = it * NW + w;
-    char* pw = pm + (((w >> 1) * 4 + 2 * (w & 1)) * 16 + rl) * 16;   // [head][..][key chunk][q]
-    uint4 vf[2][NC];
-    if (t < v.n) {
-      const int key0 = tile_of(v, t) * kTile;
-      const bool full = all_visible(pos0, pos1, key0, p.window, p.keep);
+    // ---- scores -> hi / lo weights
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+      const int t = it * KT + tw0 + u;
+      const int key0 = tile_of(v, min(t, v.n - 1)) * kTile;
+      const bool ok = t < v.n, full = ok && all_visible(pos0, pos1, key0, p.window, p.keep);
       bool vis[4] = {true, true, true, true};
       if (!full) {
 #pragma unroll
-        for (int i = 0; i < 4; ++i) vis[i] = sees(qpos, key0 + 4 * i + b, p.window, p.keep);
+        for (int i = 0; i < 4; ++i) vis[i] = ok && sees(qpos, key0 + 4 * b + i, p.window, p.keep);
       }
-      // hi / lo parts of the weights, [key i][heads pairwise]
-      unsigned xh[4][HX / 2], xl[4][HX / 2];
-      float px[4] = {0.f, 0.f, 0.f, 0.f};  // the even head of a pair
+      float x[HW][4];
 #pragma unroll
-      for (int c = 0; c < GP; ++c) {
-        if (c + 1 < GP && c + 1 < p.G) load_k(kf[(c + 1) & 1], c + 1, t);
+      for (int k = 0; k < HW; ++k) {
+        f32x4 a = {};
 #pragma unroll
-        for (int r = 0; r < RP; ++r) {
-          const int h = c * RP + r;
-          f32x4 a = {};
-          const bool real = c < p.G && r < R;
-          if (real) {
+        for (int s = 0; s < KSN; ++s) a = mfma16(as_bf16x8(kf[k / RP][u][s]), as_bf16x8(qf[k][s]), a);
 #pragma unroll
-            for (int s = 0; s < KSN; ++s)
-              if (s < nst) {
-                uint4 qf;
-                if constexpr (C::QL) qf = qs[((size_t)h * nst + s) * 64 + lane];
-                else qf = ld128(qp + (size_t)(c * R + r) * p.dk + s * 32);
-                a = mfma16(as_bf16x8(kf[c & 1][s]), as_bf16x8(qf), a);
-              }
-          }
-          const float ls = lse[h * 16 + rl];
-          float x[4];
-#pragma unroll
-          for (int i = 0; i < 4; ++i) x[i] = real && vis[i] ? __builtin_amdgcn_exp2f(a[i] * sl2 - ls) : 0.f;
-          if (HT == 1 || (h & 1)) {
-#pragma unroll
-            for (int i = 0; i < 4; ++i) {
-              const float e = HT == 1 ? x[i] : px[i], o = HT == 1 ? 0.f : x[i];
-              const unsigned hi = pack2(e, o);
-              xh[i][h >> 1] = hi;
-              xl[i][h >> 1] = pack2(e - __uint_as_float(hi << 16), o - __uint_as_float(hi & 0xffff0000u));
-            }
-          } else {
-#pragma unroll
-            for (int i = 0; i < 4; ++i) px[i] = x[i];
-          }
-          // (bounds how far ahead the query fragments are read: unbounded, their registers spill)
-          if ((r & 1) == 1 || RP == 1) __builtin_amdgcn_sched_barrier(0);
-        }
+        for (int i = 0; i < 4; ++i) x[k][i] = vis[i] ? __builtin_amdgcn_exp2f(a[i] * sl2 - ls[k]) : 0.f;
       }
-      if constexpr (HT < 4) {
-#pragma unroll
-        for (int i = 0; i < 4; ++i) xh[i][1] = xl[i][1] = 0u;
-      }
-      // next iteration's first keys, this one's first values
-      if (t + NW < v.n && it + 1 < it1) load_k(kf[0], 0, t + NW);
-      load_v(vf[0], it, 0);
-      // per key element: B operands by transposing the lane groups' blocks of 8 heads (4 registers), the
-      // mixed weights of keys 4 i .. 4 i + 3 of every head, and their bf16 quads to LDS
+      // head h, part (hi 0, lo 1) at byte: HT 32 part * 1024 + h / 8 block; 16 block 2 part + h / 8; 8 block
+      // part; 4 block 0, element 4 part + h
+      char* xw = xm + ((tw0 + u) * kTile + 4 * b) * KB + rl * 16 + (HX == 4 ? hw0 * 2 : (hw0 >> 3) * 256 + (hw0 & 7) * 2);
+      constexpr int LO = HX == 32 ? 1024 : HX == 16 ? 512 : HX == 8 ? 256 : 8;
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        uint4 bm[C::KM][4];  // [mixing step][source lane group]
+        if constexpr (HW == 1) {
+          const u16 hi = f2bf(x[0][i]);
+          *reinterpret_cast<u16*>(xw + i * KB) = hi;
+          *reinterpret_cast<u16*>(xw + i * KB + LO) = f2bf(x[0][i] - bf2f(hi));
+        } else {
+          unsigned hi[HW / 2], lo[HW / 2];
 #pragma unroll
-        for (int ks = 0; ks < C::KM; ++ks) {
-          unsigned o[4][4];  // [source group][register]
-#pragma unroll
-          for (int g = 0; g < 4; ++g) {
-            unsigned q0, q1, q2, q3;
-            if constexpr (HT == 32) {
-              const unsigned (&x)[HX / 2] = ks ? xl[i] : xh[i];
-              q0 = x[g], q1 = x[4 + g], q2 = x[8 + g], q3 = x[12 + g];
-            } else if constexpr (HT == 16) {
-              q0 = xh[i][g], q1 = xh[i][4 + g], q2 = xl[i][g], q3 = xl[i][4 + g];
-            } else if constexpr (HT == 8) {
-              q0 = xh[i][g], q1 = xl[i][g], q2 = 0u, q3 = 0u;
-            } else {
-              q0 = g < 2 ? xh[i][g & 1] : xl[i][g & 1], q1 = 0u, q2 = 0u, q3 = 0u;
-            }
-            transpose4(q0, q1, q2, q3);
-            o[0][g] = q0, o[1][g] = q1, o[2][g] = q2, o[3][g] = q3;
+          for (int k = 0; k < HW; k += 2) {
+            hi[k / 2] = pack2(x[k][i], x[k + 1][i]);
+            lo[k / 2] = pack2(x[k][i] - __uint_as_float(hi[k / 2] << 16), x[k + 1][i] - __uint_as_float(hi[k / 2] & 0xffff0000u));
           }
-#pragma unroll
-          for (int g = 0; g < 4; ++g) bm[ks][g] = make_uint4(o[g][0], o[g][1], o[g][2], o[g][3]);
-        }
-#pragma unroll
-        for (int mt = 0; mt < C::MT; ++mt) {
-          f32x4 y[4];
-#pragma unroll
-          for (int g = 0; g < 4; ++g) {
-            f32x4 a = {};
-#pragma unroll
-            for (int ks = 0; ks < C::KM; ++ks) a = mfma16(as_bf16x8(tf[mt]), as_bf16x8(bm[ks][g]), a);
-            y[g] = a;
-          }
-#pragma unroll
-          for (int e = 0; e < 4; ++e) {
-            const int h = 16 * mt + 4 * b + e;
-            if (HT >= 16 || h < HT)
-              *reinterpret_cast<uint2*>(pw + h * HS + (i >> 1) * 256 + (i & 1) * 8) =
-                  make_uint2(pack2(y[0][e], y[1][e]), pack2(y[2][e], y[3][e]));
+          if constexpr (HW == 2) {
+            *reinterpret_cast<unsigned*>(xw + i * KB) = hi[0];
+            *reinterpret_cast<unsigned*>(xw + i * KB + LO) = lo[0];
+          } else {
+            *reinterpret_cast<uint2*>(xw + i * KB) = make_uint2(hi[0], hi[1]);
+            *reinterpret_cast<uint2*>(xw + i * KB + LO) = make_uint2(lo[0], lo[1]);
           }
         }
       }
-    } else {
-      load_v(vf[0], it, 0);
-#pragma unroll
-      for (int mt = 0; mt < C::MT; ++mt)
-#pragma unroll
-        for (int ch = 0; ch < 2; ++ch)
-#pragma unroll
-          for (int i = 0; i < 4; ++i) {
-            const int h = 16 * mt + 4 * b + i;
-            if (HT >= 16 || h < HT) *reinterpret_cast<uint4*>(pw + h * HS + ch * 256) = make_uint4(0, 0, 0, 0);
-          }
     }
     lds_sync();
+    if (!C::LATE_K) load_k(kf, it + 1);
+    // ---- mixing: keys 4 kq .. 4 kq + 3
+#pragma unroll
+    for (int u = 0; u < KT / 2; ++u) {
+      const int kq = w + 8 * u;
+#pragma unroll
+      for (int mt = 0; mt < C::MT; ++mt) {
+        f32x4 y[4];
+#pragma unroll
+        for (int g = 0; g < 4; ++g) {
+          y[g] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+          for (int ks = 0; ks < C::KM; ++ks)
+            y[g] = mfma16(as_bf16x8(tf[mt]), *reinterpret_cast<const bf16x8*>(xm + (4 * kq + g) * KB + ks * 1024 + lane * 16), y[g]);
+        }
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const int h = 16 * mt + 4 * b + e;
+          if (HX >= 16 || h < HX)
+            *reinterpret_cast<uint2*>(pm + h * HS + (((kq >> 1) * 16) + rl) * 16 + (kq & 1) * 8) =
+                make_uint2(pack2(y[0][e], y[1][e]), pack2(y[2][e], y[3][e]));
+        }
+      }
+    }
+    lds_sync();
+    // ---- values
+    auto load_p = [&](uint4 (&pf)[RP], int c, int kg) {
+#pragma unroll
+      for (int r = 0; r < RP; ++r)
+        pf[r] = *reinterpret_cast<const uint4*>(pm + (c * RP + r) * HS + ((kg * 4 + b) * 16 + rl) * 16);
+    };
     uint4 pf[RP];
 #pragma unroll
     for (int st = 0; st < STEPS; ++st) {
       const int kg = st / CH;
-      if (it * NW + 2 * kg >= v.n) break;
-      if (st + 1 < STEPS && it * NW + 2 * ((st + 1) / CH) < v.n) load_v(vf[(st + 1) & 1], it, st + 1);
+      if (kg > 0 && it * KT + 2 * kg >= v.n) break;
+      uint4(&vc)[NC] = st & 1 ? vb : va;
 #pragma unroll
       for (int n = 0; n < NC; ++n) {
-        const int u = (st % CH) * NC + n, idx = v0 + u;
-        if (u >= nvw || idx >= nvt) break;
-        const int c = idx / ndv;
-        if (u == 0 || c != (idx - 1) / ndv) {  // (the kv head's mixed weights serve all of its value tiles)
+        const int u = (st % CH) * NC + n;
+        // (a kv head's mixed weights serve all of this wave's value tiles of it)
+        if (u == 0 || (!ONE && tile_at(u) / ndv != tile_at(u - 1) / ndv)) load_p(pf, tile_at(u) / ndv, kg);
 #pragma unroll
-          for (int r = 0; r < RP; ++r)
-            if (r < R) pf[r] = *reinterpret_cast<const uint4*>(pm + (c * RP + r) * HS + ((kg * 4 + b) * 16 + rl) * 16);
-        }
-#pragma unroll
-        for (int r = 0; r < RP; ++r)
-          if (r < R) acc[u][r] = mfma16(as_bf16x8(vf[st & 1][n]), as_bf16x8(pf[r]), acc[u][r]);
+        for (int r = 0; r < RP; ++r) acc[u][r] = mfma16(as_bf16x8(vc[n]), as_bf16x8(pf[r]), acc[u][r]);
       }
+      // the step after next (or the next round's) into the registers just used
+      if (STEPS == 1) load_v(vc, it + 1, 0);
+      else load_v(vc, st + 2 < STEPS ? it : it + 1, st + 2 < STEPS ? st + 2 : st + 2 - STEPS);
     }
-    lds_sync();
+    if (C::LATE_K) load_k(kf, it + 1);
   }
   if (nact > 1) {
     // ---- every split's sums out (sc1), a ticket, and the last one adds them in order
-    constexpr int kWave = NV * RP * 64 * 16, kPart = NW * kWave;     // bytes per wave / workgroup
+    constexpr int kWave = NV * RP * 64 * 16, kPart = kPW * kWave;     // bytes per wave / workgroup
     float* base = pp.part + (size_t)bt * pp.splits * (kPart / 4);
     const __amdgpu_buffer_rsrc_t rp = rsrc_f32(base, (int64_t)pp.splits * (kPart / 4));
     const int at = w * kWave + lane * 16;
@@ -700,7 +707,7 @@ __global__ __launch_bounds__(NW * 64) void talk_prefill_kernel(TalkPrefillParams
     for (int r = 0; r < RP; ++r) {
       if (r >= R) break;
       const int h = c * R + r;
-      const float g = head_gate<u16>(p, qrow, h);
+      const float g = gate[(c * RP + r) * 16 + rl];
       uint2 o;
       o.x = pack2(acc[n][r][0] * g, acc[n][r][1] * g);
       o.y = pack2(acc[n][r][2] * g, acc[n][r][3] * g);
@@ -721,34 +728,41 @@ constexpr size_t kMaxLds = 160 * 1024;
 // or the launch
 enum Want { WANT_FIT, WANT_PART, WANT_LAUNCH };
 
-template <int GP, int RP, int NV, int NW, int KSN>
+template <int GP, int RP, int NV, int KSN>
 int64_t prefill_cfg(const TalkPrefillParams& p, hipStream_t st, Want want) {
-  using C = PrefillCfg<GP, RP, NV, NW, KSN>;
-  if (C::lds(p.a.dk) > kMaxLds - 64) return -10;
+  using C = PrefillCfg<GP, RP, NV, KSN>;
+  static_assert(C::LDS <= kMaxLds - 64, "LDS");
   if (want == WANT_FIT) return 0;
-  if (want == WANT_PART) return (int64_t)NW * NV * RP * 256;
+  if (want == WANT_PART) return (int64_t)kPW * NV * RP * 256;
   const int R = p.a.H / p.a.G;
   constexpr int RB = RP < 4 ? RP : 4;
   hipLaunchKernelGGL((talk_lse_kernel<RB, KSN>), dim3(p.n_tiles * p.a.G, (R + RB - 1) / RB), dim3(256), 0, st, p);
-  hipLaunchKernelGGL((talk_prefill_kernel<GP, RP, NV, NW, KSN>), dim3(p.n_tiles, p.splits), dim3(NW * 64),
-                     (C::lds(p.a.dk)), st, p);
+  const dim3 grid(p.n_tiles, p.splits), block(kPW * 64);
+  if constexpr (KSN == 4 && NV == GP) {  // (the usual sizes)
+    const int ndv = p.a.dv >> 4, nvw = (p.a.G * ndv + kPW - 1) / kPW;
+    if (ndv % nvw == 0) {
+      hipLaunchKernelGGL((talk_prefill_kernel<GP, RP, NV, KSN, true>), grid, block, C::LDS, st, p);
+      return 0;
+    }
+  }
+  hipLaunchKernelGGL((talk_prefill_kernel<GP, RP, NV, KSN, false>), grid, block, C::LDS, st, p);
   return 0;
 }
 
 template <int GP, int RP>
 int64_t prefill_sizes(const TalkPrefillParams& p, hipStream_t st, Want want) {
-  constexpr int HT = GP * RP;
-  constexpr int NW = HT > 16 ? 4 : 8;       // 32 heads: 4 waves with twice the registers
-  constexpr int N1 = (GP * 8 + NW - 1) / NW, N2 = (GP * 16 + NW - 1) / NW;   // dv <= 128 / <= 256
-  const int need = (p.a.G * (p.a.dv >> 4) + NW - 1) / NW;
+  constexpr int N1 = GP, N2 = 2 * GP;   // value tiles per wave: dv <= 128 / <= 256
+  const int need = (p.a.G * (p.a.dv >> 4) + kPW - 1) / kPW;
   if (need <= N1) {
-    if (p.a.dk <= 128) return prefill_cfg<GP, RP, N1, NW, 4>(p, st, want);
-    return prefill_cfg<GP, RP, N1, NW, 8>(p, st, want);
+    if (p.a.dk <= 64) return prefill_cfg<GP, RP, N1, 2>(p, st, want);
+    if (p.a.dk <= 128) return prefill_cfg<GP, RP, N1, 4>(p, st, want);
+    return prefill_cfg<GP, RP, N1, 8>(p, st, want);
   }
-  if constexpr (HT <= 16) {
+  if constexpr (GP * RP <= 16) {
     if (need <= N2) {
-      if (p.a.dk <= 128) return prefill_cfg<GP, RP, N2, NW, 4>(p, st, want);
-      return prefill_cfg<GP, RP, N2, NW, 8>(p, st, want);
+      if (p.a.dk <= 64) return prefill_cfg<GP, RP, N2, 2>(p, st, want);
+      if (p.a.dk <= 128) return prefill_cfg<GP, RP, N2, 4>(p, st, want);
+      return prefill_cfg<GP, RP, N2, 8>(p, st, want);
     }
   }
   return -10;
@@ -780,7 +794,7 @@ int64_t dispatch_prefill(const TalkPrefillParams& p, hipStream_t st, Want want) 
 }
 
 int check_attn(const TalkAttnParams& p) {
-  if (p.rows < 1 || p.G < 1 || p.H < 1 || p.H % p.G || p.block_size % kTile || p.dk % 32 || p.dv % 16) return -1;
+  if (p.rows < 1 || p.G < 1 || p.H < 1 || p.H % p.G || p.block_size < kTile || (p.block_size & (p.block_size - 1)) || p.dk % 32 || p.dv % 16) return -1;
   if (p.window < 0 || p.keep < 0) return -2;
   if ((p.k_sh | p.k_sb | p.v_sh | p.v_sb | p.ldq) % 8) return -3;
   return 0;
@@ -817,6 +831,7 @@ extern "C" int64_t vwa_talk_prefill_part(int H, int G, int dk, int dv) {
 extern "C" int vwa_talk_prefill(const TalkPrefillParams* p, hipStream_t st) {
   const int rc = check_attn(p->a);
   if (rc) return rc;
+  if (p->max_tiles < 1 || p->max_tiles > kTab) return -8;  // (the kernel keeps the tiles' places in LDS)
   if (p->a.f32 || p->n_tiles < 1 || !p->tiles || !p->talk_frag || !p->lse || p->splits < 1 || p->a.ldo % 4) return -6;
   if (p->splits > 1) {
     const int64_t part = dispatch_prefill(*p, st, WANT_PART);

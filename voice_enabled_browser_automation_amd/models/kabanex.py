@@ -5,12 +5,12 @@ feed-forward, all reading one LayerNorm of an f32 residual stream.
 
 Engine contract as models/llama.py (ragged rows with their own position, slot and block-table row;
 optional logit-row selection), plus a recurrent state row per sequence (``stateful``) next to the
-paged K / V (``cache_layers``).  MI355X layout of a layer -- five launches at decode:
+paged K / V (``cache_layers``).  MI355X layout of a layer -- six launches at decode:
 
     layernorm_f32 -> ONE input projection [q | k | v | gate | z | x | g || up] whose epilogue squares the
-    feed-forward part straight into the output projection's input -> rotation + cache write ->
-    attention (gate and left_scale in its epilogue) and minGRU (right_scale in its epilogue), both into
-    that same input -> ONE output projection over [heads | recurrence | feed-forward] with the f32 residual
+    feed-forward part straight into the output projection's input -> rotation + cache write and the
+    minGRU (right_scale in its epilogue, into that same input) -> attention (two launches: scores, then
+    mixing and values; gate and left_scale in the epilogue, into that same input) -> ONE output projection over [heads | recurrence | feed-forward] with the f32 residual
     in its epilogue
 
 Sizes are arbitrary: projection sections are padded to the MFMA tiles with zero weight rows / columns
@@ -67,7 +67,10 @@ class LayerDims:
 
     @property
     def n_mix(self) -> int:
-        return self.at[5] + self.w
+        """Columns of the mixers' part; large projections are padded here to 256 columns in all (the tiled
+        GEMM's large tile)."""
+        n = self.at[5] + self.w
+        return n if n + self.f < 2048 else _up(n + self.f, 256) - self.f
 
     @property
     def heads_out(self) -> int:
@@ -183,12 +186,14 @@ class KabanexModel:
     def row_buffers(self, rows: int, max_ctx: int) -> Dict[str, object]:
         """Activation buffers of a step of ``rows`` rows (fixed addresses when the engine keeps them)."""
         dev, dt = self.device, self.dtype
-        z = lambda n, t=dt: torch.zeros(rows, n, dtype=t, device=dev)  # noqa: E731
-        # (distinct layouts have their own concatenation rows: the padding columns are never written)
-        return dict(hidden=z(self.d_pad, torch.float32), normed=z(self.d_pad),
-                    mix=torch.zeros(rows * max(D.n_mix for D in self.dims), dtype=dt, device=dev),
-                    q=torch.zeros(rows * max(D.H * D.dk for D in self.dims), dtype=dt, device=dev),
-                    cat={D: z(D.n_cat) for D in set(self.dims)})
+        e = lambda *n, t=dt: torch.empty(*n, dtype=t, device=dev)  # noqa: E731
+        # every buffer is written before it is read, but for the padding columns of a concatenation row: zeroed
+        # once, never written (so each distinct layout has rows of its own)
+        full = {D: D.n_cat == D.heads_out + L.right.width + L.ffn for L, D in zip(self.cfg.layers, self.dims)}
+        return dict(hidden=e(rows, self.d_pad, t=torch.float32), normed=e(rows, self.d_pad),
+                    mix=e(rows * max(D.n_mix for D in self.dims)), q=e(rows * max(D.H * D.dk for D in self.dims)),
+                    cat={D: e(rows, D.n_cat) if ok else torch.zeros(rows, D.n_cat, dtype=dt, device=dev)
+                         for D, ok in full.items()})
 
     def step_buffers(self, rows: int, max_ctx: int) -> Dict[str, object]:
         dev = self.device
@@ -227,16 +232,15 @@ class KabanexModel:
         cat = bufs.cat[D][:M]
         r_at, f_at = D.heads_out, D.heads_out + D.w
         ops.linear_split(h, L.w_in, y, cat[:, f_at : f_at + D.f] if D.f else None)
-        q = ops.qkv_cache_write(y, n_q_heads=D.H, rot_dims=a.rot_dims, rope=self.ropes[(a.rot_base, a.rot_dims)],
-                                positions=rows["positions"], slots=rows["slots"],
-                                q_out=bufs.q[: M * D.H * D.dk].view(M, D.H * D.dk), k_cache=kv.k[li], v_cache=kv.v[li])
+        W = C.right.width
+        q = ops.qkv_cache_mingru(y, (z0, x0, r0), L.zb, L.xb, n_q_heads=D.H, rot_dims=a.rot_dims,
+                                 rope=self.ropes[(a.rot_base, a.rot_dims)], q_out=bufs.q[: M * D.H * D.dk].view(M, D.H * D.dk),
+                                 k_cache=kv.k[li], v_cache=kv.v[li], state=kv.state[li], out_scale=C.right_scale,
+                                 out=cat[:, r_at : r_at + W], plan=plan, **rows)
         ops.talk_attention(q, kv.k[li], kv.v[li], bufs.block_table, n_q_heads=D.H, scale=a.scale, window=a.window,
                            keep=a.keep_first, talk=L.talk, talk_frag=L.talk_frag, gate=y[:, g0 : g0 + D.gate],
                            out_scale=C.left_scale, max_ctx=bufs.max_ctx, scratch=bufs.talk, out=cat[:, : D.heads_out],
                            plan=plan, **rows)
-        W = C.right.width
-        ops.mingru(y[:, z0 : z0 + W], y[:, x0 : x0 + W], y[:, r0 : r0 + W], L.zb, L.xb, state=kv.state[li],
-                   out_scale=C.right_scale, out=cat[:, r_at : r_at + W], plan=plan, **rows)
         xo = x[:, : self.n_out]
         ops.linear(cat, L.w_out, out=xo, residual=xo)
 

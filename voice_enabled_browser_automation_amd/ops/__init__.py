@@ -1183,4 +1183,4 @@ def env_int(name: str) -> int:
 
 
 from .stack import (TalkScratch, embedding_f32, layernorm_f32, linear_split, mingru, plan_runs,  # noqa: E402,F401
-                    qkv_cache_write, talk_attention, talk_fragment)
+                    qkv_cache_mingru, qkv_cache_write, talk_attention, talk_fragment)

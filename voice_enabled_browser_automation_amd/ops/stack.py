@@ -51,12 +51,15 @@ def plan_runs(runs: Sequence[Tuple[int, int]], device, max_pos: int) -> SimpleNa
                            singles=dev(singles, 1).view(-1) if singles else None)
 
 
+def visible_tiles(max_ctx: int, window: int, keep: int) -> int:
+    """16-key tiles a row can see at most."""
+    tiles = -(-max_ctx // 16)
+    return min(tiles, -(-keep // 16) + (window + 14) // 16 + 1) if window > 0 else tiles
+
+
 def visible_chunks(max_ctx: int, window: int, keep: int) -> int:
     """128-key chunks a row can see at most (vwa talk_chunks): sizes the rows-form scratch."""
-    tiles = -(-max_ctx // 16)
-    if window > 0:
-        tiles = min(tiles, -(-keep // 16) + (window + 14) // 16 + 1)
-    return -(-tiles // 8)
+    return -(-visible_tiles(max_ctx, window, keep) // 8)
 
 
 class TalkScratch:
@@ -127,6 +130,26 @@ def qkv_cache_write(x: torch.Tensor, *, n_q_heads: int, rot_dims: int, rope: tor
     return q_out
 
 
+def qkv_cache_mingru(y: torch.Tensor, at: Tuple[int, int, int], zb: torch.Tensor, xb: torch.Tensor, *, n_q_heads: int,
+                     rot_dims: int, rope: torch.Tensor, positions: torch.Tensor, seq_ids: torch.Tensor, slots: torch.Tensor,
+                     q_out: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, state: torch.Tensor,
+                     out_scale: float, out: torch.Tensor, plan: Optional[SimpleNamespace] = None) -> torch.Tensor:
+    """qkv_cache_write of a layer's projected rows and the mingru of its columns at = (z, x, g): one launch
+    for a decode step on the GPU, else the two ops."""
+    W = state.shape[1]
+    z, x, g = (y[:, a : a + W] for a in at)
+    if y.is_cuda and plan is None:
+        G, dk, dv = k_cache.shape[1], k_cache.shape[3], v_cache.shape[2]
+        _ext().qkv_mingru(y, n_q_heads, G, dk, dv, rot_dims, rope, positions, slots, q_out, k_cache, v_cache, z, x, g, zb, xb,
+                          seq_ids, state, out_scale, out)
+        return q_out
+    qkv_cache_write(y, n_q_heads=n_q_heads, rot_dims=rot_dims, rope=rope, positions=positions, slots=slots, q_out=q_out,
+                    k_cache=k_cache, v_cache=v_cache)
+    mingru(z, x, g, zb, xb, seq_ids=seq_ids, positions=positions, slots=slots, state=state, out_scale=out_scale, out=out,
+           plan=plan)
+    return q_out
+
+
 def talk_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor,
                    positions: torch.Tensor, seq_ids: torch.Tensor, slots: torch.Tensor, *, n_q_heads: int, scale: float,
                    window: int, keep: int, talk: Optional[torch.Tensor], talk_frag: Optional[torch.Tensor],
@@ -148,7 +171,7 @@ def talk_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor
 
     G, dk, dv = k_cache.shape[1], k_cache.shape[3], v_cache.shape[2]
     part = E.talk_prefill_part(n_q_heads, G, dk, dv) if plan is not None and talk_frag is not None else -1
-    if part > 0 and q.dtype == torch.bfloat16:
+    if part > 0 and q.dtype == torch.bfloat16 and visible_tiles(max_ctx, window + 15 if window > 0 else 0, keep) <= 1024:
         if plan.tiles is not None:
             from . import scratch as ws
 

@@ -25,6 +25,7 @@ from dataclasses import dataclass, field
 from types import SimpleNamespace
 from typing import Dict, List, Optional, Sequence, Tuple
 
+import numpy as np
 import torch
 
 from .. import ops
@@ -612,7 +613,7 @@ class LLMEngine:
         ``chunk`` rows: the projections then run as prompt-sized MFMA GEMMs (gemm.hip) shared by
         every request instead of one weight pass per request (reference: each /parse sends its
         prompt independently, apps/brain/src/server.ts:98-105).  No logits are computed."""
-        rows: List[Tuple[Sequence_, int]] = []
+        parts: List[Tuple[Sequence_, int]] = []
         for seq, upto in items:
             end = min(upto, len(seq.tokens))
             todo = end - seq.n_computed
@@ -621,18 +622,20 @@ class LLMEngine:
             if todo > seq.n_computed and todo > self.bufs.max_rows and not self.stateful:
                 self.prefill(seq, upto=end)
                 continue
-            rows += [(seq, t) for t in seq.tokens[seq.n_computed:end]]
-        if not rows:
+            parts.append((seq, todo))
+        n = sum(k for _, k in parts)
+        if not n:
             return
-        self.stats["prefill_tokens"] += len(rows)
+        self.stats["prefill_tokens"] += n
         self.stats["batched_prefills"] = self.stats.get("batched_prefills", 0) + 1
-        if len(rows) <= self.bufs.max_rows:
+        if n <= self.bufs.max_rows:
+            rows = [(seq, t) for seq, k in parts for t in seq.tokens[seq.n_computed : seq.n_computed + k]]
             self.run_rows(rows, logits_for=[len(rows) - 1], check=True, defer_head=True)
             self._head_rows = None
             return
         self._sync_staging()
-        for i in range(0, len(rows), chunk):
-            self._ragged_forward(rows[i : i + chunk])
+        for cut in self._cut(parts, chunk):
+            self._ragged_forward(cut)
 
     def step_batch(self, entries: List[Tuple[Sequence_, List[int]]], want: Sequence[int] = (),
                    chunk: int = 4096) -> Optional[torch.Tensor]:
@@ -640,28 +643,31 @@ class LLMEngine:
         are appended to its sequence and all of them run together (the step graphs when they fit a row
         bucket, one ragged forward otherwise).  ``want``: places in the concatenated tokens whose logits
         are returned, f32 [len(want), V] (None when there are none)."""
-        rows: List[Tuple[Sequence_, int]] = []
+        parts: List[Tuple[Sequence_, int]] = []
         for seq, toks in entries:
             if seq.n_computed != len(seq.tokens):
                 # (a prompt given to new_sequence: its next tokens are the uncomputed ones)
                 assert seq.tokens[seq.n_computed : seq.n_computed + len(toks)] == list(toks), "tokens out of order"
             else:
                 seq.tokens.extend(toks)
-            rows += [(seq, t) for t in toks]
-        want = list(want)
-        if not rows:
+            if toks:
+                parts.append((seq, len(toks)))
+        want, n = list(want), sum(k for _, k in parts)
+        if not n:
             return None
-        if len(rows) <= min(self.bufs.max_rows, BUCKETS[-1]):
+        if n <= min(self.bufs.max_rows, BUCKETS[-1]):
+            rows = [(seq, t) for seq, k in parts for t in seq.tokens[seq.n_computed : seq.n_computed + k]]
             if want:
                 return self.run_rows(rows, logits_for=want)
-            self.run_rows(rows, logits_for=[len(rows) - 1], defer_head=True)
+            self.run_rows(rows, logits_for=[n - 1], defer_head=True)
             self._head_rows = None
             return None
         self._sync_staging()
-        hidden = []
-        for i in range(0, len(rows), chunk):
-            part = rows[i : i + chunk]
-            hs = self._ragged_forward(part, [w - i for w in want if i <= w < i + len(part)])
+        hidden, at = [], 0
+        for cut in self._cut(parts, chunk):
+            m = sum(k for _, k in cut)
+            hs = self._ragged_forward(cut, [w - at for w in want if at <= w < at + m])
+            at += m
             if hs is not None:
                 hidden.append(hs)
         if not want:
@@ -669,44 +675,64 @@ class LLMEngine:
         hs = torch.cat(hidden) if len(hidden) > 1 else hidden[0]
         return self.model.lm_logits(self.bufs, hs)
 
+    @staticmethod
+    def _cut(parts: List[Tuple[Sequence_, int]], chunk: int) -> List[List[Tuple[Sequence_, int]]]:
+        """(sequence, tokens) parts cut into forwards of at most ``chunk`` rows."""
+        out: List[List[Tuple[Sequence_, int]]] = []
+        room = 0
+        for seq, k in parts:
+            while k > 0:
+                if room == 0:
+                    out.append([])
+                    room = chunk
+                take = min(k, room)
+                out[-1].append((seq, take))
+                room -= take
+                k -= take
+        return out
+
     def _sync_staging(self) -> None:
         if self._staging_inflight and self.device.type == "cuda":
             torch.cuda.current_stream().synchronize()
             self._staging_inflight = False
 
-    def _ragged_forward(self, rows: List[Tuple[Sequence_, int]], want: Sequence[int] = ()) -> Optional[torch.Tensor]:
-        """One eager forward of ragged rows (more than the step buffers hold): the decode-mode
-        model forward over scratch buffers sized for them; attention in 64-row slices, or by the
-        model's own row plan.  Returns the final hidden rows at the places ``want``."""
-        n = len(rows)
+    def _ragged_forward(self, parts: List[Tuple[Sequence_, int]], want: Sequence[int] = ()) -> Optional[torch.Tensor]:
+        """One eager forward of ragged rows (more than the step buffers hold): the next tokens of each
+        (sequence, count), concatenated; the decode-mode model forward over scratch buffers sized for
+        them, attention in 64-row slices or by the model's own row plan.  Returns the final hidden rows
+        at the places ``want``."""
         bs = self.block_size
-        pending: Dict[int, int] = {}
-        toks, poss, sids, slots = [], [], [], []
-        for seq, tok in rows:
-            pos = pending.get(seq.sid, seq.n_computed)
-            if pos // bs >= len(seq.blocks):
-                self._ensure_blocks(seq, pos + 1)
-            toks.append(tok)
+        ends: Dict[int, int] = {}
+        toks, poss, slots = [], [], []
+        for seq, k in parts:
+            start = ends.get(seq.sid, seq.n_computed)
+            self._ensure_blocks(seq, start + k)
+            pos = np.arange(start, start + k)
+            toks.append(np.asarray(seq.tokens[start : start + k], dtype=np.int32))
             poss.append(pos)
-            sids.append(seq.sid)
-            slots.append(seq.blocks[pos // bs] * bs + pos % bs)
-            pending[seq.sid] = pos + 1
+            slots.append(np.asarray(seq.blocks, dtype=np.int64)[pos // bs] * bs + pos % bs)
+            ends[seq.sid] = start + k
+        n = sum(k for _, k in parts)
+        np_meta = np.empty((4, n), dtype=np.int32)
+        np_meta[0], np_meta[1] = np.concatenate(toks), np.concatenate(poss)
+        np_meta[2] = np.repeat([seq.sid for seq, _ in parts], [k for _, k in parts])
+        np_meta[3] = np_meta[1] + 1
+        runs = self._runs(parts, poss)
         if self.bufs.table_dirty:
             self.bufs.block_table.copy_(self.bufs.h_table, non_blocking=self.device.type == "cuda")
             self.bufs.table_dirty = False
             self._staging_inflight = self.device.type == "cuda"  # (the copy reads the pinned table)
         dev, m = self.device, self.model
-        i32 = dict(dtype=torch.int32)
-        meta = torch.tensor([toks, poss, sids, [p + 1 for p in poss]], **i32)
+        meta, slot_t = torch.from_numpy(np_meta), torch.from_numpy(np.concatenate(slots))
         if dev.type == "cuda":
             meta = meta.pin_memory().to(dev, non_blocking=True)
+            slot_t = slot_t.pin_memory().to(dev, non_blocking=True)
         scratch = SimpleNamespace(
             tokens=meta[0], positions=meta[1], seq_ids=meta[2], ctx_lens=meta[3],
-            slots=torch.tensor(slots, dtype=torch.int64).to(dev, non_blocking=dev.type == "cuda"),
-            block_table=self.bufs.block_table, max_ctx=self.bufs.max_ctx, logits_local=self.bufs.logits_local)
+            slots=slot_t, block_table=self.bufs.block_table, max_ctx=self.bufs.max_ctx, logits_local=self.bufs.logits_local)
         if hasattr(m, "row_buffers"):
             vars(scratch).update(m.row_buffers(n, self.bufs.max_ctx), talk=getattr(self.bufs, "talk", None),
-                                 plan=m.plan_rows(self._runs(sids, poss), max(poss)))
+                                 plan=m.plan_rows([(a, k) for a, k, _, _ in runs], int(np_meta[1].max())))
         else:
             d = m.cfg.hidden
             vars(scratch).update(
@@ -715,9 +741,9 @@ class LLMEngine:
                 attn=torch.empty(n, m.nq * m.hd, dtype=m.dtype, device=dev),
                 act=torch.empty(n, getattr(m, "F", getattr(m.cfg, "ffn", d)), dtype=m.dtype, device=dev),
                 part_o=self.bufs.part_o, part_ml=self.bufs.part_ml, attn_cnt=self.bufs.attn_cnt,
-                logits=self.bufs.logits, flash=self._ragged_flash(sids, poss) if dev.type == "cuda" else None)
+                logits=self.bufs.logits, flash=self._ragged_flash(runs, n) if dev.type == "cuda" else None)
         hs = m.forward(scratch, n, self.kv, head=False)
-        for sid, ln in pending.items():
+        for sid, ln in ends.items():
             self.seqs[sid].n_computed = ln
         self.stats["steps"] += 1
         self.stats["rows"] += n
@@ -726,46 +752,41 @@ class LLMEngine:
         return hs.index_select(0, torch.tensor(list(want), dtype=torch.int64, device=hs.device))
 
     @staticmethod
-    def _runs(sids: List[int], poss: List[int]) -> List[Tuple[int, int]]:
-        """(first row, rows) of the runs of one sequence at consecutive positions."""
+    def _runs(parts, poss) -> List[Tuple[int, int, int, int]]:
+        """(first row, rows, sequence id, first position) of the runs of one sequence at consecutive
+        positions (adjacent parts of one sequence are one run)."""
         runs: List[List[int]] = []
-        for i, (sid, pos) in enumerate(zip(sids, poss)):
-            if runs and sids[i - 1] == sid and pos == poss[i - 1] + 1:
-                runs[-1][1] += 1
+        at = 0
+        for (seq, k), pos in zip(parts, poss):
+            if runs and runs[-1][2] == seq.sid and runs[-1][3] + runs[-1][1] == pos[0]:
+                runs[-1][1] += k
             else:
-                runs.append([i, 1])
-        return [(a, n) for a, n in runs]
+                runs.append([at, k, seq.sid, int(pos[0])])
+            at += k
+        return [tuple(r) for r in runs]
 
-    def _ragged_flash(self, sids: List[int], poss: List[int]) -> Optional[SimpleNamespace]:
+    def _ragged_flash(self, runs: List[Tuple[int, int, int, int]], n: int) -> Optional[SimpleNamespace]:
         """Ragged rows made of whole per-sequence runs (consecutive positions, one run per
         sequence -- the batched admission prefill): the batched causal flash attention layout for
         them ([B runs, S = longest run] queries at absolute offsets, each run's own block-table row)
         -- one launch per layer instead of the decode kernel over 64-row slices."""
-        if not PREFILL_FLASH:
-            return None
-        runs: List[List[int]] = []  # [sid, first row, rows, first position]
-        for i, (sid, pos) in enumerate(zip(sids, poss)):
-            if runs and runs[-1][0] == sid and pos == poss[i - 1] + 1:
-                runs[-1][2] += 1
-            else:
-                runs.append([sid, i, 1, pos])
         # (one run -- a single request's suffix -- keeps the decode kernel's key-split slices:
         # the batched flash launch then has 32 workgroups for the whole GPU, 41 vs 35 us per
         # layer on the headline's 85-row suffix, profiles/r6_prefill_flash_b1_rejected.md)
-        if len(runs) < 2 or len({r[0] for r in runs}) != len(runs):
+        if not PREFILL_FLASH or len(runs) < 2 or len({r[2] for r in runs}) != len(runs):
             return None
-        B, S = len(runs), max(r[2] for r in runs)
-        if B * S > 2 * len(sids):  # one long run among short ones: mostly padding queries -- slices
+        B, S = len(runs), max(r[1] for r in runs)
+        if B * S > 2 * n:  # one long run among short ones: mostly padding queries -- slices
             return None
-        dst = torch.empty(len(sids), dtype=torch.int64)
-        for b, (_, i0, cnt, _) in enumerate(runs):
+        dst = torch.empty(n, dtype=torch.int64)
+        for b, (i0, cnt, _, _) in enumerate(runs):
             dst[i0 : i0 + cnt] = torch.arange(b * S, b * S + cnt)
         dev = self.device
-        meta = torch.tensor([[r[3] for r in runs], [r[3] + r[2] for r in runs], [r[0] for r in runs]],
+        meta = torch.tensor([[r[3] for r in runs], [r[3] + r[1] for r in runs], [r[2] for r in runs]],
                             dtype=torch.int32).pin_memory().to(dev, non_blocking=True)
         return SimpleNamespace(B=B, S=S, dst=dst.pin_memory().to(dev, non_blocking=True), q_offsets=meta[0],
                                k_lens=meta[1], table=self.bufs.block_table.index_select(0, meta[2]),
-                               max_k=max(r[3] + r[2] for r in runs))
+                               max_k=max(r[3] + r[1] for r in runs))
 
     def prefill(self, seq: Sequence_, chunk: int = 2048, upto: Optional[int] = None) -> Optional[torch.Tensor]:
         """Compute K/V for seq.tokens[n_computed:upto] (default: all tokens); returns f32 logits
@@ -785,7 +806,7 @@ class LLMEngine:
                 continue
             if hasattr(self.model, "row_buffers"):
                 self._sync_staging()
-                hs = self._ragged_forward([(seq, t) for t in seq.tokens[start : start + n]], [n - 1])
+                hs = self._ragged_forward([(seq, n)], [n - 1])
                 logits = self.model.lm_logits(self.bufs, hs)
                 continue
             self._ensure_blocks(seq, start + n)
