@@ -221,8 +221,6 @@ int64_t max_tiles(int64_t max_ctx, int64_t window, int64_t keep) {
   return std::min(all, (keep + 15) / 16 + (window + 14) / 16 + 1);
 }
 
-int64_t talk_chunks(int64_t max_ctx, int64_t window, int64_t keep) { return (max_tiles(max_ctx, window, keep) + 7) / 8; }
-
 void talk_attention(Tensor q, Tensor k, Tensor v, Tensor table, Tensor positions, Tensor seq_ids, Tensor slots,
                     c10::optional<Tensor> row_list, int64_t n_rows, int64_t H, double scale, int64_t window, int64_t keep,
                     c10::optional<Tensor> talk, c10::optional<Tensor> gate, double out_scale, int64_t max_ctx, Tensor s,
@@ -234,7 +232,7 @@ void talk_attention(Tensor q, Tensor k, Tensor v, Tensor table, Tensor positions
   TORCH_CHECK(max_ctx >= 1 && max_ctx <= table.size(1) * k.size(2), "max_ctx exceeds the block table");
   if (row_list.has_value()) p.row_list = i32p(*row_list, n_rows, "row_list");
   p.rows = (int)n_rows;
-  const int64_t nch = talk_chunks(max_ctx, window, keep), R = H / p.G;
+  const int64_t nch = (max_tiles(max_ctx, window, keep) + 7) / 8, R = H / p.G;
   p.nch = (int)nch;
   p.s = f32p(s, n_rows * H * nch * 128, "s");
   p.stat = f32p(stat, n_rows * H * nch * 2, "stat");
@@ -349,7 +347,6 @@ void bind_stack(py::module_& m) {
   m.def("embedding_f32", &embedding_f32);
   m.def("qkv_cache", &qkv_cache);
   m.def("qkv_mingru", &qkv_mingru);
-  m.def("talk_chunks", &talk_chunks);
   m.def("talk_prefill_part", [](int64_t H, int64_t G, int64_t dk, int64_t dv) {
     return vwa_talk_prefill_part((int)H, (int)G, (int)dk, (int)dv);
   });

@@ -34,7 +34,7 @@ struct QkvCacheParams {
 // Attention over the visible keys of each row (j <= i and (i - j < window or j < keep); window 0: all)
 // with the heads' softmax weights mixed across heads (talk [H][H]; null: not mixed), an optional
 // per-head output gate sigmoid(gate[row][h]) and a constant output scale.
-// Keys are walked in 16-key tiles (a tile never crosses a cache block), 8 tiles per workgroup chunk.
+// Keys are walked in 16-key tiles (a tile never crosses a cache block), dealt to workgroups in chunks of at most 8.
 struct TalkAttnParams {
   const void* q; int ldq;           // [rows, H * dk]
   const void* k; const void* v; int64_t k_sb, k_sh, v_sb, v_sh;

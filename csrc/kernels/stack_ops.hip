@@ -27,37 +27,40 @@ VWA_DEVICE float block_sum(float v, float* red) {
   return (red[0] + red[1]) + (red[2] + red[3]);
 }
 
-// one workgroup per row, the row held in registers (D <= 8192): 4 columns per thread and step
+// one workgroup per row, the row held in registers: STEPS x 1024 columns, 4 per thread and step, all
+// loads in flight at once (columns past the row repeat its last quad and count as zero)
 constexpr int kLnSteps = 8;
-template <class T>
+template <class T, int STEPS>
 __global__ __launch_bounds__(256) void layernorm_f32_kernel(const float* __restrict__ x, int ldx,
                                                             const float* __restrict__ w, const float* __restrict__ b,
                                                             T* __restrict__ y, int ldy, int D, int Dpad, float eps) {
   __shared__ float red[4];
   const float* xr = x + (size_t)blockIdx.x * ldx;
   T* yr = y + (size_t)blockIdx.x * ldy;
-  float v[kLnSteps][4];
+  float v[STEPS][4];
+  const int last = (D - 1) & ~3;
+#pragma unroll
+  for (int i = 0; i < STEPS; ++i) {
+    const float4 f = *reinterpret_cast<const float4*>(xr + min((i * 256 + (int)threadIdx.x) * 4, last));
+    v[i][0] = f.x;
+    v[i][1] = f.y;
+    v[i][2] = f.z;
+    v[i][3] = f.w;
+  }
   float s = 0.f;
 #pragma unroll
-  for (int i = 0; i < kLnSteps; ++i) {
+  for (int i = 0; i < STEPS; ++i) {
     const int c = (i * 256 + threadIdx.x) * 4;
-    if (i * 1024 >= D) break;
-    if (c < D) {  // (rows are padded to a multiple of 4 and the padding is zero or never read back)
-      const float4 f = *reinterpret_cast<const float4*>(xr + c);
-      v[i][0] = f.x;
-      v[i][1] = c + 1 < D ? f.y : 0.f;
-      v[i][2] = c + 2 < D ? f.z : 0.f;
-      v[i][3] = c + 3 < D ? f.w : 0.f;
-    } else {
-      v[i][0] = v[i][1] = v[i][2] = v[i][3] = 0.f;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      v[i][j] = c + j < D ? v[i][j] : 0.f;
+      s += v[i][j];
     }
-    s += (v[i][0] + v[i][1]) + (v[i][2] + v[i][3]);
   }
   const float mu = block_sum(s, red) / (float)D;
   float q = 0.f;
 #pragma unroll
-  for (int i = 0; i < kLnSteps; ++i) {
-    if (i * 1024 >= D) break;
+  for (int i = 0; i < STEPS; ++i) {
     const int c = (i * 256 + threadIdx.x) * 4;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
@@ -67,16 +70,28 @@ __global__ __launch_bounds__(256) void layernorm_f32_kernel(const float* __restr
   }
   const float rstd = 1.f / sqrtf(block_sum(q, red) / (float)D + eps);
 #pragma unroll
-  for (int i = 0; i < kLnSteps; ++i) {
-    if (i * 1024 >= D) break;
+  for (int i = 0; i < STEPS; ++i) {
     const int c = (i * 256 + threadIdx.x) * 4;
     if (c >= D) continue;
     float o[4];
 #pragma unroll
-    for (int j = 0; j < 4; ++j) o[j] = c + j < D ? (v[i][j] - mu) * rstd * w[c + j] + b[c + j] : 0.f;
+    for (int j = 0; j < 4; ++j) {
+      const int cj = min(c + j, D - 1);
+      o[j] = c + j < D ? (v[i][j] - mu) * rstd * w[cj] + b[cj] : 0.f;
+    }
     st4(yr + c, o);
   }
   for (int c = ((D + 3) & ~3) + threadIdx.x; c < Dpad; c += 256) stv(yr + c, 0.f);
+}
+
+template <class T>
+void launch_ln(const float* x, int ldx, const float* w, const float* b, T* y, int ldy, int rows, int D, int Dpad, float eps,
+               hipStream_t st) {
+  const dim3 grid(rows), block(256);
+  if (D <= 1024) hipLaunchKernelGGL((layernorm_f32_kernel<T, 1>), grid, block, 0, st, x, ldx, w, b, y, ldy, D, Dpad, eps);
+  else if (D <= 2048) hipLaunchKernelGGL((layernorm_f32_kernel<T, 2>), grid, block, 0, st, x, ldx, w, b, y, ldy, D, Dpad, eps);
+  else if (D <= 4096) hipLaunchKernelGGL((layernorm_f32_kernel<T, 4>), grid, block, 0, st, x, ldx, w, b, y, ldy, D, Dpad, eps);
+  else hipLaunchKernelGGL((layernorm_f32_kernel<T, 8>), grid, block, 0, st, x, ldx, w, b, y, ldy, D, Dpad, eps);
 }
 
 template <class T>
@@ -86,7 +101,8 @@ __global__ __launch_bounds__(256) void embedding_f32_kernel(const int* __restric
   const int row = blockIdx.x;
   const int id = ids[row];
   const bool ok = id >= 0 && id < vocab;
-  for (int c = threadIdx.x; c < Dpad; c += 256)
+  const int c = blockIdx.y * 256 + threadIdx.x;
+  if (c < Dpad)
     out[(size_t)row * ldo + c] = ok && c < D ? ldv(table + (size_t)id * ld + c) : 0.f;
 }
 
@@ -164,12 +180,8 @@ extern "C" int vwa_layernorm_f32(const float* x, int ldx, const float* w, const 
   if (rows < 1 || D < 1 || D > kLnSteps * 1024 || Dpad < D || ldx % 4 || ldy % 4 || ldx < ((D + 3) & ~3) || ldy < Dpad ||
       Dpad % 4)
     return -1;
-  if (f32)
-    hipLaunchKernelGGL((layernorm_f32_kernel<float>), dim3(rows), dim3(256), 0, st, x, ldx, w, b,
-                       reinterpret_cast<float*>(y), ldy, D, Dpad, eps);
-  else
-    hipLaunchKernelGGL((layernorm_f32_kernel<u16>), dim3(rows), dim3(256), 0, st, x, ldx, w, b,
-                       reinterpret_cast<u16*>(y), ldy, D, Dpad, eps);
+  if (f32) launch_ln(x, ldx, w, b, reinterpret_cast<float*>(y), ldy, rows, D, Dpad, eps, st);
+  else launch_ln(x, ldx, w, b, reinterpret_cast<u16*>(y), ldy, rows, D, Dpad, eps, st);
   return (int)hipGetLastError();
 }
 
@@ -177,10 +189,10 @@ extern "C" int vwa_embedding_f32(const int* ids, const void* table, int ld, floa
                                  int vocab, int f32, hipStream_t st) {
   if (rows < 1 || D < 1 || ld < D || Dpad < D || ldo < Dpad) return -1;
   if (f32)
-    hipLaunchKernelGGL((embedding_f32_kernel<float>), dim3(rows), dim3(256), 0, st, ids,
+    hipLaunchKernelGGL((embedding_f32_kernel<float>), dim3(rows, (Dpad + 255) / 256), dim3(256), 0, st, ids,
                        reinterpret_cast<const float*>(table), ld, out, ldo, D, Dpad, vocab);
   else
-    hipLaunchKernelGGL((embedding_f32_kernel<u16>), dim3(rows), dim3(256), 0, st, ids,
+    hipLaunchKernelGGL((embedding_f32_kernel<u16>), dim3(rows, (Dpad + 255) / 256), dim3(256), 0, st, ids,
                        reinterpret_cast<const u16*>(table), ld, out, ldo, D, Dpad, vocab);
   return (int)hipGetLastError();
 }

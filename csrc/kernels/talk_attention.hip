@@ -27,8 +27,6 @@ using namespace vwa;
 namespace {
 
 constexpr int kTile = 16;                  // keys per tile
-constexpr int kChunkTiles = 8;             // tiles per workgroup of the rows form
-constexpr int kChunk = kTile * kChunkTiles;
 constexpr float kLog2e = 1.4426950408889634f;
 
 template <class T> struct MM;
@@ -76,43 +74,57 @@ VWA_DEVICE f32x4 ld_sc1_x4(__amdgpu_buffer_rsrc_t r, int off) {
 }
 
 // ------------------------------------------------------------------------------------------ rows form
+constexpr int kChunkTiles = 8;             // most tiles of a workgroup's chunk
+constexpr int kChunk = kTile * kChunkTiles;
+
+// A row's visible tiles are dealt evenly to the fewest chunks; chunk c holds tiles c * per ..
+struct Chunks {
+  int per, n;
+};
+VWA_DEVICE Chunks chunks_of(int tiles) {
+  const int k = (tiles + kChunkTiles - 1) / kChunkTiles, per = (tiles + k - 1) / k;
+  return Chunks{per, (tiles + per - 1) / per};
+}
+
 template <class T>
 __global__ __launch_bounds__(256) void talk_scores_kernel(TalkAttnParams p) {
   using M = MM<T>;
+  constexpr int NU = kChunkTiles / 4;                // tiles per wave
   __shared__ float sm[4][16][2];
   const int ri = blockIdx.x / p.G, c = blockIdx.x % p.G, chunk = blockIdx.y, r0 = blockIdx.z * 16;
   const int row = p.row_list ? p.row_list[ri] : ri;
   if (p.slots[row] < 0) return;
   const int pos = p.positions[row], seq = p.seq_ids[row];
   const Vis v = vis_tiles(pos, pos, p.window, p.keep);
-  if (chunk * kChunkTiles >= v.n) return;
+  const Chunks ck = chunks_of(v.n);
+  if (chunk >= ck.n) return;
   const int R = p.H / p.G, Rb = min(16, R - r0);
   const int lane = lane_id(), w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), rl = lane & 15, b = lane >> 4;
   const T* q = reinterpret_cast<const T*>(p.q) + (size_t)row * p.ldq + (size_t)(c * R + r0 + min(rl, Rb - 1)) * p.dk + b * M::EPL;
   const int lb = __builtin_ctz(p.block_size);
-  const T* kp[2];
-  int key0[2];
-  bool ok[2];
+  const T* kp[NU];
+  int key0[NU];
+  bool ok[NU];
 #pragma unroll
-  for (int u = 0; u < 2; ++u) {
-    const int t = chunk * kChunkTiles + w * 2 + u;
-    ok[u] = t < v.n;
+  for (int u = 0; u < NU; ++u) {
+    const int lt = w + 4 * u, t = chunk * ck.per + lt;
+    ok[u] = lt < ck.per && t < v.n;
     key0[u] = tile_of(v, ok[u] ? t : v.n - 1) * kTile;
     const int64_t blk = p.block_table[(int64_t)seq * p.table_stride + (key0[u] >> lb)];
     kp[u] = reinterpret_cast<const T*>(p.k) + blk * p.k_sb + (int64_t)c * p.k_sh +
             (int64_t)((key0[u] & (p.block_size - 1)) + rl) * p.dk + b * M::EPL;
   }
-  f32x4 acc[2] = {};
+  f32x4 acc[NU] = {};
 #pragma unroll 4
   for (int k = 0; k < p.dk; k += M::KS) {
     const uint4 qf = *reinterpret_cast<const uint4*>(q + k);
 #pragma unroll
-    for (int u = 0; u < 2; ++u) acc[u] = M::mma(*reinterpret_cast<const uint4*>(kp[u] + k), qf, acc[u]);
+    for (int u = 0; u < NU; ++u) acc[u] = M::mma(*reinterpret_cast<const uint4*>(kp[u] + k), qf, acc[u]);
   }
   // lane (column rl = head, keys 4b .. 4b+3 of both tiles): mask, store, chunk statistics
   float mx = -INFINITY;
 #pragma unroll
-  for (int u = 0; u < 2; ++u)
+  for (int u = 0; u < NU; ++u)
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const bool vis = ok[u] && sees(pos, key0[u] + 4 * b + i, p.window, p.keep);
@@ -121,17 +133,17 @@ __global__ __launch_bounds__(256) void talk_scores_kernel(TalkAttnParams p) {
     }
   if (rl < Rb) {
 #pragma unroll
-    for (int u = 0; u < 2; ++u)
+    for (int u = 0; u < NU; ++u)
       if (ok[u])
         *reinterpret_cast<float4*>(p.s + ((size_t)ri * p.H + c * R + r0 + rl) * p.nch * kChunk +
-                                   (chunk * kChunkTiles + w * 2 + u) * kTile + 4 * b) =
+                                   chunk * kChunk + (w + 4 * u) * kTile + 4 * b) =
             make_float4(acc[u][0], acc[u][1], acc[u][2], acc[u][3]);
   }
   mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
   mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
   float l = 0.f;
 #pragma unroll
-  for (int u = 0; u < 2; ++u)
+  for (int u = 0; u < NU; ++u)
 #pragma unroll
     for (int i = 0; i < 4; ++i) l += acc[u][i] == -INFINITY ? 0.f : __expf(acc[u][i] - mx);
   l += __shfl_xor(l, 16, 64);
@@ -160,13 +172,15 @@ VWA_DEVICE float head_gate(const TalkAttnParams& p, int row, int h) {
   return p.out_scale / (1.f + __expf(-ldv(reinterpret_cast<const T*>(p.gate) + (size_t)row * p.ldg + h)));
 }
 
-// LDS: statistics [H][2], weights [H][128] f32, mixed weights [128 / KS][64][16 B]
+// LDS: statistics [H][2], weights [H][keys] f32, mixed weights [keys / KS][64][16 B]
 template <class T>
 size_t mix_lds(int H) { return (size_t)H * (2 + kChunk) * 4 + kChunk * 16 * sizeof(T); }
 
 template <class T>
 __global__ __launch_bounds__(256) void talk_mix_kernel(TalkAttnParams p) {
   using M = MM<T>;
+  constexpr int HP = 256 / kChunk;                   // heads side by side over the threads
+  static_assert(HP == 2);
   extern __shared__ __attribute__((aligned(16))) char smem[];
   __shared__ int s_last;
   const int ri = blockIdx.x / p.G, c = blockIdx.x % p.G, chunk = blockIdx.y, r0 = blockIdx.z * 16;
@@ -180,23 +194,23 @@ __global__ __launch_bounds__(256) void talk_mix_kernel(TalkAttnParams p) {
   }
   const int pos = p.positions[row], seq = p.seq_ids[row];
   const Vis v = vis_tiles(pos, pos, p.window, p.keep);
-  if (chunk * kChunkTiles >= v.n) return;
-  const int nact = (v.n + kChunkTiles - 1) / kChunkTiles;
-  const int nt = min(kChunkTiles, v.n - chunk * kChunkTiles), nkey = nt * kTile;
+  const Chunks ck = chunks_of(v.n);
+  if (chunk >= ck.n) return;
+  const int nact = ck.n, t0 = chunk * ck.per, nt = min(ck.per, v.n - t0), nkey = nt * kTile;
   T* pf = reinterpret_cast<T*>(smem);                                   // mixed weights, B-operand order
-  float* wt = reinterpret_cast<float*>(smem + kChunk * 16 * sizeof(T));  // [H][128]
+  float* wt = reinterpret_cast<float*>(smem + kChunk * 16 * sizeof(T));  // [H][keys]
   float* hm = wt + p.H * kChunk;                                        // [H] max
   float* hl = hm + p.H;                                                 // [H] 1 / sum
   const int g0 = p.talk ? 0 : h0, g1 = p.talk ? p.H : h0 + Rb;          // heads whose weights are needed
   const int lane = lane_id(), w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), rl = lane & 15, b = lane >> 4;
   // ---- everything that is read is requested first: the scores of this thread's (key, heads), the first
   // value tiles of this wave (16-column tiles w, w + 4, ...), the chunk statistics
-  constexpr int kPre = 8;
-  const int j = threadIdx.x & (kChunk - 1), hp = w >> 1;                // key, head parity
+  constexpr int kPre = 16 / HP;
+  const int j = threadIdx.x & (kChunk - 1), hp = w >> 1;                // key, first head
   const float* srow = p.s + (size_t)ri * p.H * p.nch * kChunk + chunk * kChunk + j;
   float sv[kPre];
 #pragma unroll
-  for (int k = 0; k < kPre; ++k) sv[k] = srow[(size_t)min(g0 + hp + 2 * k, g1 - 1) * p.nch * kChunk];
+  for (int k = 0; k < kPre; ++k) sv[k] = srow[(size_t)min(g0 + hp + HP * k, g1 - 1) * p.nch * kChunk];
   constexpr int TPS = M::KS / kTile;                 // tiles per step (bf16 2, f32 1)
   constexpr int NST = kChunkTiles / TPS;
   const int lb = __builtin_ctz(p.block_size);
@@ -204,9 +218,9 @@ __global__ __launch_bounds__(256) void talk_mix_kernel(TalkAttnParams p) {
   bool vok[NST];
 #pragma unroll
   for (int s = 0; s < NST; ++s) {
-    const int t = chunk * kChunkTiles + s * TPS + (TPS == 2 ? b >> 1 : 0);
-    vok[s] = t < v.n;
-    const int key = tile_of(v, vok[s] ? t : v.n - 1) * kTile;
+    const int lt = s * TPS + (TPS == 2 ? b >> 1 : 0);
+    vok[s] = lt < nt;
+    const int key = tile_of(v, vok[s] ? t0 + lt : v.n - 1) * kTile;
     const int64_t blk = p.block_table[(int64_t)seq * p.table_stride + (key >> lb)];
     vb[s] = reinterpret_cast<const T*>(p.v) + blk * p.v_sb + (int64_t)c * p.v_sh + (int64_t)rl * p.block_size +
             (key & (p.block_size - 1)) + (TPS == 2 ? (b & 1) : b) * M::EPL;
@@ -245,13 +259,13 @@ __global__ __launch_bounds__(256) void talk_mix_kernel(TalkAttnParams p) {
   auto weight = [&](int h, float s) { wt[h * kChunk + j] = j < nkey && s != -INFINITY ? __expf(s - hm[h]) * hl[h] : 0.f; };
 #pragma unroll
   for (int k = 0; k < kPre; ++k)
-    if (g0 + hp + 2 * k < g1) weight(g0 + hp + 2 * k, sv[k]);
-  for (int h = g0 + hp + 2 * kPre; h < g1; h += 2) weight(h, srow[(size_t)h * p.nch * kChunk]);
+    if (g0 + hp + HP * k < g1) weight(g0 + hp + HP * k, sv[k]);
+  for (int h = g0 + hp + HP * kPre; h < g1; h += HP) weight(h, srow[(size_t)h * p.nch * kChunk]);
   __syncthreads();
   // ---- mixed weights of this kv head's query heads
   {
     const int idx = ((j / M::KS) * 64 + 16 * ((j % M::KS) / M::EPL)) * M::EPL + j % M::EPL;
-    for (int r = hp; r < Rb; r += 2) {
+    for (int r = hp; r < Rb; r += HP) {
       float x = 0.f;
       if (p.talk) {
         const float* tk = p.talk + (size_t)(h0 + r) * p.H;  // (uniform per wave: scalar loads)
@@ -800,23 +814,24 @@ int check_attn(const TalkAttnParams& p) {
   return 0;
 }
 
+template <class T>
+int launch_rows(const TalkAttnParams& p, hipStream_t st) {
+  const size_t lds = mix_lds<T>(p.H);
+  if (lds > kMaxLds - 64) return -5;
+  const dim3 grid(p.rows * p.G, p.nch, (p.H / p.G + 15) / 16), block(256);
+  hipLaunchKernelGGL((talk_scores_kernel<T>), grid, block, 0, st, p);
+  hipLaunchKernelGGL((talk_mix_kernel<T>), grid, block, lds, st, p);
+  return (int)hipGetLastError();
+}
+
 }  // namespace
 
 extern "C" int vwa_talk_attention(const TalkAttnParams* p, hipStream_t st) {
   const int rc = check_attn(*p);
   if (rc) return rc;
   if (p->nch < 1 || !p->s || !p->stat || !p->part || !p->counters) return -4;
-  const size_t lds = p->f32 ? mix_lds<float>(p->H) : mix_lds<u16>(p->H);
-  if (lds > kMaxLds - 64 || (int64_t)p->nch * p->H * p->dv * 4 >= (1ll << 31)) return -5;
-  const dim3 grid(p->rows * p->G, p->nch, (p->H / p->G + 15) / 16), block(256);
-  if (p->f32) {
-    hipLaunchKernelGGL((talk_scores_kernel<float>), grid, block, 0, st, *p);
-    hipLaunchKernelGGL((talk_mix_kernel<float>), grid, block, lds, st, *p);
-  } else {
-    hipLaunchKernelGGL((talk_scores_kernel<u16>), grid, block, 0, st, *p);
-    hipLaunchKernelGGL((talk_mix_kernel<u16>), grid, block, lds, st, *p);
-  }
-  return (int)hipGetLastError();
+  if ((int64_t)p->nch * p->H * p->dv * 4 >= (1ll << 31)) return -5;
+  return p->f32 ? launch_rows<float>(*p, st) : launch_rows<u16>(*p, st);
 }
 
 extern "C" int64_t vwa_talk_prefill_part(int H, int G, int dk, int dv) {

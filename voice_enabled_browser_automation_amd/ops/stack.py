@@ -58,7 +58,7 @@ def visible_tiles(max_ctx: int, window: int, keep: int) -> int:
 
 
 def visible_chunks(max_ctx: int, window: int, keep: int) -> int:
-    """128-key chunks a row can see at most (vwa talk_chunks): sizes the rows-form scratch."""
+    """128-key chunks a row can see at most: sizes the rows-form scratch."""
     return -(-visible_tiles(max_ctx, window, keep) // 8)
 
 
