@@ -10,6 +10,7 @@
 
 // bindings_stack.cpp: the ops of layer stacks with an f32 residual stream
 void bind_stack(pybind11::module_& m);
+void bind_mixers(pybind11::module_& m);
 
 namespace {
 
@@ -1579,4 +1580,5 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("attention_split_tokens", []() { return vwa_attention_split_tokens(); });
   m.def("set_attention_impl", [](int64_t impl) { vwa_set_attention_impl((int)impl); });
   bind_stack(m);
+  bind_mixers(m);
 }

@@ -1,37 +1,10 @@
 // Torch bindings of the layer-stack kernels (stack_kernels.h): f32 residual rows, T = bf16 or f32
 // activations / caches / weights.  Shapes, dtypes and strides are checked here, before any launch.
-#include "bindings_common.h"
+#include "bindings_checks.h"
+#include "kernels/mixer_kernels.h"
 #include "kernels/stack_kernels.h"
 
 namespace {
-
-bool t_is_f32(const Tensor& t, const char* name) {
-  TORCH_CHECK(t.is_cuda(), name, " must be a GPU tensor");
-  TORCH_CHECK(t.scalar_type() == at::kBFloat16 || t.scalar_type() == at::kFloat, name, " must be bf16 or f32");
-  return t.scalar_type() == at::kFloat;
-}
-void check_t(const Tensor& t, bool f32, const char* name) {
-  TORCH_CHECK(t_is_f32(t, name) == f32, name, ": dtype differs from the other operands'");
-}
-void check_rows(const Tensor& t, int64_t rows, int64_t cols, const char* name) {
-  TORCH_CHECK(t.is_cuda() && t.dim() == 2 && t.stride(1) == 1 && t.size(0) >= rows && t.size(1) >= cols && t.stride(0) >= cols,
-              name, " must be [>= ", rows, ", >= ", cols, "] with contiguous columns");
-}
-void check_aligned(const Tensor& t, const char* name) {
-  TORCH_CHECK((reinterpret_cast<uintptr_t>(t.data_ptr()) & 15) == 0, name, " must be 16-byte aligned");
-}
-const int* i32p(const Tensor& t, int64_t n, const char* name) {
-  TORCH_CHECK(t.is_cuda() && t.scalar_type() == at::kInt && t.is_contiguous() && t.numel() >= n, name, ": int32 [>= ", n, "]");
-  return t.data_ptr<int>();
-}
-const int64_t* i64p(const Tensor& t, int64_t n, const char* name) {
-  TORCH_CHECK(t.is_cuda() && t.scalar_type() == at::kLong && t.is_contiguous() && t.numel() >= n, name, ": int64 [>= ", n, "]");
-  return t.data_ptr<int64_t>();
-}
-float* f32p(const Tensor& t, int64_t n, const char* name) {
-  TORCH_CHECK(t.is_cuda() && t.scalar_type() == at::kFloat && t.is_contiguous() && t.numel() >= n, name, ": f32 [>= ", n, "]");
-  return t.data_ptr<float>();
-}
 
 void gemm_f32(Tensor x, Tensor w, Tensor y, int64_t epi, c10::optional<Tensor> residual, c10::optional<Tensor> y2) {
   c10::DeviceGuard g(x.device());
@@ -54,7 +27,9 @@ void gemm_f32(Tensor x, Tensor w, Tensor y, int64_t epi, c10::optional<Tensor> r
   TORCH_CHECK(y.dim() == 2 && y.size(0) == M, "y rows");
   p.Y = y.data_ptr<float>();
   p.ldy = (int)y.stride(0);
-  if (epi == 6) {
+  if (epi == 2) {
+    TORCH_CHECK(N % 32 == 0 && y.size(1) * 2 == N && y.stride(1) == 1, "SwiGLU epilogue: y [M, N / 2], N a multiple of 32");
+  } else if (epi == 6) {
     TORCH_CHECK(y2.has_value(), "split epilogue needs y2");
     check_t(*y2, true, "y2");
     check_rows(*y2, M, 1, "y2");
@@ -75,23 +50,48 @@ void gemm_f32(Tensor x, Tensor w, Tensor y, int64_t epi, c10::optional<Tensor> r
   check_rc(vwa_gemm_f32((int)epi, &p, cur_stream(x)), "gemm_f32");
 }
 
-void layernorm_f32(Tensor x, Tensor w, Tensor b, Tensor y, double eps) {
+void layernorm_f32(Tensor x, Tensor w, c10::optional<Tensor> b, Tensor y, double eps) {
   c10::DeviceGuard g(x.device());
   check_t(x, true, "x");
   const bool f32 = t_is_f32(y, "y");
   const int64_t D = w.numel(), rows = y.size(0);
   f32p(w, D, "w");
-  f32p(b, D, "b");
   check_rows(x, rows, D, "x");
   check_rows(y, rows, D, "y");
   check_aligned(x, "x");
   check_aligned(y, "y");
-  check_rc(vwa_layernorm_f32(x.data_ptr<float>(), (int)x.stride(0), w.data_ptr<float>(), b.data_ptr<float>(), y.data_ptr(),
+  check_rc(vwa_layernorm_f32(x.data_ptr<float>(), (int)x.stride(0), w.data_ptr<float>(),
+                             b.has_value() ? f32p(*b, D, "b") : nullptr, y.data_ptr(),
                              (int)y.stride(0), (int)rows, (int)D, (int)y.size(1), (float)eps, f32, cur_stream(x)),
            "layernorm_f32");
 }
 
-void embedding_f32(Tensor ids, Tensor table, Tensor out) {
+// x (f32 rows) += norm(sum of the row's n_parts branch rows) * w1; h = norm(x) * w2 (no w2: no h)
+void add_norm(Tensor x, Tensor br, int64_t n_parts, Tensor w1, c10::optional<Tensor> w2, c10::optional<Tensor> h, double eps) {
+  c10::DeviceGuard g(x.device());
+  check_t(x, true, "x");
+  const bool f32 = t_is_f32(br, "branch");
+  const int64_t D = w1.numel(), rows = x.size(0), q = (D + 3) / 4 * 4;
+  TORCH_CHECK(n_parts >= 1, "n_parts");
+  check_rows(x, rows, q, "x");
+  check_rows(br, rows * n_parts, q, "branch");
+  check_aligned(x, "x");
+  check_aligned(br, "branch");
+  const float* p1 = f32p(w1, D, "w1");
+  const float* p2 = w2.has_value() ? f32p(*w2, D, "w2") : nullptr;
+  if (p2) {
+    TORCH_CHECK(h.has_value(), "w2 needs h");
+    check_t(*h, f32, "h");
+    check_rows(*h, rows, q, "h");
+    check_aligned(*h, "h");
+  }
+  check_rc(vwa_add_norm(x.data_ptr<float>(), (int)x.stride(0), br.data_ptr(), (int)br.stride(0), (int)n_parts, p1, p2,
+                        p2 ? h->data_ptr() : nullptr, p2 ? (int)h->stride(0) : 0, (int)rows, (int)D, p2 ? (int)h->size(1) : 0,
+                        (float)eps, f32, cur_stream(x)),
+           "add_norm");
+}
+
+void embedding_f32(Tensor ids, Tensor table, Tensor out, double scale) {
   c10::DeviceGuard g(out.device());
   const bool f32 = t_is_f32(table, "table");
   check_t(out, true, "out");
@@ -99,8 +99,8 @@ void embedding_f32(Tensor ids, Tensor table, Tensor out) {
   const int64_t rows = out.size(0);
   check_rows(out, rows, table.size(1), "out");
   check_rc(vwa_embedding_f32(i32p(ids, rows, "ids"), table.data_ptr(), (int)table.stride(0), out.data_ptr<float>(),
-                             (int)out.stride(0), (int)rows, (int)table.size(1), (int)out.size(1), (int)table.size(0), f32,
-                             cur_stream(out)),
+                             (int)out.stride(0), (int)rows, (int)table.size(1), (int)out.size(1), (int)table.size(0),
+                             (float)scale, f32, cur_stream(out)),
            "embedding_f32");
 }
 
@@ -344,6 +344,7 @@ void bind_stack(py::module_& m) {
   m.def("gemm_f32", &gemm_f32, py::arg("x"), py::arg("w"), py::arg("y"), py::arg("epi"), py::arg("residual") = py::none(),
         py::arg("y2") = py::none());
   m.def("layernorm_f32", &layernorm_f32);
+  m.def("add_norm", &add_norm);
   m.def("embedding_f32", &embedding_f32);
   m.def("qkv_cache", &qkv_cache);
   m.def("qkv_mingru", &qkv_mingru);

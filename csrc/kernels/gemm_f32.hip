@@ -52,6 +52,10 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(GemmF32Params p) {
     for (int r = 0; r < 4; ++r) {
       const int m = m0 + 16 * i + 4 * g + r;
       if (m >= p.M) continue;
+      if constexpr (EPI == 2) {  // (the wave's two column tiles are gate and up of the same 16 features)
+        p.Y[(size_t)m * p.ldy + (n0 >> 1) + rl] = silu(acc[i][0][r]) * acc[i][1][r];
+        continue;
+      }
 #pragma unroll
       for (int j = 0; j < 2; ++j) {
         const int n = n0 + 16 * j + rl;
@@ -75,12 +79,14 @@ extern "C" int vwa_gemm_f32(int epi, const GemmF32Params* p, hipStream_t st) {
   if ((reinterpret_cast<uintptr_t>(p->X) & 15) || (reinterpret_cast<uintptr_t>(p->W) & 15)) return -2;
   if (epi == 1 && !p->R) return -3;
   if (epi == 6 && (!p->Y2 || p->n_split < 0 || p->n_split > p->N)) return -4;
+  if (epi == 2 && p->N % 32) return -5;
   const dim3 grid((p->N + 63) / 64, (p->M + 63) / 64), block(256);
   switch (epi) {
     case 0: hipLaunchKernelGGL((gemm_f32_kernel<0>), grid, block, 0, st, *p); break;
     case 1: hipLaunchKernelGGL((gemm_f32_kernel<1>), grid, block, 0, st, *p); break;
+    case 2: hipLaunchKernelGGL((gemm_f32_kernel<2>), grid, block, 0, st, *p); break;
     case 6: hipLaunchKernelGGL((gemm_f32_kernel<6>), grid, block, 0, st, *p); break;
-    default: return -5;
+    default: return -6;
   }
   return (int)hipGetLastError();
 }

@@ -1,0 +1,216 @@
+// Routed experts.
+//
+//  moe_route : sigmoid router scores (MFMA, f32 sums), the best ``top`` experts of every row, and the pairs
+//              (row, choice) grouped by expert into tiles of at most ``tile`` pairs -- by the last workgroup
+//  moe_gemm  : the experts' matrices over such a tile.  First launch: the tile's rows times gate and up, scaled
+//              by the pair's score ahead of the activation (w (W h) = W (w h)); second: down, one row per pair.
+//              (The pairs of a row are added, in the order of its choices, by add_norm.)
+// A row's results do not depend on the tile it lands in, so the order inside an expert is free.
+#include "mixer_kernels.h"
+#include "stack_types.h"
+
+using namespace vwa;
+
+namespace {
+
+constexpr size_t kMaxLds = 160 * 1024 - 8192;
+constexpr int kRouteWaves = 8, kRouteThreads = kRouteWaves * 64, kMaxExperts = 256;
+
+// pairs -> tiles of one expert each (the whole workgroup)
+VWA_DEVICE void group_pairs(const MoeRouteParams& p, const int* ids) {
+  __shared__ int cnt[kMaxExperts], first[kMaxExperts], s_total;
+  const int tid = threadIdx.x, P = p.rows * p.top;
+  for (int e = tid; e < p.E; e += kRouteThreads) cnt[e] = 0;
+  __syncthreads();
+  auto id_of = [&](int i) { return __hip_atomic_load(const_cast<int*>(ids) + i, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT); };
+  for (int i = tid; i < P; i += kRouteThreads) {
+    const int e = id_of(i);
+    if (e >= 0) atomicAdd(&cnt[e], 1);
+  }
+  __syncthreads();
+  if (tid < 64) {                                    // exclusive prefix of the experts' tile counts
+    int base = 0;
+    for (int e0 = 0; e0 < p.E; e0 += 64) {
+      const int e = e0 + tid, n = e < p.E ? (cnt[e] + p.tile - 1) / p.tile : 0;
+      int x = n;
+#pragma unroll
+      for (int o = 1; o < 64; o <<= 1) {
+        const int y = __shfl_up(x, o, 64);
+        if (tid >= o) x += y;
+      }
+      if (e < p.E) first[e] = base + x - n;
+      base += __shfl(x, 63, 64);
+    }
+    if (tid == 0) s_total = base;
+  }
+  __syncthreads();
+  for (int e = tid; e < p.E; e += kRouteThreads) {
+    const int n = cnt[e];
+    for (int k = 0; k * p.tile < n; ++k) {
+      int* t = p.tiles + 1 + 3 * (first[e] + k);
+      t[0] = e;
+      t[1] = (first[e] + k) * p.tile;
+      t[2] = min(p.tile, n - k * p.tile);
+    }
+  }
+  if (tid == 0) p.tiles[0] = s_total;
+  __syncthreads();
+  for (int e = tid; e < p.E; e += kRouteThreads) cnt[e] = first[e] * p.tile;
+  __syncthreads();
+  for (int i = tid; i < P; i += kRouteThreads) {
+    const int e = id_of(i);
+    if (e >= 0) p.order[atomicAdd(&cnt[e], 1)] = i;
+  }
+}
+
+template <class T>
+__global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(MoeRouteParams p) {
+  using M = MM<T>;
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  __shared__ int s_last;
+  const int tid = threadIdx.x, lane = lane_id(), w = __builtin_amdgcn_readfirstlane(tid >> 6), rl = lane & 15, g = lane >> 4;
+  const int r0 = blockIdx.x * 16, nr = min(16, p.rows - r0), et = (p.E + 15) / 16, Ep = et * 16, steps = p.K / M::KS;
+  float* red = reinterpret_cast<float*>(smem);       // [waves][Ep][16 rows]
+  float* sc = red + kRouteWaves * Ep * 16;           // [16 rows][Ep + 1]
+  const T* h = reinterpret_cast<const T*>(p.h) + (size_t)(r0 + min(rl, nr - 1)) * p.ldh + g * M::EPL;
+  const uint4* wf = reinterpret_cast<const uint4*>(p.w) + lane;
+  for (int e = 0; e < et; ++e) {                     // D[expert 4 g + i][row rl], every wave a part of K
+    f32x4 acc = {};
+#pragma unroll 4
+    for (int s = w; s < steps; s += kRouteWaves)
+      acc = M::mma(wf[((size_t)e * steps + s) * 64], *reinterpret_cast<const uint4*>(h + s * M::KS), acc);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) red[(w * Ep + e * 16 + 4 * g + i) * 16 + rl] = acc[i];
+  }
+  __syncthreads();
+  for (int i = tid; i < Ep * 16; i += kRouteThreads) {
+    float z = 0.f;
+#pragma unroll
+    for (int k = 0; k < kRouteWaves; ++k) z += red[k * Ep * 16 + i];
+    sc[(i & 15) * (Ep + 1) + (i >> 4)] = (i >> 4) < p.E ? 1.f / (1.f + expf(-z)) : -2.f;
+  }
+  __syncthreads();
+  const int r = tid >> 5, q = tid & 31, row = r0 + r;  // 32 lanes per row
+  for (int k = 0; k < p.top; ++k) {
+    float best = -3.f;
+    int at = 0;
+    for (int e = q; e < p.E; e += 32) {
+      const float v = sc[r * (Ep + 1) + e];
+      if (v > best) {
+        best = v;
+        at = e;
+      }
+    }
+#pragma unroll
+    for (int o = 16; o > 0; o >>= 1) {
+      const float bo = __shfl_xor(best, o, 32);
+      const int ao = __shfl_xor(at, o, 32);
+      if (bo > best || (bo == best && ao < at)) {
+        best = bo;
+        at = ao;
+      }
+    }
+    if (q == 0 && r < nr) {
+      const bool live = p.slots[row] >= 0;
+      sc[r * (Ep + 1) + at] = -1.f;                  // (taken; scores are positive)
+      p.wts[row * p.top + k] = live ? best : 0.f;
+      __hip_atomic_store(p.ids + row * p.top + k, live ? at : -1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    }
+    __syncthreads();
+  }
+  // ---- the last workgroup groups the pairs
+  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+  __syncthreads();
+  if (tid == 0) {
+    const int t = __hip_atomic_fetch_add(p.ticket, 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    s_last = t == (int)gridDim.x - 1;
+    if (s_last) __hip_atomic_store(p.ticket, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  }
+  __syncthreads();
+  if (!s_last) return;
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+  group_pairs(p, p.ids);
+}
+
+// ------------------------------------------------------------------------------------------ small tiles (16 pairs)
+// A workgroup per (tile, 16 features | 16 columns); its 4 waves split K, the sums meet in LDS.
+template <class T, bool DOWN>
+__global__ __launch_bounds__(256) void moe_gemm16_kernel(MoeGemmParams p) {
+  using M = MM<T>;
+  constexpr int NA = DOWN ? 1 : 2;
+  __shared__ float red[4][NA][64][4];
+  const int tile = blockIdx.y;
+  if (tile >= p.tiles[0]) return;
+  const int e = p.tiles[1 + 3 * tile], place = p.tiles[2 + 3 * tile], n = p.tiles[3 + 3 * tile];
+  const int lane = lane_id(), w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), rl = lane & 15, g = lane >> 4;
+  const int KG = p.K / (16 * M::EPL), unit = blockIdx.x;
+  const int src = place + min(rl, n - 1);
+  const T* x = reinterpret_cast<const T*>(p.x) + (size_t)(DOWN ? src : p.order[src] / p.top) * p.ldx + 4 * M::EPL * g;
+  const uint4* wp = reinterpret_cast<const uint4*>(reinterpret_cast<const T*>(p.w) + e * p.w_expert) + (size_t)unit * NA * KG * 256 + lane;
+  f32x4 acc[NA] = {};
+#pragma unroll 2
+  for (int kg = w; kg < KG; kg += 4) {
+    uint4 f[NA][4], a[4];
+#pragma unroll
+    for (int s = 0; s < 4; ++s) {
+#pragma unroll
+      for (int j = 0; j < NA; ++j) f[j][s] = wp[((size_t)j * KG + kg) * 256 + s * 64];
+      a[s] = *reinterpret_cast<const uint4*>(x + kg * 16 * M::EPL + s * M::EPL);
+    }
+#pragma unroll
+    for (int s = 0; s < 4; ++s)
+#pragma unroll
+      for (int j = 0; j < NA; ++j) acc[j] = M::mma(a[s], f[j][s], acc[j]);
+  }
+#pragma unroll
+  for (int j = 0; j < NA; ++j) *reinterpret_cast<f32x4*>(red[w][j][lane]) = acc[j];
+  __syncthreads();
+  // thread (lane, i = wave): pair 4 g + i, column rl
+  const int q = 4 * g + w;
+  if (q >= n) return;
+  float v[NA];
+#pragma unroll
+  for (int j = 0; j < NA; ++j) v[j] = (red[0][j][lane][w] + red[1][j][lane][w]) + (red[2][j][lane][w] + red[3][j][lane][w]);
+  const int pair = p.order[place + q];
+  T* y = reinterpret_cast<T*>(p.y);
+  if constexpr (DOWN) {
+    stv(y + (size_t)pair * p.ldy + unit * 16 + rl, v[0]);
+  } else {
+    const float s = p.wts[pair];
+    stv(y + (size_t)(place + q) * p.ldy + unit * 16 + rl, silu(s * v[0]) * (s * v[1]));
+  }
+}
+
+}  // namespace
+
+extern "C" int vwa_moe_route(const MoeRouteParams* p, hipStream_t st) {
+  if (p->rows < 1 || p->E < 1 || p->E > kMaxExperts || p->top < 1 || p->top > p->E || p->K % 32 || p->ldh % 8 || p->tile < 1 ||
+      !p->wts || !p->ids || !p->tiles || !p->order || !p->ticket)
+    return -1;
+  // (every expert's last tile may be partly filled)
+  const int64_t P = (int64_t)p->rows * p->top;
+  if (p->max_tiles < (P < p->E ? P : p->E) + P / p->tile) return -2;
+  const int Ep = (p->E + 15) / 16 * 16;
+  const size_t lds = (size_t)kRouteWaves * Ep * 16 * 4 + 16 * (Ep + 1) * 4;
+  if (lds > kMaxLds) return -10;
+  const dim3 grid((p->rows + 15) / 16), block(kRouteThreads);
+  if (p->f32) hipLaunchKernelGGL((moe_route_kernel<float>), grid, block, lds, st, *p);
+  else hipLaunchKernelGGL((moe_route_kernel<u16>), grid, block, lds, st, *p);
+  return (int)hipGetLastError();
+}
+
+extern "C" int vwa_moe_gemm(const MoeGemmParams* p, hipStream_t st) {
+  if (p->max_tiles < 1 || p->N % (p->down ? 16 : 32) || p->K % 128 || p->ldx % 8 || p->tile != 16 || !p->tiles || !p->order ||
+      (!p->down && !p->wts))
+    return -1;
+  if ((reinterpret_cast<uintptr_t>(p->x) | reinterpret_cast<uintptr_t>(p->w)) & 15) return -2;
+  const dim3 grid(p->N / (p->down ? 16 : 32), p->max_tiles), block(256);
+  if (p->f32) {
+    if (p->down) hipLaunchKernelGGL((moe_gemm16_kernel<float, true>), grid, block, 0, st, *p);
+    else hipLaunchKernelGGL((moe_gemm16_kernel<float, false>), grid, block, 0, st, *p);
+  } else {
+    if (p->down) hipLaunchKernelGGL((moe_gemm16_kernel<u16, true>), grid, block, 0, st, *p);
+    else hipLaunchKernelGGL((moe_gemm16_kernel<u16, false>), grid, block, 0, st, *p);
+  }
+  return (int)hipGetLastError();
+}

@@ -3,17 +3,10 @@
 #pragma once
 #include "common.h"
 #include "stack_kernels.h"
+#include "stack_types.h"
 
 namespace {
 using namespace vwa;
-
-template <class T> VWA_DEVICE float ldv(const T* p);
-template <> VWA_DEVICE float ldv<u16>(const u16* p) { return bf2f(*p); }
-template <> VWA_DEVICE float ldv<float>(const float* p) { return *p; }
-VWA_DEVICE void stv(u16* p, float v) { *p = f2bf(v); }
-VWA_DEVICE void stv(float* p, float v) { *p = v; }
-
-VWA_DEVICE float sigm(float x) { return 1.f / (1.f + __expf(-x)); }
 
 struct Gate {
   float z, c;

@@ -1,0 +1,370 @@
+// Real-gated linear recurrence behind a short causal convolution (RgLruParams), f32 state.
+//
+// One workgroup handles whole blocks of channels: it forms u = conv(x) of up to RT rows in LDS, multiplies
+// it by the block's two gate matrices on the MFMA (D[row][channel]: a lane holds 4 consecutive rows of one
+// channel) and scans S <- a S + b over the rows in registers -- in the lane, over the four lane groups,
+// over the 16-row tiles.  A row that starts a run of its sequence folds the state it starts from into b and
+// takes a = 0, so one scan serves any mix of runs.
+//
+//  * rows form (decode steps, <= 64 rows): a workgroup per block; runs are found from the sequence ids.
+//    The block's workgroup is the only reader and writer of its channels' state rows.
+//  * scan form (prompt-sized runs): workgroups per (chunk of a run, block, 128 channels).  Launch 1 reduces
+//    every chunk to S_end = A S_start + B; launch 2 folds the chunks in front of its own, scans again and
+//    writes the outputs; the run's last chunk writes the state.
+//
+// A run that starts at position 0 starts from zeros whatever its slot holds.
+#include "mixer_kernels.h"
+#include "stack_types.h"
+
+using namespace vwa;
+
+namespace {
+
+constexpr size_t kMaxLds = 160 * 1024 - 2048;
+constexpr int kPad = 16;                             // bytes between LDS rows of u: 16 rows hit different banks
+
+VWA_DEVICE float gelu_tanh(float z) {
+  return z / (1.f + __expf(-1.5957691216057308f * (z + 0.044715f * z * z * z)));
+}
+
+struct Step {
+  float a, b;
+};
+// the recurrence's step from the gates' pre-activations; a and 1 - a^2 both from expm1 of log a
+VWA_DEVICE Step lru_step(float rp, float ip, float decay, float u) {
+  const float em = expm1f(decay * sigm(rp));
+  const float a = 1.f + em;
+  return Step{a, sqrtf(-em * (1.f + a)) * sigm(ip) * u};
+}
+
+template <class T> VWA_DEVICE int u_stride(int bs) { return bs * (int)sizeof(T) + kPad; }
+
+// r, i pre-activations of RT rows for 16 channels: u in LDS, gate fragments from global memory
+template <class T, int NT>
+VWA_DEVICE void gate_products(const char* us, int stride, const T* gw, int steps, f32x4 (&ar)[NT], f32x4 (&ai)[NT]) {
+  using M = MM<T>;
+  const int lane = lane_id(), rl = lane & 15, b = lane >> 4;
+#pragma unroll
+  for (int t = 0; t < NT; ++t) ar[t] = ai[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+  const uint4* wr = reinterpret_cast<const uint4*>(gw) + lane;
+  const uint4* wi = wr + (size_t)steps * 64;
+  const char* ua = us + rl * stride + b * 16;
+#pragma unroll 4
+  for (int s = 0; s < steps; ++s) {
+    const uint4 fr = wr[s * 64], fi = wi[s * 64];
+#pragma unroll
+    for (int t = 0; t < NT; ++t) {
+      const uint4 a = *reinterpret_cast<const uint4*>(ua + t * 16 * stride + s * 64);
+      ar[t] = M::mma(a, fr, ar[t]);
+      ai[t] = M::mma(a, fi, ai[t]);
+    }
+  }
+}
+
+// inclusive scan of the 16 rows of a tile (row 4 b + i in lane group b, register i): s[i] <- the state after
+// row i given the state ``carry`` before the tile; A, B: the tile as one step.  Returns the state after it.
+VWA_DEVICE float scan_tile(const float (&a)[4], const float (&bb)[4], float carry, float (&s)[4], float& A, float& B) {
+  const int lane = lane_id(), g = lane >> 4;
+  float pa[4], pb[4];
+  pa[0] = a[0];
+  pb[0] = bb[0];
+#pragma unroll
+  for (int i = 1; i < 4; ++i) {
+    pa[i] = a[i] * pa[i - 1];
+    pb[i] = a[i] * pb[i - 1] + bb[i];
+  }
+  // the lane groups in front: (ea, eb)
+  float ea = 1.f, eb = 0.f, ta = 1.f, tb = 0.f;
+#pragma unroll
+  for (int k = 0; k < 4; ++k) {
+    const float ka = __shfl(pa[3], (lane & 15) + 16 * k, 64), kb = __shfl(pb[3], (lane & 15) + 16 * k, 64);
+    tb = ka * tb + kb;
+    ta = ka * ta;
+    if (k + 1 == g) {
+      ea = ta;
+      eb = tb;
+    }
+  }
+  const float s0 = ea * carry + eb;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) s[i] = pa[i] * s0 + pb[i];
+  A = ta;
+  B = tb;
+  return ta * carry + tb;
+}
+
+// eight channels of the input xp + xb of row r (an input row of this step)
+template <class T>
+VWA_DEVICE void input8(const RgLruParams& p, int r, int ch, float (&v)[8]) {
+  ld8(reinterpret_cast<const T*>(p.yx) + (size_t)r * p.ld + p.nb * p.bs + ch, v);
+#pragma unroll
+  for (int e = 0; e < 8; ++e) v[e] += p.xb[ch + e];
+}
+
+// eight channels of u of row r: j rows of the run lie in front of r in this step, the inputs before them
+// come from the state row st (null: zeros)
+template <class T>
+VWA_DEVICE void conv8(const RgLruParams& p, int r, int j, const float* st, int ch, float (&u)[8]) {
+  const int W = p.nb * p.bs;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) u[e] = p.cb[ch + e];
+  for (int k = 0; k < p.taps; ++k) {                 // k tokens back
+    float v[8];
+    if (k <= j) {
+      input8<T>(p, r - k, ch, v);
+    } else if (st) {
+      ld8(st + (size_t)(p.taps - (k - j)) * W + ch, v);
+    } else {
+      break;
+    }
+    const float* w = p.cw + (size_t)(p.taps - 1 - k) * W + ch;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) u[e] += w[e] * v[e];
+  }
+}
+
+// the last taps - 1 inputs of a run of n rows ending at row r -> its state row (n rows shift the old ones)
+template <class T>
+VWA_DEVICE void save_inputs8(const RgLruParams& p, int r, int n, bool fresh, float* st, int ch) {
+  const int W = p.nb * p.bs;
+  for (int i = 1; i < p.taps; ++i) {                 // place i: the input taps - i tokens before the next one
+    const int back = p.taps - 1 - i;                 // rows before r
+    float v[8];
+    if (back < n) {
+      input8<T>(p, r - back, ch, v);
+    } else if (!fresh) {
+      ld8(st + (size_t)(i + n) * W + ch, v);         // (read before a lower place is written)
+    } else {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[e] = 0.f;
+    }
+    st8(st + (size_t)i * W + ch, v);
+  }
+}
+
+// ------------------------------------------------------------------------------------------ rows form
+template <class T, int NT>
+__global__ __launch_bounds__(1024) void rglru_rows_kernel(RgLruParams p) {
+  constexpr int RT = NT * 16;
+  extern __shared__ __attribute__((aligned(16))) char us[];
+  __shared__ int s_first[64], s_len[64];             // of the row's run: first row; rows (at its last row, else 0)
+  const int blk = blockIdx.x, bs = p.bs, W = p.nb * bs, c0 = blk * bs;
+  const int tid = threadIdx.x, nthr = blockDim.x, lane = lane_id(), w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int rl = lane & 15, g = lane >> 4, stride = u_stride<T>(bs), steps = bs / MM<T>::KS;
+  T* out = reinterpret_cast<T*>(p.out);
+  if (tid < p.rows && tid < 64) {
+    const int r = tid;
+    int f = r, len = 0;
+    if (p.slots[r] >= 0) {
+      const int seq = p.seq_ids[r];
+      while (f > 0 && p.slots[f - 1] >= 0 && p.seq_ids[f - 1] == seq) --f;
+      const bool end = r + 1 >= p.rows || p.slots[r + 1] < 0 || p.seq_ids[r + 1] != seq;
+      len = end ? r + 1 - f : 0;
+    } else {
+      f = -1;
+    }
+    s_first[r] = f;
+    s_len[r] = len;
+  }
+  __syncthreads();
+  const int oct = bs / 8;
+  for (int r0 = 0; r0 < p.rows; r0 += RT) {
+    const int n = min(RT, p.rows - r0);
+    for (int x = tid; x < RT * oct; x += nthr) {
+      const int i = x / oct, ch = (x % oct) * 8, r = r0 + i;
+      float u[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+      if (i < n && s_first[r] >= 0) {
+        const int f = s_first[r];
+        const float* st = p.positions[f] > 0 ? p.state + (size_t)p.seq_ids[r] * p.state_ld : nullptr;
+        conv8<T>(p, r, r - f, st, c0 + ch, u);
+      }
+      st8(reinterpret_cast<T*>(us + i * stride) + ch, u);
+    }
+    __syncthreads();                                 // (every read of the old inputs is done as well)
+    for (int x = tid; x < n * oct; x += nthr) {
+      const int i = x / oct, r = r0 + i, len = s_len[r];
+      if (len == 0) continue;
+      save_inputs8<T>(p, r, len, p.positions[s_first[r]] == 0, p.state + (size_t)p.seq_ids[r] * p.state_ld, c0 + (x % oct) * 8);
+    }
+    for (int ct = w; ct < bs / 16; ct += nthr >> 6) {
+      f32x4 ar[NT], ai[NT];
+      gate_products<T, NT>(us, stride, reinterpret_cast<const T*>(p.gw) + (size_t)(blk * (bs / 16) + ct) * 32 * bs, steps, ar, ai);
+      const int ch = c0 + ct * 16 + rl;
+      const float rb = p.rb[ch], ib = p.ib[ch], dec = p.decay[ch], yb = p.yb[ch];
+      float carry = 0.f;
+#pragma unroll
+      for (int t = 0; t < NT; ++t) {
+        float a[4], b[4], s[4], A, B;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int li = t * 16 + 4 * g + i, r = r0 + li;
+          a[i] = b[i] = 0.f;
+          if (li < n && s_first[r] >= 0) {
+            const float u = ldv(reinterpret_cast<const T*>(us + li * stride) + ct * 16 + rl);
+            const Step st = lru_step(ar[t][i] + rb, ai[t][i] + ib, dec, u);
+            a[i] = st.a;
+            b[i] = st.b;
+            if (s_first[r] == r || li == 0) {        // (a run that goes on from the rows before: its state was saved)
+              if (p.positions[r] > 0) b[i] += st.a * p.state[(size_t)p.seq_ids[r] * p.state_ld + ch];
+              a[i] = 0.f;
+            }
+          }
+        }
+        carry = scan_tile(a, b, carry, s, A, B);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int li = t * 16 + 4 * g + i, r = r0 + li;
+          if (li >= n) continue;
+          float o = 0.f;
+          if (s_first[r] >= 0) {
+            o = s[i] * gelu_tanh(ldv(reinterpret_cast<const T*>(p.yx) + (size_t)r * p.ld + ch) + yb);
+            if (s_len[r] > 0 || li == n - 1) p.state[(size_t)p.seq_ids[r] * p.state_ld + ch] = s[i];
+          }
+          stv(out + (size_t)r * p.ldo + ch, o);
+        }
+      }
+    }
+    __syncthreads();                                 // u is overwritten; saved states are read by the next rows
+  }
+}
+
+// ------------------------------------------------------------------------------------------ scan form
+constexpr int kScanWaves = 8;
+
+template <class T, int PASS, int NT>
+__global__ __launch_bounds__(kScanWaves * 64) void rglru_scan_kernel(RgLruParams p) {
+  constexpr int RT = NT * 16;
+  extern __shared__ __attribute__((aligned(16))) char us[];
+  const int ck = blockIdx.x, blk = blockIdx.y, bs = p.bs, W = p.nb * bs, c0 = blk * bs;
+  const int tid = threadIdx.x, lane = lane_id(), w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int rl = lane & 15, g = lane >> 4, stride = u_stride<T>(bs), steps = bs / MM<T>::KS;
+  const int row0 = p.chunks[4 * ck], n = p.chunks[4 * ck + 1], idx = p.chunks[4 * ck + 2], cnt = p.chunks[4 * ck + 3];
+  const int run0 = idx > 0 ? p.chunks[4 * (ck - idx)] : row0;  // first row of the run
+  const int pos0 = p.positions[run0];
+  float* st = p.state + (size_t)p.seq_ids[row0] * p.state_ld;
+  const int ct = blockIdx.z * kScanWaves + w;
+  const bool active = ct < bs / 16;
+  const int ch = c0 + (active ? ct : 0) * 16 + rl;
+  const float rb = p.rb[ch], ib = p.ib[ch], dec = p.decay[ch], yb = p.yb[ch];
+  float carry = 0.f, Ac = 1.f, Bc = 0.f;
+  if (PASS == 2 && active) {
+    carry = p.cS[(size_t)(ck - idx) * W + ch];
+    for (int k = ck - idx; k < ck; ++k) carry = p.cA[(size_t)k * W + ch] * carry + p.cB[(size_t)k * W + ch];
+  }
+  const int oct = bs / 8;
+  for (int r0 = 0; r0 < n; r0 += RT) {
+    const int m = min(RT, n - r0);
+    for (int x = tid; x < RT * oct; x += kScanWaves * 64) {
+      const int i = x / oct, c = (x % oct) * 8, r = row0 + r0 + i;
+      float u[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+      if (i < m) conv8<T>(p, r, r - run0, pos0 > 0 ? st : nullptr, c0 + c, u);
+      st8(reinterpret_cast<T*>(us + i * stride) + c, u);
+    }
+    __syncthreads();
+    if (active) {
+      f32x4 ar[NT], ai[NT];
+      gate_products<T, NT>(us, stride, reinterpret_cast<const T*>(p.gw) + (size_t)(blk * (bs / 16) + ct) * 32 * bs, steps, ar, ai);
+#pragma unroll
+      for (int t = 0; t < NT; ++t) {
+        float a[4], b[4], s[4], A, B;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int li = t * 16 + 4 * g + i;
+          const float u = ldv(reinterpret_cast<const T*>(us + li * stride) + ct * 16 + rl);
+          const Step q = lru_step(ar[t][i] + rb, ai[t][i] + ib, dec, u);
+          a[i] = li < m ? q.a : 1.f;
+          b[i] = li < m ? q.b : 0.f;
+        }
+        carry = scan_tile(a, b, carry, s, A, B);
+        if (PASS == 1) {
+          Bc = A * Bc + B;
+          Ac = A * Ac;
+        } else {
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            const int li = t * 16 + 4 * g + i, r = row0 + r0 + li;
+            if (li >= m) continue;
+            const float y = gelu_tanh(ldv(reinterpret_cast<const T*>(p.yx) + (size_t)r * p.ld + ch) + yb);
+            stv(reinterpret_cast<T*>(p.out) + (size_t)r * p.ldo + ch, s[i] * y);
+          }
+        }
+      }
+    }
+    __syncthreads();
+  }
+  if (active && g == 0) {
+    if (PASS == 1) {
+      p.cA[(size_t)ck * W + ch] = Ac;
+      p.cB[(size_t)ck * W + ch] = Bc;
+      if (idx == 0) p.cS[(size_t)ck * W + ch] = pos0 > 0 ? st[ch] : 0.f;
+    } else if (idx == cnt - 1) {
+      st[ch] = carry;
+    }
+  }
+}
+
+// the runs' last inputs (after the scan: its first chunks read the old ones)
+template <class T>
+__global__ __launch_bounds__(256) void rglru_inputs_kernel(RgLruParams p) {
+  const int ck = blockIdx.y, ch = (blockIdx.x * 256 + threadIdx.x) * 8;
+  const int row0 = p.chunks[4 * ck], n = p.chunks[4 * ck + 1], idx = p.chunks[4 * ck + 2], cnt = p.chunks[4 * ck + 3];
+  if (idx != cnt - 1 || ch >= p.nb * p.bs) return;
+  const int run0 = idx > 0 ? p.chunks[4 * (ck - idx)] : row0;
+  save_inputs8<T>(p, row0 + n - 1, row0 + n - run0, p.positions[run0] == 0, p.state + (size_t)p.seq_ids[row0] * p.state_ld, ch);
+}
+
+int check(const RgLruParams& p) {
+  if (p.rows < 1 || p.nb < 1 || p.bs < 32 || p.bs % 32 || p.taps < 1 || p.ld % 8 || p.state_ld % 4) return -1;
+  if ((int64_t)p.ld < 2ll * p.nb * p.bs || p.ldo < p.nb * p.bs || p.state_ld < (int64_t)p.taps * p.nb * p.bs) return -2;
+  if ((reinterpret_cast<uintptr_t>(p.yx) | reinterpret_cast<uintptr_t>(p.state) | reinterpret_cast<uintptr_t>(p.gw)) & 15) return -3;
+  return 0;
+}
+
+template <class T>
+size_t u_bytes(int rows, int bs) { return (size_t)rows * (bs * sizeof(T) + kPad); }
+
+template <class T>
+int launch_rows(const RgLruParams& p, hipStream_t st) {
+  const dim3 grid(p.nb), block(64 * (p.bs / 16 < 16 ? p.bs / 16 : 16));
+  if (p.rows > 16 && u_bytes<T>(64, p.bs) <= kMaxLds)
+    hipLaunchKernelGGL((rglru_rows_kernel<T, 4>), grid, block, u_bytes<T>(64, p.bs), st, p);
+  else if (u_bytes<T>(16, p.bs) <= kMaxLds)
+    hipLaunchKernelGGL((rglru_rows_kernel<T, 1>), grid, block, u_bytes<T>(16, p.bs), st, p);
+  else
+    return -10;
+  return (int)hipGetLastError();
+}
+
+template <class T, int NT>
+int launch_scan_nt(const RgLruParams& p, hipStream_t st) {
+  const dim3 grid(p.n_chunks, p.nb, (p.bs / 16 + kScanWaves - 1) / kScanWaves), block(kScanWaves * 64);
+  const size_t lds = u_bytes<T>(16 * NT, p.bs);
+  hipLaunchKernelGGL((rglru_scan_kernel<T, 1, NT>), grid, block, lds, st, p);
+  hipLaunchKernelGGL((rglru_scan_kernel<T, 2, NT>), grid, block, lds, st, p);
+  if (p.taps > 1)
+    hipLaunchKernelGGL((rglru_inputs_kernel<T>), dim3((p.nb * p.bs / 8 + 255) / 256, p.n_chunks), dim3(256), 0, st, p);
+  return (int)hipGetLastError();
+}
+
+template <class T>
+int launch_scan(const RgLruParams& p, hipStream_t st) {
+  if (u_bytes<T>(64, p.bs) <= 80 * 1024) return launch_scan_nt<T, 4>(p, st);
+  if (u_bytes<T>(16, p.bs) <= kMaxLds) return launch_scan_nt<T, 1>(p, st);
+  return -10;
+}
+
+}  // namespace
+
+extern "C" int vwa_rglru_rows(const RgLruParams* p, hipStream_t st) {
+  const int rc = check(*p);
+  if (rc) return rc;
+  if (p->rows > 64) return -4;
+  return p->f32 ? launch_rows<float>(*p, st) : launch_rows<u16>(*p, st);
+}
+
+extern "C" int vwa_rglru_scan(const RgLruParams* p, hipStream_t st) {
+  const int rc = check(*p);
+  if (rc) return rc;
+  if (p->n_chunks < 1 || !p->chunks || !p->cA || !p->cB || !p->cS) return -4;
+  return p->f32 ? launch_scan<float>(*p, st) : launch_scan<u16>(*p, st);
+}

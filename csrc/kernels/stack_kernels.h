@@ -6,7 +6,7 @@
 #include <stdint.h>
 
 // Y[M, N] = epi(X[M, K] . W[N, K]^T) in 32-bit (f32 MFMA).  epi as gemm.hip: 0 store, 1 residual add,
-// 6 split (columns >= n_split: relu(v)^2 -> Y2)
+// 2 SwiGLU over gate / up rows interleaved per 16 (Y [M, N / 2]), 6 split (columns >= n_split: relu(v)^2 -> Y2)
 struct GemmF32Params {
   const float* X; int ldx;
   const float* W;                   // row-major [N, K]
@@ -91,12 +91,12 @@ struct MinGruParams {
 extern "C" {
 #endif
 int vwa_gemm_f32(int epi, const GemmF32Params* p, hipStream_t st);
-// y (T) [rows, ldy] = layer norm of x f32 rows over D columns; columns D .. Dpad-1 of y are zeroed
+// y (T) [rows, ldy] = layer norm of x f32 rows over D columns (b null: no bias); columns D .. Dpad-1 of y are zeroed
 int vwa_layernorm_f32(const float* x, int ldx, const float* w, const float* b, void* y, int ldy, int rows, int D, int Dpad,
                       float eps, int f32, hipStream_t st);
-// out f32 [rows, ldo] = table (T) rows; ids outside the table give zeros; columns D .. Dpad-1 are zeroed
+// out f32 [rows, ldo] = table (T) rows * scale; ids outside the table give zeros; columns D .. Dpad-1 are zeroed
 int vwa_embedding_f32(const int* ids, const void* table, int ld, float* out, int ldo, int rows, int D, int Dpad, int vocab,
-                      int f32, hipStream_t st);
+                      float scale, int f32, hipStream_t st);
 int vwa_qkv_cache(const QkvCacheParams* p, hipStream_t st);
 // a decode step's qkv_cache and mingru_rows over the same rows, one launch
 int vwa_qkv_mingru(const QkvCacheParams* p, const MinGruParams* g, hipStream_t st);

@@ -1,23 +1,16 @@
 // Row kernels of layer stacks with an f32 residual stream.
 //
-//  layernorm_f32 : y (T) = (x - mean) * rstd * w + b of f32 rows, two-pass statistics in f32
-//  embedding_f32 : f32 residual rows from a T table
+//  layernorm_f32 : y (T) = (x - mean) * rstd * w (+ b) of f32 rows, two-pass statistics in f32
+//  add_norm      : x += norm(branch) * w1, h = norm(x) * w2 -- the end of a sublayer and the start of the next
+//  embedding_f32 : f32 residual rows from a T table, scaled
 //  qkv_cache     : partial rotation of q / k heads + paged cache write (V transposed inside a block)
 //  qkv_mingru    : qkv_cache and the recurrence's rows form of a decode step in one launch
+#include "mixer_kernels.h"
 #include "recurrence.h"
 
 using namespace vwa;
 
 namespace {
-
-// four consecutive values
-VWA_DEVICE void st4(u16* p, const float (&v)[4]) {
-  uint2 o;
-  o.x = pack2(v[0], v[1]);
-  o.y = pack2(v[2], v[3]);
-  *reinterpret_cast<uint2*>(p) = o;
-}
-VWA_DEVICE void st4(float* p, const float (&v)[4]) { *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]); }
 
 VWA_DEVICE float block_sum(float v, float* red) {
   v = wave_sum(v);
@@ -77,7 +70,7 @@ __global__ __launch_bounds__(256) void layernorm_f32_kernel(const float* __restr
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int cj = min(c + j, D - 1);
-      o[j] = c + j < D ? (v[i][j] - mu) * rstd * w[cj] + b[cj] : 0.f;
+      o[j] = c + j < D ? (v[i][j] - mu) * rstd * w[cj] + (b ? b[cj] : 0.f) : 0.f;
     }
     st4(yr + c, o);
   }
@@ -94,16 +87,108 @@ void launch_ln(const float* x, int ldx, const float* w, const float* b, T* y, in
   else hipLaunchKernelGGL((layernorm_f32_kernel<T, 8>), grid, block, 0, st, x, ldx, w, b, y, ldy, D, Dpad, eps);
 }
 
+// mean and 1 / std of the row held as STEPS x 4 values per thread (columns past D are zero)
+template <int STEPS>
+VWA_DEVICE float2 row_stats(const float (&v)[STEPS][4], int D, float eps, float* red) {
+  float s = 0.f;
+#pragma unroll
+  for (int i = 0; i < STEPS; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) s += v[i][j];
+  const float mu = block_sum(s, red) / (float)D;
+  float q = 0.f;
+#pragma unroll
+  for (int i = 0; i < STEPS; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const float d = (i * 256 + (int)threadIdx.x) * 4 + j < D ? v[i][j] - mu : 0.f;
+      q += d * d;
+    }
+  return make_float2(mu, 1.f / sqrtf(block_sum(q, red) / (float)D + eps));
+}
+
+// four weights from column c (0 past D)
+VWA_DEVICE void w4(const float* w, int c, int D, float (&v)[4]) {
+#pragma unroll
+  for (int j = 0; j < 4; ++j) v[j] = c + j < D ? w[min(c + j, D - 1)] : 0.f;
+}
+
+// one workgroup per row: x += norm(sum of the branch rows) * w1; h = norm(x) * w2.  Loads of the branch
+// and of the residual are in flight together.
+template <class T, int STEPS>
+__global__ __launch_bounds__(256) void add_norm_kernel(float* __restrict__ x, int ldx, const T* __restrict__ br, int ldb,
+                                                       int n_parts, const float* __restrict__ w1, const float* __restrict__ w2,
+                                                       T* __restrict__ h, int ldh, int D, int Dpad, float eps) {
+  __shared__ float red[4];
+  float* xr = x + (size_t)blockIdx.x * ldx;
+  const T* b = br + (size_t)blockIdx.x * n_parts * ldb;
+  const int last = (D - 1) & ~3;
+  float v[STEPS][4], xs[STEPS][4];
+#pragma unroll
+  for (int i = 0; i < STEPS; ++i) {
+    const int c = min((i * 256 + (int)threadIdx.x) * 4, last);
+    ld4(b + c, v[i]);
+    ld4(xr + c, xs[i]);
+  }
+  for (int k = 1; k < n_parts; ++k)
+#pragma unroll
+    for (int i = 0; i < STEPS; ++i) {
+      float u[4];
+      ld4(b + (size_t)k * ldb + min((i * 256 + (int)threadIdx.x) * 4, last), u);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) v[i][j] += u[j];
+    }
+#pragma unroll
+  for (int i = 0; i < STEPS; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if ((i * 256 + (int)threadIdx.x) * 4 + j >= D) v[i][j] = xs[i][j] = 0.f;
+  const float2 sb = row_stats<STEPS>(v, D, eps, red);
+#pragma unroll
+  for (int i = 0; i < STEPS; ++i) {
+    const int c = (i * 256 + threadIdx.x) * 4;
+    float w[4];
+    w4(w1, c, D, w);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) xs[i][j] += c + j < D ? (v[i][j] - sb.x) * sb.y * w[j] : 0.f;
+    if (c < D) st4(xr + c, xs[i]);  // (columns past D of the last quad stay zero)
+  }
+  if (!w2) return;
+  T* hr = h + (size_t)blockIdx.x * ldh;
+  const float2 sx = row_stats<STEPS>(xs, D, eps, red);
+#pragma unroll
+  for (int i = 0; i < STEPS; ++i) {
+    const int c = (i * 256 + threadIdx.x) * 4;
+    if (c >= D) continue;
+    float w[4], o[4];
+    w4(w2, c, D, w);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) o[j] = c + j < D ? (xs[i][j] - sx.x) * sx.y * w[j] : 0.f;
+    st4(hr + c, o);
+  }
+  for (int c = ((D + 3) & ~3) + threadIdx.x; c < Dpad; c += 256) stv(hr + c, 0.f);
+}
+
+template <class T>
+void launch_add_norm(float* x, int ldx, const T* br, int ldb, int parts, const float* w1, const float* w2, T* h, int ldh,
+                     int rows, int D, int Dpad, float eps, hipStream_t st) {
+  const dim3 grid(rows), block(256);
+  if (D <= 1024) hipLaunchKernelGGL((add_norm_kernel<T, 1>), grid, block, 0, st, x, ldx, br, ldb, parts, w1, w2, h, ldh, D, Dpad, eps);
+  else if (D <= 2048) hipLaunchKernelGGL((add_norm_kernel<T, 2>), grid, block, 0, st, x, ldx, br, ldb, parts, w1, w2, h, ldh, D, Dpad, eps);
+  else if (D <= 4096) hipLaunchKernelGGL((add_norm_kernel<T, 4>), grid, block, 0, st, x, ldx, br, ldb, parts, w1, w2, h, ldh, D, Dpad, eps);
+  else hipLaunchKernelGGL((add_norm_kernel<T, 8>), grid, block, 0, st, x, ldx, br, ldb, parts, w1, w2, h, ldh, D, Dpad, eps);
+}
+
 template <class T>
 __global__ __launch_bounds__(256) void embedding_f32_kernel(const int* __restrict__ ids, const T* __restrict__ table,
                                                             int ld, float* __restrict__ out, int ldo, int D, int Dpad,
-                                                            int vocab) {
+                                                            int vocab, float scale) {
   const int row = blockIdx.x;
   const int id = ids[row];
   const bool ok = id >= 0 && id < vocab;
   const int c = blockIdx.y * 256 + threadIdx.x;
   if (c < Dpad)
-    out[(size_t)row * ldo + c] = ok && c < D ? ldv(table + (size_t)id * ld + c) : 0.f;
+    out[(size_t)row * ldo + c] = ok && c < D ? ldv(table + (size_t)id * ld + c) * scale : 0.f;
 }
 
 // Part of one row.  VEC consecutive dimensions per thread (8 when the half rotation is a
@@ -185,15 +270,29 @@ extern "C" int vwa_layernorm_f32(const float* x, int ldx, const float* w, const 
   return (int)hipGetLastError();
 }
 
+extern "C" int vwa_add_norm(float* x, int ldx, const void* br, int ldb, int n_parts, const float* w1, const float* w2, void* h,
+                            int ldh, int rows, int D, int Dpad, float eps, int f32, hipStream_t st) {
+  const int q = (D + 3) & ~3;
+  if (rows < 1 || D < 1 || D > kLnSteps * 1024 || n_parts < 1 || ldx % 4 || ldb % 4 || ldx < q || ldb < q || !w1) return -1;
+  if (w2 && (Dpad < q || Dpad % 4 || ldh % 4 || ldh < Dpad)) return -2;
+  if (f32)
+    launch_add_norm(x, ldx, reinterpret_cast<const float*>(br), ldb, n_parts, w1, w2, reinterpret_cast<float*>(h), ldh, rows, D,
+                    Dpad, eps, st);
+  else
+    launch_add_norm(x, ldx, reinterpret_cast<const u16*>(br), ldb, n_parts, w1, w2, reinterpret_cast<u16*>(h), ldh, rows, D,
+                    Dpad, eps, st);
+  return (int)hipGetLastError();
+}
+
 extern "C" int vwa_embedding_f32(const int* ids, const void* table, int ld, float* out, int ldo, int rows, int D, int Dpad,
-                                 int vocab, int f32, hipStream_t st) {
+                                 int vocab, float scale, int f32, hipStream_t st) {
   if (rows < 1 || D < 1 || ld < D || Dpad < D || ldo < Dpad) return -1;
   if (f32)
     hipLaunchKernelGGL((embedding_f32_kernel<float>), dim3(rows, (Dpad + 255) / 256), dim3(256), 0, st, ids,
-                       reinterpret_cast<const float*>(table), ld, out, ldo, D, Dpad, vocab);
+                       reinterpret_cast<const float*>(table), ld, out, ldo, D, Dpad, vocab, scale);
   else
     hipLaunchKernelGGL((embedding_f32_kernel<u16>), dim3(rows, (Dpad + 255) / 256), dim3(256), 0, st, ids,
-                       reinterpret_cast<const u16*>(table), ld, out, ldo, D, Dpad, vocab);
+                       reinterpret_cast<const u16*>(table), ld, out, ldo, D, Dpad, vocab, scale);
   return (int)hipGetLastError();
 }
 

@@ -21,6 +21,7 @@
 #include "common.h"
 #include "mq_attention.h"
 #include "stack_kernels.h"
+#include "stack_types.h"
 
 using namespace vwa;
 
@@ -28,27 +29,6 @@ namespace {
 
 constexpr int kTile = 16;                  // keys per tile
 constexpr float kLog2e = 1.4426950408889634f;
-
-template <class T> struct MM;
-template <> struct MM<u16> {               // 16-byte fragments: 8 k per lane, 32 per step
-  static constexpr int KS = 32, EPL = 8;
-  static VWA_DEVICE f32x4 mma(const uint4& a, const uint4& b, const f32x4& c) { return mfma16(as_bf16x8(a), as_bf16x8(b), c); }
-};
-template <> struct MM<float> {             // 4 k per lane, 16 per step: element j of every lane group per MFMA
-  static constexpr int KS = 16, EPL = 4;
-  static VWA_DEVICE f32x4 mma(const uint4& a, const uint4& b, f32x4 c) {
-    c = __builtin_amdgcn_mfma_f32_16x16x4f32(__uint_as_float(a.x), __uint_as_float(b.x), c, 0, 0, 0);
-    c = __builtin_amdgcn_mfma_f32_16x16x4f32(__uint_as_float(a.y), __uint_as_float(b.y), c, 0, 0, 0);
-    c = __builtin_amdgcn_mfma_f32_16x16x4f32(__uint_as_float(a.z), __uint_as_float(b.z), c, 0, 0, 0);
-    return __builtin_amdgcn_mfma_f32_16x16x4f32(__uint_as_float(a.w), __uint_as_float(b.w), c, 0, 0, 0);
-  }
-};
-
-template <class T> VWA_DEVICE float ldv(const T* p);
-template <> VWA_DEVICE float ldv<u16>(const u16* p) { return bf2f(*p); }
-template <> VWA_DEVICE float ldv<float>(const float* p) { return *p; }
-VWA_DEVICE void stv(u16* p, float v) { *p = f2bf(v); }
-VWA_DEVICE void stv(float* p, float v) { *p = v; }
 
 struct Vis {
   int sink, first, n;                      // kept tiles 0 .. sink-1, then tiles first ..; n in all

@@ -3,7 +3,7 @@
 
 def model_class(cfg):
     """The model class that runs a configuration."""
-    from .config import GPT2Config, KabanexConfig, LlamaConfig
+    from .config import GPT2Config, KabanexConfig, LlamaConfig, RipupelConfig
 
     if isinstance(cfg, LlamaConfig):
         from .llama import LlamaModel
@@ -17,4 +17,8 @@ def model_class(cfg):
         from .kabanex import KabanexModel
 
         return KabanexModel
+    if isinstance(cfg, RipupelConfig):
+        from .ripupel import RipupelModel
+
+        return RipupelModel
     raise TypeError(f"no language model class for {type(cfg).__name__}")

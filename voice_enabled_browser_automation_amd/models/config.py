@@ -168,6 +168,127 @@ def kabanex_stack(name: str, *, vocab: int, hidden: int, n_layers: int, heads: i
     return KabanexConfig(name=name, vocab_size=vocab, hidden=hidden, layers=(L,) * n_layers, **kw)
 
 
+@dataclass(frozen=True)
+class RgLruConfig:
+    """Gated branch beside a short causal convolution and a real-gated linear recurrence, whose gates are
+    block-diagonal in the recurrence's channels."""
+    width: int
+    blocks: int
+    conv: int                # taps
+
+    @property
+    def block(self) -> int:
+        return self.width // self.blocks
+
+
+@dataclass(frozen=True)
+class LatentAttentionConfig:
+    """Attention whose keys and values are projections of one cached latent, with a shared rotated key part,
+    a softmax sink per head and an output gate per element."""
+    heads: int
+    dim: int                 # unrotated query / key size of a head
+    rot_dim: int             # rotated query / key size of a head
+    vdim: int
+    kv_rank: int
+    scale: float
+    rot_base: float
+    kv_from: Optional[int] = None    # the layer whose cached latent this one reads (None: its own)
+
+
+@dataclass(frozen=True)
+class DenseFFConfig:
+    ff: int
+
+
+@dataclass(frozen=True)
+class MoEConfig:
+    """``experts`` feed-forwards of size ff, of which a token uses the ``top`` with the largest sigmoid scores;
+    the score scales the expert's input."""
+    experts: int
+    top: int
+    ff: int
+
+
+@dataclass(frozen=True)
+class SerialLayerConfig:
+    """A mixer, then a feed-forward (None: none), each between two norms."""
+    mixer: object            # RgLruConfig | LatentAttentionConfig
+    mlp: object = None       # DenseFFConfig | MoEConfig | None
+
+
+@dataclass(frozen=True)
+class RipupelConfig:
+    name: str
+    vocab_size: int
+    hidden: int
+    layers: tuple            # of SerialLayerConfig, in order (sizes may differ from layer to layer)
+    embed_scale: float = 1.0
+    norm_eps: float = 1e-6
+    max_pos: int = 8192      # rotation table length to start with (it grows with the engine's contexts)
+    bos_id: int = 0
+    eos_ids: tuple = ()
+    init_std: float = 0.02
+
+    @property
+    def n_layers(self) -> int:
+        return len(self.layers)
+
+    @staticmethod
+    def from_json(j: dict, name: str = "ripupel") -> "RipupelConfig":
+        """The checkpoint's config.json.  A mixer or feed-forward kind this design does not have is an error,
+        never ignored."""
+        layers = []
+        for i, L in enumerate(j["layers"]):
+            m, mlp = L["mixer"], L.get("mlp")
+            if L["type"] == "rglru":
+                mixer = RgLruConfig(width=m["width"], blocks=m["blocks"], conv=m["conv"])
+                if mixer.blocks < 1 or mixer.width % mixer.blocks or mixer.conv < 1:
+                    raise ValueError(f"layer {i}: recurrence width, blocks or convolution taps do not fit")
+            elif L["type"] == "latent_attention":
+                mixer = LatentAttentionConfig(heads=m["heads"], dim=m["dim"], rot_dim=m["rot_dim"], vdim=m["vdim"],
+                                              kv_rank=m["kv_rank"], scale=float(m["scale"]), rot_base=float(m["rot"]["base"]),
+                                              kv_from=m.get("kv_from"))
+                if mixer.rot_dim < 2 or mixer.rot_dim % 2 or m["rot"]["dims"] != mixer.rot_dim:
+                    raise ValueError(f"layer {i}: rotated dimensions do not fit")
+                if mixer.kv_from is not None:
+                    src = layers[mixer.kv_from].mixer if 0 <= mixer.kv_from < i else None
+                    if not isinstance(src, LatentAttentionConfig) or src.kv_from is not None or \
+                            (src.kv_rank, src.rot_dim, src.rot_base) != (mixer.kv_rank, mixer.rot_dim, mixer.rot_base):
+                        raise ValueError(f"layer {i}: layer {mixer.kv_from} has no latent it could share")
+            else:
+                raise ValueError(f"layer {i}: unknown mixer type {L['type']!r}")
+            if mlp is None:
+                ff = None
+            elif mlp["kind"] == "dense":
+                ff = DenseFFConfig(ff=mlp["ff"])
+            elif mlp["kind"] == "moe":
+                ff = MoEConfig(experts=mlp["router"]["experts"], top=mlp["router"]["top"], ff=mlp["expert"]["ff"])
+                if not 1 <= ff.top <= ff.experts:
+                    raise ValueError(f"layer {i}: {ff.top} of {ff.experts} experts")
+            else:
+                raise ValueError(f"layer {i}: unknown feed-forward kind {mlp['kind']!r}")
+            layers.append(SerialLayerConfig(mixer=mixer, mlp=ff))
+        return RipupelConfig(name=name, vocab_size=j["vocab"], hidden=j["width"], layers=tuple(layers),
+                             embed_scale=float(j["embedding"]["scale"]), norm_eps=float(j["norm"]["eps"]))
+
+
+def ripupel_stack(name: str, *, vocab: int, hidden: int, n_layers: int, heads: int, dim: int, rot_dim: int, vdim: int,
+                  kv_rank: int, width: int, blocks: int, ffn: int, experts: int, top: int, expert_ff: int, conv: int = 4,
+                  rot_base: float = 500000.0, **kw) -> RipupelConfig:
+    """Recurrent layers with a dense feed-forward and attention layers with routed experts in turn, every second
+    attention layer on the latent of the one before (presets, benchmarks)."""
+    layers = []
+    for i in range(n_layers):
+        if i % 2 == 0:
+            layers.append(SerialLayerConfig(RgLruConfig(width=width, blocks=blocks, conv=conv), DenseFFConfig(ffn)))
+        else:
+            layers.append(SerialLayerConfig(
+                LatentAttentionConfig(heads=heads, dim=dim, rot_dim=rot_dim, vdim=vdim, kv_rank=kv_rank,
+                                      scale=(dim + rot_dim) ** -0.5, rot_base=rot_base, kv_from=i - 2 if i % 4 == 3 else None),
+                MoEConfig(experts=experts, top=top, ff=expert_ff)))
+    return RipupelConfig(name=name, vocab_size=vocab, hidden=hidden, layers=tuple(layers), **kw)
+
+
 LLAMA_PRESETS = {
     "llama3-8b": LlamaConfig(),
     "llama3-70b": LlamaConfig(name="llama3-70b", hidden=8192, n_layers=80, n_heads=64, n_kv_heads=8, ffn=28672),
@@ -205,6 +326,18 @@ KABANEX_PRESETS = {
 }
 
 
+RIPUPEL_PRESETS = {
+    # Llama-3.2-1B-sized layers (bench.py --design): its residual width, feed-forward and vocabulary
+    "ripupel-1b": ripupel_stack("ripupel-1b", vocab=128256, hidden=2048, n_layers=16, heads=16, dim=128, rot_dim=64, vdim=128,
+                                kv_rank=512, width=2048, blocks=16, ffn=8192, experts=32, top=4, expert_ff=1024, bos_id=128000,
+                                eos_ids=(128001, 128009)),
+    # small shapes for tests (vocab kept at the real tokenizer size so the grammar works)
+    "ripupel-tiny": ripupel_stack("ripupel-tiny", vocab=128256, hidden=192, n_layers=4, heads=3, dim=32, rot_dim=16, vdim=48,
+                                  kv_rank=64, width=192, blocks=3, ffn=256, experts=6, top=2, expert_ff=64, bos_id=128000,
+                                  eos_ids=(128001, 128009)),
+}
+
+
 def _llama_from_json(j: dict, name: str) -> LlamaConfig:
     hd = j.get("head_dim") or j["hidden_size"] // j["num_attention_heads"]
     return LlamaConfig(name=name, vocab_size=j["vocab_size"], hidden=j["hidden_size"], n_layers=j["num_hidden_layers"],
@@ -217,6 +350,7 @@ def _llama_from_json(j: dict, name: str) -> LlamaConfig:
 ARCHITECTURES = {
     "Kabanex": KabanexConfig.from_json,
     "LlamaForCausalLM": _llama_from_json,
+    "Ripupel": RipupelConfig.from_json,
 }
 
 
@@ -234,7 +368,7 @@ def get_config(name: str):
     """A preset by name, or the configuration of a checkpoint folder."""
     if os.path.isfile(os.path.join(name, "config.json")):
         return config_from_dir(name)
-    for table in (LLAMA_PRESETS, GPT2_PRESETS, KABANEX_PRESETS, WHISPER_PRESETS):
+    for table in (LLAMA_PRESETS, GPT2_PRESETS, KABANEX_PRESETS, RIPUPEL_PRESETS, WHISPER_PRESETS):
         if name in table:
             return table[name]
     raise KeyError(f"unknown model preset {name!r}")

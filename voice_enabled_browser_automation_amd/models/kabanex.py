@@ -95,6 +95,7 @@ class KabanexLayerWeights:
 
 class KabanexModel:
     stateful = True          # recurrent state per sequence: prefix-cached blocks alone cannot resume one
+    shared_buffers = ("talk",)   # step buffers that ragged forwards use as well
 
     def __init__(self, cfg: KabanexConfig, *, device="cpu", dtype: Optional[torch.dtype] = None,
                  tp: Optional[TPContext] = None, seed: int = 0, weights: Optional[dict] = None):
@@ -205,7 +206,7 @@ class KabanexModel:
                                        for L, D in zip(self.cfg.layers, self.dims)], max_ctx, dev))
         return b
 
-    def plan_rows(self, runs: Sequence[Tuple[int, int]], max_pos: int) -> SimpleNamespace:
+    def plan_rows(self, runs: Sequence[Tuple[int, int, int, int]], max_pos: int) -> SimpleNamespace:
         return ops.plan_runs(runs, self.device, max_pos)
 
     # ------------------------------------------------------------------ forward

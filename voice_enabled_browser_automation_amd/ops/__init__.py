@@ -690,6 +690,10 @@ def linear_swiglu(x: torch.Tensor, w_gu: torch.Tensor, *, fuse_rms: bool = False
     F = w_gu.shape[0] // 2
     if out is None:
         out = torch.empty((M, F), dtype=x.dtype, device=x.device)
+    if _gpu(x) and x.dtype == torch.float32:  # 32-bit models
+        assert not fuse_rms, "f32 linear_swiglu: no fused norm"
+        ext().gemm_f32(x, w_gu, out, 2)
+        return out
     if isinstance(w_gu, TiledWeight):
         if _gpu(x) and _stream_ok(x, w_gu):
             ext().skinny_gemm_swiglu(x, w_gu.t, None, out, fuse_rms, eps, None, True)
@@ -1182,5 +1186,7 @@ def env_int(name: str) -> int:
     return int(knob(name))
 
 
-from .stack import (TalkScratch, embedding_f32, layernorm_f32, linear_split, mingru, plan_runs,  # noqa: E402,F401
+from .mixers import (LatentScratch, LatentWeights, MoeWeights, RgLruWeights, fragments, gate_fragments,  # noqa: E402,F401
+                     latent_attention, latent_qkv, moe, moe_buffers, rglru, tile_weights)
+from .stack import (TalkScratch, add_norm, embedding_f32, layernorm_f32, linear_split, mingru, plan_runs,  # noqa: E402,F401
                     qkv_cache_mingru, qkv_cache_write, talk_attention, talk_fragment)

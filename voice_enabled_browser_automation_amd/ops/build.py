@@ -5,7 +5,7 @@
   ``csrc/bindings.cpp`` is compiled against the torch headers, and the lot is linked against
   torch's own HIP runtime (same ``libamdhip64.so.7`` soname, so one HIP runtime per process).
 * ``_vwa_core.so`` -- the same bindings over the kernels of CORE only (GEMMs, elementwise, sampling,
-  windowed attention, recurrences); the launchers of the other files are stubs that fail with a code
+  windowed and latent attention, recurrences, routed experts); the launchers of the other files are stubs that fail with a code
   (csrc/core_stubs.cpp).  The command-line entry points build it when a checkout has no library at
   all and the model at hand runs no chained launch: seconds instead of the minutes chain.hip takes.
 * ``_vwa_native.so`` -- the CPU runtime library (grammar engine, KV block manager): plain C++17
@@ -86,7 +86,8 @@ def _run(cmd: list[str]) -> None:
 
 
 # kernel files the core library holds; launchers of the others are stubs there
-CORE = ("gemm", "gemm_f32", "skinny_stream", "elementwise", "stack_ops", "talk_attention", "recurrence", "sample")
+CORE = ("gemm", "gemm_f32", "skinny_stream", "elementwise", "stack_ops", "talk_attention", "recurrence", "rglru", "latent", "moe",
+        "sample")
 
 
 def build_kernels(force: bool = False, jobs: int = 8, core: bool = False) -> str:
@@ -121,7 +122,7 @@ def _build_kernels(force: bool, jobs: int, core: bool) -> str:
         objs.append(obj)
         if force or not _newer(obj, _deps(src)):
             jobs_list.append(common + ["-c", src, "-o", obj])
-    for name in ("bindings", "bindings_stack"):
+    for name in ("bindings", "bindings_stack", "bindings_mixers"):
         src, obj = os.path.join(CSRC, name + ".cpp"), os.path.join(BUILD, name + ".o")
         objs.append(obj)
         if force or not _newer(obj, _deps(src)):

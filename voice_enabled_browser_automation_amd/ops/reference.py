@@ -112,17 +112,25 @@ def layernorm(x, w, b, *, eps=1e-5, residual=None, residual_out=None, out):
 # ----------------------------------------------------------------------------- layer stacks (ops/stack.py)
 def layernorm_f32(x, w, b, *, eps, out):
     D = w.shape[0]
-    y = F.layer_norm(x[:, :D].float(), (D,), w.float(), b.float(), eps)
+    y = F.layer_norm(x[:, :D].float(), (D,), w.float(), None if b is None else b.float(), eps)
     out.zero_()
     out[:, :D] = y.to(out.dtype)
     return out
 
 
-def embedding_f32(ids, table, *, out):
+def add_norm(x, branch, w1, w2, *, eps, out=None, n_parts=1):
+    D = w1.shape[0]
+    y = branch[: x.shape[0] * n_parts, :D].float().view(x.shape[0], n_parts, D).sum(1)
+    x[:, :D] += F.layer_norm(y, (D,), w1, None, eps)
+    if w2 is not None:
+        layernorm_f32(x, w2, None, eps=eps, out=out)
+
+
+def embedding_f32(ids, table, *, out, scale=1.0):
     idl = ids[: out.shape[0]].long()
     ok = (idl >= 0) & (idl < table.shape[0])
     out.zero_()
-    out[:, : table.shape[1]] = table[idl.clamp(0, table.shape[0] - 1)].float() * ok[:, None]
+    out[:, : table.shape[1]] = table[idl.clamp(0, table.shape[0] - 1)].float() * scale * ok[:, None]
     return out
 
 
@@ -193,6 +201,101 @@ def mingru(z, x, g, zb, xb, *, seq_ids, positions, slots, state, out_scale, out)
         S = (1 - zf[m]) * S + zf[m] * cand[m]
         state[sid] = S
         out[m, :W] = (S * F.silu(gf[m]) * out_scale).to(out.dtype)
+    return out
+
+
+# ----------------------------------------------------------------------------- mixers (ops/mixers.py)
+def rglru(yx, w, *, seq_ids, positions, slots, state, out):
+    W, taps = w.decay.shape[0], w.conv.shape[0]
+    rows = out.shape[0]
+    out.zero_()
+    r0 = 0
+    while r0 < rows:
+        if int(slots[r0]) < 0:
+            r0 += 1
+            continue
+        seq, r1 = int(seq_ids[r0]), r0 + 1
+        while r1 < rows and int(seq_ids[r1]) == seq and int(slots[r1]) >= 0:
+            r1 += 1
+        st = state[seq, : taps * W].view(taps, W)
+        if int(positions[r0]) == 0:
+            st.zero_()
+        xs = torch.cat([st[1:], yx[r0:r1, W : 2 * W].float() + w.xb])
+        n = r1 - r0
+        u = sum(xs[k : k + n] * w.conv[k] for k in range(taps)) + w.conv_b
+        u = u.to(yx.dtype).float()
+        pre = torch.einsum("nbi,bgoi->gnbo", u.view(n, w.nb, -1), w.gates.float()).reshape(2, n, W)
+        em = torch.expm1(w.decay * torch.sigmoid(pre[0] + w.rb))
+        b = torch.sqrt(-em * (2.0 + em)) * torch.sigmoid(pre[1] + w.ib) * u
+        y = F.gelu(yx[r0:r1, :W].float() + w.yb, approximate="tanh")
+        S = st[0].clone()
+        for t in range(n):
+            S = (1.0 + em[t]) * S + b[t]
+            out[r0 + t] = (S * y[t]).to(out.dtype)
+        st[0], st[1:] = S, xs[n:]
+        r0 = r1
+    return out
+
+
+def _rotate_half(x, cs):
+    """x [rows, heads, r], cs [rows, r / 2, 2]."""
+    half = x.shape[-1] // 2
+    c, s = cs[:, None, :, 0], cs[:, None, :, 1]
+    u, v = x[..., :half], x[..., half:]
+    return torch.cat([u * c - v * s, v * c + u * s], -1)
+
+
+def latent_qkv(y, w, *, rope, positions, slots, q_out, cache):
+    M, hq, rot = q_out.shape[0], w.dim_p + w.rot_p, 2 * rope.shape[1]
+    cs = rope[positions[:M].long()]
+    q = y[:M, : w.H * hq].float().view(M, w.H, hq)
+    o = torch.zeros(M, w.H, w.rank_p + w.rot_p)
+    o[..., : w.rank_p] = torch.einsum("mhi,hoi->mho", q[..., : w.dim_p], w.uk.float())
+    o[..., w.rank_p : w.rank_p + rot] = _rotate_half(q[..., w.dim_p : w.dim_p + rot], cs)
+    q_out.copy_(o.view(M, -1).to(q_out.dtype))
+    if cache is None:
+        return q_out
+    rank, at = w.norm.shape[0], w.H * hq
+    c = y[:M, at : at + rank].float()
+    row = torch.zeros(M, w.rank_p + w.rot_p)
+    row[:, :rank] = c * torch.rsqrt(c.pow(2).mean(-1, keepdim=True) + w.eps) * w.norm
+    row[:, w.rank_p : w.rank_p + rot] = _rotate_half(y[:M, None, at + w.rank_p : at + w.rank_p + rot].float(), cs)[:, 0]
+    bs = cache.shape[2]
+    for m in range(M):
+        sl = int(slots[m])
+        if sl >= 0:
+            cache[sl // bs, 0, sl % bs] = row[m].to(cache.dtype)
+    return q_out
+
+
+def latent_attention(q, w, *, cache, block_table, positions, seq_ids, slots, gate, out):
+    dk, bs = w.rank_p + w.rot_p, cache.shape[2]
+    out.zero_()
+    for m in range(q.shape[0]):
+        if int(slots[m]) < 0:
+            continue
+        n = int(positions[m]) + 1
+        blocks = block_table[int(seq_ids[m]), : -(-n // bs)].long()
+        k = cache[blocks, 0].reshape(-1, dk)[:n].float()
+        s = (q[m].float().view(w.H, dk) @ k.t()) * w.scale
+        p = torch.softmax(torch.cat([s, w.sink[:, None]], -1), -1)[:, :n]
+        o = torch.einsum("hr,hvr->hv", p @ k[:, : w.rank_p], w.uv.float()).reshape(-1)
+        out[m] = (o * torch.sigmoid(gate[m].float())).to(out.dtype)
+    return out
+
+
+def moe(h, w, *, slots, out):
+    F_, rows = w.down.shape[2], h.shape[0]
+    s = torch.sigmoid(h.float() @ w.router[: w.E].float().t())
+    val, idx = torch.topk(s, w.top, dim=-1)
+    for m in range(rows):
+        if int(slots[m]) < 0:
+            continue
+        for k in range(w.top):
+            e = int(idx[m, k])
+            gu = (val[m, k] * (w.gate_up[e].float() @ h[m].float())).view(F_ // 16, 2, 16)
+            a = (F.silu(gu[:, 0]) * gu[:, 1]).reshape(-1).to(h.dtype).float()
+            out[m * w.top + k] = (w.down[e].float() @ a).to(out.dtype)
     return out
 
 

@@ -27,21 +27,21 @@ def _ext():
 
 
 # ----------------------------------------------------------------------------- row plans
-def plan_runs(runs: Sequence[Tuple[int, int]], device, max_pos: int) -> SimpleNamespace:
-    """Launch tables of a ragged step with many rows.  runs: (first row, rows), each of one sequence at
+def plan_runs(runs: Sequence[Tuple[int, int]], device, max_pos: int, scan_rows: int = SCAN_ROWS) -> SimpleNamespace:
+    """Launch tables of a ragged step with many rows.  runs: (first row, rows, ..), each of one sequence at
     consecutive positions; max_pos: the largest position of the step.  tiles: prefill attention tiles of the runs longer than one row; singles:
     the rows that are a run of their own (decoded tokens beside prompt portions); chunks: recurrence
-    scan chunks of every run."""
+    scan chunks (of scan_rows rows) of every run."""
     tiles: List[List[int]] = []
     singles: List[int] = []
     chunks: List[List[int]] = []
-    for r0, n in runs:
+    for r0, n, *_ in runs:
         if n == 1:
             singles.append(r0)
         else:
             tiles += [[r0 + i, min(TILE_ROWS, n - i)] for i in range(0, n, TILE_ROWS)]
-        k = -(-n // SCAN_ROWS)
-        chunks += [[r0 + i * SCAN_ROWS, min(SCAN_ROWS, n - i * SCAN_ROWS), i, k] for i in range(k)]
+        k = -(-n // scan_rows)
+        chunks += [[r0 + i * scan_rows, min(scan_rows, n - i * scan_rows), i, k] for i in range(k)]
 
     def dev(x, cols):
         t = torch.tensor(x, dtype=torch.int32).view(-1, cols)
@@ -81,19 +81,28 @@ class TalkScratch:
 
 
 # ----------------------------------------------------------------------------- ops
-def layernorm_f32(x: torch.Tensor, w: torch.Tensor, b: torch.Tensor, *, eps: float, out: torch.Tensor) -> torch.Tensor:
-    """out = (x - mean) / sqrt(var + eps) * w + b of f32 rows; out may be wider than w (zero columns)."""
+def layernorm_f32(x: torch.Tensor, w: torch.Tensor, b: Optional[torch.Tensor], *, eps: float, out: torch.Tensor) -> torch.Tensor:
+    """out = (x - mean) / sqrt(var + eps) * w (+ b) of f32 rows; out may be wider than w (zero columns)."""
     if not x.is_cuda:
         return ref.layernorm_f32(x, w, b, eps=eps, out=out)
     _ext().layernorm_f32(x, w, b, out, eps)
     return out
 
 
-def embedding_f32(ids: torch.Tensor, table: torch.Tensor, *, out: torch.Tensor) -> torch.Tensor:
-    """f32 residual rows from the embedding table; out may be wider than the table (zero columns)."""
+def add_norm(x: torch.Tensor, branch: torch.Tensor, w1: torch.Tensor, w2: Optional[torch.Tensor], *, eps: float,
+             out: Optional[torch.Tensor] = None, n_parts: int = 1) -> None:
+    """The end of a sublayer and the start of the next: x (f32 rows) += norm(branch) * w1, out = norm(x) * w2
+    (w2 None: not computed).  branch rows n_parts * i .. are added up for row i; layer norms without bias."""
+    if not x.is_cuda:
+        return ref.add_norm(x, branch, w1, w2, eps=eps, out=out, n_parts=n_parts)
+    _ext().add_norm(x, branch, n_parts, w1, w2, out, eps)
+
+
+def embedding_f32(ids: torch.Tensor, table: torch.Tensor, *, out: torch.Tensor, scale: float = 1.0) -> torch.Tensor:
+    """f32 residual rows from the embedding table, scaled; out may be wider than the table (zero columns)."""
     if not out.is_cuda:
-        return ref.embedding_f32(ids, table, out=out)
-    _ext().embedding_f32(ids, table, out)
+        return ref.embedding_f32(ids, table, out=out, scale=scale)
+    _ext().embedding_f32(ids, table, out, scale)
     return out
 
 

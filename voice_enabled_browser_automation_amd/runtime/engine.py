@@ -186,6 +186,8 @@ class LLMEngine:
             PagedKVCache.bytes_per_block(cfg.n_layers, model.nkv, model.hd, block_size)
         if hasattr(model, "ensure_positions"):
             model.ensure_positions(max_model_len)
+        if not per_block and kv_blocks is None:  # (a stack without attention keeps no pages: no budget to divide)
+            kv_blocks = max_seqs * -(-max_model_len // block_size) + 1
         if layers and kv_blocks is None and kv_gb is None and knob("VWA_KV_GB").strip().lower() == "auto":
             # what is free now, minus headroom for step buffers, graphs, prompt scratch and a co-located service
             free, _total = torch.cuda.mem_get_info(self.device) if self.device.type == "cuda" else (0, 0)
@@ -731,8 +733,8 @@ class LLMEngine:
             tokens=meta[0], positions=meta[1], seq_ids=meta[2], ctx_lens=meta[3],
             slots=slot_t, block_table=self.bufs.block_table, max_ctx=self.bufs.max_ctx, logits_local=self.bufs.logits_local)
         if hasattr(m, "row_buffers"):
-            vars(scratch).update(m.row_buffers(n, self.bufs.max_ctx), talk=getattr(self.bufs, "talk", None),
-                                 plan=m.plan_rows([(a, k) for a, k, _, _ in runs], int(np_meta[1].max())))
+            vars(scratch).update({name: getattr(self.bufs, name) for name in m.shared_buffers})
+            vars(scratch).update(m.row_buffers(n, self.bufs.max_ctx), plan=m.plan_rows(runs, int(np_meta[1].max())))
         else:
             d = m.cfg.hidden
             vars(scratch).update(

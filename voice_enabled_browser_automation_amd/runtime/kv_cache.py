@@ -21,12 +21,15 @@ import torch
 
 @dataclass(frozen=True)
 class CacheLayer:
-    """What one layer keeps of a sequence: paged keys and values, and ``state`` f32 channels."""
-    n_kv_heads: int
-    k_dim: int
-    v_dim: int
+    """What one layer keeps of a sequence: paged keys and values (v_dim 0: the values are projections of the
+    key rows), and ``state`` f32 channels.  shared: the layer reads the pages of that earlier layer and has
+    none of its own."""
+    n_kv_heads: int = 0
+    k_dim: int = 0
+    v_dim: int = 0
     v_transposed: bool = False
     state: int = 0
+    shared: Optional[int] = None
 
 
 class PagedKVCache:
@@ -55,14 +58,17 @@ class PagedKVCache:
             shape = (num_blocks, L.n_kv_heads) + ((dim, block_size) if transposed else (block_size, dim))
             return torch.zeros(shape, dtype=dtype, device=device)
 
-        self.k = [pages(L, L.k_dim, False) for L in layers]
-        self.v = [pages(L, L.v_dim, L.v_transposed) for L in layers]
+        self.k, self.v = [], []
+        for L in layers:
+            own = L.shared is None
+            self.k.append(pages(L, L.k_dim, False) if own else self.k[L.shared])
+            self.v.append(pages(L, L.v_dim, L.v_transposed) if own else self.v[L.shared])
         self.state = [torch.zeros(n_slots, L.state, dtype=torch.float32, device=device) for L in layers]
         return self
 
     @staticmethod
     def layer_bytes_per_block(layers: Sequence["CacheLayer"], block_size: int, elem: int = 2) -> int:
-        return sum(L.n_kv_heads * block_size * (L.k_dim + L.v_dim) * elem for L in layers)
+        return sum(L.n_kv_heads * block_size * (L.k_dim + L.v_dim) * elem for L in layers if L.shared is None)
 
     @staticmethod
     def bytes_per_block(n_layers: int, n_kv_heads: int, head_dim: int, block_size: int, elem: int = 2) -> int:

@@ -64,14 +64,14 @@ def load_llm(name: str, *, device, tp=None, seed: int = 0, weights_path: Optiona
     the Llama projections to OCP e4m3 on load; ``dtype`` overrides the compute dtype (torch.float32:
     everything in 32-bit, for the models that have it)."""
     from ..models import model_class
-    from ..models.config import GPT2Config, KabanexConfig, get_config
+    from ..models.config import GPT2Config, KabanexConfig, RipupelConfig, get_config
 
     cfg = get_config(name)
     if weights_path is None and os.path.isdir(name):
         weights_path = name
     w = LazySafetensors(weights_path) if weights_path else None
     cls = model_class(cfg)
-    if isinstance(cfg, (GPT2Config, KabanexConfig)):
+    if isinstance(cfg, (GPT2Config, KabanexConfig, RipupelConfig)):
         return cls(cfg, device=device, seed=seed, weights=w, dtype=dtype)
     if dtype not in (None, torch.bfloat16):
         raise NotImplementedError(f"{cls.__name__} has no {dtype} kernels")
