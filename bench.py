@@ -199,10 +199,10 @@ def main():
                          "intent decoding); reported under 'concurrent', outside the headline value")
     ap.add_argument("--dtype", default=knob("VWA_DTYPE"), choices=("bf16", "fp8"),
                     help="LLM weight dtype: bf16 (headline config) or fp8 (W8A8 on the fp8 MFMA, config 5)")
-    ap.add_argument("--design", choices=("kabanex",), help="instead of the headline: prefill / decode throughput of a model "
-                    "design beside Llama layers of equal size (tools/design_bench.py)")
+    ap.add_argument("--design", choices=("ripupel", "kabanex"), help="instead of the headline: prefill / decode "
+                    "throughput of a model design beside the closest model at equal size (tools/design_bench.py)")
     ap.add_argument("--design-size", default="s1,s2,s4")
-    ap.add_argument("--design-only", choices=("kabanex", "llama"))
+    ap.add_argument("--design-only", choices=("ripupel", "kabanex", "llama"))
     ap.add_argument("--design-rounds", type=int, default=3)
     ap.add_argument("--no-graphs", action="store_true")
     ap.add_argument("--verbose", action="store_true")

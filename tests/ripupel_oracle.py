@@ -166,3 +166,103 @@ def forward(cfg, weights, tokens, layers=False):
         res.append(x)
     logits = layer_norm(x, w["final.norm"], eps) @ w["embed"].T
     return (logits, res) if layers else logits
+
+
+# ----------------------------------------------------------------------------- test models
+def rglru_layer(width, blocks, conv, mlp):
+    return {"type": "rglru", "mixer": {"width": width, "blocks": blocks, "conv": conv}, "mlp": mlp}
+
+
+def latent_layer(heads, dim, rot_dim, vdim, kv_rank, mlp, base=10000.0, scale=None, kv_from=None):
+    m = {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "kv_rank": kv_rank,
+         "rot": {"base": base, "dims": rot_dim}, "scale": (dim + rot_dim) ** -0.5 if scale is None else scale}
+    if kv_from is not None:
+        m["kv_from"] = kv_from
+    return {"type": "latent_attention", "mixer": m, "mlp": mlp}
+
+
+def dense(ff):
+    return {"kind": "dense", "ff": ff}
+
+
+def moe(experts, top, ff):
+    return {"kind": "moe", "router": {"experts": experts, "top": top}, "expert": {"ff": ff}}
+
+
+def model_config(width, vocab, layers, eps=1e-5, scale=0.7):
+    return {"architecture": "Ripupel", "vocab": vocab, "width": width, "norm": {"eps": eps}, "embedding": {"scale": scale},
+            "layers": layers}
+
+
+def random_weights(cfg, seed=0, dtype=torch.bfloat16):
+    """Weights that keep every mechanism visible: spread-out attention scores, sinks of the scores' size, strong
+    gates, slow and fast recurrent channels.  The first coordinates of a token's embedding rank the experts with
+    wide margins and the branches hardly touch them, so no choice of experts is a close call."""
+    gen = torch.Generator().manual_seed(seed)
+    r = lambda *s, std=1.0, mean=0.0: (mean + torch.randn(*s, generator=gen) * std).to(dtype)  # noqa: E731
+    d, V = cfg["width"], cfg["vocab"]
+    s = d ** -0.5
+    n_exp = max([0] + [L["mlp"]["router"]["experts"] for L in cfg["layers"] if L["mlp"] and L["mlp"]["kind"] == "moe"])
+    embed = r(V, d, std=1.5).float()
+    for t in range(V):
+        for k in range(n_exp):
+            embed[t, (t * 7 + k) % n_exp] = 4.0 - 8.0 * k / max(1, n_exp - 1)
+    w = {"embed": embed.to(dtype), "final.norm": r(d, mean=1, std=0.2)}
+
+    def out_norm():
+        n = r(d, mean=1, std=0.2)
+        n[:n_exp] = n[:n_exp] * 0.02
+        return n
+
+    for i, L in enumerate(cfg["layers"]):
+        p, m, c = f"l{i}.", f"l{i}.mix.", L["mixer"]
+        w[p + "norm1"], w[p + "norm1b"] = r(d, mean=1, std=0.2), out_norm()
+        if L["type"] == "rglru":
+            W, nb = c["width"], c["blocks"]
+            k = W // nb
+            w.update({m + "y": r(W, d, std=s), m + "y.b": r(W, std=0.3), m + "x": r(W, d, std=s), m + "x.b": r(W, std=0.3),
+                      m + "conv": r(W, c["conv"], std=0.6), m + "conv.b": r(W, std=0.3), m + "ra": r(nb, k, k, std=2 * k ** -0.5),
+                      m + "ra.b": r(nb, k), m + "ri": r(nb, k, k, std=2 * k ** -0.5), m + "ri.b": r(nb, k),
+                      m + "lam": r(W, mean=-4.0, std=2.0), m + "o": r(d, W, std=W ** -0.5)})
+        else:
+            H, n = c["heads"], c["kv_rank"]
+            w.update({m + "q": r(H * (c["dim"] + c["rot_dim"]), d, std=1.6 * s), m + "uk": r(H * c["dim"], n, std=1.6 * n ** -0.5),
+                      m + "uv": r(H * c["vdim"], n, std=n ** -0.5), m + "sink": r(H, mean=1.0), m + "g": r(H * c["vdim"], d, std=s),
+                      m + "o": r(d, H * c["vdim"], std=(H * c["vdim"]) ** -0.5)})
+            if "kv_from" not in c:
+                w.update({m + "dkv": r(n + c["rot_dim"], d, std=1.6 * s), m + "dkv.norm": r(n, mean=1, std=0.2)})
+        f = L["mlp"]
+        if not f:
+            continue
+        w[p + "norm2"], w[p + "norm2b"] = r(d, mean=1, std=0.2), out_norm()
+        w[p + "norm2"][:n_exp] = 1.0
+        names, ff = [p + "mlp."], f.get("ff")
+        if f["kind"] == "moe":
+            E, ff = f["router"]["experts"], f["expert"]["ff"]
+            router = r(E, d, std=0.02 * s).float()
+            for e in range(E):
+                router[e, e] += 1.0
+            w[p + "mlp.router"] = router.to(dtype)
+            names = [p + f"mlp.e{e}." for e in range(E)]
+        for q in names:
+            w.update({q + "gate": r(ff, d, std=s), q + "up": r(ff, d, std=s), q + "down": r(d, ff, std=ff ** -0.5)})
+    return w
+
+
+def save_model(path, cfg, weights):
+    import json
+    import os
+
+    from safetensors.torch import save_file
+
+    os.makedirs(path, exist_ok=True)
+    with open(os.path.join(path, "config.json"), "w") as fh:
+        json.dump(cfg, fh)
+    save_file({k: v.contiguous() for k, v in weights.items()}, os.path.join(path, "model.safetensors"))
+
+
+def logit_error(got, want):
+    """Per row: RMS over the vocabulary of the difference (its mean taken off), relative to the logits' spread."""
+    d = got.double().cpu() - want
+    d = d - d.mean(-1, keepdim=True)
+    return d.pow(2).mean(-1).sqrt() / want.std()

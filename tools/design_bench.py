@@ -1,7 +1,7 @@
 """Prefill and decode throughput of one model design beside the framework's closest model at equal size
 (bench.py --design; random weights, a few layers of a real model's sizes).
 
-    python bench.py --design kabanex [--design-size s1,s2,s4] [--design-only kabanex|llama]
+    python bench.py --design ripupel|kabanex [--design-size s1,s2,s4] [--design-only ripupel|kabanex|llama]
 
 Per size: prompt tokens/s of one 2048-token prompt, and generated tokens/s of 1 / 16 / 64 sequences decoding
 at ~1.5k tokens of context through the captured step graphs (LM head included, sampling not).  The two
@@ -17,23 +17,31 @@ import torch
 
 VOCAB = 32768
 LAYERS = 8
+CLOSEST = {"ripupel": "kabanex", "kabanex": "llama"}  # the model a design is timed beside
 PROMPT = 2048
 CONTEXT = 1536
 
-# width, heads, kv heads, head size, feed-forward: Kabanex layers and Llama layers of (nearly) equal bytes
+# width, heads, kv heads, head size, feed-forward: layers of (nearly) equal bytes.  Ripupel: ``top`` of ``experts``
+# feed-forwards of size expert_ff in every second layer, together as wide as the dense one
 SIZES = {
-    "s1": dict(hidden=1024, heads=8, kv_heads=4, dim=128, ffn=4096),
-    "s2": dict(hidden=2048, heads=16, kv_heads=4, dim=128, ffn=8192),
-    "s4": dict(hidden=4096, heads=32, kv_heads=8, dim=128, ffn=14336),
+    "s1": dict(hidden=1024, heads=8, kv_heads=4, dim=128, ffn=4096, experts=16, top=4, expert_ff=1024),
+    "s2": dict(hidden=2048, heads=16, kv_heads=4, dim=128, ffn=8192, experts=16, top=4, expert_ff=2048),
+    "s4": dict(hidden=4096, heads=32, kv_heads=8, dim=128, ffn=14336, experts=16, top=4, expert_ff=3584),
 }
 
 
 def build(design: str, size: str, dev):
-    from voice_enabled_browser_automation_amd.models.config import LlamaConfig, kabanex_stack
+    from voice_enabled_browser_automation_amd.models.config import LlamaConfig, kabanex_stack, ripupel_stack
     from voice_enabled_browser_automation_amd.models.kabanex import KabanexModel
     from voice_enabled_browser_automation_amd.models.llama import LlamaModel
+    from voice_enabled_browser_automation_amd.models.ripupel import RipupelModel
 
     s = SIZES[size]
+    if design == "ripupel":
+        return RipupelModel(ripupel_stack(size, vocab=VOCAB, hidden=s["hidden"], n_layers=LAYERS, heads=s["heads"], dim=s["dim"],
+                                          rot_dim=64, vdim=s["dim"], kv_rank=512, width=s["hidden"], blocks=s["hidden"] // 256,
+                                          ffn=s["ffn"], experts=s["experts"], top=s["top"], expert_ff=s["expert_ff"]),
+                            device=dev, seed=1)
     if design == "llama":
         return LlamaModel(LlamaConfig(name=size, vocab_size=VOCAB, hidden=s["hidden"], n_layers=LAYERS, n_heads=s["heads"],
                                       n_kv_heads=s["kv_heads"], head_dim=s["dim"], ffn=s["ffn"]), device=dev, seed=1)
@@ -103,7 +111,7 @@ class Bed:
 def run(args) -> None:
     dev = torch.device("cuda", 0)
     torch.cuda.set_device(dev)
-    designs = [args.design_only] if args.design_only else [args.design, "llama"]
+    designs = [args.design_only] if args.design_only else [args.design, CLOSEST[args.design]]
     res = {"metric": "prefill / decode throughput (tokens/s) of a model design beside the closest model at equal size",
            "unit": "tokens/s", "n_gpus": 1, "dtype": "bf16", "data": "random weights, random tokens", "layers": LAYERS,
            "prompt": PROMPT, "context": CONTEXT, "sizes": {}}
