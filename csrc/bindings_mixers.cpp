@@ -72,7 +72,7 @@ void rglru(Tensor yx, Tensor yb, Tensor xb, Tensor cw, Tensor cb, Tensor gw, Ten
 }
 
 HeadLinearParams lin_params(const Tensor& x, int64_t xs, const Tensor& w, int64_t nb, int64_t N, int64_t K, const Tensor& y,
-                            int64_t ys, int64_t rows) {
+                            int64_t ys, int64_t rows, const OptTensor& row_list = c10::nullopt) {
   const bool f32 = t_is_f32(x, "x");
   TORCH_CHECK(nb >= 1 && N >= 16 && N % 16 == 0 && K >= 32 && K % 32 == 0 && xs >= 0 && ys >= N, "head_linear sizes");
   check_rows(x, rows, (nb - 1) * xs + K, "x");
@@ -81,6 +81,10 @@ HeadLinearParams lin_params(const Tensor& x, int64_t xs, const Tensor& w, int64_
   check_t(y, f32, "y");
   check_rows(y, rows, (nb - 1) * ys + N, "y");
   HeadLinearParams p{};
+  if (row_list.has_value()) {
+    p.row_list = i32p(*row_list, 1, "row_list");
+    rows = row_list->numel();
+  }
   p.x = x.data_ptr();
   p.ldx = (int)x.stride(0);
   p.xs = (int)xs;
@@ -96,9 +100,10 @@ HeadLinearParams lin_params(const Tensor& x, int64_t xs, const Tensor& w, int64_
   return p;
 }
 
-void head_linear(Tensor x, int64_t xs, Tensor w, int64_t nb, int64_t N, int64_t K, Tensor y, int64_t ys) {
+// row_list: the rows of x and y it serves (entries below both tensors' rows)
+void head_linear(Tensor x, int64_t xs, Tensor w, int64_t nb, int64_t N, int64_t K, Tensor y, int64_t ys, OptTensor row_list) {
   c10::DeviceGuard g(x.device());
-  const HeadLinearParams p = lin_params(x, xs, w, nb, N, K, y, ys, y.size(0));
+  const HeadLinearParams p = lin_params(x, xs, w, nb, N, K, y, ys, y.size(0), row_list);
   check_rc(vwa_head_linear(&p, cur_stream(x)), "head_linear");
 }
 
@@ -241,6 +246,81 @@ void latent_out(Tensor part, Tensor stat, int64_t nch, Tensor slots, OptTensor r
   check_rc(vwa_latent_out(&p, cur_stream(out)), "latent_out");
 }
 
+// context rows of segs [n, 3] (block-table row, first key, keys of the run) -> lat [64 n, kp], krot [64 n, rot_p]
+void latent_gather(Tensor cache, Tensor table, Tensor segs, Tensor lat, Tensor krot) {
+  c10::DeviceGuard g(cache.device());
+  LatentPrefillParams p{};
+  for (const Tensor* t : {&cache, &lat, &krot}) {
+    check_bf16(*t, "cache / lat / krot");
+    check_aligned(*t, "cache / lat / krot");
+  }
+  TORCH_CHECK(segs.dim() == 2 && segs.size(1) == 3 && segs.size(0) >= 1, "segs int32 [n, 3]");
+  const int64_t n = segs.size(0), rot_p = krot.size(1);
+  TORCH_CHECK(lat.dim() == 2 && krot.dim() == 2 && lat.is_contiguous() && krot.is_contiguous() && lat.size(0) >= 64 * n && krot.size(0) >= 64 * n,
+              "lat / krot [64 n, ..]");
+  TORCH_CHECK(cache.dim() == 4 && cache.size(1) == 1 && cache.stride(3) == 1 && cache.stride(2) == cache.size(3) &&
+                  cache.size(3) > rot_p && lat.size(1) >= cache.size(3) - rot_p && cache.stride(0) % 8 == 0,
+              "cache [blocks, 1, block_size, rank_p + rot_p]");
+  TORCH_CHECK(table.is_cuda() && table.scalar_type() == at::kInt && table.dim() == 2 && table.stride(1) == 1, "block table int32");
+  p.cache = cache.data_ptr();
+  p.c_sb = cache.stride(0);
+  p.block_table = table.data_ptr<int>();
+  p.table_stride = (int)table.stride(0);
+  p.block_size = (int)cache.size(2);
+  p.segs = i32p(segs, 3 * n, "segs");
+  p.n_segs = (int)n;
+  p.rot_p = (int)rot_p;
+  p.rank_p = (int)(cache.size(3) - rot_p);
+  p.kp = (int)lat.size(1);
+  p.lat = bfp_mut(lat);
+  p.krot = bfp_mut(krot);
+  check_rc(vwa_latent_gather(&p, cur_stream(cache)), "latent_gather");
+}
+
+// tiles [n, 4]: first row, rows, row of its run's key 0 in kv, position of the first row (all inside the tensors)
+void latent_prefill(Tensor y, Tensor q, int64_t H, int64_t dim_p, int64_t q_head, int64_t q_at, Tensor kv, Tensor krot, Tensor tiles,
+                    double scale, Tensor sink, Tensor gate, int64_t vd, Tensor out) {
+  c10::DeviceGuard g(y.device());
+  LatentPrefillParams p{};
+  for (const Tensor* t : {&y, &q, &kv, &krot, &gate, &out}) {
+    check_bf16(*t, "operand");
+    TORCH_CHECK(t->dim() == 2 && t->stride(1) == 1, "operands must be 2-D with contiguous columns");
+  }
+  for (const Tensor* t : {&y, &q, &kv, &krot}) check_aligned(*t, "operand");
+  const int64_t rows = out.size(0), rot_p = krot.size(1), cols = kv.size(1) - H * dim_p;
+  TORCH_CHECK(H >= 1 && cols > 0 && cols % H == 0 && krot.is_contiguous(), "kv [T, H (dim_p + vdk)]");
+  check_rows(y, rows, H * (dim_p + rot_p), "y");
+  check_rows(q, rows, (H - 1) * q_head + q_at + rot_p, "q");
+  check_rows(gate, rows, H * vd, "gate");
+  check_rows(out, rows, H * vd, "out");
+  TORCH_CHECK(((reinterpret_cast<uintptr_t>(gate.data_ptr()) | reinterpret_cast<uintptr_t>(out.data_ptr())) & 7) == 0,
+              "gate / out rows must be 8-byte aligned");
+  TORCH_CHECK(tiles.dim() == 2 && tiles.size(1) == 4 && tiles.size(0) >= 1, "tiles int32 [n, 4]");
+  p.q_tiles = i32p(tiles, tiles.numel(), "tiles");
+  p.n_tiles = (int)tiles.size(0);
+  p.H = (int)H;
+  p.dim_p = (int)dim_p;
+  p.rot_p = (int)rot_p;
+  p.vdk = (int)(cols / H);
+  p.vd = (int)vd;
+  p.scale = (float)scale;
+  p.qn = y.data_ptr();
+  p.ldqn = (int)y.stride(0);
+  p.qr = q.data_ptr();
+  p.ldqr = (int)q.stride(0);
+  p.qr_head = (int)q_head;
+  p.qr_at = (int)q_at;
+  p.kv = kv.data_ptr();
+  p.ldkv = (int)kv.stride(0);
+  p.krot = bfp_mut(krot);
+  p.sink = f32p(sink, H, "sink");
+  p.gate = gate.data_ptr();
+  p.ldg = (int)gate.stride(0);
+  p.out = out.data_ptr();
+  p.ldo = (int)out.stride(0);
+  check_rc(vwa_latent_prefill(&p, cur_stream(y)), "latent_prefill");
+}
+
 void moe_route(Tensor h, Tensor w, int64_t E, int64_t top, Tensor slots, Tensor wts, Tensor ids, int64_t tile, Tensor tiles,
                Tensor order, Tensor ticket) {
   c10::DeviceGuard g(h.device());
@@ -300,6 +380,11 @@ void moe_gemm(Tensor x, Tensor w, int64_t rows, int64_t top, bool down, Tensor w
   p.tiles = i32p(tiles, 4, "tiles");
   p.order = i32p(order, places, "order");
   p.tile = (int)tile;
+  p.x_rows = (int)(down ? places : rows);
+  if (tile == 128) {
+    check_aligned(y, "y");
+    TORCH_CHECK(y.stride(0) % 8 == 0, "y rows must be 16-byte aligned");
+  }
   p.y = y.data_ptr();
   p.ldy = (int)y.stride(0);
   check_rc(vwa_moe_gemm(&p, cur_stream(x)), "moe_gemm");
@@ -311,11 +396,15 @@ void bind_mixers(py::module_& m) {
   m.def("rglru", &rglru, py::arg("yx"), py::arg("yb"), py::arg("xb"), py::arg("cw"), py::arg("cb"), py::arg("gw"), py::arg("rb"),
         py::arg("ib"), py::arg("decay"), py::arg("nb"), py::arg("seq_ids"), py::arg("positions"), py::arg("slots"), py::arg("state"),
         py::arg("out"), py::arg("chunks") = py::none(), py::arg("scratch") = py::none());
-  m.def("head_linear", &head_linear);
+  m.def("head_linear", &head_linear, py::arg("x"), py::arg("xs"), py::arg("w"), py::arg("nb"), py::arg("N"), py::arg("K"), py::arg("y"),
+        py::arg("ys"), py::arg("row_list") = py::none());
   m.def("latent_rows", &latent_rows);
   m.def("latent_qkv", &latent_qkv);
   m.def("latent_attention", &latent_attention);
   m.def("latent_out", &latent_out);
+  m.def("latent_prefill_fits", [](int64_t dim_p, int64_t rot_p, int64_t vdk) { return vwa_latent_prefill_fits((int)dim_p, (int)rot_p, (int)vdk) != 0; });
+  m.def("latent_gather", &latent_gather);
+  m.def("latent_prefill", &latent_prefill);
   m.def("moe_route", &moe_route);
   m.def("moe_gemm", &moe_gemm);
 }

@@ -34,6 +34,10 @@
 //   5 QKV (rotary + paged KV write)   6 split: the first n_split columns stored, relu^2 of the others
 //   to a second matrix (one projection feeding a layer's mixers and its feed-forward)
 //
+// Grouped launches (routed experts, GemmParams::g_*): a row block is a tile of (row, expert) pairs of one
+// expert; its X rows are gathered (or taken in place order) by the LDS-DMA's per-lane addresses, W is the
+// expert's, and the per-row scale is the pair's score.
+//
 // Implicit-GEMM convolution (K3, ops.conv1d_gelu): X rows are ldx apart and K long, so a k=3
 // conv over a zero-padded channels-last buffer is X row t = padded rows t*stride .. t*stride+2
 // (ldx = stride*Cin, K = 3*Cin) -- the A tiles are staged through the same LDS-DMA pipeline.
@@ -108,9 +112,10 @@ VWA_DEVICE void dma16(__amdgpu_buffer_rsrc_t r, char* lds_wave_base, unsigned vo
 // above) and B the fp8 tiled k-group of every tile verbatim ([tile][s2][lane][16 B]: block s2 = h
 // holds the lane's k 32 g + 16 h .. + 16, both sub-steps of half h), converted to bf16 fragments on
 // the LDS read -- no quantised copy of X, half the weight bytes of bf16.
-template <class C, bool WT, bool F8, bool W8 = false>
+// rows (grouped launches): X rows of this thread's pieces (< 0: none)
+template <class C, bool WT, bool F8, bool W8 = false, bool GRP = false>
 VWA_DEVICE void issue_stage(const GemmParams& p, __amdgpu_buffer_rsrc_t rx, __amdgpu_buffer_rsrc_t rw, int bm,
-                            int bn, int hs, char* buf) {
+                            int bn, int hs, char* buf, const int (&rows)[C::BM / 8 / C::NW]) {
   const int w = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int kg = F8 || W8 ? hs : hs >> 1;
 #pragma unroll
@@ -120,13 +125,13 @@ VWA_DEVICE void issue_stage(const GemmParams& p, __amdgpu_buffer_rsrc_t rx, __am
   for (int it = 0; it < C::BM / 8 / C::NW; ++it) {
     const int q = it * C::NW + w;  // wave-instruction index: rows 8q .. 8q + 7
     const int r = 8 * q + (lane >> 3), c = (lane & 7) ^ swz((r >> 1) & 7);
-    const int m = bm + r;
+    const int m = GRP ? rows[it] : bm + r;
     unsigned off;
     if constexpr (F8)
       off = (unsigned)((size_t)m * p.ldx + (size_t)kg * BKG + 32 * (c >> 1) + 16 * (c & 1));
     else
       off = (unsigned)(((size_t)m * p.ldx + (size_t)kg * BKG + 32 * (c >> 1) + 16 * ha + 8 * (c & 1)) * 2);
-    dma16(rx, buf + hh * C::A_BYTES + q * 1024, m < p.M ? off : 0xFFFFFFF0u);
+    dma16(rx, buf + hh * C::A_BYTES + q * 1024, (GRP ? m >= 0 : m < p.M) ? off : 0xFFFFFFF0u);
   }
   }
   const int kgn = p.K / BKG;
@@ -516,11 +521,12 @@ VWA_DEVICE float reduce_item(const GemmParams& p, __amdgpu_buffer_rsrc_t rws, in
 // (round 4's 4-stage variant for one-row-block GEMMs measured slower in whole decode steps -- 128 KB
 // of LDS leaves one workgroup per CU, so split-K grids above 256 workgroups ran in two rounds:
 // fp8 32 rows 4.97 vs 4.36 ms, profiles/r4_gemm_ab.md -- and was removed in round 5)
-template <class C, int EPI, bool WT, bool F8 = false, bool P8 = false, bool W8 = false>
+template <class C, int EPI, bool WT, bool F8 = false, bool P8 = false, bool W8 = false, bool GRP = false>
 __global__ __launch_bounds__(C::THREADS, C::NW == 4 ? 2 : 1) void gemm_kernel(GemmParams p) {
   extern __shared__ __attribute__((aligned(16))) char lds[];
   constexpr int FM = C::FM, FN = C::FN;
-  const int mb = (p.M + C::BM - 1) / C::BM, nb = (p.N + C::BN - 1) / C::BN;
+  static_assert(!GRP || (C::BM == 128 && WT && !F8 && !P8 && !W8 && (EPI == EPI_SWIGLU || EPI == EPI_STORE)), "grouped: bf16 128-row tiles");
+  const int mb = GRP ? p.g_max : (p.M + C::BM - 1) / C::BM, nb = (p.N + C::BN - 1) / C::BN;
   const int tiles = mb * nb;
   const int split = blockIdx.x / tiles % p.splits;  // split-K slice (blocks of one slice are contiguous)
   if (p.nbatch > 1) {  // batch z = blockIdx.x / (tiles * splits), splits == 1 (vwa_gemm)
@@ -534,7 +540,24 @@ __global__ __launch_bounds__(C::THREADS, C::NW == 4 ? 2 : 1) void gemm_kernel(Ge
   if (p.ss_zero && blockIdx.x == 0)
     for (int i = threadIdx.x; i < p.ss_zero_n; i += C::THREADS) p.ss_zero[i] = 0ull;
   const int lt = xcd_remap((int)(blockIdx.x % tiles), tiles);
-  const int bn = (lt / mb) * C::BN, bm = (lt % mb) * C::BM;
+  const int bn = (lt / mb) * C::BN;
+  int bm = (lt % mb) * C::BM, place = 0;
+  int rows[C::BM / 8 / C::NW];
+  size_t x_rows = 0;
+  if constexpr (GRP) {
+    const int gt = lt % mb;
+    if (gt >= p.g_tiles[0]) return;
+    p.W += (size_t)p.g_tiles[1 + 3 * gt] * p.g_wstride;
+    place = p.g_tiles[2 + 3 * gt];
+    x_rows = (size_t)p.M;                            // (X rows the buffer holds)
+    p.M = p.g_tiles[3 + 3 * gt];
+    bm = 0;
+#pragma unroll
+    for (int it = 0; it < C::BM / 8 / C::NW; ++it) {
+      const int r = 8 * (it * C::NW + (threadIdx.x >> 6)) + ((threadIdx.x & 63) >> 3);
+      rows[it] = r < p.M ? (p.g_down ? place + r : p.g_order[place + r] / p.g_top) : -1;
+    }
+  }
   const int KG = p.K / BKG;
   const int kg0 = split * p.kg_per_split, kg1 = min(KG, kg0 + p.kg_per_split);
   const int w = threadIdx.x >> 6, wm = w / C::WN, wn = w % C::WN;
@@ -551,7 +574,7 @@ __global__ __launch_bounds__(C::THREADS, C::NW == 4 ? 2 : 1) void gemm_kernel(Ge
                 "8 LDS-DMA instructions per thread per stage (the counted vmcnt)");
   const int h0 = SPG * kg0, nh = SPG * (kg1 - kg0);
   // X extent: the last row starts at (M-1)*ldx and is K long (rows may overlap: conv views)
-  const __amdgpu_buffer_rsrc_t rx = rsrc(p.X, ((size_t)(p.M - 1) * p.ldx + p.K) * (F8 ? 1 : 2));
+  const __amdgpu_buffer_rsrc_t rx = rsrc(p.X, ((GRP ? x_rows - 1 : (size_t)(p.M - 1)) * p.ldx + p.K) * (F8 ? 1 : 2));
   const __amdgpu_buffer_rsrc_t rw = rsrc(p.W, (size_t)p.N * p.K * (F8 || W8 ? 1 : 2));
   if constexpr (P8) {
     static_assert(C::BM == 256 && C::BN == 256 && C::NW == 8 && WT && !F8, "8-phase pipeline: CfgP8, tiled bf16");
@@ -629,8 +652,8 @@ __global__ __launch_bounds__(C::THREADS, C::NW == 4 ? 2 : 1) void gemm_kernel(Ge
     }
     if (wm == 0) asm volatile("s_barrier" ::: "memory");  // (group 1 started one barrier later)
   } else {
-  if (nh > 0) issue_stage<C, WT, F8, W8>(p, rx, rw, bm, bn, h0, lds);
-  if (nh > 1) issue_stage<C, WT, F8, W8>(p, rx, rw, bm, bn, h0 + 1, lds + STG);
+  if (nh > 0) issue_stage<C, WT, F8, W8, GRP>(p, rx, rw, bm, bn, h0, lds, rows);
+  if (nh > 1) issue_stage<C, WT, F8, W8, GRP>(p, rx, rw, bm, bn, h0 + 1, lds + STG, rows);
   for (int i = 0; i < nh; ++i) {
     if (i + 1 < nh)
       asm volatile("s_waitcnt vmcnt(8)\n\ts_barrier" ::: "memory");  // this stage landed everywhere
@@ -638,7 +661,7 @@ __global__ __launch_bounds__(C::THREADS, C::NW == 4 ? 2 : 1) void gemm_kernel(Ge
       asm volatile("s_waitcnt vmcnt(0)\n\ts_barrier" ::: "memory");
     compute_stage<C, F8, W8>(lds + (i & 1) * STG, acc, wm, wn);
     asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");  // every wave done reading it
-    if (i + 2 < nh) issue_stage<C, WT, F8, W8>(p, rx, rw, bm, bn, h0 + i + 2, lds + (i & 1) * STG);
+    if (i + 2 < nh) issue_stage<C, WT, F8, W8, GRP>(p, rx, rw, bm, bn, h0 + i + 2, lds + (i & 1) * STG, rows);
   }
   }
   const int l = lane_id();
@@ -679,7 +702,8 @@ __global__ __launch_bounds__(C::THREADS, C::NW == 4 ? 2 : 1) void gemm_kernel(Ge
 #pragma unroll
     for (int i = 0; i < FM; ++i)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) rsv[i][r] = row0 + i * 16 + r < p.M ? row_scale(p, row0 + i * 16 + r) : 1.f;
+      for (int r = 0; r < 4; ++r)
+        rsv[i][r] = row0 + i * 16 + r < p.M ? row_scale(p, GRP ? p.g_order[place + row0 + i * 16 + r] : row0 + i * 16 + r) : 1.f;
   }
   // W8A8: acc * sx[m] * sw[n] (SwiGLU: gate / up columns scale before the activation); W8A16: sw only
   if constexpr (F8 || W8) {
@@ -773,7 +797,7 @@ __global__ __launch_bounds__(C::THREADS, C::NW == 4 ? 2 : 1) void gemm_kernel(Ge
     if (EPI == EPI_SPLIT && n >= p.n_split)
       *reinterpret_cast<uint4*>(p.Y2 + (size_t)m * p.ldy2 + n - p.n_split) = v;
     else
-      *reinterpret_cast<uint4*>(reinterpret_cast<u16*>(p.Y) + (size_t)m * p.ldy + n) = v;
+      *reinterpret_cast<uint4*>(reinterpret_cast<u16*>(p.Y) + (size_t)(GRP ? (p.g_down ? p.g_order[place + m] : place + m) : m) * p.ldy + n) = v;
   }
   if (kResid<EPI> && p.ss_out) {  // one atomic per (row, wave): the CPR lanes of a row reduce first
 #pragma unroll
@@ -931,6 +955,28 @@ extern "C" int vwa_gemm(int epi, const GemmParams* pp, hipStream_t st) {
     case EPI_SPLIT: return launch_epi<EPI_SPLIT>(p, st, p8);
     default: return -3;
   }
+}
+
+extern "C" int vwa_gemm_grouped(int epi, const GemmParams* pp, hipStream_t st) {
+  GemmParams p = *pp;
+  if (p.M < 1 || p.N % 16 || p.N < 16 || p.K < BKG || p.K % BKG || p.ldx % 8 || p.ldy % 8 || p.y_f32 || p.bias || p.R || p.sw || p.sx ||
+      p.ss_in || p.ss_out || p.ss_zero || !p.w_tiled || p.nbatch > 1 || !p.g_tiles || !p.g_order || p.g_max < 1 || p.g_top < 1)
+    return -10;
+  if ((reinterpret_cast<uintptr_t>(p.X) | reinterpret_cast<uintptr_t>(p.W) | reinterpret_cast<uintptr_t>(p.Y)) & 15) return -11;
+  if (epi == EPI_SWIGLU && (p.N % 32 || !p.rstd)) return -12;
+  if ((int64_t)p.M * p.ldx * 2 >= 0x7FFFFFF0ll || (int64_t)p.N * p.K * 2 >= 0x7FFFFFF0ll) return -13;  // (32-bit offsets)
+  p.splits = 1;
+  p.nbatch = 1;
+  p.kg_per_split = p.K / BKG;
+  using C = CfgS;
+  const dim3 grid(p.g_max * ((p.N + C::BN - 1) / C::BN)), block(C::THREADS);
+  const int lds = 2 * C::STAGE > C::LDS ? 2 * C::STAGE : C::LDS;
+  switch (epi) {
+    case EPI_SWIGLU: hipLaunchKernelGGL((gemm_kernel<C, EPI_SWIGLU, true, false, false, false, true>), grid, block, lds, st, p); break;
+    case EPI_STORE: hipLaunchKernelGGL((gemm_kernel<C, EPI_STORE, true, false, false, false, true>), grid, block, lds, st, p); break;
+    default: return -3;
+  }
+  return (int)hipGetLastError();
 }
 
 extern "C" int vwa_row_rstd(const uint16_t* x, int ldx, int M, int K, float eps, float* rstd, hipStream_t st) {

@@ -29,10 +29,11 @@ VWA_DEVICE void head_linear_wg(const HeadLinearParams& p, int b, int cg, int r0)
   const int lane = lane_id(), w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), rl = lane & 15, g = lane >> 4;
   const int nt = p.N >> 4, t0 = (cg * 4 + w) * kHlTiles, steps = p.K / M::KS;
   if (t0 >= nt) return;
+  auto row_of = [&](int r) { return p.row_list ? p.row_list[r] : r; };
   const T* xp[NT];
 #pragma unroll
   for (int t = 0; t < NT; ++t)
-    xp[t] = reinterpret_cast<const T*>(p.x) + (size_t)min(r0 + 16 * t + rl, p.rows - 1) * p.ldx + (size_t)b * p.xs + g * M::EPL;
+    xp[t] = reinterpret_cast<const T*>(p.x) + (size_t)row_of(min(r0 + 16 * t + rl, p.rows - 1)) * p.ldx + (size_t)b * p.xs + g * M::EPL;
   const uint4* wp[kHlTiles];
 #pragma unroll
   for (int j = 0; j < kHlTiles; ++j)
@@ -60,9 +61,7 @@ VWA_DEVICE void head_linear_wg(const HeadLinearParams& p, int b, int cg, int r0)
       for (int j = 0; j < kHlTiles; ++j) {
         if (t0 + j >= nt) continue;
         const int c = b * p.ys + (t0 + j) * 16 + rl;
-        float v = acc[t][j][i];
-        if (p.gate) v *= sigm(ldv(reinterpret_cast<const T*>(p.gate) + (size_t)r * p.ldg + c));
-        stv(reinterpret_cast<T*>(p.y) + (size_t)r * p.ldy + c, v);
+        stv(reinterpret_cast<T*>(p.y) + (size_t)row_of(r) * p.ldy + c, acc[t][j][i]);
       }
     }
 }

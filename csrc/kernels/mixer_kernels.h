@@ -32,13 +32,12 @@ struct RgLruParams {
 };
 
 // y[m][b * ys ..] = W_b . x[m][b * xs ..] for every head / block b (K inputs, N outputs)
-// gate: y *= sigmoid(gate[m][same column])
 struct HeadLinearParams {
+  const int* row_list;              // rows of x and y this launch serves (null: 0 .. rows - 1)
   const void* x; int ldx; int xs;
   const void* w;                    // T fragment order per block [nb][N / 16][K steps][64][EPL]
   int nb, N, K, rows, f32;
   void* y; int ldy; int ys;
-  const void* gate; int ldg;        // (null: none)
 };
 
 // Row part of latent attention: rotation of the heads' rotated query parts, norm of the latent, rotation
@@ -82,6 +81,26 @@ struct LatentOutParams {
   void* out; int ldo;
 };
 
+// Latent attention of prompt-sized runs (bf16) over expanded keys and values (latent_prefill.hip).
+// gather: segs [n_segs][3] = block-table row, first key, keys of its run -- 64 rows of lat / krot each;
+// prefill: q_tiles [n_tiles][4] = first row, rows (<= 128), row of the run's key 0 in kv / krot, position of the
+// first row.  kv rows: [keys H x dim_p | values H x vdk]; runs' contexts are padded to 64 rows.
+struct LatentPrefillParams {
+  const void* cache; int64_t c_sb; const int* block_table; int table_stride, block_size;
+  const int* segs; int n_segs;
+  int rank_p, rot_p, kp;
+  uint16_t* lat; uint16_t* krot;    // [64 n_segs][kp], [64 n_segs][rot_p]
+  const int* q_tiles; int n_tiles;
+  int H, dim_p, vdk, vd;            // value columns in kv (a multiple of 32) and in out / gate
+  float scale;
+  const void* qn; int ldqn;         // projected rows, head h at h * (dim_p + rot_p)
+  const void* qr; int ldqr; int qr_head, qr_at;   // rotated parts
+  const void* kv; int ldkv;
+  const float* sink;
+  const void* gate; int ldg;
+  void* out; int ldo;
+};
+
 // Routed experts.  A pair is (row, k): row's k-th choice, pair id = row * top + k.
 struct MoeRouteParams {
   const void* h; int ldh; int K;    // [rows, K] T (K a multiple of the fragment step)
@@ -102,7 +121,8 @@ struct MoeGemmParams {
   const void* w; int64_t w_expert;  // elements per expert; pre-tiled order (ops.mixers.tile_weight)
   int N, K, top, f32, down;         // N: rows of one expert's matrix (gate / up interleaved by 16: 2 x ff)
   const float* wts;
-  const int* tiles; const int* order; int max_tiles, tile;
+  const int* tiles; const int* order; int max_tiles, tile;   // tile: 16, or 128 (bf16: the LDS-tiled GEMM)
+  int x_rows;                       // rows of x
   void* y; int ldy;
 };
 
@@ -117,6 +137,9 @@ int vwa_latent_rows(const LatentRowsParams* p, hipStream_t st);
 int vwa_latent_qkv(const LatentRowsParams* p, const HeadLinearParams* q, hipStream_t st);
 int vwa_latent_attention(const LatentAttnParams* p, hipStream_t st);
 int vwa_latent_out(const LatentOutParams* p, hipStream_t st);
+int vwa_latent_prefill_fits(int dim_p, int rot_p, int vdk);
+int vwa_latent_gather(const LatentPrefillParams* p, hipStream_t st);
+int vwa_latent_prefill(const LatentPrefillParams* p, hipStream_t st);
 int vwa_moe_route(const MoeRouteParams* p, hipStream_t st);
 int vwa_moe_gemm(const MoeGemmParams* p, hipStream_t st);
 // x (f32 rows) += norm(sum of the row's n_parts branch rows) * w1; h (T) = norm(x) * w2 (w2 null: no h)

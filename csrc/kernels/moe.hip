@@ -2,12 +2,14 @@
 //
 //  moe_route : sigmoid router scores (MFMA, f32 sums), the best ``top`` experts of every row, and the pairs
 //              (row, choice) grouped by expert into tiles of at most ``tile`` pairs -- by the last workgroup
-//  moe_gemm  : the experts' matrices over such a tile.  First launch: the tile's rows times gate and up, scaled
+//  moe_gemm  : the experts' matrices over such a tile (here tiles of 16 pairs, streaming; tiles of 128 go to
+//              gemm.hip's grouped launch).  First launch: the tile's rows times gate and up, scaled
 //              by the pair's score ahead of the activation (w (W h) = W (w h)); second: down, one row per pair.
 //              (The pairs of a row are added, in the order of its choices, by add_norm.)
 // A row's results do not depend on the tile it lands in, so the order inside an expert is free.
 #include "mixer_kernels.h"
 #include "stack_types.h"
+#include "vwa_kernels.h"
 
 using namespace vwa;
 
@@ -200,10 +202,31 @@ extern "C" int vwa_moe_route(const MoeRouteParams* p, hipStream_t st) {
 }
 
 extern "C" int vwa_moe_gemm(const MoeGemmParams* p, hipStream_t st) {
-  if (p->max_tiles < 1 || p->N % (p->down ? 16 : 32) || p->K % 128 || p->ldx % 8 || p->tile != 16 || !p->tiles || !p->order ||
+  if (p->max_tiles < 1 || p->N % (p->down ? 16 : 32) || p->K % 128 || p->ldx % 8 || (p->tile != 16 && p->tile != 128) || !p->tiles || !p->order ||
       (!p->down && !p->wts))
     return -1;
   if ((reinterpret_cast<uintptr_t>(p->x) | reinterpret_cast<uintptr_t>(p->w)) & 15) return -2;
+  if (p->tile == 128) {
+    if (p->f32) return -3;
+    GemmParams q{};
+    q.X = reinterpret_cast<const uint16_t*>(p->x);
+    q.ldx = p->ldx;
+    q.W = reinterpret_cast<const uint16_t*>(p->w);
+    q.w_tiled = 1;
+    q.M = p->x_rows;
+    q.N = p->N;
+    q.K = p->K;
+    q.Y = p->y;
+    q.ldy = p->ldy;
+    q.rstd = p->down ? nullptr : p->wts;
+    q.g_tiles = p->tiles;
+    q.g_order = p->order;
+    q.g_max = p->max_tiles;
+    q.g_top = p->top;
+    q.g_down = p->down;
+    q.g_wstride = p->w_expert;
+    return vwa_gemm_grouped(p->down ? 0 : 2, &q, st);
+  }
   const dim3 grid(p->N / (p->down ? 16 : 32), p->max_tiles), block(256);
   if (p->f32) {
     if (p->down) hipLaunchKernelGGL((moe_gemm16_kernel<float, true>), grid, block, 0, st, *p);

@@ -189,6 +189,11 @@ struct GemmParams {
   // epilogue 6 (split, bf16): columns n < n_split (a multiple of 16) go to Y, the others as relu(v)^2
   // to Y2[m][n - n_split] -- one projection of a normed row feeding the mixers and the feed-forward
   int n_split; uint16_t* Y2; int ldy2;
+  // grouped launch (tiles != null; vwa_gemm_grouped): every 128-row block is one tile of (row, expert) pairs
+  // of one expert -- tiles [1 + 3 g_max] int32: count, then (expert, first place, pairs); order: place -> pair.
+  // X row of a place: pair / top (g_down: the place itself); Y row: the place (g_down: the pair); rstd: per
+  // PAIR; W + expert * g_wstride
+  const int* g_tiles; const int* g_order; int g_max, g_top, g_down; int64_t g_wstride;
 };
 
 struct FlashAttnParams {
@@ -263,6 +268,8 @@ int vwa_chain_launch(const ChainParams* d_cp, int seq, int n_phases, int attn_g,
 // -10: a shape / role table the kernel does not take (the caller keeps per-kernel launches)
 int vwa_wdec_launch(const WdecParams* p, int grid, hipStream_t st);
 int vwa_gemm(int epi, const GemmParams* p, hipStream_t st);
+// routed experts' products over 128-pair tiles (GemmParams::g_*): epi 2 SwiGLU, 0 store
+int vwa_gemm_grouped(int epi, const GemmParams* p, hipStream_t st);
 int vwa_gemm_splits(int M, int N, int K, int cus, int64_t ws_floats, int f8);
 void vwa_gemm_set_split_fill(int pct);  // split-K while tiles x splits < pct % of the CUs (0: bf16 75, fp8 100)
 void vwa_gemm_set_p8(int mode);  // 0: 128^2 kernel only, 1: 256^2 8-phase wherever eligible, 2: measured rule

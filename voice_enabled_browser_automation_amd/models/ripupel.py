@@ -13,6 +13,8 @@ Launches of a decode step (T activations, f32 residual, branch outputs T):
     latent attention  input projection [q | latent | key part | gate] -> queries into latent space, rotation,
                       latent norm, cache write -> attention over the cached latents -> merge with the sinks,
                       value projection, gate -> output projection
+                      (prompt-sized runs instead expand their context's keys and values once: gather -> GEMM ->
+                      flash attention with sinks and gate)
     dense ff          gate / up with SwiGLU in the epilogue -> down
     routed experts    router + grouping -> gate / up of the chosen experts -> down, a row per (token, expert)
 
@@ -31,7 +33,7 @@ from typing import Dict, List, Optional, Sequence, Tuple
 import torch
 
 from .. import ops
-from ..ops.mixers import SCAN_ROWS, LatentScratch, LatentWeights, MoeWeights, RgLruWeights
+from ..ops.mixers import SCAN_ROWS, LatentScratch, LatentWeights, MoeWeights, RgLruWeights, plan_latent
 from ..parallel.tp import TPContext
 from ..runtime.kv_cache import CacheLayer
 from .config import DenseFFConfig, LatentAttentionConfig, MoEConfig, RgLruConfig, RipupelConfig
@@ -166,7 +168,7 @@ class RipupelModel:
             if isinstance(D, RgLruDims):
                 mixer = self._build_rglru(L.mixer, D, m, mat, vec, zeros, w_in, w_out, gpu)
             else:
-                mixer = self._build_latent(L.mixer, D, m, mat, vec, zeros, w_in, w_out, frag)
+                mixer = self._build_latent(L.mixer, D, m, mat, vec, zeros, w_in, w_out, frag, tiled)
             lw = RipupelLayerWeights(norm1=vec(p + "norm1", d), norm1b=vec(p + "norm1b", d), norm2=None, norm2b=None,
                                      w_in=place(w_in), w_out=place(w_out), mixer=mixer)
             if L.mlp is not None:
@@ -218,7 +220,8 @@ class RipupelModel:
                             gates=ops.gate_fragments(gates) if gpu else gates, rb=chan(vec(m + "ra.b", nb, k).view(-1)),
                             ib=chan(vec(m + "ri.b", nb, k).view(-1)), decay=chan(decay))
 
-    def _build_latent(self, c: LatentAttentionConfig, D: LatentDims, m: str, mat, vec, zeros, w_in, w_out, frag) -> LatentWeights:
+    def _build_latent(self, c: LatentAttentionConfig, D: LatentDims, m: str, mat, vec, zeros, w_in, w_out, frag,
+                      tiled: bool) -> LatentWeights:
         d, H, hq = self.cfg.hidden, c.heads, c.dim + c.rot_dim
         kv_at, g_at = D.at
         q = mat(m + "q", H * hq, d).view(H, hq, d)
@@ -233,9 +236,16 @@ class RipupelModel:
         uk, uv = zeros(H, D.rank, D.dim), zeros(H, D.vd, D.rank)
         uk[:, : c.kv_rank, : c.dim] = mat(m + "uk", H * c.dim, c.kv_rank).view(H, c.dim, c.kv_rank).transpose(1, 2)
         uv[:, : c.vdim, : c.kv_rank] = mat(m + "uv", H * c.vdim, c.kv_rank).view(H, c.vdim, c.kv_rank)
+        w_kv = None
+        if tiled:  # the same projections for prompts: keys of all heads, then values (32-column heads)
+            vdk = _up(D.vd, 32)
+            w_kv = zeros(_columns(H * (D.dim + vdk)), _up(D.rank, 128))
+            w_kv[: H * D.dim, : D.rank].view(H, D.dim, D.rank).copy_(uk.transpose(1, 2))
+            w_kv[H * D.dim : H * (D.dim + vdk), : D.rank].view(H, vdk, D.rank)[:, : D.vd] = uv
+            w_kv = ops.TiledWeight(w_kv)
         return LatentWeights(H=H, dim_p=D.dim, rot_p=D.rot, rank_p=D.rank, vd=D.vd, scale=c.scale, eps=self.cfg.norm_eps,
                              norm=vec(m + "dkv.norm", c.kv_rank) if D.own else None, sink=vec(m + "sink", H), uk=frag(uk),
-                             uv=frag(uv))
+                             uv=frag(uv), w_kv=w_kv)
 
     def weight_bytes(self) -> int:
         ts = [self.lm_head]
@@ -298,7 +308,7 @@ class RipupelModel:
         return b
 
     def plan_rows(self, runs: Sequence[Tuple[int, int, int, int]], max_pos: int) -> SimpleNamespace:
-        return ops.plan_runs(runs, self.device, max_pos, scan_rows=SCAN_ROWS)
+        return plan_latent(runs, self.device, ops.plan_runs(runs, self.device, max_pos, scan_rows=SCAN_ROWS))
 
     # ------------------------------------------------------------------ forward
     def forward(self, bufs, M: int, kv, *, n_sel: Optional[int] = None, head: bool = True) -> torch.Tensor:
@@ -324,7 +334,7 @@ class RipupelModel:
         if isinstance(D, RgLruDims):
             ops.rglru(y, L.mixer, state=kv.state[li], out=cat[:, : D.cols], plan=plan, **rows)
         else:
-            self._attend(li, y, cat[:, : D.cols], bufs, M, kv, rows)
+            self._attend(li, y, cat[:, : D.cols], bufs, M, kv, rows, plan)
         ops.linear(cat, L.w_out, out=br[:M])
         after = self.layers[li + 1].norm1 if li + 1 < self.cfg.n_layers else None
         if C.mlp is None:
@@ -341,13 +351,13 @@ class RipupelModel:
             ops.linear(act, L.down, out=br[:M])
         ops.add_norm(x, br[: M * parts], L.norm2b, after, eps=eps, out=h, n_parts=parts)
 
-    def _attend(self, li: int, y, out, bufs, M: int, kv, rows) -> None:
+    def _attend(self, li: int, y, out, bufs, M: int, kv, rows, plan) -> None:
         a, D, w = self.cfg.layers[li].mixer, self.dims[li], self.layers[li].mixer
         g = D.at[1]
         q = ops.latent_qkv(y, w, rope=self.ropes[(a.rot_base, a.rot_dim)], positions=rows["positions"], slots=rows["slots"],
-                           q_out=bufs.q[: M * D.H * D.dk].view(M, D.H * D.dk), cache=kv.k[li] if D.own else None)
+                           q_out=bufs.q[: M * D.H * D.dk].view(M, D.H * D.dk), cache=kv.k[li] if D.own else None, plan=plan)
         ops.latent_attention(q, w, cache=kv.k[li], block_table=bufs.block_table, gate=y[:, g : g + D.cols], max_ctx=bufs.max_ctx,
-                             scratch=bufs.latent, out=out, **rows)
+                             scratch=bufs.latent, out=out, y=y, plan=plan, **rows)
 
     def lm_logits(self, bufs, hs: torch.Tensor, col_mask: Optional[torch.Tensor] = None, mask_rows: int = 1,
                   gather: bool = True) -> torch.Tensor:

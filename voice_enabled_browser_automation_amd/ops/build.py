@@ -86,7 +86,7 @@ def _run(cmd: list[str]) -> None:
 
 
 # kernel files the core library holds; launchers of the others are stubs there
-CORE = ("gemm", "gemm_f32", "skinny_stream", "elementwise", "stack_ops", "talk_attention", "recurrence", "rglru", "latent", "moe",
+CORE = ("gemm", "gemm_f32", "skinny_stream", "elementwise", "stack_ops", "talk_attention", "recurrence", "rglru", "latent", "latent_prefill", "moe",
         "sample")
 
 

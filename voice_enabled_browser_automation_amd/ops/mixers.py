@@ -23,7 +23,9 @@ from .stack import ROW_SLICE, _ext
 SCAN_ROWS = 128     # rows per chunk of the recurrence scan
 ATTN_KEYS = 64      # keys per round of the latent attention
 ATTN_GROUPS = 512   # workgroups a latent attention launch is cut into
-MOE_TILE = 16       # pairs per tile of the experts' products
+EXPAND_ROWS = 32    # runs of fewer rows attend in latent space ...
+EXPAND_CONTEXT = 128  # ... and so do runs behind more than this many tokens of context per row
+MOE_TILES = (16, 128)  # pairs per tile of the experts' products: streaming kernel, LDS-tiled GEMM
 
 
 # ----------------------------------------------------------------------------- weight layouts
@@ -98,6 +100,12 @@ class LatentWeights:
     sink: torch.Tensor             # f32 [H]
     uk: torch.Tensor
     uv: torch.Tensor
+    w_kv: object = None            # prompts: the keys' and values' projections [H (dim_p + vdk), rank to 128] (TiledWeight)
+
+    @property
+    def vdk(self) -> int:
+        """Value columns of a head in the expanded rows."""
+        return -(-self.vd // 32) * 32
 
 
 def latent_chunks(rows: int, H: int, max_ctx: int) -> int:
@@ -119,33 +127,91 @@ class LatentScratch:
         self.stat = torch.zeros(stat, dtype=torch.float32, device=device)
 
 
+def plan_latent(runs: Sequence[Tuple[int, int, int, int]], device, plan: SimpleNamespace) -> SimpleNamespace:
+    """Attention tables of a ragged step, added to ``plan``.  runs: (first row, rows, block-table row, first
+    position).  Runs worth expanding their context go to the prefill form: q_tiles (the longest contexts
+    first) and segs (64 context rows each, one run after the other); short: the rows of the others."""
+    tiles, segs, short = [], [], []
+    for r0, n, sid, pos in runs:
+        ctx = pos + n
+        if n < EXPAND_ROWS or ctx > EXPAND_CONTEXT * n:
+            short += range(r0, r0 + n)
+            continue
+        t0 = 64 * len(segs)
+        segs += [[sid, k, ctx] for k in range(0, ctx, 64)]
+        tiles += [[r0 + i, min(128, n - i), t0, pos + i] for i in range(0, n, 128)]
+    tiles.sort(key=lambda t: -t[3])
+    cuda = torch.device(device).type == "cuda"
+
+    def dev(x, *shape):
+        if not x:
+            return None
+        t = torch.tensor(x, dtype=torch.int32).view(*shape)
+        return t.pin_memory().to(device, non_blocking=True) if cuda else t
+
+    plan.q_tiles, plan.segs, plan.short = dev(tiles, -1, 4), dev(segs, -1, 3), dev(short, -1)
+    return plan
+
+
+def _expands(w: LatentWeights, y: torch.Tensor, plan) -> bool:
+    """This step's long runs take the prefill form."""
+    return (plan is not None and plan.q_tiles is not None and w.w_kv is not None and y.dtype == torch.bfloat16
+            and _ext().latent_prefill_fits(w.dim_p, w.rot_p, w.vdk))
+
+
 def latent_qkv(y: torch.Tensor, w: LatentWeights, *, rope: torch.Tensor, positions: torch.Tensor, slots: torch.Tensor,
-               q_out: torch.Tensor, cache: Optional[torch.Tensor]) -> torch.Tensor:
+               q_out: torch.Tensor, cache: Optional[torch.Tensor], plan: Optional[SimpleNamespace] = None) -> torch.Tensor:
     """Projected rows [q | latent | key part | ..]: the queries in latent space, rotated parts behind them
     (q_out [rows, H (rank_p + rot_p)]); latent normed, key part rotated, both to the cache (slot < 0: not
-    written; ``cache`` None: the layer reads another layer's)."""
+    written; ``cache`` None: the layer reads another layer's).  Rows of the prefill form get their rotated
+    parts only."""
     if not y.is_cuda:
         return ref.latent_qkv(y, w, rope=rope, positions=positions, slots=slots, q_out=q_out, cache=cache)
-    _ext().latent_qkv(y, w.H, w.dim_p, w.rot_p, w.rank_p, rope, positions, slots, q_out, w.norm if cache is not None else None,
-                      w.eps, cache, w.uk)
+    E, norm, dk, hq = _ext(), w.norm if cache is not None else None, w.rank_p + w.rot_p, w.dim_p + w.rot_p
+    if not _expands(w, y, plan):
+        E.latent_qkv(y, w.H, w.dim_p, w.rot_p, w.rank_p, rope, positions, slots, q_out, norm, w.eps, cache, w.uk)
+        return q_out
+    E.latent_rows(y, w.H, w.dim_p, w.rot_p, rope, positions, slots, q_out, dk, w.rank_p, norm, w.eps, cache)
+    if plan.short is not None:
+        E.head_linear(y, hq, w.uk, w.H, w.rank_p, w.dim_p, q_out, dk, plan.short)
     return q_out
 
 
 def latent_attention(q: torch.Tensor, w: LatentWeights, *, cache: torch.Tensor, block_table: torch.Tensor, positions: torch.Tensor,
                      seq_ids: torch.Tensor, slots: torch.Tensor, gate: torch.Tensor, max_ctx: int, scratch: LatentScratch,
-                     out: torch.Tensor) -> torch.Tensor:
-    """Causal softmax with a sink per head over the cached latents, value projection, output gate."""
+                     out: torch.Tensor, y: Optional[torch.Tensor] = None, plan: Optional[SimpleNamespace] = None) -> torch.Tensor:
+    """Causal softmax with a sink per head over the cached latents, value projection, output gate.  y: the
+    projected rows (the prefill form reads the unrotated query parts there)."""
     if not q.is_cuda:
         return ref.latent_attention(q, w, cache=cache, block_table=block_table, positions=positions, seq_ids=seq_ids,
                                     slots=slots, gate=gate, out=out)
     E, rows = _ext(), q.shape[0]
-    for i in range(0, rows, ROW_SLICE):
-        n = min(ROW_SLICE, rows - i)
+
+    def rows_form(row_list, i, n):
         nch = latent_chunks(n, w.H, max_ctx)
-        s = slice(i, i + n)
-        E.latent_attention(q[s], cache, block_table, positions[s], seq_ids[s], slots[s], None, n, w.H, w.rank_p, w.scale, nch,
+        s = slice(i, i + n) if row_list is None else slice(None)
+        E.latent_attention(q[s], cache, block_table, positions[s], seq_ids[s], slots[s], row_list, n, w.H, w.rank_p, w.scale, nch,
                            scratch.part, scratch.stat)
-        E.latent_out(scratch.part, scratch.stat, nch, slots[s], None, n, w.H, w.rank_p, w.sink, w.uv, gate[s], out[s])
+        E.latent_out(scratch.part, scratch.stat, nch, slots[s], row_list, n, w.H, w.rank_p, w.sink, w.uv, gate[s], out[s])
+
+    if y is None or not _expands(w, y, plan):
+        for i in range(0, rows, ROW_SLICE):
+            rows_form(None, i, min(ROW_SLICE, rows - i))
+        return out
+    if plan.short is not None:
+        for i in range(0, plan.short.shape[0], ROW_SLICE):
+            lst = plan.short[i : i + ROW_SLICE]
+            rows_form(lst, 0, lst.shape[0])
+    from . import linear, scratch as ws
+
+    T, kp, n_kv, bf = 64 * plan.segs.shape[0], w.w_kv.shape[1], w.w_kv.shape[0], torch.bfloat16
+    lat = ws(q.device, "latent_ctx", T * kp, bf).view(T, kp)
+    krot = ws(q.device, "latent_rot", T * w.rot_p, bf).view(T, w.rot_p)
+    kv = ws(q.device, "latent_kv", T * n_kv, bf).view(T, n_kv)
+    E.latent_gather(cache, block_table, plan.segs, lat, krot)
+    linear(lat, w.w_kv, out=kv)
+    E.latent_prefill(y, q, w.H, w.dim_p, w.rank_p + w.rot_p, w.rank_p, kv[:, : w.H * (w.dim_p + w.vdk)], krot, plan.q_tiles, w.scale,
+                     w.sink, gate, w.vd, out)
     return out
 
 
@@ -166,15 +232,23 @@ def moe_tiles(pairs: int, E: int, tile: int) -> int:
     return min(pairs, E) + pairs // tile
 
 
+def moe_tile(rows: int, E: int, top: int, dtype) -> int:
+    """The tile size of a step: the LDS-tiled GEMM once its tiles are a quarter full on average."""
+    return MOE_TILES[1] if dtype == torch.bfloat16 and rows * top >= 32 * E else MOE_TILES[0]
+
+
 def moe_buffers(rows: int, layers: Sequence[Tuple[int, int, int]], dtype, device) -> SimpleNamespace:
-    """Routing tables and expert activations of a step of ``rows`` rows; layers: (E, top, F) of every layer."""
+    """Routing tables and expert activations of a step of up to ``rows`` rows; layers: (E, top, F) of every layer."""
     top = max(t for _, t, _ in layers)
-    tiles = max(moe_tiles(rows * t, E, MOE_TILE) for E, t, _ in layers)
-    F = max(f for _, _, f in layers)
+    # (fewer rows may take the smaller tiles)
+    sizes = [(moe_tiles(rows * t, E, tile), tile, f) for E, t, f in layers for tile in MOE_TILES if tile <= moe_tile(rows, E, t, dtype)]
+    tiles = max(n for n, _, _ in sizes)
+    places = max(n * t for n, t, _ in sizes)
+    act = max(n * t * f for n, t, f in sizes)
     i32 = dict(dtype=torch.int32, device=device)
     return SimpleNamespace(wts=torch.zeros(rows * top, dtype=torch.float32, device=device), ids=torch.zeros(rows * top, **i32),
-                           tiles=torch.zeros(1 + 3 * tiles, **i32), order=torch.zeros(tiles * MOE_TILE, **i32),
-                           ticket=torch.zeros(1, **i32), act=torch.zeros(tiles * MOE_TILE * F, dtype=dtype, device=device))
+                           tiles=torch.zeros(1 + 3 * tiles, **i32), order=torch.zeros(places, **i32),
+                           ticket=torch.zeros(1, **i32), act=torch.empty(act, dtype=dtype, device=device))
 
 
 def moe(h: torch.Tensor, w: MoeWeights, *, slots: torch.Tensor, bufs: SimpleNamespace, out: torch.Tensor) -> torch.Tensor:
@@ -182,11 +256,11 @@ def moe(h: torch.Tensor, w: MoeWeights, *, slots: torch.Tensor, bufs: SimpleName
     rows = h.shape[0]
     if not h.is_cuda:
         return ref.moe(h, w, slots=slots, out=out)
-    E, F = _ext(), w.down.shape[2]
-    n = moe_tiles(rows * w.top, w.E, MOE_TILE)
-    tiles, order = bufs.tiles[: 1 + 3 * n], bufs.order[: n * MOE_TILE]
-    act = bufs.act[: n * MOE_TILE * F].view(-1, F)
-    E.moe_route(h, w.router, w.E, w.top, slots, bufs.wts, bufs.ids, MOE_TILE, tiles, order, bufs.ticket)
-    E.moe_gemm(h, w.gate_up, rows, w.top, False, bufs.wts, MOE_TILE, tiles, order, act)
-    E.moe_gemm(act, w.down, rows, w.top, True, bufs.wts, MOE_TILE, tiles, order, out)
+    E, F, tile = _ext(), w.down.shape[2], moe_tile(rows, w.E, w.top, h.dtype)
+    n = moe_tiles(rows * w.top, w.E, tile)
+    tiles, order = bufs.tiles[: 1 + 3 * n], bufs.order[: n * tile]
+    act = bufs.act[: n * tile * F].view(-1, F)
+    E.moe_route(h, w.router, w.E, w.top, slots, bufs.wts, bufs.ids, tile, tiles, order, bufs.ticket)
+    E.moe_gemm(h, w.gate_up, rows, w.top, False, bufs.wts, tile, tiles, order, act)
+    E.moe_gemm(act, w.down, rows, w.top, True, bufs.wts, tile, tiles, order, out)
     return out
