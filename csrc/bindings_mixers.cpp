@@ -15,7 +15,8 @@ const void* frag(const Tensor& w, bool f32, int64_t n, const char* name) {
 
 // y | x projections [rows, 2 width]; conv [taps, width]; state [slots, taps * width]; chunks / scratch: scan form
 void rglru(Tensor yx, Tensor yb, Tensor xb, Tensor cw, Tensor cb, Tensor gw, Tensor rb, Tensor ib, Tensor decay, int64_t nb,
-           Tensor seq_ids, Tensor positions, Tensor slots, Tensor state, Tensor out, OptTensor chunks, OptTensor scratch) {
+           Tensor seq_ids, Tensor positions, Tensor slots, Tensor state, Tensor out, OptTensor chunks, OptTensor scratch,
+           OptTensor u) {
   c10::DeviceGuard g(yx.device());
   const bool f32 = t_is_f32(yx, "yx");
   const int64_t rows = out.size(0), W = decay.numel();
@@ -63,7 +64,10 @@ void rglru(Tensor yx, Tensor yb, Tensor xb, Tensor cw, Tensor cb, Tensor gw, Ten
   TORCH_CHECK(chunks->dim() == 2 && chunks->size(1) == 4 && chunks->size(0) >= 1, "chunks int32 [n, 4]");
   p.chunks = i32p(*chunks, chunks->numel(), "chunks");
   p.n_chunks = (int)chunks->size(0);
-  TORCH_CHECK(scratch.has_value(), "scan form needs scratch");
+  TORCH_CHECK(scratch.has_value() && u.has_value(), "scan form needs scratch and u");
+  check_t(*u, f32, "u");
+  TORCH_CHECK(u->is_contiguous() && u->numel() >= rows * W, "u [rows, width]");
+  p.u = u->data_ptr();
   float* s = f32p(*scratch, 3 * (int64_t)p.n_chunks * W, "scratch");
   p.cA = s;
   p.cB = s + (size_t)p.n_chunks * W;
@@ -395,7 +399,7 @@ void moe_gemm(Tensor x, Tensor w, int64_t rows, int64_t top, bool down, Tensor w
 void bind_mixers(py::module_& m) {
   m.def("rglru", &rglru, py::arg("yx"), py::arg("yb"), py::arg("xb"), py::arg("cw"), py::arg("cb"), py::arg("gw"), py::arg("rb"),
         py::arg("ib"), py::arg("decay"), py::arg("nb"), py::arg("seq_ids"), py::arg("positions"), py::arg("slots"), py::arg("state"),
-        py::arg("out"), py::arg("chunks") = py::none(), py::arg("scratch") = py::none());
+        py::arg("out"), py::arg("chunks") = py::none(), py::arg("scratch") = py::none(), py::arg("u") = py::none());
   m.def("head_linear", &head_linear, py::arg("x"), py::arg("xs"), py::arg("w"), py::arg("nb"), py::arg("N"), py::arg("K"), py::arg("y"),
         py::arg("ys"), py::arg("row_list") = py::none());
   m.def("latent_rows", &latent_rows);

@@ -26,9 +26,10 @@ struct RgLruParams {
   float* state; int64_t state_ld;   // [state slots][taps * width]: S, then the last taps - 1 inputs (oldest first)
   void* out; int ldo;
   // scan form: chunks [n_chunks][4] = first row, rows, index in its run, chunks of the run;
-  // cA / cB / cS [n_chunks][width] f32 scratch
+  // cA / cB / cS [n_chunks][width] f32 scratch, u [rows][width] T scratch
   const int* chunks; int n_chunks;
   float* cA; float* cB; float* cS;
+  void* u;
 };
 
 // y[m][b * ys ..] = W_b . x[m][b * xs ..] for every head / block b (K inputs, N outputs)

@@ -78,9 +78,18 @@ __global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(MoeRouteParams
   const uint4* wf = reinterpret_cast<const uint4*>(p.w) + lane;
   for (int e = 0; e < et; ++e) {                     // D[expert 4 g + i][row rl], every wave a part of K
     f32x4 acc = {};
-#pragma unroll 4
-    for (int s = w; s < steps; s += kRouteWaves)
-      acc = M::mma(wf[((size_t)e * steps + s) * 64], *reinterpret_cast<const uint4*>(h + s * M::KS), acc);
+    for (int s0 = w; s0 < steps; s0 += 8 * kRouteWaves) {
+      uint4 a[8], b[8];
+#pragma unroll
+      for (int u = 0; u < 8; ++u) {
+        const int s = min(s0 + u * kRouteWaves, steps - 1);
+        a[u] = wf[((size_t)e * steps + s) * 64];
+        b[u] = *reinterpret_cast<const uint4*>(h + s * M::KS);
+      }
+#pragma unroll
+      for (int u = 0; u < 8; ++u)
+        if (s0 + u * kRouteWaves < steps) acc = M::mma(a[u], b[u], acc);
+    }
 #pragma unroll
     for (int i = 0; i < 4; ++i) red[(w * Ep + e * 16 + 4 * g + i) * 16 + rl] = acc[i];
   }
@@ -150,7 +159,6 @@ __global__ __launch_bounds__(256) void moe_gemm16_kernel(MoeGemmParams p) {
   const T* x = reinterpret_cast<const T*>(p.x) + (size_t)(DOWN ? src : p.order[src] / p.top) * p.ldx + 4 * M::EPL * g;
   const uint4* wp = reinterpret_cast<const uint4*>(reinterpret_cast<const T*>(p.w) + e * p.w_expert) + (size_t)unit * NA * KG * 256 + lane;
   f32x4 acc[NA] = {};
-#pragma unroll 2
   for (int kg = w; kg < KG; kg += 4) {
     uint4 f[NA][4], a[4];
 #pragma unroll

@@ -6,11 +6,11 @@
 // over the 16-row tiles.  A row that starts a run of its sequence folds the state it starts from into b and
 // takes a = 0, so one scan serves any mix of runs.
 //
-//  * rows form (decode steps, <= 64 rows): a workgroup per block; runs are found from the sequence ids.
-//    The block's workgroup is the only reader and writer of its channels' state rows.
-//  * scan form (prompt-sized runs): workgroups per (chunk of a run, block, 128 channels).  Launch 1 reduces
-//    every chunk to S_end = A S_start + B; launch 2 folds the chunks in front of its own, scans again and
-//    writes the outputs; the run's last chunk writes the state.
+//  * rows form (decode steps, <= 64 rows): a workgroup per block and 16 rows, for the runs that start there; runs
+//    are found from the sequence ids.  It is the only reader and writer of its runs' state in the block.
+//  * scan form (prompt-sized runs): workgroups per (chunk of a run, block, 128 channels).  Launch 1 forms u and
+//    reduces every chunk to S_end = A S_start + B; launch 2 folds the chunks in front of its own, scans again
+//    and writes the outputs; the run's last chunk writes the state.
 //
 // A run that starts at position 0 starts from zeros whatever its slot holds.
 #include "mixer_kernels.h"
@@ -23,41 +23,66 @@ namespace {
 constexpr size_t kMaxLds = 160 * 1024 - 2048;
 constexpr int kPad = 16;                             // bytes between LDS rows of u: 16 rows hit different banks
 
-VWA_DEVICE float gelu_tanh(float z) {
-  return z / (1.f + __expf(-1.5957691216057308f * (z + 0.044715f * z * z * z)));
-}
+VWA_DEVICE float rcp_sigm(float x) { return __builtin_amdgcn_rcpf(1.f + __expf(-x)); }
+VWA_DEVICE float gelu_tanh(float z) { return z * rcp_sigm(1.5957691216057308f * (z + 0.044715f * z * z * z)); }
 
 struct Step {
   float a, b;
 };
-// the recurrence's step from the gates' pre-activations; a and 1 - a^2 both from expm1 of log a
+// The recurrence's step from the gates' pre-activations: a = exp(x), b = sqrt(1 - a^2) i u.  1 - a^2 = -expm1(2 x)
+// by its series where a is near 1 (the difference would lose the small decays), directly elsewhere.
 VWA_DEVICE Step lru_step(float rp, float ip, float decay, float u) {
-  const float em = expm1f(decay * sigm(rp));
-  const float a = 1.f + em;
-  return Step{a, sqrtf(-em * (1.f + a)) * sigm(ip) * u};
+  const float x = decay * rcp_sigm(rp), y = 2.f * x;
+  const float a = __expf(x);
+  float q = 1.f / 5040.f;                            // (|y| < 1/4: the next term is below 2e-9 of y)
+  q = q * y + 1.f / 720.f;
+  q = q * y + 1.f / 120.f;
+  q = q * y + 1.f / 24.f;
+  q = q * y + 1.f / 6.f;
+  q = q * y + 0.5f;
+  q = q * y + 1.f;
+  const float d = y > -0.25f ? -y * q : 1.f - a * a;
+  return Step{a, __builtin_amdgcn_sqrtf(d) * rcp_sigm(ip) * u};
 }
 
 template <class T> VWA_DEVICE int u_stride(int bs) { return bs * (int)sizeof(T) + kPad; }
 
-// r, i pre-activations of RT rows for 16 channels: u in LDS, gate fragments from global memory
-template <class T, int NT>
-VWA_DEVICE void gate_products(const char* us, int stride, const T* gw, int steps, f32x4 (&ar)[NT], f32x4 (&ai)[NT]) {
+// gate fragments of 16 channels, steps s0 .. s0 + PRE
+template <int PRE>
+struct GateFrags {
+  uint4 r[PRE], i[PRE];
+  template <class T> VWA_DEVICE void load(const T* gw, int steps, int s0) {
+    const uint4* wr = reinterpret_cast<const uint4*>(gw) + lane_id();
+    const uint4* wi = wr + (size_t)steps * 64;
+#pragma unroll
+    for (int s = 0; s < PRE; ++s) {
+      const int k = min(s0 + s, steps - 1) * 64;
+      r[s] = wr[k];
+      i[s] = wi[k];
+    }
+  }
+};
+// r, i pre-activations of 16 NT rows for 16 channels: u in LDS; f holds the first fragments
+template <class T, int NT, int PRE>
+VWA_DEVICE void gate_products(const char* us, int stride, const T* gw, int steps, GateFrags<PRE>& f, f32x4 (&ar)[NT], f32x4 (&ai)[NT]) {
   using M = MM<T>;
   const int lane = lane_id(), rl = lane & 15, b = lane >> 4;
 #pragma unroll
   for (int t = 0; t < NT; ++t) ar[t] = ai[t] = f32x4{0.f, 0.f, 0.f, 0.f};
-  const uint4* wr = reinterpret_cast<const uint4*>(gw) + lane;
-  const uint4* wi = wr + (size_t)steps * 64;
   const char* ua = us + rl * stride + b * 16;
-#pragma unroll 4
-  for (int s = 0; s < steps; ++s) {
-    const uint4 fr = wr[s * 64], fi = wi[s * 64];
+  for (int s0 = 0; s0 < steps; s0 += PRE) {
 #pragma unroll
-    for (int t = 0; t < NT; ++t) {
-      const uint4 a = *reinterpret_cast<const uint4*>(ua + t * 16 * stride + s * 64);
-      ar[t] = M::mma(a, fr, ar[t]);
-      ai[t] = M::mma(a, fi, ai[t]);
+    for (int s = 0; s < PRE; ++s) {
+      if (s0 + s < steps) {
+#pragma unroll
+        for (int t = 0; t < NT; ++t) {
+          const uint4 a = *reinterpret_cast<const uint4*>(ua + t * 16 * stride + (s0 + s) * 64);
+          ar[t] = M::mma(a, f.r[s], ar[t]);
+          ai[t] = M::mma(a, f.i[s], ai[t]);
+        }
+      }
     }
+    if (s0 + PRE < steps) f.load(gw, steps, s0 + PRE);
   }
 }
 
@@ -143,84 +168,94 @@ VWA_DEVICE void save_inputs8(const RgLruParams& p, int r, int n, bool fresh, flo
 }
 
 // ------------------------------------------------------------------------------------------ rows form
-template <class T, int NT>
+// Workgroup (block, tile): the runs whose first row lies in rows 16 tile .. 16 tile + 15, 16 rows at a time to
+// their ends (other runs' rows count as inert).
+template <class T>
 __global__ __launch_bounds__(1024) void rglru_rows_kernel(RgLruParams p) {
-  constexpr int RT = NT * 16;
   extern __shared__ __attribute__((aligned(16))) char us[];
   __shared__ int s_first[64], s_len[64];             // of the row's run: first row; rows (at its last row, else 0)
-  const int blk = blockIdx.x, bs = p.bs, W = p.nb * bs, c0 = blk * bs;
+  const int blk = blockIdx.x, lo = blockIdx.y * 16, bs = p.bs, c0 = blk * bs;
   const int tid = threadIdx.x, nthr = blockDim.x, lane = lane_id(), w = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int rl = lane & 15, g = lane >> 4, stride = u_stride<T>(bs), steps = bs / MM<T>::KS;
+  const int rl = lane & 15, g = lane >> 4, stride = u_stride<T>(bs), steps = bs / MM<T>::KS, waves = nthr >> 6;
   T* out = reinterpret_cast<T*>(p.out);
-  if (tid < p.rows && tid < 64) {
+  const T* gw0 = reinterpret_cast<const T*>(p.gw) + (size_t)blk * (bs / 16) * 32 * bs;
+  GateFrags<4> f;                                    // (requested ahead of everything that waits)
+  f.load(gw0 + (size_t)w * 32 * bs, steps, 0);
+  if (tid < 64) {                                    // (one wave: runs from the rows' ids)
     const int r = tid;
-    int f = r, len = 0;
-    if (p.slots[r] >= 0) {
-      const int seq = p.seq_ids[r];
-      while (f > 0 && p.slots[f - 1] >= 0 && p.seq_ids[f - 1] == seq) --f;
-      const bool end = r + 1 >= p.rows || p.slots[r + 1] < 0 || p.seq_ids[r + 1] != seq;
-      len = end ? r + 1 - f : 0;
-    } else {
-      f = -1;
-    }
-    s_first[r] = f;
-    s_len[r] = len;
+    const bool in = r < p.rows;
+    const bool live = in && p.slots[r] >= 0;
+    const int seq = live ? p.seq_ids[r] : -1 - r;
+    const int before = __shfl_up(seq, 1, 64), after = __shfl_down(seq, 1, 64);
+    const unsigned long long heads = __ballot(live && (r == 0 || before != seq));
+    const unsigned long long mine = heads & ((2ull << r) - 1ull);
+    const int first = live && mine ? 63 - __builtin_clzll(mine) : -1;
+    s_first[r] = first;
+    s_len[r] = live && (r == 63 || after != seq) ? r + 1 - first : 0;
   }
   __syncthreads();
-  const int oct = bs / 8;
-  for (int r0 = 0; r0 < p.rows; r0 += RT) {
-    const int n = min(RT, p.rows - r0);
-    for (int x = tid; x < RT * oct; x += nthr) {
+  const int oct = bs / 8, hi = min(lo + 16, p.rows);
+  auto owned = [&](int r) { return s_first[r] >= lo && s_first[r] < hi; };
+  for (int r0 = lo; r0 < p.rows; r0 += 16) {
+    if (r0 > lo && !owned(r0)) break;                // (a run that goes past the tile owns the next row)
+    const int n = min(16, p.rows - r0);
+    for (int x = tid; x < 16 * oct; x += nthr) {
       const int i = x / oct, ch = (x % oct) * 8, r = r0 + i;
       float u[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-      if (i < n && s_first[r] >= 0) {
-        const int f = s_first[r];
-        const float* st = p.positions[f] > 0 ? p.state + (size_t)p.seq_ids[r] * p.state_ld : nullptr;
-        conv8<T>(p, r, r - f, st, c0 + ch, u);
+      if (i < n && owned(r)) {
+        const int fr = s_first[r];
+        const float* st = p.positions[fr] > 0 ? p.state + (size_t)p.seq_ids[r] * p.state_ld : nullptr;
+        conv8<T>(p, r, r - fr, st, c0 + ch, u);
       }
       st8(reinterpret_cast<T*>(us + i * stride) + ch, u);
     }
     __syncthreads();                                 // (every read of the old inputs is done as well)
     for (int x = tid; x < n * oct; x += nthr) {
       const int i = x / oct, r = r0 + i, len = s_len[r];
-      if (len == 0) continue;
+      if (len == 0 || !owned(r)) continue;
       save_inputs8<T>(p, r, len, p.positions[s_first[r]] == 0, p.state + (size_t)p.seq_ids[r] * p.state_ld, c0 + (x % oct) * 8);
     }
-    for (int ct = w; ct < bs / 16; ct += nthr >> 6) {
-      f32x4 ar[NT], ai[NT];
-      gate_products<T, NT>(us, stride, reinterpret_cast<const T*>(p.gw) + (size_t)(blk * (bs / 16) + ct) * 32 * bs, steps, ar, ai);
+    for (int ct = w; ct < bs / 16; ct += waves) {
+      const T* gw = gw0 + (size_t)ct * 32 * bs;
       const int ch = c0 + ct * 16 + rl;
       const float rb = p.rb[ch], ib = p.ib[ch], dec = p.decay[ch], yb = p.yb[ch];
-      float carry = 0.f;
+      float y[4], s_in[4];
 #pragma unroll
-      for (int t = 0; t < NT; ++t) {
-        float a[4], b[4], s[4], A, B;
+      for (int i = 0; i < 4; ++i) {                  // (requested ahead of the products)
+        const int li = min(4 * g + i, n - 1), r = r0 + li;
+        y[i] = ldv(reinterpret_cast<const T*>(p.yx) + (size_t)r * p.ld + ch);
+        const bool head = owned(r) && (s_first[r] == r || li == 0) && p.positions[r] > 0;
+        s_in[i] = head ? p.state[(size_t)p.seq_ids[r] * p.state_ld + ch] : 0.f;
+      }
+      f32x4 ar[1], ai[1];
+      if (r0 > lo || ct != w) f.load(gw, steps, 0);
+      gate_products<T, 1, 4>(us, stride, gw, steps, f, ar, ai);
+      float a[4], b[4], s[4], A, B;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const int li = t * 16 + 4 * g + i, r = r0 + li;
-          a[i] = b[i] = 0.f;
-          if (li < n && s_first[r] >= 0) {
-            const float u = ldv(reinterpret_cast<const T*>(us + li * stride) + ct * 16 + rl);
-            const Step st = lru_step(ar[t][i] + rb, ai[t][i] + ib, dec, u);
-            a[i] = st.a;
-            b[i] = st.b;
-            if (s_first[r] == r || li == 0) {        // (a run that goes on from the rows before: its state was saved)
-              if (p.positions[r] > 0) b[i] += st.a * p.state[(size_t)p.seq_ids[r] * p.state_ld + ch];
-              a[i] = 0.f;
-            }
+      for (int i = 0; i < 4; ++i) {
+        const int li = 4 * g + i, r = r0 + li;
+        a[i] = b[i] = 0.f;
+        if (li < n && owned(r)) {
+          const float u = ldv(reinterpret_cast<const T*>(us + li * stride) + ct * 16 + rl);
+          const Step st = lru_step(ar[0][i] + rb, ai[0][i] + ib, dec, u);
+          a[i] = st.a;
+          b[i] = st.b;
+          if (s_first[r] == r || li == 0) {          // (a run that goes on from the rows before: its state was saved)
+            b[i] += st.a * s_in[i];
+            a[i] = 0.f;
           }
         }
-        carry = scan_tile(a, b, carry, s, A, B);
+      }
+      scan_tile(a, b, 0.f, s, A, B);
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const int li = t * 16 + 4 * g + i, r = r0 + li;
-          if (li >= n) continue;
-          float o = 0.f;
-          if (s_first[r] >= 0) {
-            o = s[i] * gelu_tanh(ldv(reinterpret_cast<const T*>(p.yx) + (size_t)r * p.ld + ch) + yb);
-            if (s_len[r] > 0 || li == n - 1) p.state[(size_t)p.seq_ids[r] * p.state_ld + ch] = s[i];
-          }
-          stv(out + (size_t)r * p.ldo + ch, o);
+      for (int i = 0; i < 4; ++i) {
+        const int li = 4 * g + i, r = r0 + li;
+        if (li >= n) continue;
+        if (owned(r)) {
+          stv(out + (size_t)r * p.ldo + ch, s[i] * gelu_tanh(y[i] + yb));
+          if (s_len[r] > 0 || li == n - 1) p.state[(size_t)p.seq_ids[r] * p.state_ld + ch] = s[i];
+        } else if (s_first[r] < 0 && r0 == lo) {
+          stv(out + (size_t)r * p.ldo + ch, 0.f);    // inert row of a padded step
         }
       }
     }
@@ -231,6 +266,7 @@ __global__ __launch_bounds__(1024) void rglru_rows_kernel(RgLruParams p) {
 // ------------------------------------------------------------------------------------------ scan form
 constexpr int kScanWaves = 8;
 
+// Pass 1 forms u by the convolution and leaves it in p.u for pass 2.
 template <class T, int PASS, int NT>
 __global__ __launch_bounds__(kScanWaves * 64) void rglru_scan_kernel(RgLruParams p) {
   constexpr int RT = NT * 16;
@@ -240,30 +276,54 @@ __global__ __launch_bounds__(kScanWaves * 64) void rglru_scan_kernel(RgLruParams
   const int rl = lane & 15, g = lane >> 4, stride = u_stride<T>(bs), steps = bs / MM<T>::KS;
   const int row0 = p.chunks[4 * ck], n = p.chunks[4 * ck + 1], idx = p.chunks[4 * ck + 2], cnt = p.chunks[4 * ck + 3];
   const int run0 = idx > 0 ? p.chunks[4 * (ck - idx)] : row0;  // first row of the run
-  const int pos0 = p.positions[run0];
-  float* st = p.state + (size_t)p.seq_ids[row0] * p.state_ld;
   const int ct = blockIdx.z * kScanWaves + w;
   const bool active = ct < bs / 16;
   const int ch = c0 + (active ? ct : 0) * 16 + rl;
+  const T* gw = reinterpret_cast<const T*>(p.gw) + (size_t)(blk * (bs / 16) + (active ? ct : 0)) * 32 * bs;
+  GateFrags<8> f;
+  f.load(gw, steps, 0);
+  const int pos0 = p.positions[run0];
+  float* st = p.state + (size_t)p.seq_ids[row0] * p.state_ld;
   const float rb = p.rb[ch], ib = p.ib[ch], dec = p.decay[ch], yb = p.yb[ch];
   float carry = 0.f, Ac = 1.f, Bc = 0.f;
-  if (PASS == 2 && active) {
-    carry = p.cS[(size_t)(ck - idx) * W + ch];
-    for (int k = ck - idx; k < ck; ++k) carry = p.cA[(size_t)k * W + ch] * carry + p.cB[(size_t)k * W + ch];
+  if (PASS == 2) {
+    const int k0 = ck - idx;
+    carry = p.cS[(size_t)k0 * W + ch];
+    for (int k = k0; k < ck; k += 8) {
+      float ca[8], cb[8];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const size_t o = (size_t)min(k + e, ck - 1) * W + ch;
+        ca[e] = p.cA[o];
+        cb[e] = p.cB[o];
+      }
+#pragma unroll
+      for (int e = 0; e < 8; ++e) carry = k + e < ck ? ca[e] * carry + cb[e] : carry;
+    }
   }
   const int oct = bs / 8;
+  T* ug = reinterpret_cast<T*>(p.u);
   for (int r0 = 0; r0 < n; r0 += RT) {
     const int m = min(RT, n - r0);
     for (int x = tid; x < RT * oct; x += kScanWaves * 64) {
       const int i = x / oct, c = (x % oct) * 8, r = row0 + r0 + i;
+      T* d = reinterpret_cast<T*>(us + i * stride) + c;
+      if (PASS == 2) {                               // (rows past the chunk repeat its last one; their steps are dropped)
+        const T* src = ug + (size_t)(row0 + r0 + min(i, m - 1)) * W + c0 + c;
+#pragma unroll
+        for (int e = 0; e < (int)sizeof(T) / 2; ++e) reinterpret_cast<uint4*>(d)[e] = reinterpret_cast<const uint4*>(src)[e];
+        continue;
+      }
       float u[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
       if (i < m) conv8<T>(p, r, r - run0, pos0 > 0 ? st : nullptr, c0 + c, u);
-      st8(reinterpret_cast<T*>(us + i * stride) + c, u);
+      st8(d, u);
+      if (i < m && blockIdx.z == 0) st8(ug + (size_t)r * W + c0 + c, u);
     }
     __syncthreads();
     if (active) {
       f32x4 ar[NT], ai[NT];
-      gate_products<T, NT>(us, stride, reinterpret_cast<const T*>(p.gw) + (size_t)(blk * (bs / 16) + ct) * 32 * bs, steps, ar, ai);
+      if (r0 > 0) f.load(gw, steps, 0);
+      gate_products<T, NT, 8>(us, stride, gw, steps, f, ar, ai);
 #pragma unroll
       for (int t = 0; t < NT; ++t) {
         float a[4], b[4], s[4], A, B;
@@ -325,13 +385,9 @@ size_t u_bytes(int rows, int bs) { return (size_t)rows * (bs * sizeof(T) + kPad)
 
 template <class T>
 int launch_rows(const RgLruParams& p, hipStream_t st) {
-  const dim3 grid(p.nb), block(64 * (p.bs / 16 < 16 ? p.bs / 16 : 16));
-  if (p.rows > 16 && u_bytes<T>(64, p.bs) <= kMaxLds)
-    hipLaunchKernelGGL((rglru_rows_kernel<T, 4>), grid, block, u_bytes<T>(64, p.bs), st, p);
-  else if (u_bytes<T>(16, p.bs) <= kMaxLds)
-    hipLaunchKernelGGL((rglru_rows_kernel<T, 1>), grid, block, u_bytes<T>(16, p.bs), st, p);
-  else
-    return -10;
+  if (u_bytes<T>(16, p.bs) > kMaxLds) return -10;
+  const dim3 grid(p.nb, (p.rows + 15) / 16), block(64 * (p.bs / 16 < 16 ? p.bs / 16 : 16));
+  hipLaunchKernelGGL((rglru_rows_kernel<T>), grid, block, u_bytes<T>(16, p.bs), st, p);
   return (int)hipGetLastError();
 }
 
@@ -365,6 +421,6 @@ extern "C" int vwa_rglru_rows(const RgLruParams* p, hipStream_t st) {
 extern "C" int vwa_rglru_scan(const RgLruParams* p, hipStream_t st) {
   const int rc = check(*p);
   if (rc) return rc;
-  if (p->n_chunks < 1 || !p->chunks || !p->cA || !p->cB || !p->cS) return -4;
+  if (p->n_chunks < 1 || !p->chunks || !p->cA || !p->cB || !p->cS || !p->u || (reinterpret_cast<uintptr_t>(p->u) & 15)) return -4;
   return p->f32 ? launch_scan<float>(*p, st) : launch_scan<u16>(*p, st);
 }

@@ -175,6 +175,8 @@ LATENT = [  # H, dim, rot, vd, rank, block size, n
     (8, 128, 64, 128, 512, 16, 200),
     (4, 96, 64, 80, 200, 16, 140),
     (6, 33, 66, 17, 64, 16, 70),         # a rotated part larger than the other
+    (2, 32, 32, 32, 300, 16, 100),
+    (3, 40, 16, 24, 700, 16, 90),
 ]
 
 

@@ -20,7 +20,7 @@ import torch
 from . import reference as ref
 from .stack import ROW_SLICE, _ext
 
-SCAN_ROWS = 128     # rows per chunk of the recurrence scan
+SCAN_ROWS = 64      # rows per chunk of the recurrence scan
 ATTN_KEYS = 64      # keys per round of the latent attention
 ATTN_GROUPS = 512   # workgroups a latent attention launch is cut into
 EXPAND_ROWS = 32    # runs of fewer rows attend in latent space ...
@@ -81,7 +81,9 @@ def rglru(yx: torch.Tensor, w: RgLruWeights, *, seq_ids: torch.Tensor, positions
     else:
         from . import scratch
 
-        _ext().rglru(*args, plan.chunks, scratch(yx.device, "scan", 3 * plan.chunks.shape[0] * w.decay.numel()))
+        W = w.decay.numel()
+        _ext().rglru(*args, plan.chunks, scratch(yx.device, "scan", 3 * plan.chunks.shape[0] * W),
+                     scratch(yx.device, "rglru_u", out.shape[0] * W, yx.dtype))
     return out
 
 
