@@ -53,6 +53,7 @@ template <int EPI> constexpr bool kResid = EPI == EPI_RESID || EPI == EPI_GELU_R
 template <int EPI> constexpr bool kGelu = EPI == EPI_GELU || EPI == EPI_GELU_RESID;
 
 constexpr int BKG = 128;
+constexpr int kGroup = 4;  // row blocks of a grouped launch that walk the columns together
 
 // Workgroup shapes: BM x BN output tile, WM x WN waves, each wave (BM/WM) x (BN/WN).
 //   Cfg<128, 128, 2, 2>: 4 waves of 64 x 64, 64 KB LDS -> 2 workgroups per CU -- the one in use.
@@ -263,8 +264,10 @@ using CfgP8 = Cfg<256, 256, 2, 4>;
 
 // half-tile `which` (0 A-lo, 1 A-hi, 2 B-lo, 3 B-hi) of stage hs into the stage image `st`:
 // 16 wave-instructions of 1 KB = 2 per wave (tiled bf16 weights only)
+// (rows: as issue_stage)
+template <bool GRP>
 VWA_DEVICE void p8_issue(const GemmParams& p, __amdgpu_buffer_rsrc_t rx, __amdgpu_buffer_rsrc_t rw, int bm, int bn,
-                         int hs, int which, char* st) {
+                         int hs, int which, char* st, const int (&rows)[4]) {
   const int w = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int kg = hs >> 1, h = hs & 1;
   const int kgn = p.K / BKG;
@@ -274,10 +277,10 @@ VWA_DEVICE void p8_issue(const GemmParams& p, __amdgpu_buffer_rsrc_t rx, __amdgp
     if (which < 2) {
       const int qa = 16 * which + q;  // rows 8 qa .. 8 qa + 7
       const int r = 8 * qa + (lane >> 3), c = (lane & 7) ^ swz((r >> 1) & 7);
-      const int m = bm + r;
+      const int m = GRP ? rows[2 * which + it] : bm + r;
       const unsigned off =
           (unsigned)(((size_t)m * p.ldx + (size_t)kg * BKG + 32 * (c >> 1) + 16 * h + 8 * (c & 1)) * 2);
-      dma16(rx, st + qa * 1024, m < p.M ? off : 0xFFFFFFF0u);
+      dma16(rx, st + qa * 1024, (GRP ? m >= 0 : m < p.M) ? off : 0xFFFFFFF0u);
     } else {
       const int tile = 8 * (which - 2) + (q >> 1), sp = q & 1;
       const int T = (bn >> 4) + tile;
@@ -525,8 +528,8 @@ template <class C, int EPI, bool WT, bool F8 = false, bool P8 = false, bool W8 =
 __global__ __launch_bounds__(C::THREADS, C::NW == 4 ? 2 : 1) void gemm_kernel(GemmParams p) {
   extern __shared__ __attribute__((aligned(16))) char lds[];
   constexpr int FM = C::FM, FN = C::FN;
-  static_assert(!GRP || (C::BM == 128 && WT && !F8 && !P8 && !W8 && (EPI == EPI_SWIGLU || EPI == EPI_STORE)), "grouped: bf16 128-row tiles");
-  const int mb = GRP ? p.g_max : (p.M + C::BM - 1) / C::BM, nb = (p.N + C::BN - 1) / C::BN;
+  static_assert(!GRP || (WT && !F8 && !W8 && (EPI == EPI_SWIGLU || EPI == EPI_STORE)), "grouped: tiled bf16");
+  const int mb = GRP ? p.g_tiles[0] : (p.M + C::BM - 1) / C::BM, nb = (p.N + C::BN - 1) / C::BN;
   const int tiles = mb * nb;
   const int split = blockIdx.x / tiles % p.splits;  // split-K slice (blocks of one slice are contiguous)
   if (p.nbatch > 1) {  // batch z = blockIdx.x / (tiles * splits), splits == 1 (vwa_gemm)
@@ -539,14 +542,16 @@ __global__ __launch_bounds__(C::THREADS, C::NW == 4 ? 2 : 1) void gemm_kernel(Ge
   // share the column block's weight tile in L2
   if (p.ss_zero && blockIdx.x == 0)
     for (int i = threadIdx.x; i < p.ss_zero_n; i += C::THREADS) p.ss_zero[i] = 0ull;
+  if (GRP && (int)blockIdx.x >= tiles) return;       // (the grid is sized for the most row blocks there can be)
   const int lt = xcd_remap((int)(blockIdx.x % tiles), tiles);
-  const int bn = (lt / mb) * C::BN;
-  int bm = (lt % mb) * C::BM, place = 0;
+  // (grouped: column blocks of kGroup row blocks -- mostly one expert's -- after one another)
+  const int band = GRP ? lt / (kGroup * nb) * kGroup : 0, bh = GRP ? min(kGroup, mb - band) : mb, bt = lt - band * nb;
+  const int bn = (bt / bh) * C::BN;
+  int bm = (bt % bh) * C::BM, place = 0;
   int rows[C::BM / 8 / C::NW];
   size_t x_rows = 0;
   if constexpr (GRP) {
-    const int gt = lt % mb;
-    if (gt >= p.g_tiles[0]) return;
+    const int gt = band + bt % bh;
     p.W += (size_t)p.g_tiles[1 + 3 * gt] * p.g_wstride;
     place = p.g_tiles[2 + 3 * gt];
     x_rows = (size_t)p.M;                            // (X rows the buffer holds)
@@ -582,9 +587,9 @@ __global__ __launch_bounds__(C::THREADS, C::NW == 4 ? 2 : 1) void gemm_kernel(Ge
     auto stage = [&](int s) { return lds + (s & 1) * C::STAGE; };
     if (nh > 0) {
 #pragma unroll
-      for (int hq = 0; hq < 4; ++hq) p8_issue(p, rx, rw, bm, bn, h0, hq, stage(0));
+      for (int hq = 0; hq < 4; ++hq) p8_issue<GRP>(p, rx, rw, bm, bn, h0, hq, stage(0), rows);
     }
-    if (nh > 1) p8_issue(p, rx, rw, bm, bn, h0 + 1, 0, stage(1));
+    if (nh > 1) p8_issue<GRP>(p, rx, rw, bm, bn, h0 + 1, 0, stage(1), rows);
     if (nh > 1) asm volatile("s_waitcnt vmcnt(2)\n\ts_barrier" ::: "memory");
     else asm volatile("s_waitcnt vmcnt(0)\n\ts_barrier" ::: "memory");
     bf16x8 a[4][2], b[2][2];
@@ -614,8 +619,8 @@ __global__ __launch_bounds__(C::THREADS, C::NW == 4 ? 2 : 1) void gemm_kernel(Ge
       read_a(0);
       read_b(0);
       if (n1) {
-        p8_issue(p, rx, rw, bm, bn, h0 + s + 1, 1, stage(s + 1));
-        p8_issue(p, rx, rw, bm, bn, h0 + s + 1, 2, stage(s + 1));
+        p8_issue<GRP>(p, rx, rw, bm, bn, h0 + s + 1, 1, stage(s + 1), rows);
+        p8_issue<GRP>(p, rx, rw, bm, bn, h0 + s + 1, 2, stage(s + 1), rows);
       }
       __builtin_amdgcn_sched_barrier(0);
       asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
@@ -624,7 +629,7 @@ __global__ __launch_bounds__(C::THREADS, C::NW == 4 ? 2 : 1) void gemm_kernel(Ge
       asm volatile("s_barrier" ::: "memory");
       // P1
       read_b(2);
-      if (n1) p8_issue(p, rx, rw, bm, bn, h0 + s + 1, 3, stage(s + 1));
+      if (n1) p8_issue<GRP>(p, rx, rw, bm, bn, h0 + s + 1, 3, stage(s + 1), rows);
       __builtin_amdgcn_sched_barrier(0);
       asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
       p8_mfma<0, 2>(acc, a, b);
@@ -642,7 +647,7 @@ __global__ __launch_bounds__(C::THREADS, C::NW == 4 ? 2 : 1) void gemm_kernel(Ge
       // barrier; with the groups a barrier apart every wave has waited by the barrier that ends the
       // phase, and the next stage is read only after it
       read_b(0);
-      if (n2) p8_issue(p, rx, rw, bm, bn, h0 + s + 2, 0, stage(s + 2));
+      if (n2) p8_issue<GRP>(p, rx, rw, bm, bn, h0 + s + 2, 0, stage(s + 2), rows);
       __builtin_amdgcn_sched_barrier(0);
       if (n2) asm volatile("s_waitcnt vmcnt(2) lgkmcnt(0)\n\ts_barrier" ::: "memory");
       else asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)\n\ts_barrier" ::: "memory");
@@ -886,6 +891,14 @@ int launch_epi(const GemmParams& p, hipStream_t st, bool p8) {
   return (int)hipGetLastError();
 }
 
+template <class C, int EPI, bool P8>
+int launch_grouped(const GemmParams& p, hipStream_t st) {
+  const dim3 grid(p.g_max * ((p.N + C::BN - 1) / C::BN)), block(C::THREADS);
+  const int lds = 2 * C::STAGE > C::LDS ? 2 * C::STAGE : C::LDS;
+  hipLaunchKernelGGL((gemm_kernel<C, EPI, true, false, P8, false, true>), grid, block, lds, st, p);
+  return (int)hipGetLastError();
+}
+
 }  // namespace
 
 // Split-K slices for a shape: enough workgroups to cover the CUs ~2x when the output tiles
@@ -968,15 +981,10 @@ extern "C" int vwa_gemm_grouped(int epi, const GemmParams* pp, hipStream_t st) {
   p.splits = 1;
   p.nbatch = 1;
   p.kg_per_split = p.K / BKG;
-  using C = CfgS;
-  const dim3 grid(p.g_max * ((p.N + C::BN - 1) / C::BN)), block(C::THREADS);
-  const int lds = 2 * C::STAGE > C::LDS ? 2 * C::STAGE : C::LDS;
-  switch (epi) {
-    case EPI_SWIGLU: hipLaunchKernelGGL((gemm_kernel<C, EPI_SWIGLU, true, false, false, false, true>), grid, block, lds, st, p); break;
-    case EPI_STORE: hipLaunchKernelGGL((gemm_kernel<C, EPI_STORE, true, false, false, false, true>), grid, block, lds, st, p); break;
-    default: return -3;
-  }
-  return (int)hipGetLastError();
+  if (epi != EPI_SWIGLU && epi != EPI_STORE) return -3;
+  if (p.g_tile == CfgS::BM) return epi == EPI_SWIGLU ? launch_grouped<CfgS, EPI_SWIGLU, false>(p, st) : launch_grouped<CfgS, EPI_STORE, false>(p, st);
+  if (p.g_tile == CfgP8::BM) return epi == EPI_SWIGLU ? launch_grouped<CfgP8, EPI_SWIGLU, true>(p, st) : launch_grouped<CfgP8, EPI_STORE, true>(p, st);
+  return -4;
 }
 
 extern "C" int vwa_row_rstd(const uint16_t* x, int ldx, int M, int K, float eps, float* rstd, hipStream_t st) {

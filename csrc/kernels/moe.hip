@@ -2,8 +2,8 @@
 //
 //  moe_route : sigmoid router scores (MFMA, f32 sums), the best ``top`` experts of every row, and the pairs
 //              (row, choice) grouped by expert into tiles of at most ``tile`` pairs -- by the last workgroup
-//  moe_gemm  : the experts' matrices over such a tile (here tiles of 16 pairs, streaming; tiles of 128 go to
-//              gemm.hip's grouped launch).  First launch: the tile's rows times gate and up, scaled
+//  moe_gemm  : the experts' matrices over such a tile (here tiles of 16 pairs, streaming; tiles of 128 or 256
+//              go to gemm.hip's grouped launch).  First launch: the tile's rows times gate and up, scaled
 //              by the pair's score ahead of the activation (w (W h) = W (w h)); second: down, one row per pair.
 //              (The pairs of a row are added, in the order of its choices, by add_norm.)
 // A row's results do not depend on the tile it lands in, so the order inside an expert is free.
@@ -210,11 +210,11 @@ extern "C" int vwa_moe_route(const MoeRouteParams* p, hipStream_t st) {
 }
 
 extern "C" int vwa_moe_gemm(const MoeGemmParams* p, hipStream_t st) {
-  if (p->max_tiles < 1 || p->N % (p->down ? 16 : 32) || p->K % 128 || p->ldx % 8 || (p->tile != 16 && p->tile != 128) || !p->tiles || !p->order ||
+  if (p->max_tiles < 1 || p->N % (p->down ? 16 : 32) || p->K % 128 || p->ldx % 8 || (p->tile != 16 && p->tile != 128 && p->tile != 256) || !p->tiles || !p->order ||
       (!p->down && !p->wts))
     return -1;
   if ((reinterpret_cast<uintptr_t>(p->x) | reinterpret_cast<uintptr_t>(p->w)) & 15) return -2;
-  if (p->tile == 128) {
+  if (p->tile > 16) {
     if (p->f32) return -3;
     GemmParams q{};
     q.X = reinterpret_cast<const uint16_t*>(p->x);
@@ -230,6 +230,7 @@ extern "C" int vwa_moe_gemm(const MoeGemmParams* p, hipStream_t st) {
     q.g_tiles = p->tiles;
     q.g_order = p->order;
     q.g_max = p->max_tiles;
+    q.g_tile = p->tile;
     q.g_top = p->top;
     q.g_down = p->down;
     q.g_wstride = p->w_expert;

@@ -23,6 +23,12 @@ namespace {
 constexpr size_t kMaxLds = 160 * 1024 - 2048;
 constexpr int kPad = 16;                             // bytes between LDS rows of u: 16 rows hit different banks
 
+// v, with nothing known about it
+VWA_DEVICE int opaque(int v) {
+  asm volatile("" : "+v"(v));
+  return v;
+}
+
 VWA_DEVICE float rcp_sigm(float x) { return __builtin_amdgcn_rcpf(1.f + __expf(-x)); }
 VWA_DEVICE float gelu_tanh(float z) { return z * rcp_sigm(1.5957691216057308f * (z + 0.044715f * z * z * z)); }
 
@@ -51,14 +57,15 @@ template <class T> VWA_DEVICE int u_stride(int bs) { return bs * (int)sizeof(T) 
 template <int PRE>
 struct GateFrags {
   uint4 r[PRE], i[PRE];
-  template <class T> VWA_DEVICE void load(const T* gw, int steps, int s0) {
-    const uint4* wr = reinterpret_cast<const uint4*>(gw) + lane_id();
-    const uint4* wi = wr + (size_t)steps * 64;
+  template <class T> VWA_DEVICE void load(const T* gw, int steps, int s0, int beg = 0, int end = PRE) {
+    const uint4* wr = reinterpret_cast<const uint4*>(gw);
+    const unsigned l = lane_id();                    // (uniform bases: one offset register)
 #pragma unroll
     for (int s = 0; s < PRE; ++s) {
-      const int k = min(s0 + s, steps - 1) * 64;
-      r[s] = wr[k];
-      i[s] = wi[k];
+      if (s < beg || s >= end) continue;
+      const uint4* ws = wr + min(s0 + s, steps - 1) * 64;
+      r[s] = ws[l];
+      i[s] = (ws + steps * 64)[l];
     }
   }
 };
@@ -70,6 +77,7 @@ VWA_DEVICE void gate_products(const char* us, int stride, const T* gw, int steps
 #pragma unroll
   for (int t = 0; t < NT; ++t) ar[t] = ai[t] = f32x4{0.f, 0.f, 0.f, 0.f};
   const char* ua = us + rl * stride + b * 16;
+#pragma unroll 1
   for (int s0 = 0; s0 < steps; s0 += PRE) {
 #pragma unroll
     for (int s = 0; s < PRE; ++s) {
@@ -81,6 +89,7 @@ VWA_DEVICE void gate_products(const char* us, int stride, const T* gw, int steps
           ai[t] = M::mma(a, f.i[s], ai[t]);
         }
       }
+      if (NT == 1 && (s & 1)) __builtin_amdgcn_sched_barrier(0);  // (bounds the operands read ahead)
     }
     if (s0 + PRE < steps) f.load(gw, steps, s0 + PRE);
   }
@@ -118,52 +127,91 @@ VWA_DEVICE float scan_tile(const float (&a)[4], const float (&bb)[4], float carr
   return ta * carry + tb;
 }
 
-// eight channels of the input xp + xb of row r (an input row of this step)
+// row r's inputs (without xb)
 template <class T>
-VWA_DEVICE void input8(const RgLruParams& p, int r, int ch, float (&v)[8]) {
-  ld8(reinterpret_cast<const T*>(p.yx) + (size_t)r * p.ld + p.nb * p.bs + ch, v);
-#pragma unroll
-  for (int e = 0; e < 8; ++e) v[e] += p.xb[ch + e];
+VWA_DEVICE const T* input_at(const RgLruParams& p, int r, int ch) {
+  return reinterpret_cast<const T*>(p.yx) + (size_t)r * p.ld + p.nb * p.bs + ch;
 }
 
-// eight channels of u of row r: j rows of the run lie in front of r in this step, the inputs before them
-// come from the state row st (null: zeros)
-template <class T>
-VWA_DEVICE void conv8(const RgLruParams& p, int r, int j, const float* st, int ch, float (&u)[8]) {
+// four channels of u of row r: j rows of the run lie in front of r in this step, the inputs before them come from
+// the state row st (fresh: zeros).  Both places of a tap are requested, whichever it takes: no load waits for another.
+template <class T, int G>
+VWA_DEVICE void conv4(const RgLruParams& p, int r, int j, const float* st, bool fresh, int ch, float (&u)[4]) {
   const int W = p.nb * p.bs;
+  float xb[4];
+  ld4(p.cb + ch, u);
+  ld4(p.xb + ch, xb);
+#pragma unroll 1
+  for (int k0 = 0; k0 < p.taps; k0 += G) {           // k tokens back
+    float x[G][4], s[G][4], w[G][4];
 #pragma unroll
-  for (int e = 0; e < 8; ++e) u[e] = p.cb[ch + e];
-  for (int k = 0; k < p.taps; ++k) {                 // k tokens back
-    float v[8];
-    if (k <= j) {
-      input8<T>(p, r - k, ch, v);
-    } else if (st) {
-      ld8(st + (size_t)(p.taps - (k - j)) * W + ch, v);
-    } else {
-      break;
+    for (int e = 0; e < G; ++e) {
+      const int k = min(k0 + e, p.taps - 1);
+      ld4(input_at<T>(p, r - min(k, j), ch), x[e]);
+      ld4(st + (size_t)min(p.taps - (k - j), p.taps - 1) * W + ch, s[e]);
+      ld4(p.cw + (size_t)(p.taps - 1 - k) * W + ch, w[e]);
     }
-    const float* w = p.cw + (size_t)(p.taps - 1 - k) * W + ch;
 #pragma unroll
-    for (int e = 0; e < 8; ++e) u[e] += w[e] * v[e];
+    for (int e = 0; e < G; ++e) {
+      if (k0 + e >= p.taps) break;
+#pragma unroll
+      for (int c = 0; c < 4; ++c) u[c] += w[e][c] * (k0 + e <= j ? x[e][c] + xb[c] : fresh ? 0.f : s[e][c]);
+    }
+  }
+}
+
+// the same for rows r .. r + 3, all their taps among the inputs of this step's rows r_min .. r_max
+template <class T>
+VWA_DEVICE void conv_strip(const RgLruParams& p, int r, int r_min, int r_max, int ch, float (&u)[4][4]) {
+  const int W = p.nb * p.bs;
+  float xb[4];
+  ld4(p.xb + ch, xb);
+#pragma unroll
+  for (int i = 0; i < 4; ++i) ld4(p.cb + ch, u[i]);
+#pragma unroll 1
+  for (int k0 = 0; k0 < p.taps; k0 += 4) {
+    float x[7][4], w[4][4];
+#pragma unroll
+    for (int e = 0; e < 7; ++e) ld4(input_at<T>(p, min(max(r + 3 - k0 - e, r_min), r_max), ch), x[e]);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) ld4(p.cw + (size_t)max(p.taps - 1 - k0 - e, 0) * W + ch, w[e]);
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+#pragma unroll
+      for (int c = 0; c < 4; ++c) w[e][c] = k0 + e < p.taps ? w[e][c] : 0.f;
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+#pragma unroll
+        for (int c = 0; c < 4; ++c) u[i][c] += w[e][c] * (x[3 - i + e][c] + xb[c]);
   }
 }
 
 // the last taps - 1 inputs of a run of n rows ending at row r -> its state row (n rows shift the old ones)
 template <class T>
-VWA_DEVICE void save_inputs8(const RgLruParams& p, int r, int n, bool fresh, float* st, int ch) {
+VWA_DEVICE void save_inputs4(const RgLruParams& p, int r, int n, bool fresh, float* st, int ch) {
+  constexpr int G = 3;
   const int W = p.nb * p.bs;
-  for (int i = 1; i < p.taps; ++i) {                 // place i: the input taps - i tokens before the next one
-    const int back = p.taps - 1 - i;                 // rows before r
-    float v[8];
-    if (back < n) {
-      input8<T>(p, r - back, ch, v);
-    } else if (!fresh) {
-      ld8(st + (size_t)(i + n) * W + ch, v);         // (read before a lower place is written)
-    } else {
+  float xb[4];
+  ld4(p.xb + ch, xb);
+#pragma unroll 1
+  for (int i0 = 1; i0 < p.taps; i0 += G) {           // place i: the input taps - i tokens before the next one
+    float x[G][4], s[G][4];
 #pragma unroll
-      for (int e = 0; e < 8; ++e) v[e] = 0.f;
+    for (int e = 0; e < G; ++e) {
+      const int i = min(i0 + e, p.taps - 1), back = p.taps - 1 - i;  // rows before r
+      ld4(input_at<T>(p, r - min(back, n - 1), ch), x[e]);
+      ld4(st + (size_t)min(i + n, p.taps - 1) * W + ch, s[e]);       // (read before a lower place is written)
     }
-    st8(st + (size_t)i * W + ch, v);
+#pragma unroll
+    for (int e = 0; e < G; ++e) {
+      const int i = i0 + e;
+      if (i >= p.taps) break;
+#pragma unroll
+      for (int c = 0; c < 4; ++c) x[e][c] = p.taps - 1 - i < n ? x[e][c] + xb[c] : fresh ? 0.f : s[e][c];
+      st4(st + (size_t)i * W + ch, x[e]);
+    }
   }
 }
 
@@ -172,79 +220,81 @@ VWA_DEVICE void save_inputs8(const RgLruParams& p, int r, int n, bool fresh, flo
 // their ends (other runs' rows count as inert).
 template <class T>
 __global__ __launch_bounds__(1024) void rglru_rows_kernel(RgLruParams p) {
+  constexpr int PRE = 8;
   extern __shared__ __attribute__((aligned(16))) char us[];
-  __shared__ int s_first[64], s_len[64];             // of the row's run: first row; rows (at its last row, else 0)
+  // of a row: its sequence; its run's first row (-1: inert); its run's rows (at the run's last row, else 0); whether
+  // tokens precede it / its run
+  __shared__ int s_seq[64], s_first[64], s_len[64], s_old[64], s_run_old[64];
   const int blk = blockIdx.x, lo = blockIdx.y * 16, bs = p.bs, c0 = blk * bs;
-  const int tid = threadIdx.x, nthr = blockDim.x, lane = lane_id(), w = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int rl = lane & 15, g = lane >> 4, stride = u_stride<T>(bs), steps = bs / MM<T>::KS, waves = nthr >> 6;
+  const int tid0 = threadIdx.x, nthr = blockDim.x, w = __builtin_amdgcn_readfirstlane(tid0 >> 6);
+  const int stride = u_stride<T>(bs), steps = bs / MM<T>::KS, tiles = bs / 16, waves = nthr >> 6;
   T* out = reinterpret_cast<T*>(p.out);
-  const T* gw0 = reinterpret_cast<const T*>(p.gw) + (size_t)blk * (bs / 16) * 32 * bs;
-  GateFrags<4> f;                                    // (requested ahead of everything that waits)
-  f.load(gw0 + (size_t)w * 32 * bs, steps, 0);
-  if (tid < 64) {                                    // (one wave: runs from the rows' ids)
-    const int r = tid;
-    const bool in = r < p.rows;
-    const bool live = in && p.slots[r] >= 0;
-    const int seq = live ? p.seq_ids[r] : -1 - r;
+  const T* gw0 = reinterpret_cast<const T*>(p.gw) + (size_t)blk * tiles * 32 * bs;
+  if (tid0 < 64) {                                   // (one wave: runs from the rows' ids)
+    const int r = tid0, rc = min(r, p.rows - 1), id = p.seq_ids[rc], old = p.positions[rc] > 0;
+    const bool live = p.slots[rc] >= 0 && r < p.rows;
+    const int seq = live ? id : -1 - r;
     const int before = __shfl_up(seq, 1, 64), after = __shfl_down(seq, 1, 64);
     const unsigned long long heads = __ballot(live && (r == 0 || before != seq));
     const unsigned long long mine = heads & ((2ull << r) - 1ull);
     const int first = live && mine ? 63 - __builtin_clzll(mine) : -1;
+    s_seq[r] = max(seq, 0);
     s_first[r] = first;
     s_len[r] = live && (r == 63 || after != seq) ? r + 1 - first : 0;
+    s_old[r] = old;
+    s_run_old[r] = __shfl(old, max(first, 0), 64);
   }
   __syncthreads();
-  const int oct = bs / 8, hi = min(lo + 16, p.rows);
+  const int quads = bs / 4, hi = min(lo + 16, p.rows);
   auto owned = [&](int r) { return s_first[r] >= lo && s_first[r] < hi; };
+  auto state_of = [&](int r) { return p.state + (size_t)s_seq[r] * p.state_ld; };
+#pragma unroll 1
   for (int r0 = lo; r0 < p.rows; r0 += 16) {
     if (r0 > lo && !owned(r0)) break;                // (a run that goes past the tile owns the next row)
     const int n = min(16, p.rows - r0);
-    for (int x = tid; x < 16 * oct; x += nthr) {
-      const int i = x / oct, ch = (x % oct) * 8, r = r0 + i;
-      float u[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-      if (i < n && owned(r)) {
-        const int fr = s_first[r];
-        const float* st = p.positions[fr] > 0 ? p.state + (size_t)p.seq_ids[r] * p.state_ld : nullptr;
-        conv8<T>(p, r, r - fr, st, c0 + ch, u);
-      }
-      st8(reinterpret_cast<T*>(us + i * stride) + ch, u);
-    }
-    __syncthreads();                                 // (every read of the old inputs is done as well)
-    for (int x = tid; x < n * oct; x += nthr) {
-      const int i = x / oct, r = r0 + i, len = s_len[r];
-      if (len == 0 || !owned(r)) continue;
-      save_inputs8<T>(p, r, len, p.positions[s_first[r]] == 0, p.state + (size_t)p.seq_ids[r] * p.state_ld, c0 + (x % oct) * 8);
-    }
-    for (int ct = w; ct < bs / 16; ct += waves) {
+#pragma unroll 1
+    for (int t0 = 0; t0 < tiles; t0 += waves) {
+      // (mostly the only pass: addresses are formed where they are used, not kept across passes)
+      const int tid = opaque(tid0), lane = tid & 63, rl = lane & 15, g = lane >> 4;
+      const int ct = min(t0 + w, tiles - 1), ch = c0 + ct * 16 + rl;
+      // ---- requested ahead of the convolution
       const T* gw = gw0 + (size_t)ct * 32 * bs;
-      const int ch = c0 + ct * 16 + rl;
+      GateFrags<PRE> f;
+      f.load(gw, steps, 0, 0, PRE / 2);
       const float rb = p.rb[ch], ib = p.ib[ch], dec = p.decay[ch], yb = p.yb[ch];
-      float y[4], s_in[4];
+      T yv[4];
+      float s_in[4];
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {                  // (requested ahead of the products)
-        const int li = min(4 * g + i, n - 1), r = r0 + li;
-        y[i] = ldv(reinterpret_cast<const T*>(p.yx) + (size_t)r * p.ld + ch);
-        const bool head = owned(r) && (s_first[r] == r || li == 0) && p.positions[r] > 0;
-        s_in[i] = head ? p.state[(size_t)p.seq_ids[r] * p.state_ld + ch] : 0.f;
+      for (int i = 0; i < 4; ++i) {
+        const int r = r0 + min(4 * g + i, n - 1);
+        yv[i] = reinterpret_cast<const T*>(p.yx)[(size_t)r * p.ld + ch];
+        s_in[i] = state_of(r)[ch];
       }
+      if (t0 == 0) {
+#pragma unroll 1
+        for (int x = tid; x < 16 * quads; x += nthr) {
+          const int i = x / quads, c = (x % quads) * 4, r = r0 + i;
+          float u[4] = {0.f, 0.f, 0.f, 0.f};
+          if (i < n && owned(r)) conv4<T, 4>(p, r, r - s_first[r], state_of(r), !s_run_old[r], c0 + c, u);
+          st4(reinterpret_cast<T*>(us + i * stride) + c, u);
+        }
+      }
+      __builtin_amdgcn_sched_barrier(0);             // (the convolution's registers are free from here)
+      f.load(gw, steps, 0, PRE / 2, PRE);
+      __syncthreads();                               // (every read of the old inputs is done as well)
+      if (t0 + w >= tiles) continue;
       f32x4 ar[1], ai[1];
-      if (r0 > lo || ct != w) f.load(gw, steps, 0);
-      gate_products<T, 1, 4>(us, stride, gw, steps, f, ar, ai);
+      gate_products<T, 1, PRE>(us, stride, gw, steps, f, ar, ai);
       float a[4], b[4], s[4], A, B;
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        const int li = 4 * g + i, r = r0 + li;
-        a[i] = b[i] = 0.f;
-        if (li < n && owned(r)) {
-          const float u = ldv(reinterpret_cast<const T*>(us + li * stride) + ct * 16 + rl);
-          const Step st = lru_step(ar[0][i] + rb, ai[0][i] + ib, dec, u);
-          a[i] = st.a;
-          b[i] = st.b;
-          if (s_first[r] == r || li == 0) {          // (a run that goes on from the rows before: its state was saved)
-            b[i] += st.a * s_in[i];
-            a[i] = 0.f;
-          }
-        }
+        const int li = 4 * g + i, r = r0 + min(li, n - 1);
+        const bool mine = li < n && owned(r), head = s_first[r] == r || li == 0;
+        const float u = ldv(reinterpret_cast<const T*>(us + li * stride) + ct * 16 + rl);
+        const Step st = lru_step(ar[0][i] + rb, ai[0][i] + ib, dec, u);
+        // (a run that goes on from the rows before: its state was saved)
+        b[i] = !mine ? 0.f : head && s_old[r] ? st.b + st.a * s_in[i] : st.b;
+        a[i] = mine && !head ? st.a : 0.f;
       }
       scan_tile(a, b, 0.f, s, A, B);
 #pragma unroll
@@ -252,12 +302,17 @@ __global__ __launch_bounds__(1024) void rglru_rows_kernel(RgLruParams p) {
         const int li = 4 * g + i, r = r0 + li;
         if (li >= n) continue;
         if (owned(r)) {
-          stv(out + (size_t)r * p.ldo + ch, s[i] * gelu_tanh(y[i] + yb));
-          if (s_len[r] > 0 || li == n - 1) p.state[(size_t)p.seq_ids[r] * p.state_ld + ch] = s[i];
+          stv(out + (size_t)r * p.ldo + ch, s[i] * gelu_tanh(ldv(&yv[i]) + yb));
+          if (s_len[r] > 0 || li == n - 1) state_of(r)[ch] = s[i];
         } else if (s_first[r] < 0 && r0 == lo) {
           stv(out + (size_t)r * p.ldo + ch, 0.f);    // inert row of a padded step
         }
       }
+    }
+#pragma unroll 1
+    for (int x = opaque(tid0); x < n * quads; x += nthr) {
+      const int r = r0 + x / quads, len = s_len[r];
+      if (len > 0 && owned(r)) save_inputs4<T>(p, r, len, !s_run_old[r], state_of(r), c0 + (x % quads) * 4);
     }
     __syncthreads();                                 // u is overwritten; saved states are read by the next rows
   }
@@ -268,7 +323,7 @@ constexpr int kScanWaves = 8;
 
 // Pass 1 forms u by the convolution and leaves it in p.u for pass 2.
 template <class T, int PASS, int NT>
-__global__ __launch_bounds__(kScanWaves * 64) void rglru_scan_kernel(RgLruParams p) {
+__global__ __launch_bounds__(kScanWaves * 64, NT == 4 ? 4 : 2) void rglru_scan_kernel(RgLruParams p) {
   constexpr int RT = NT * 16;
   extern __shared__ __attribute__((aligned(16))) char us[];
   const int ck = blockIdx.x, blk = blockIdx.y, bs = p.bs, W = p.nb * bs, c0 = blk * bs;
@@ -280,8 +335,8 @@ __global__ __launch_bounds__(kScanWaves * 64) void rglru_scan_kernel(RgLruParams
   const bool active = ct < bs / 16;
   const int ch = c0 + (active ? ct : 0) * 16 + rl;
   const T* gw = reinterpret_cast<const T*>(p.gw) + (size_t)(blk * (bs / 16) + (active ? ct : 0)) * 32 * bs;
-  GateFrags<8> f;
-  f.load(gw, steps, 0);
+  constexpr int PRE = 4;
+  GateFrags<PRE> f;
   const int pos0 = p.positions[run0];
   float* st = p.state + (size_t)p.seq_ids[row0] * p.state_ld;
   const float rb = p.rb[ch], ib = p.ib[ch], dec = p.decay[ch], yb = p.yb[ch];
@@ -301,29 +356,57 @@ __global__ __launch_bounds__(kScanWaves * 64) void rglru_scan_kernel(RgLruParams
       for (int e = 0; e < 8; ++e) carry = k + e < ck ? ca[e] * carry + cb[e] : carry;
     }
   }
-  const int oct = bs / 8;
+  const int quads = bs / 4;
   T* ug = reinterpret_cast<T*>(p.u);
-  for (int r0 = 0; r0 < n; r0 += RT) {
-    const int m = min(RT, n - r0);
+  for (int r0 = 0; r0 < (NT == 4 ? 1 : n); r0 += RT) {   // (NT = 4: a chunk is one tile)
+    const int m = min(RT, n - r0);                   // (rows past the chunk repeat its last one; their steps are dropped)
+    T yv[PASS == 2 ? NT : 1][4];
+    if constexpr (PASS == 2) {
+      const int oct = bs / 8;
+      const T* yr = reinterpret_cast<const T*>(p.yx) + (size_t)(row0 + r0) * p.ld;
+#pragma unroll
+      for (int t = 0; t < NT; ++t)
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          yv[t][i] = yr[(unsigned)(min(t * 16 + 4 * g + i, m - 1) * p.ld + ch)];
+  #pragma unroll 1
     for (int x = tid; x < RT * oct; x += kScanWaves * 64) {
-      const int i = x / oct, c = (x % oct) * 8, r = row0 + r0 + i;
-      T* d = reinterpret_cast<T*>(us + i * stride) + c;
-      if (PASS == 2) {                               // (rows past the chunk repeat its last one; their steps are dropped)
+        const int i = x / oct, c = (x % oct) * 8;
+        T* d = reinterpret_cast<T*>(us + i * stride) + c;
         const T* src = ug + (size_t)(row0 + r0 + min(i, m - 1)) * W + c0 + c;
 #pragma unroll
         for (int e = 0; e < (int)sizeof(T) / 2; ++e) reinterpret_cast<uint4*>(d)[e] = reinterpret_cast<const uint4*>(src)[e];
-        continue;
       }
-      float u[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-      if (i < m) conv8<T>(p, r, r - run0, pos0 > 0 ? st : nullptr, c0 + c, u);
-      st8(d, u);
-      if (i < m && blockIdx.z == 0) st8(ug + (size_t)r * W + c0 + c, u);
+    } else {
+  #pragma unroll 1
+    for (int x = tid; x < RT / 4 * quads; x += kScanWaves * 64) {
+        const int i0 = x / quads * 4, c = (x % quads) * 4, r = row0 + r0 + i0, last = row0 + r0 + m - 1;
+        float u[4][4];
+        if (r - run0 >= p.taps - 1) {
+          conv_strip<T>(p, r, run0, last, c0 + c, u);
+        } else {
+#pragma unroll 1
+          for (int i = 0; i < 4; ++i) {
+            float v[4];
+            conv4<T, 4>(p, min(r + i, last), min(r + i, last) - run0, st, pos0 <= 0, c0 + c, v);
+            st4(reinterpret_cast<T*>(us + (i0 + i) * stride) + c, v);
+            if (i0 + i < m && blockIdx.z == 0) st4(ug + (size_t)(r + i) * W + c0 + c, v);
+          }
+          continue;
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          st4(reinterpret_cast<T*>(us + (i0 + i) * stride) + c, u[i]);
+          if (i0 + i < m && blockIdx.z == 0) st4(ug + (size_t)(r + i) * W + c0 + c, u[i]);
+        }
+      }
     }
+    __builtin_amdgcn_sched_barrier(0);               // (the convolution's registers are free from here)
+    f.load(gw, steps, 0);
     __syncthreads();
     if (active) {
       f32x4 ar[NT], ai[NT];
-      if (r0 > 0) f.load(gw, steps, 0);
-      gate_products<T, NT, 8>(us, stride, gw, steps, f, ar, ai);
+      gate_products<T, NT, PRE>(us, stride, gw, steps, f, ar, ai);
 #pragma unroll
       for (int t = 0; t < NT; ++t) {
         float a[4], b[4], s[4], A, B;
@@ -342,12 +425,13 @@ __global__ __launch_bounds__(kScanWaves * 64) void rglru_scan_kernel(RgLruParams
         } else {
 #pragma unroll
           for (int i = 0; i < 4; ++i) {
-            const int li = t * 16 + 4 * g + i, r = row0 + r0 + li;
+            const int li = t * 16 + 4 * g + i;
             if (li >= m) continue;
-            const float y = gelu_tanh(ldv(reinterpret_cast<const T*>(p.yx) + (size_t)r * p.ld + ch) + yb);
-            stv(reinterpret_cast<T*>(p.out) + (size_t)r * p.ldo + ch, s[i] * y);
+            const float y = gelu_tanh(ldv(&yv[t][i]) + yb);
+            stv(reinterpret_cast<T*>(p.out) + (size_t)(row0 + r0) * p.ldo + (unsigned)(li * p.ldo + ch), s[i] * y);
           }
         }
+        __builtin_amdgcn_sched_barrier(0);           // (one tile's registers at a time)
       }
     }
     __syncthreads();
@@ -366,11 +450,11 @@ __global__ __launch_bounds__(kScanWaves * 64) void rglru_scan_kernel(RgLruParams
 // the runs' last inputs (after the scan: its first chunks read the old ones)
 template <class T>
 __global__ __launch_bounds__(256) void rglru_inputs_kernel(RgLruParams p) {
-  const int ck = blockIdx.y, ch = (blockIdx.x * 256 + threadIdx.x) * 8;
+  const int ck = blockIdx.y, ch = (blockIdx.x * 256 + threadIdx.x) * 4;
   const int row0 = p.chunks[4 * ck], n = p.chunks[4 * ck + 1], idx = p.chunks[4 * ck + 2], cnt = p.chunks[4 * ck + 3];
   if (idx != cnt - 1 || ch >= p.nb * p.bs) return;
   const int run0 = idx > 0 ? p.chunks[4 * (ck - idx)] : row0;
-  save_inputs8<T>(p, row0 + n - 1, row0 + n - run0, p.positions[run0] == 0, p.state + (size_t)p.seq_ids[row0] * p.state_ld, ch);
+  save_inputs4<T>(p, row0 + n - 1, row0 + n - run0, p.positions[run0] == 0, p.state + (size_t)p.seq_ids[row0] * p.state_ld, ch);
 }
 
 int check(const RgLruParams& p) {
@@ -398,7 +482,7 @@ int launch_scan_nt(const RgLruParams& p, hipStream_t st) {
   hipLaunchKernelGGL((rglru_scan_kernel<T, 1, NT>), grid, block, lds, st, p);
   hipLaunchKernelGGL((rglru_scan_kernel<T, 2, NT>), grid, block, lds, st, p);
   if (p.taps > 1)
-    hipLaunchKernelGGL((rglru_inputs_kernel<T>), dim3((p.nb * p.bs / 8 + 255) / 256, p.n_chunks), dim3(256), 0, st, p);
+    hipLaunchKernelGGL((rglru_inputs_kernel<T>), dim3((p.nb * p.bs / 4 + 255) / 256, p.n_chunks), dim3(256), 0, st, p);
   return (int)hipGetLastError();
 }
 

@@ -113,8 +113,8 @@ VWA_DEVICE void w4(const float* w, int c, int D, float (&v)[4]) {
   for (int j = 0; j < 4; ++j) v[j] = c + j < D ? w[min(c + j, D - 1)] : 0.f;
 }
 
-// one workgroup per row: x += norm(sum of the branch rows) * w1; h = norm(x) * w2.  Loads of the branch
-// and of the residual are in flight together.
+// one workgroup per row: x += norm(sum of the branch rows) * w1; h = norm(x) * w2.  Loads of the branch,
+// of the residual and of the weights are in flight together.
 template <class T, int STEPS>
 __global__ __launch_bounds__(256) void add_norm_kernel(float* __restrict__ x, int ldx, const T* __restrict__ br, int ldb,
                                                        int n_parts, const float* __restrict__ w1, const float* __restrict__ w2,
@@ -123,21 +123,38 @@ __global__ __launch_bounds__(256) void add_norm_kernel(float* __restrict__ x, in
   float* xr = x + (size_t)blockIdx.x * ldx;
   const T* b = br + (size_t)blockIdx.x * n_parts * ldb;
   const int last = (D - 1) & ~3;
-  float v[STEPS][4], xs[STEPS][4];
+  float v[STEPS][4], xs[STEPS][4], wa[STEPS][4], wb[STEPS][4];
 #pragma unroll
   for (int i = 0; i < STEPS; ++i) {
     const int c = min((i * 256 + (int)threadIdx.x) * 4, last);
     ld4(b + c, v[i]);
     ld4(xr + c, xs[i]);
   }
-  for (int k = 1; k < n_parts; ++k)
+  auto weights = [&](const float* w, float (&o)[STEPS][4]) {
+    if (D % 4 == 0) {
 #pragma unroll
-    for (int i = 0; i < STEPS; ++i) {
-      float u[4];
-      ld4(b + (size_t)k * ldb + min((i * 256 + (int)threadIdx.x) * 4, last), u);
+      for (int i = 0; i < STEPS; ++i) ld4(w + min((i * 256 + (int)threadIdx.x) * 4, last), o[i]);
+    } else {
 #pragma unroll
-      for (int j = 0; j < 4; ++j) v[i][j] += u[j];
+      for (int i = 0; i < STEPS; ++i) w4(w, (i * 256 + (int)threadIdx.x) * 4, D, o[i]);
     }
+  };
+  weights(w1, wa);
+  weights(w2 ? w2 : w1, wb);
+  for (int k = 1; k < n_parts; k += 3) {
+    float u[3][STEPS][4];
+#pragma unroll
+    for (int e = 0; e < 3; ++e)
+#pragma unroll
+      for (int i = 0; i < STEPS; ++i)
+        ld4(b + (size_t)min(k + e, n_parts - 1) * ldb + min((i * 256 + (int)threadIdx.x) * 4, last), u[e][i]);
+#pragma unroll
+    for (int e = 0; e < 3; ++e)
+#pragma unroll
+      for (int i = 0; i < STEPS; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) v[i][j] += k + e < n_parts ? u[e][i][j] : 0.f;
+  }
 #pragma unroll
   for (int i = 0; i < STEPS; ++i)
 #pragma unroll
@@ -147,10 +164,8 @@ __global__ __launch_bounds__(256) void add_norm_kernel(float* __restrict__ x, in
 #pragma unroll
   for (int i = 0; i < STEPS; ++i) {
     const int c = (i * 256 + threadIdx.x) * 4;
-    float w[4];
-    w4(w1, c, D, w);
 #pragma unroll
-    for (int j = 0; j < 4; ++j) xs[i][j] += c + j < D ? (v[i][j] - sb.x) * sb.y * w[j] : 0.f;
+    for (int j = 0; j < 4; ++j) xs[i][j] += c + j < D ? (v[i][j] - sb.x) * sb.y * wa[i][j] : 0.f;
     if (c < D) st4(xr + c, xs[i]);  // (columns past D of the last quad stay zero)
   }
   if (!w2) return;
@@ -160,10 +175,9 @@ __global__ __launch_bounds__(256) void add_norm_kernel(float* __restrict__ x, in
   for (int i = 0; i < STEPS; ++i) {
     const int c = (i * 256 + threadIdx.x) * 4;
     if (c >= D) continue;
-    float w[4], o[4];
-    w4(w2, c, D, w);
+    float o[4];
 #pragma unroll
-    for (int j = 0; j < 4; ++j) o[j] = c + j < D ? (xs[i][j] - sx.x) * sx.y * w[j] : 0.f;
+    for (int j = 0; j < 4; ++j) o[j] = c + j < D ? (xs[i][j] - sx.x) * sx.y * wb[i][j] : 0.f;
     st4(hr + c, o);
   }
   for (int c = ((D + 3) & ~3) + threadIdx.x; c < Dpad; c += 256) stv(hr + c, 0.f);

@@ -191,9 +191,9 @@ struct GemmParams {
   int n_split; uint16_t* Y2; int ldy2;
   // grouped launch (tiles != null; vwa_gemm_grouped): every 128-row block is one tile of (row, expert) pairs
   // of one expert -- tiles [1 + 3 g_max] int32: count, then (expert, first place, pairs); order: place -> pair.
-  // X row of a place: pair / top (g_down: the place itself); Y row: the place (g_down: the pair); rstd: per
+  // g_tile: most pairs of a tile (128 or 256); X row of a place: pair / top (g_down: the place itself); Y row: the place (g_down: the pair); rstd: per
   // PAIR; W + expert * g_wstride
-  const int* g_tiles; const int* g_order; int g_max, g_top, g_down; int64_t g_wstride;
+  const int* g_tiles; const int* g_order; int g_max, g_top, g_down, g_tile; int64_t g_wstride;
 };
 
 struct FlashAttnParams {

@@ -361,8 +361,9 @@ MOE = [(8, 2, 40, 72), (5, 1, 128, 130), (16, 4, 96, 256), (3, 3, 64, 100), (40,
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("E,top,ff,d", MOE)
 @pytest.mark.parametrize("M", [1, 7, 16, 40, 64, 150, 700])
-def test_moe(dtype, E, top, ff, d, M):
-    """Every row's experts, their scores on the input side, the tables' bounds; some rows inert."""
+def test_moe(dtype, E, top, ff, d, M, monkeypatch):
+    """Every row's experts, their scores on the input side, the tables' bounds; some rows inert.  Every tile size
+    that could serve the rows."""
     K, F, N = up(d, 128), up(ff, 128), up(d, 16)
     h = rnd(M, d, seed=1, dtype=dtype)
     router = rnd(E, d, seed=2, std=2 * d ** -0.5, dtype=dtype)
@@ -391,16 +392,18 @@ def test_moe(dtype, E, top, ff, d, M):
     slots = torch.zeros(M, dtype=torch.int64, device=DEV)
     inert = [t for t in (2, M - 1) if M > 4]
     slots[inert] = -1
-    bufs = ops.moe_buffers(M, [(E, top, F)], dtype, DEV)
-    for _ in range(2):  # (the tables are used again)
-        out = torch.full((M * top, N), 7.0, dtype=dtype, device=DEV)
-        ops.moe(hp.to(DEV), p, slots=slots, bufs=bufs, out=out)
-        got = out.cpu().view(M, top, N)
-        live = [t for t in range(M) if t not in inert]
-        # (equal scores may come in either order: compare the sum, and each where the order is certain)
-        assert rel(got[live][..., :d].double().sum(1), want[live].sum(1)) < (1e-5 if dtype == F32 else 2e-2)
-        assert (got[inert] == 7.0).all()               # inert rows choose nothing
-        assert int(bufs.ticket) == 0
+    for tile in [t for t in mixers.MOE_TILES if t == 16 or (dtype == BF16 and M >= 40)]:
+        monkeypatch.setattr(mixers, "moe_tile", lambda *_: tile)  # noqa: B023
+        bufs = ops.moe_buffers(M, [(E, top, F)], dtype, DEV)
+        for _ in range(2):  # (the tables are used again)
+            out = torch.full((M * top, N), 7.0, dtype=dtype, device=DEV)
+            ops.moe(hp.to(DEV), p, slots=slots, bufs=bufs, out=out)
+            got = out.cpu().view(M, top, N)
+            live = [t for t in range(M) if t not in inert]
+            # (equal scores may come in either order: compare the sum, and each where the order is certain)
+            assert rel(got[live][..., :d].double().sum(1), want[live].sum(1)) < (1e-5 if dtype == F32 else 2e-2)
+            assert (got[inert] == 7.0).all()           # inert rows choose nothing
+            assert int(bufs.ticket) == 0
 
 
 # ----------------------------------------------------------------------------- the model through the engine
