@@ -385,7 +385,7 @@ void moe_gemm(Tensor x, Tensor w, int64_t rows, int64_t top, bool down, Tensor w
   p.order = i32p(order, places, "order");
   p.tile = (int)tile;
   p.x_rows = (int)(down ? places : rows);
-  if (tile > 16) {
+  if (tile > 32) {
     check_aligned(y, "y");
     TORCH_CHECK(y.stride(0) % 8 == 0, "y rows must be 16-byte aligned");
   }

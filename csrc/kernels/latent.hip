@@ -374,17 +374,17 @@ __global__ __launch_bounds__(256) void latent_attn_f32_kernel(LatentAttnParams p
 }
 
 // ------------------------------------------------------------------------------------------ merge + value projection
-// A workgroup per (head, 16 rows, 64 value columns): 4 column tiles x 2 halves of the latent.  The weights' first
+// A workgroup per (head, rb <= 16 rows, 64 value columns): 4 column tiles x 2 halves of the latent.  The weights' first
 // fragments are requested ahead of the merge; few rows spread a merge over the threads by chunks as well.
 constexpr int kOutThreads = 512, kOutPre = 8;
 template <class T>
 size_t out_lds(int rank_p, int nch) { return 16 * ((size_t)rank_p * sizeof(T) + 16) + 16 * (size_t)nch * 4 + kOutThreads * 16; }
 
 template <class T>
-__global__ __launch_bounds__(kOutThreads) void latent_out_kernel(LatentOutParams p) {
+__global__ __launch_bounds__(kOutThreads) void latent_out_kernel(LatentOutParams p, int rb) {
   using M = MM<T>;
   extern __shared__ __attribute__((aligned(16))) char smem[];
-  const int h = blockIdx.x, r0 = blockIdx.y * 16, tid = threadIdx.x, nr = min(16, p.rows - r0);
+  const int h = blockIdx.x, r0 = blockIdx.y * rb, tid = threadIdx.x, nr = min(rb, p.rows - r0);
   const int lane = lane_id(), w = __builtin_amdgcn_readfirstlane(tid >> 6), rl = lane & 15, g = lane >> 4;
   const int stride = p.rank_p * (int)sizeof(T) + 16;
   float4* red = reinterpret_cast<float4*>(smem + 16 * stride);               // [512]
@@ -582,8 +582,11 @@ extern "C" int vwa_latent_out(const LatentOutParams* p, hipStream_t st) {
   if (p->rows < 1 || p->H < 1 || p->vd % 16 || p->rank_p % 32 || p->nch < 1 || !p->part || !p->stat || !p->sink) return -1;
   const size_t lds = p->f32 ? out_lds<float>(p->rank_p, p->nch) : out_lds<u16>(p->rank_p, p->nch);
   if (lds > kMaxLds) return -10;
-  const dim3 grid(p->H, (p->rows + 15) / 16, (p->vd + 63) / 64), block(kOutThreads);
-  if (p->f32) hipLaunchKernelGGL((latent_out_kernel<float>), grid, block, lds, st, *p);
-  else hipLaunchKernelGGL((latent_out_kernel<u16>), grid, block, lds, st, *p);
+  // (the merges are the work: fewer rows each while the launch is short of workgroups)
+  int rb = 16;
+  while (rb > 2 && p->H * ((p->vd + 63) / 64) * ((p->rows + rb - 1) / rb) < 256) rb /= 2;
+  const dim3 grid(p->H, (p->rows + rb - 1) / rb, (p->vd + 63) / 64), block(kOutThreads);
+  if (p->f32) hipLaunchKernelGGL((latent_out_kernel<float>), grid, block, lds, st, *p, rb);
+  else hipLaunchKernelGGL((latent_out_kernel<u16>), grid, block, lds, st, *p, rb);
   return (int)hipGetLastError();
 }

@@ -109,7 +109,7 @@ struct MoeRouteParams {
   int rows, E, top, f32;
   const int64_t* slots;             // rows with slot < 0 choose nothing
   float* wts; int* ids;             // [rows * top]: score and expert of every pair (inert: -1)
-  int tile;                         // pairs per tile (16, 128 or 256)
+  int tile;                         // pairs per tile (16, 32, 128 or 256)
   int max_tiles;
   int* tiles;                       // [1 + 3 * max_tiles]: count, then (expert, first sorted place, pairs)
   int* order;                       // [max_tiles * tile]: sorted place -> pair
@@ -122,7 +122,7 @@ struct MoeGemmParams {
   const void* w; int64_t w_expert;  // elements per expert; pre-tiled order (ops.mixers.tile_weight)
   int N, K, top, f32, down;         // N: rows of one expert's matrix (gate / up interleaved by 16: 2 x ff)
   const float* wts;
-  const int* tiles; const int* order; int max_tiles, tile;   // tile: 16, or 128 / 256 (bf16: the LDS-tiled GEMM)
+  const int* tiles; const int* order; int max_tiles, tile;   // tile: 16, 32, or 128 / 256 (bf16: the LDS-tiled GEMM)
   int x_rows;                       // rows of x
   void* y; int ldy;
 };

@@ -2,7 +2,7 @@
 //
 //  moe_route : sigmoid router scores (MFMA, f32 sums), the best ``top`` experts of every row, and the pairs
 //              (row, choice) grouped by expert into tiles of at most ``tile`` pairs -- by the last workgroup
-//  moe_gemm  : the experts' matrices over such a tile (here tiles of 16 pairs, streaming; tiles of 128 or 256
+//  moe_gemm  : the experts' matrices over such a tile (here tiles of 16 or 32 pairs, streaming; of 128 or 256
 //              go to gemm.hip's grouped launch).  First launch: the tile's rows times gate and up, scaled
 //              by the pair's score ahead of the activation (w (W h) = W (w h)); second: down, one row per pair.
 //              (The pairs of a row are added, in the order of its choices, by add_norm.)
@@ -25,10 +25,18 @@ VWA_DEVICE void group_pairs(const MoeRouteParams& p, const int* ids) {
   for (int e = tid; e < p.E; e += kRouteThreads) cnt[e] = 0;
   __syncthreads();
   auto id_of = [&](int i) { return __hip_atomic_load(const_cast<int*>(ids) + i, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT); };
-  for (int i = tid; i < P; i += kRouteThreads) {
-    const int e = id_of(i);
-    if (e >= 0) atomicAdd(&cnt[e], 1);
-  }
+  constexpr int B = 8;                               // ids whose loads are in flight together
+  auto for_pairs = [&](auto&& fn) {
+    for (int i0 = tid; i0 < P; i0 += B * kRouteThreads) {
+      int e[B];
+#pragma unroll
+      for (int k = 0; k < B; ++k) e[k] = id_of(min(i0 + k * kRouteThreads, P - 1));
+#pragma unroll
+      for (int k = 0; k < B; ++k)
+        if (i0 + k * kRouteThreads < P && e[k] >= 0) fn(i0 + k * kRouteThreads, e[k]);
+    }
+  };
+  for_pairs([&](int, int e) { atomicAdd(&cnt[e], 1); });
   __syncthreads();
   if (tid < 64) {                                    // exclusive prefix of the experts' tile counts
     int base = 0;
@@ -59,10 +67,7 @@ VWA_DEVICE void group_pairs(const MoeRouteParams& p, const int* ids) {
   __syncthreads();
   for (int e = tid; e < p.E; e += kRouteThreads) cnt[e] = first[e] * p.tile;
   __syncthreads();
-  for (int i = tid; i < P; i += kRouteThreads) {
-    const int e = id_of(i);
-    if (e >= 0) p.order[atomicAdd(&cnt[e], 1)] = i;
-  }
+  for_pairs([&](int i, int e) { p.order[atomicAdd(&cnt[e], 1)] = i; });
 }
 
 template <class T>
@@ -143,52 +148,86 @@ __global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(MoeRouteParams
   group_pairs(p, p.ids);
 }
 
-// ------------------------------------------------------------------------------------------ small tiles (16 pairs)
-// A workgroup per (tile, 16 features | 16 columns); its 4 waves split K, the sums meet in LDS.
-template <class T, bool DOWN>
-__global__ __launch_bounds__(256) void moe_gemm16_kernel(MoeGemmParams p) {
+// ------------------------------------------------------------------------------------------ small tiles (16 NP pairs)
+// A workgroup per (tile, NU x 16 features | columns); its 4 waves split K, the sums meet in LDS.
+template <class T, bool DOWN, int NP, int NU>
+__global__ __launch_bounds__(256) void moe_small_kernel(MoeGemmParams p) {
   using M = MM<T>;
-  constexpr int NA = DOWN ? 1 : 2;
-  __shared__ float red[4][NA][64][4];
+  constexpr int NA = DOWN ? 1 : 2;                   // 16-row tiles of the matrix per unit
+  __shared__ float red[4][NP][NU][NA][64][4];
   const int tile = blockIdx.y;
   if (tile >= p.tiles[0]) return;
   const int e = p.tiles[1 + 3 * tile], place = p.tiles[2 + 3 * tile], n = p.tiles[3 + 3 * tile];
   const int lane = lane_id(), w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), rl = lane & 15, g = lane >> 4;
-  const int KG = p.K / (16 * M::EPL), unit = blockIdx.x;
-  const int src = place + min(rl, n - 1);
-  const T* x = reinterpret_cast<const T*>(p.x) + (size_t)(DOWN ? src : p.order[src] / p.top) * p.ldx + 4 * M::EPL * g;
-  const uint4* wp = reinterpret_cast<const uint4*>(reinterpret_cast<const T*>(p.w) + e * p.w_expert) + (size_t)unit * NA * KG * 256 + lane;
-  f32x4 acc[NA] = {};
+  const int KG = p.K / (16 * M::EPL), units = p.N / (16 * NA), unit0 = blockIdx.x * NU;
+  const T* x[NP];
+#pragma unroll
+  for (int t = 0; t < NP; ++t) {
+    const int src = place + min(16 * t + rl, n - 1);
+    x[t] = reinterpret_cast<const T*>(p.x) + (size_t)(DOWN ? src : p.order[src] / p.top) * p.ldx + 4 * M::EPL * g;
+  }
+  const uint4* wp[NU];                               // (a unit past the matrix repeats its last one)
+#pragma unroll
+  for (int u = 0; u < NU; ++u)
+    wp[u] = reinterpret_cast<const uint4*>(reinterpret_cast<const T*>(p.w) + e * p.w_expert) + (size_t)min(unit0 + u, units - 1) * NA * KG * 256;
+  f32x4 acc[NP][NU][NA] = {};
   for (int kg = w; kg < KG; kg += 4) {
-    uint4 f[NA][4], a[4];
+    uint4 f[NU][NA][4], a[NP][4];
 #pragma unroll
     for (int s = 0; s < 4; ++s) {
 #pragma unroll
-      for (int j = 0; j < NA; ++j) f[j][s] = wp[((size_t)j * KG + kg) * 256 + s * 64];
-      a[s] = *reinterpret_cast<const uint4*>(x + kg * 16 * M::EPL + s * M::EPL);
+      for (int u = 0; u < NU; ++u)
+#pragma unroll
+        for (int j = 0; j < NA; ++j) f[u][j][s] = (wp[u] + ((size_t)j * KG + kg) * 256 + s * 64)[(unsigned)lane];
+#pragma unroll
+      for (int t = 0; t < NP; ++t) a[t][s] = *reinterpret_cast<const uint4*>(x[t] + kg * 16 * M::EPL + s * M::EPL);
     }
 #pragma unroll
     for (int s = 0; s < 4; ++s)
 #pragma unroll
-      for (int j = 0; j < NA; ++j) acc[j] = M::mma(a[s], f[j][s], acc[j]);
+      for (int t = 0; t < NP; ++t)
+#pragma unroll
+        for (int u = 0; u < NU; ++u)
+#pragma unroll
+          for (int j = 0; j < NA; ++j) acc[t][u][j] = M::mma(a[t][s], f[u][j][s], acc[t][u][j]);
   }
 #pragma unroll
-  for (int j = 0; j < NA; ++j) *reinterpret_cast<f32x4*>(red[w][j][lane]) = acc[j];
+  for (int t = 0; t < NP; ++t)
+#pragma unroll
+    for (int u = 0; u < NU; ++u)
+#pragma unroll
+      for (int j = 0; j < NA; ++j) *reinterpret_cast<f32x4*>(red[w][t][u][j][lane]) = acc[t][u][j];
   __syncthreads();
-  // thread (lane, i = wave): pair 4 g + i, column rl
-  const int q = 4 * g + w;
-  if (q >= n) return;
-  float v[NA];
-#pragma unroll
-  for (int j = 0; j < NA; ++j) v[j] = (red[0][j][lane][w] + red[1][j][lane][w]) + (red[2][j][lane][w] + red[3][j][lane][w]);
-  const int pair = p.order[place + q];
+  // thread (lane, i = wave): pairs 16 t + 4 g + i, column rl
   T* y = reinterpret_cast<T*>(p.y);
-  if constexpr (DOWN) {
-    stv(y + (size_t)pair * p.ldy + unit * 16 + rl, v[0]);
-  } else {
-    const float s = p.wts[pair];
-    stv(y + (size_t)(place + q) * p.ldy + unit * 16 + rl, silu(s * v[0]) * (s * v[1]));
+#pragma unroll
+  for (int t = 0; t < NP; ++t) {
+    const int q = 16 * t + 4 * g + w;
+    if (q >= n) continue;
+    const int pair = p.order[place + q];
+    const float score = DOWN ? 1.f : p.wts[pair];
+    T* yr = y + (size_t)(DOWN ? pair : place + q) * p.ldy + unit0 * 16 + rl;
+#pragma unroll
+    for (int u = 0; u < NU; ++u) {
+      if (unit0 + u >= units) continue;
+      float v[NA];
+#pragma unroll
+      for (int j = 0; j < NA; ++j)
+        v[j] = (red[0][t][u][j][lane][w] + red[1][t][u][j][lane][w]) + (red[2][t][u][j][lane][w] + red[3][t][u][j][lane][w]);
+      if constexpr (DOWN) stv(yr + u * 16, v[0]);
+      else stv(yr + u * 16, silu(score * v[0]) * (score * v[1]));
+    }
   }
+}
+
+// (units: as many matrix tiles per row of x read, gate / up or down)
+template <class T, int NP>
+void launch_small(const MoeGemmParams& p, hipStream_t st) {
+  constexpr int NG = NP, ND = NP == 1 ? 1 : 2 * NP;
+  const int units = p.N / (p.down ? 16 : 32), nu = p.down ? ND : NG;
+  const dim3 grid((units + nu - 1) / nu, p.max_tiles), block(256);
+  if (p.down) hipLaunchKernelGGL((moe_small_kernel<T, true, NP, ND>), grid, block, 0, st, p);
+  else hipLaunchKernelGGL((moe_small_kernel<T, false, NP, NG>), grid, block, 0, st, p);
 }
 
 }  // namespace
@@ -210,11 +249,11 @@ extern "C" int vwa_moe_route(const MoeRouteParams* p, hipStream_t st) {
 }
 
 extern "C" int vwa_moe_gemm(const MoeGemmParams* p, hipStream_t st) {
-  if (p->max_tiles < 1 || p->N % (p->down ? 16 : 32) || p->K % 128 || p->ldx % 8 || (p->tile != 16 && p->tile != 128 && p->tile != 256) || !p->tiles || !p->order ||
+  if (p->max_tiles < 1 || p->N % (p->down ? 16 : 32) || p->K % 128 || p->ldx % 8 || (p->tile != 16 && p->tile != 32 && p->tile != 128 && p->tile != 256) || !p->tiles || !p->order ||
       (!p->down && !p->wts))
     return -1;
   if ((reinterpret_cast<uintptr_t>(p->x) | reinterpret_cast<uintptr_t>(p->w)) & 15) return -2;
-  if (p->tile > 16) {
+  if (p->tile > 32) {
     if (p->f32) return -3;
     GemmParams q{};
     q.X = reinterpret_cast<const uint16_t*>(p->x);
@@ -236,13 +275,7 @@ extern "C" int vwa_moe_gemm(const MoeGemmParams* p, hipStream_t st) {
     q.g_wstride = p->w_expert;
     return vwa_gemm_grouped(p->down ? 0 : 2, &q, st);
   }
-  const dim3 grid(p->N / (p->down ? 16 : 32), p->max_tiles), block(256);
-  if (p->f32) {
-    if (p->down) hipLaunchKernelGGL((moe_gemm16_kernel<float, true>), grid, block, 0, st, *p);
-    else hipLaunchKernelGGL((moe_gemm16_kernel<float, false>), grid, block, 0, st, *p);
-  } else {
-    if (p->down) hipLaunchKernelGGL((moe_gemm16_kernel<u16, true>), grid, block, 0, st, *p);
-    else hipLaunchKernelGGL((moe_gemm16_kernel<u16, false>), grid, block, 0, st, *p);
-  }
+  if (p->f32) p->tile == 16 ? launch_small<float, 1>(*p, st) : launch_small<float, 2>(*p, st);
+  else p->tile == 16 ? launch_small<u16, 1>(*p, st) : launch_small<u16, 2>(*p, st);
   return (int)hipGetLastError();
 }

@@ -392,7 +392,7 @@ def test_moe(dtype, E, top, ff, d, M, monkeypatch):
     slots = torch.zeros(M, dtype=torch.int64, device=DEV)
     inert = [t for t in (2, M - 1) if M > 4]
     slots[inert] = -1
-    for tile in [t for t in mixers.MOE_TILES if t == 16 or (dtype == BF16 and M >= 40)]:
+    for tile in [t for t in mixers.MOE_TILES if t <= 32 or (dtype == BF16 and M >= 40)]:
         monkeypatch.setattr(mixers, "moe_tile", lambda *_: tile)  # noqa: B023
         bufs = ops.moe_buffers(M, [(E, top, F)], dtype, DEV)
         for _ in range(2):  # (the tables are used again)

@@ -25,7 +25,7 @@ ATTN_KEYS = 64      # keys per round of the latent attention
 ATTN_GROUPS = 512   # workgroups a latent attention launch is cut into
 EXPAND_ROWS = 32    # runs of fewer rows attend in latent space ...
 EXPAND_CONTEXT = 128  # ... and so do runs behind more than this many tokens of context per row
-MOE_TILES = (16, 128, 256)  # pairs per tile of the experts' products: streaming kernel, the LDS-tiled GEMM's two tiles
+MOE_TILES = (16, 32, 128, 256)  # pairs per tile of the experts' products: streaming kernel, LDS-tiled GEMM
 
 
 # ----------------------------------------------------------------------------- weight layouts
@@ -235,10 +235,12 @@ def moe_tiles(pairs: int, E: int, tile: int) -> int:
 
 
 def moe_tile(rows: int, E: int, top: int, dtype) -> int:
-    """The tile size of a step: the LDS-tiled GEMM once its small tiles are a quarter full on average, its large
-    ones once an expert fills one."""
-    per = rows * top // E if dtype == torch.bfloat16 else 0
-    return MOE_TILES[2] if per >= 256 else MOE_TILES[1] if per >= 32 else MOE_TILES[0]
+    """The tile size of a step: the larger streaming tile where many experts would fill two small ones, the
+    LDS-tiled GEMM once its small tiles are a quarter full on average, its large ones once an expert fills one."""
+    per = rows * top / E
+    if dtype != torch.bfloat16 or per <= 8:
+        return 16
+    return 256 if per >= 256 else 128 if per >= 32 else 32
 
 
 def moe_buffers(rows: int, layers: Sequence[Tuple[int, int, int]], dtype, device) -> SimpleNamespace:
