@@ -18,13 +18,13 @@ namespace {
 constexpr size_t kMaxLds = 160 * 1024 - 8192;
 constexpr int kRouteWaves = 8, kRouteThreads = kRouteWaves * 64, kMaxExperts = 256;
 
-// pairs -> tiles of one expert each (the whole workgroup)
-VWA_DEVICE void group_pairs(const MoeRouteParams& p, const int* ids) {
+// pairs -> tiles of one expert each (the whole workgroup); id_of(pair): its expert
+template <class F>
+VWA_DEVICE void group_pairs(const MoeRouteParams& p, F&& id_of) {
   __shared__ int cnt[kMaxExperts], first[kMaxExperts], s_total;
   const int tid = threadIdx.x, P = p.rows * p.top;
   for (int e = tid; e < p.E; e += kRouteThreads) cnt[e] = 0;
   __syncthreads();
-  auto id_of = [&](int i) { return __hip_atomic_load(const_cast<int*>(ids) + i, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT); };
   constexpr int B = 8;                               // ids whose loads are in flight together
   auto for_pairs = [&](auto&& fn) {
     for (int i0 = tid; i0 < P; i0 += B * kRouteThreads) {
@@ -81,6 +81,7 @@ __global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(MoeRouteParams
   float* sc = red + kRouteWaves * Ep * 16;           // [16 rows][Ep + 1]
   const T* h = reinterpret_cast<const T*>(p.h) + (size_t)(r0 + min(rl, nr - 1)) * p.ldh + g * M::EPL;
   const uint4* wf = reinterpret_cast<const uint4*>(p.w) + lane;
+  const bool live = p.slots[r0 + min(tid >> 5, nr - 1)] >= 0;  // (of the row whose experts this thread chooses)
   for (int e = 0; e < et; ++e) {                     // D[expert 4 g + i][row rl], every wave a part of K
     f32x4 acc = {};
     for (int s0 = w; s0 < steps; s0 += 8 * kRouteWaves) {
@@ -105,8 +106,9 @@ __global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(MoeRouteParams
     for (int k = 0; k < kRouteWaves; ++k) z += red[k * Ep * 16 + i];
     sc[(i & 15) * (Ep + 1) + (i >> 4)] = (i >> 4) < p.E ? 1.f / (1.f + expf(-z)) : -2.f;
   }
+  int* lds_ids = reinterpret_cast<int*>(red);        // (a launch of one workgroup groups from here)
   __syncthreads();
-  const int r = tid >> 5, q = tid & 31, row = r0 + r;  // 32 lanes per row
+  const int r = tid >> 5, q = tid & 31, row = r0 + r;  // 32 lanes per row: the choices stay inside a wave
   for (int k = 0; k < p.top; ++k) {
     float best = -3.f;
     int at = 0;
@@ -127,12 +129,18 @@ __global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(MoeRouteParams
       }
     }
     if (q == 0 && r < nr) {
-      const bool live = p.slots[row] >= 0;
       sc[r * (Ep + 1) + at] = -1.f;                  // (taken; scores are positive)
       p.wts[row * p.top + k] = live ? best : 0.f;
+      lds_ids[r * p.top + k] = live ? at : -1;
       __hip_atomic_store(p.ids + row * p.top + k, live ? at : -1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
     }
-    __syncthreads();
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+  }
+  __syncthreads();
+  if (gridDim.x == 1) {
+    group_pairs(p, [&](int i) { return lds_ids[i]; });
+    return;
   }
   // ---- the last workgroup groups the pairs
   asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
@@ -145,7 +153,7 @@ __global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(MoeRouteParams
   __syncthreads();
   if (!s_last) return;
   __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
-  group_pairs(p, p.ids);
+  group_pairs(p, [&](int i) { return __hip_atomic_load(p.ids + i, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT); });
 }
 
 // ------------------------------------------------------------------------------------------ small tiles (16 NP pairs)
